@@ -9,7 +9,8 @@ Host decisions (which page, which slot) are made by the native allocator
 * per run with state, one float32 arena [max_seqs, elems], zeroed when a request opens.
 
 A request is `open()`ed into a slot, `reserve()`s pages as it grows (all groups or nothing),
-is `trim()`med after each step (windowed groups give back pages the window has passed) and
+is `trim()`med after each step (windowed groups give back pages the window has passed, but for a
+request's first positions that a group keeps readable) and
 `close()`d at its end.  Block table rows that changed are uploaded before a step by
 `sync_tables()`.  With `device=None` nothing is allocated on a device: the bookkeeping alone,
 for tests and planning.
@@ -49,7 +50,7 @@ def host_lib():
         lib = ctypes.CDLL(build.build_host())
         IP, LP, I64P = POINTER(c_int), POINTER(c_long), POINTER(ctypes.c_int64)
         sig = {
-            "axh_cache_create": (c_void_p, [c_int, IP, IP, IP, c_int, c_int, c_long]),
+            "axh_cache_create": (c_void_p, [c_int, IP, IP, IP, IP, c_int, c_int, c_long]),
             "axh_cache_destroy": (None, [c_void_p]),
             "axh_cache_error": (c_char_p, [c_void_p]),
             "axh_cache_open": (c_int, [c_void_p]),
@@ -63,7 +64,7 @@ def host_lib():
             "axh_cache_pages_of": (c_int, [c_void_p, c_int, c_int]),
             "axh_cache_length": (c_long, [c_void_p, c_int]),
             "axh_cache_check": (c_int, [c_void_p]),
-            "axh_sched_create": (c_void_p, [c_int, IP, IP, IP, c_int, c_int, c_long]),
+            "axh_sched_create": (c_void_p, [c_int, IP, IP, IP, IP, c_int, c_int, c_long]),
             "axh_sched_destroy": (None, [c_void_p]),
             "axh_sched_error": (c_char_p, [c_void_p]),
             "axh_sched_add": (c_int, [c_void_p, ctypes.c_int64, c_long, c_long]),
@@ -150,8 +151,8 @@ class CacheManager:
         n = len(groups)
         arr = lambda vals: (c_int * max(n, 1))(*vals)
         self._h = self.lib.axh_cache_create(n, arr([g.n_pages for g in groups]), arr([g.page_size for g in groups]),
-                                            arr([g.spec.window for g in groups]), max_seqs, self.max_pages_per_seq,
-                                            shuffle_seed)
+                                            arr([g.spec.window for g in groups]), arr([g.spec.keep for g in groups]), max_seqs,
+                                            self.max_pages_per_seq, shuffle_seed)
         if not self._h:
             raise CacheError(f"bad cache geometry: {[(g.n_pages, g.page_size, g.spec.window) for g in groups]}")
         self.plans = list(groups)

@@ -203,7 +203,7 @@ def run_info(args) -> int:
     plan = model.cache_plan
     for s, layers in zip(plan.group_specs, plan.group_layers):
         print(f"cache group: {layers} layers x {s.entries} x {s.heads} heads x {s.head_dim}"
-              + (f", window {s.window}" if s.window else ""))
+              + (f", window {s.window}" if s.window else "") + (f", the first {s.keep} kept" if s.keep else ""))
     return 0
 
 

@@ -155,6 +155,14 @@ class ModelConfig:
     def with_vocab(self, vocab_size: int) -> "ModelConfig":
         raise NotImplementedError
 
+    def size_tensors(self) -> List[str]:
+        """Tensors whose shapes give sizes that config.json does not (the loader then calls
+        `with_sizes` with the shapes of those the checkpoint has)."""
+        return []
+
+    def with_sizes(self, shapes: Dict[str, tuple]) -> "ModelConfig":
+        raise NotImplementedError
+
     def ignores_tensor(self, name: str) -> bool:
         """Tensors a checkpoint may hold that the model does not read (tables that are
         recomputed, say): they are neither unexpected nor loaded."""

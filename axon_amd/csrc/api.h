@@ -221,6 +221,14 @@ int axk_round_rows(const float* x, void* out, long n, void* stream);
 int axk_concat_round(const float* a, int wa, const float* b, int wb, void* out, int n_rows, void* stream);
 // In place on elem values; kind 0: the tanh form of GELU; kind 1: the exact (erf) GELU.
 int axk_activation(void* v, long n, int kind, void* stream);
+// A norm without statistics, n(x) = tanh(alpha x) w + b.  axk_tanh_norm: out elem [n_rows, dim] = n of the rows
+// x[rows[r]] (rows null: of row r).  axk_tanh_norm_add: x += n(y) (both float32), and next elem = the next norm of the
+// new x (next null: none).
+int axk_tanh_norm(const float* x, const int32_t* rows, float alpha, const void* w, int w_is_f32, const void* b, int b_is_f32,
+                  void* out, int n_rows, int dim, void* stream);
+int axk_tanh_norm_add(const float* y, float alpha, const void* w, int w_is_f32, const void* b, int b_is_f32, float* x, void* next,
+                      float next_alpha, const void* next_w, int next_w_is_f32, const void* next_b, int next_b_is_f32, int n_rows,
+                      int dim, void* stream);
 // out[t, f] = g sigmoid(alpha g) (u + 1), g = min(gate_up[t, f], limit), u = clamp(gate_up[t, F + f], -limit, limit).
 int axk_clamped_glu(const void* gate_up, void* out, int n_tokens, int n_ffn, float limit, float alpha, void* stream);
 
@@ -249,27 +257,30 @@ int axk_grouped_gemm(const void* x, int x_is_f32, long x_row_stride, long x_grou
 
 // Routing (csrc/moe.hip).  axk_route_topk: for each token the `top` largest of its n_experts
 // logits (the largest first; of equal ones the lower expert) and the softmax over these.
-// axk_route_scored: scores s = sigmoid(logits) that do not compete; chosen by s + correction (float32
+// axk_route_scored: scores s = sigmoid(logits) that do not compete, or with `softmax` the softmax over all
+// n_experts; chosen by s + correction (float32
 // [n_experts], or null) among the experts of the `keep` best of `groups` equal groups of neighbours (a
 // group's score: the sum of its two largest choice scores), weights s / (sum of the chosen s + 1e-20)
 // * scale (without `normalize`: s * scale); rows of logits are logits_stride apart.  Up to 1,024 experts in up to
 // 64 groups, up to 64 a token.
 // axk_route_sort: the pairs p = t top + k in expert order (sorted, and each one's token in
 // sorted_tokens) and the tiles (of up to tile_rows rows) of the grouped product, at most
-// axk_route_max_tiles of them.
+// axk_route_max_tiles of them; pairs of experts from n_experts on (identities) are not listed.
 // place_of [n_pairs] (or null): where each pair stands in `sorted`; first_of [n_experts + 1] (or
 // null): where each expert's pairs start there.
 // axk_route_combine: y[t, :] (+)= sum_k weights[t, k] rows[t top + k, :], k ascending (with
 // place_of: rows[place_of[t top + k], :]); weights may be null (all 1); extra (float32 [n_tokens, width], or null) is
-// a further row a token, times sigmoid(extra_gate[t extra_gate_stride]) if extra_gate is given.  axk_gather_rows: out[r, :] = x[rows[r], :] (elem).
+// a further row a token, times sigmoid(extra_gate[t extra_gate_stride]) if extra_gate is given; input (elem rows, or
+// null): the row of a pair whose expert (experts[pair]) is n_experts or more is input[t, :].  axk_gather_rows: out[r, :] = x[rows[r], :] (elem).
 int axk_route_topk(const float* logits, int n_tokens, int n_experts, int top, int32_t* experts, float* weights, void* stream);
 int axk_route_scored(const float* logits, long logits_stride, const float* correction, int n_tokens, int n_experts, int top,
-                     int groups, int keep, float scale, int normalize, int32_t* experts, float* weights, void* stream);
+                     int groups, int keep, float scale, int normalize, int softmax, int32_t* experts, float* weights, void* stream);
 int axk_route_max_tiles(int n_pairs, int n_experts, int tile_rows);
 int axk_route_sort(const int32_t* experts, int n_pairs, int n_experts, int top, int32_t* sorted, int32_t* sorted_tokens,
                    int32_t* tiles, int32_t* n_tiles, int32_t* place_of, int32_t* first_of, int tile_rows, void* stream);
 int axk_route_combine(const float* rows, const float* weights, float* y, int n_tokens, int top, int width, int accumulate,
-                      const int32_t* place_of, const float* extra, const float* extra_gate, long extra_gate_stride, void* stream);
+                      const int32_t* place_of, const float* extra, const float* extra_gate, long extra_gate_stride, const int32_t* experts,
+                      int n_experts, const void* input, long input_stride, void* stream);
 int axk_gather_rows(const void* x, long x_stride, const int32_t* rows, void* out, int n_rows, int width, void* stream);
 
 // A short causal convolution per channel and a gated linear recurrence (csrc/recurrent.hip).  A
@@ -322,6 +333,49 @@ int axk_state_space_scan(const float* u, const float* terms, const void* d_skip,
 int axk_gated_group_norm(const float* y, const float* z, long z_stride, const void* gain, int gain_is_f32, float eps, void* out,
                          int n_tokens, int width, int parts, void* stream);
 
+// Time mixing with a state matrix a head (csrc/time_mix.hip).  A request's state row (float32, rows state_stride apart)
+// holds two copies of copy_elems floats: the heads' states [heads][P][N], and from tail_at its last row of the mixer's
+// input; the state behind position p is in copy p & 1.
+// axk_token_shift: out elem [n_mix, n_tokens, width], out[s, t] = h[t] + (h'[t] - h[t]) mu[s], h' the request's row
+// before (from the state where the step does not hold it).  Reads the state only.
+// axk_time_mix_decay: w[t, c] = exp(-exp(w0[c] + sum_k w2[c, k] tanh(low[t, k]))), float32; w2 elem [channels, rank].
+// axk_wkv_scan: per request of the step (spans, as below) and head, over its tokens in order,
+// y_t = (S + diag(u) k v^T)^T r, S = diag(w) S + k v^T; r, k [T, heads N] and v [T, heads P] are float32 columns of rows
+// `stride` apart, w [T, heads N], u [heads, N], y [T, heads P] float32; then the state row is brought up to date (S, and
+// the last row of h_in).  segs, spans5 as in axk_state_space_scan, with ends float32 [n_segs, heads, P, N], decays float32
+// [n_segs, heads, N] and rc float32 [T, heads N]: segments side by side, folded (sums in another order, by rounding).
+int axk_token_shift(const void* h, const float* mu, int n_mix, const float* state, long state_stride, long copy_elems,
+                    long tail_at, const int32_t* positions, const int32_t* seq_rows, void* out, int n_tokens, int width,
+                    void* stream);
+int axk_time_mix_decay(const float* low, const void* w2, const void* w0, int w0_is_f32, float* w, int n_tokens, int channels,
+                       int rank, void* stream);
+int axk_wkv_scan(const float* rows, long stride, long r_at, long k_at, long v_at, const float* w, const float* u, float* state,
+                 long state_stride, long copy_elems, long tail_at, const int32_t* spans, int n_spans, const int32_t* positions,
+                 const int32_t* seq_rows, const void* h_in, int width, float* y, int heads, int N, int P, const int32_t* segs,
+                 int n_segs, int longest_seg, const int32_t* spans5, float* ends, float* decays, float* rc, void* stream);
+
+// The gated delta rule (csrc/delta_rule.hip).  A copy of the state row: the heads' states [heads][P][N], then from
+// tail_at [taps - 1][channels] of the convolutions' last inputs, oldest first; channels = [q: kv_heads N | k: kv_heads N |
+// v: heads P].
+// axk_delta_prepare: from the float32 rows of the projections (the channels first, the heads' logits of beta from
+// beta_at and of the decay from decay_at) u [T, channels], convolved, through silu, queries and keys of length 1 a head
+// (x / sqrt(sum x^2 + 1e-6)), queries times q_scale; terms [T, heads, 2] = (g, beta), g = exp(-exp(a_log) softplus(. +
+// dt_bias)), beta = sigmoid(.).  Reads the state only.
+// axk_delta_scan: per request of the step (spans [n][3] = (slot, first token, tokens); null: each token a request of its
+// own in slot seq_rows[t]) and head, over its tokens in order, S = g S, c = beta (v - S^T k), S = S + k c^T, y = S^T q;
+// then the state row is brought up to date (S, and the convolutions' inputs from conv_in, rows conv_in_stride apart).
+// axk_head_norm_gate: out elem [T, heads P] = (y / sqrt(mean y^2 + eps)) gain silu(gate), the mean over a head's P; gain
+// of P numbers, or with gain_per_head of heads P.
+int axk_delta_prepare(const float* in, long in_stride, const void* w, int taps, const float* state, long state_stride,
+                      long copy_elems, long tail_at, const int32_t* positions, const int32_t* seq_rows, int beta_at, int decay_at,
+                      const void* a_log, int a_log_is_f32, const void* dt_bias, int dt_bias_is_f32, float* u, float* terms,
+                      int n_tokens, int heads, int kv_heads, int N, int P, float q_scale, void* stream);
+int axk_delta_scan(const float* u, const float* terms, float* state, long state_stride, long copy_elems, long tail_at,
+                   const int32_t* spans, int n_spans, const int32_t* positions, const int32_t* seq_rows, const float* conv_in,
+                   long conv_in_stride, float* y, int heads, int kv_heads, int N, int P, int taps, void* stream);
+int axk_head_norm_gate(const float* y, const float* gate, long gate_stride, const void* gain, int gain_is_f32, int gain_per_head,
+                       float eps, void* out, int n_tokens, int heads, int P, void* stream);
+
 // Attention over a latent cache (csrc/latent_attention.hip); a page is [page_size][rank + rot] elem
 // (the latent and the rotated key part of each position), then [rank][page_size] (the latents again,
 // the positions of one dim side by side): 2 rank + rot elements a position.
@@ -358,17 +412,19 @@ int axk_latent_attention(const float* q_full, const void* cache, const int32_t* 
 // norm), the first `rot` dims rotated by table [T, rot / 2, 2] (sin, cos; both scaled by `magnitude`) in
 // pairs (2i, 2i + 1) if `neighbours` else (i, i + rot / 2); queries into q_out elem [T, n_q dim], keys and
 // values into the page (if write_kv).  q_temp_every > 0: a query at position p is multiplied by
-// 1 + q_temp_coef ln(floor((p + 1) / q_temp_every) + 1).
+// 1 + q_temp_coef ln(floor((p + 1) / q_temp_every) + 1).  norm_rows: the norm goes over all query units (all key
+// units) of a token at once, its gains hold n_q dim (n_k dim) numbers.  Without write_kv the key and value columns
+// need not be there.
 int axk_heads_prepare(const float* proj, long stride, int q_at, int n_q, int k_at, int n_k, int v_at, int v_width, int dim,
                       const void* q_gain, int q_gain_is_f32, const void* k_gain, int k_gain_is_f32, float eps, int rot,
                       int neighbours, float magnitude, const float* table, const int32_t* positions, const int32_t* seq_rows,
                       const int32_t* block_table, int table_stride, void* cache, int page_size, void* q_out, int n_tokens,
-                      int write_kv, float q_temp_coef, int q_temp_every, void* stream);
+                      int write_kv, float q_temp_coef, int q_temp_every, int norm_rows, void* stream);
 // axk_masked_attention: q elem [T, heads maps dim] -> out elem [T, heads vdim].  mask_kind 0: all earlier
-// positions; 1: the last mask_size positions; 2: the earlier positions of the same chunk of mask_size.
+// positions; 1: the last mask_size positions and, whatever their distance, the first `keep`; 2: the earlier positions of the same chunk of mask_size.
 // softcap > 0: s <- softcap tanh(s / softcap).  maps 2: o = rms(a_1 - lambda a_2, eps) out_scale.  gate
 // (float32 rows of gate_stride, or null): o *= sigmoid(gate), heads vdim numbers a row, or with gate_per_head
-// one a head.  sink > -inf: the softmax's sum also holds exp(sink), a key of that score without a value.  tiles (int32 [n_tiles, 2]: first token,
+// one a head.  sink > -inf: the softmax's sum also holds exp(sink), a key of that score without a value; sinks (float32 [heads], or null): one a head instead.  tiles (int32 [n_tiles, 2]: first token,
 // count; up to 16 consecutive tokens of one request each) or null (every token a tile of its own) are
 // what the matrix-core kernel works on where axk_masked_attention_uses_mfma says 1.
 // partial: axk_masked_attention_workspace floats (steps of few tokens: the blocks of 64 positions of a single token
@@ -376,13 +432,13 @@ int axk_heads_prepare(const float* proj, long stride, int q_at, int n_q, int k_a
 // the step's longest row sees, make: 0 there means no such split), or null.
 int axk_masked_attention_uses_mfma(int heads, int kv_heads, int maps, int dim, int vdim, int page_size);
 long axk_masked_attention_workspace(int n_tokens, int heads, int kv_heads, int maps, int dim, int vdim, int page_size,
-                                    int mask_kind, int mask_size, int span);
+                                    int mask_kind, int mask_size, int keep, int span);
 int axk_masked_attention(const void* q, const void* cache, const int32_t* block_table, int table_stride,
                          const int32_t* positions, const int32_t* seq_rows, const float* gate, long gate_stride, void* out,
                          int n_tokens, int heads, int kv_heads, int maps, int dim, int vdim, int page_size, int mask_kind,
                          int mask_size, float scale, float softcap, float lambda, float out_scale, float eps,
-                         const int32_t* tiles, int n_tiles, float* partial, long partial_floats, float sink, int gate_per_head,
-                         int span, void* stream);
+                         const int32_t* tiles, int n_tiles, float* partial, long partial_floats, float sink, const float* sinks,
+                         int gate_per_head, int keep, int span, void* stream);
 
 #ifdef __cplusplus
 }

@@ -1,0 +1,255 @@
+// The gated delta rule (the linear attention of Gated-DeltaNet-like models): per request and head a state matrix
+// S [N, P] that each token decays, corrects along its key and reads,
+//
+//   S <- g_t S,  u = beta_t (v_t - S^T k_t),  S <- S + k_t u^T,  o_t = S^T q_t,
+//
+// behind short causal convolutions with silu over the channels [q | k | v], queries and keys of length 1 a head.
+// Head a reads query and key head a / (heads / kv_heads).  Everything here is 32-bit in both builds but the
+// convolutions' weights as stored.
+//
+// A copy of the state row (see recurrence.h) holds the heads' states [heads][P][N], then [taps - 1][channels] of the
+// convolutions' last inputs, oldest first (zeros for a new request, which is what they read before the first token).
+#include "api.h"
+#include "recurrence.h"
+
+namespace {
+
+// A wave a unit of a token: a query or key head (convolution, silu, length 1; queries also times N^(-1/2)), a value
+// head (convolution, silu), or the token's step sizes, terms[t, a] = (g, beta) with
+// g = exp(-exp(A_log_a) softplus(decay_in_a + dt_bias_a)), beta = sigmoid(beta_in_a).  in [T, in_stride]: the
+// projections' rows, [q: kv_heads N | k: kv_heads N | v: heads P] first.
+#define DP_KEPT 4        // channels of a query or key head a lane holds: N up to 256
+__global__ void __launch_bounds__(256)
+delta_prepare_kernel(const float* __restrict__ in, long in_stride, const elem_t* __restrict__ w, int taps,
+                     const float* __restrict__ state, long state_stride, long copy_elems, long tail_at,
+                     const int32_t* __restrict__ positions, const int32_t* __restrict__ seq_rows, int beta_at, int decay_at,
+                     const void* __restrict__ a_log, int a_log_is_f32, const void* __restrict__ dt_bias, int dt_bias_is_f32,
+                     float* __restrict__ u, float* __restrict__ terms, int heads, int kv_heads, int N, int P, float q_scale) {
+  const int t = blockIdx.x, unit = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const float* row = in + (long)t * in_stride;
+  if (unit > 2 * kv_heads + heads) return;
+  if (unit == 2 * kv_heads + heads) {
+    for (int a = lane; a < heads; a += 64) {
+      const float step = rec_softplus(row[decay_at + a] + load_vec(dt_bias, dt_bias_is_f32, a));
+      terms[((long)t * heads + a) * 2] = expf(-(expf(load_vec(a_log, a_log_is_f32, a)) * step));
+      terms[((long)t * heads + a) * 2 + 1] = rec_sigmoid(row[beta_at + a]);
+    }
+    return;
+  }
+  const int channels = 2 * kv_heads * N + heads * P;
+  const bool is_v = unit >= 2 * kv_heads;
+  const int c0 = is_v ? 2 * kv_heads * N + (unit - 2 * kv_heads) * P : unit * N, size = is_v ? P : N;
+  const int inside = rec_inside(seq_rows, t, taps - 1);
+  const float* kept = rec_copy_before(state, state_stride, copy_elems, seq_rows[t], positions[t] - inside) + tail_at;
+  auto conv = [&](int c) {
+    float acc = 0.0f;
+    for (int k = 0; k < taps; ++k) {
+      const int back = taps - 1 - k;            // the input `back` tokens before this one
+      const float v = back <= inside ? row[c - (long)back * in_stride]
+                                     : kept[(long)(taps - 1 - (back - inside)) * channels + c];
+      acc = fmaf(to_float(w[(long)c * taps + k]), v, acc);
+    }
+    return rec_silu(acc);
+  };
+  float* dst = u + (long)t * channels;
+  if (is_v) {
+    for (int i = lane; i < size; i += 64) dst[c0 + i] = conv(c0 + i);
+    return;
+  }
+  float v[DP_KEPT], ss = 0.0f;
+#pragma unroll
+  for (int j = 0; j < DP_KEPT; ++j) {
+    v[j] = lane + 64 * j < size ? conv(c0 + lane + 64 * j) : 0.0f;
+    ss = fmaf(v[j], v[j], ss);
+  }
+  const float inv = (1.0f / sqrtf(wave_sum(ss) + 1e-6f)) * (unit < kv_heads ? q_scale : 1.0f);
+#pragma unroll
+  for (int j = 0; j < DP_KEPT; ++j)
+    if (lane + 64 * j < size) dst[c0 + lane + 64 * j] = v[j] * inv;
+}
+
+// The walk.  grid (requests of the step, heads, blocks of value dims); LK lanes share a value dim, OWN rows of the
+// state a lane.  With a = S^T k and b = S^T q of the state as the token finds it, u = beta (v - g a) and the read-out
+// behind the token's write is o = g b + (k . q) u: both sums leave for the lanes' permutations together.  The operands
+// of AHEAD tokens are asked for while those before them are worked on.
+template <int OWN, int AHEAD>
+struct DeltaOperands {
+  float q[AHEAD][OWN], k[AHEAD][OWN], v[AHEAD], g[AHEAD], beta[AHEAD];
+};
+
+template <int LK, int OWN, bool VEC>
+__global__ void __launch_bounds__(REC_THREADS)
+delta_scan_kernel(const float* __restrict__ u, const float* __restrict__ terms, float* __restrict__ state, long state_stride,
+                  long copy_elems, long tail_at, const int32_t* __restrict__ spans, const int32_t* __restrict__ positions,
+                  const int32_t* __restrict__ seq_rows, const float* __restrict__ conv_in, long conv_in_stride,
+                  float* __restrict__ y, int heads, int kv_heads, int N, int P, int taps) {
+  constexpr int AHEAD = OWN >= 16 ? 2 : 4;
+  const RecStretch s = rec_stretch(nullptr, spans, seq_rows, blockIdx.x);
+  const int h = blockIdx.y, g = h / (heads / kv_heads), ns = threadIdx.x % LK, n0 = ns * OWN;
+  const int p = blockIdx.z * (REC_THREADS / LK) + threadIdx.x / LK;
+  const bool has_p = p < P;
+  const int start = positions[s.first];
+  const float* from = rec_copy_before(state, state_stride, copy_elems, s.slot, start);
+  float* to = rec_copy_behind(state, state_stride, copy_elems, s.slot, start + s.count - 1);
+  const long s_at = (long)h * N * P + (long)p * N;
+  float S[OWN];
+  if (has_p) rec_load<OWN, VEC>(S, from + s_at, n0, N);
+  else {
+#pragma unroll
+    for (int i = 0; i < OWN; ++i) S[i] = 0.0f;
+  }
+  const int channels = 2 * kv_heads * N + heads * P, last = s.first + s.count;
+  const long q_col = (long)g * N, k_col = (long)(kv_heads + g) * N, v_col = 2L * kv_heads * N + (long)h * P + (has_p ? p : 0);
+  typedef DeltaOperands<OWN, AHEAD> Ops;
+  auto fetch = [&](Ops& o, int t0) {
+#pragma unroll
+    for (int a = 0; a < AHEAD; ++a) {
+      const int t = min(t0 + a, last - 1);             // behind the last token: the last again, not used
+      const float* row = u + (long)t * channels;
+      rec_load<OWN, VEC>(o.q[a], row + q_col, n0, N);
+      rec_load<OWN, VEC>(o.k[a], row + k_col, n0, N);
+      o.v[a] = row[v_col];
+      o.g[a] = terms[((long)t * heads + h) * 2];
+      o.beta[a] = terms[((long)t * heads + h) * 2 + 1];
+    }
+  };
+  auto work = [&](const Ops& o, int t0) {
+#pragma unroll
+    for (int a = 0; a < AHEAD; ++a) {
+      if (t0 + a >= last) break;
+      float sk = 0.0f, sq = 0.0f, kq = 0.0f;
+#pragma unroll
+      for (int i = 0; i < OWN; ++i) {
+        sk = fmaf(S[i], o.k[a][i], sk);
+        sq = fmaf(S[i], o.q[a][i], sq);
+        kq = fmaf(o.k[a][i], o.q[a][i], kq);
+      }
+      sk = rec_row_sum<LK>(sk);
+      sq = rec_row_sum<LK>(sq);
+      kq = rec_row_sum<LK>(kq);
+      const float c = o.beta[a] * (o.v[a] - o.g[a] * sk);
+#pragma unroll
+      for (int i = 0; i < OWN; ++i) S[i] = fmaf(o.k[a][i], c, o.g[a] * S[i]);
+      if (ns == 0 && has_p) y[((long)(t0 + a) * heads + h) * P + p] = fmaf(kq, c, o.g[a] * sq);
+    }
+  };
+  Ops even, odd;
+  fetch(even, s.first);
+  for (int t = s.first; t < last; t += 2 * AHEAD) {
+    if (t + AHEAD < last) fetch(odd, t + AHEAD);
+    work(even, t);
+    if (t + AHEAD >= last) break;
+    if (t + 2 * AHEAD < last) fetch(even, t + 2 * AHEAD);
+    work(odd, t + AHEAD);
+  }
+  if (has_p) rec_store<OWN, VEC>(to + s_at, S, n0, N);
+  if (blockIdx.y != 0 || blockIdx.z != 0) return;
+  // the convolutions' last taps - 1 inputs: of (what was kept, this step's inputs) the last taps - 1; place i takes
+  // what lies `count` places later (where both copies are one: read before it is written, ascending)
+  float* kept = to + tail_at;
+  const float* kept_from = from + tail_at;
+  for (int c = threadIdx.x; c < channels; c += REC_THREADS)
+    for (int i = 0; i < taps - 1; ++i) {
+      const int at = i + s.count;
+      kept[(long)i * channels + c] = at < taps - 1 ? kept_from[(long)at * channels + c]
+                                                   : conv_in[(long)(s.first + at - (taps - 1)) * conv_in_stride + c];
+    }
+}
+
+// out[t, a] = (y[t, a] / sqrt(mean(y[t, a]^2) + eps)) gain silu(gate[t, a]) head by head; the gain holds P numbers
+// shared by the heads, or one for every channel (gain_per_head).  A wave a (token, head).
+#define HN_KEPT 4
+__global__ void __launch_bounds__(256)
+head_norm_gate_kernel(const float* __restrict__ y, const float* __restrict__ gate, long gate_stride, const void* __restrict__ gain,
+                      int gain_is_f32, int gain_per_head, float eps, elem_t* __restrict__ out, long items, int heads, int P) {
+  const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= items) return;
+  const int lane = threadIdx.x & 63, h = (int)(item % heads);
+  const long t = item / heads;
+  const float* src = y + item * P;
+  const float* g = gate + t * gate_stride + (long)h * P;
+  elem_t* dst = out + item * P;
+  const int gain_at = gain_per_head ? h * P : 0;
+  float kept[HN_KEPT], ss = 0.0f;
+#pragma unroll
+  for (int j = 0; j < HN_KEPT; ++j) {
+    kept[j] = lane + 64 * j < P ? src[lane + 64 * j] : 0.0f;
+    ss = fmaf(kept[j], kept[j], ss);
+  }
+  for (int i = lane + 64 * HN_KEPT; i < P; i += 64) ss = fmaf(src[i], src[i], ss);
+  const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)P + eps);
+#pragma unroll
+  for (int j = 0; j < HN_KEPT; ++j) {
+    const int i = lane + 64 * j;
+    if (i < P) dst[i] = from_float(((kept[j] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * rec_silu(g[i]));
+  }
+  for (int i = lane + 64 * HN_KEPT; i < P; i += 64)
+    dst[i] = from_float(((src[i] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * rec_silu(g[i]));
+}
+
+}  // namespace
+
+extern "C" int axk_delta_prepare(const float* in, long in_stride, const void* w, int taps, const float* state, long state_stride,
+                                 long copy_elems, long tail_at, const int32_t* positions, const int32_t* seq_rows, int beta_at,
+                                 int decay_at, const void* a_log, int a_log_is_f32, const void* dt_bias, int dt_bias_is_f32, float* u,
+                                 float* terms, int n_tokens, int heads, int kv_heads, int N, int P, float q_scale, void* stream) {
+  AXK_REQUIRE(n_tokens >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && N > 0 && N <= 256 && P > 0 && taps >= 1,
+              "delta_prepare: bad sizes T=%d heads=%d kv heads=%d keys=%d (at most 256) values=%d taps=%d", n_tokens, heads, kv_heads,
+              N, P, taps);
+  const long channels = 2L * kv_heads * N + (long)heads * P;
+  AXK_REQUIRE(in_stride >= channels && beta_at >= 0 && decay_at >= 0 && beta_at + heads <= in_stride && decay_at + heads <= in_stride,
+              "delta_prepare: the parts do not fit rows of %ld", in_stride);
+  AXK_REQUIRE(tail_at >= 0 && copy_elems >= tail_at + (taps - 1) * channels && state_stride >= 2 * copy_elems,
+              "delta_prepare: a state row of %ld floats does not hold two copies of %ld with %d x %ld kept inputs from %ld",
+              state_stride, copy_elems, taps - 1, channels, tail_at);
+  if (n_tokens == 0) return 0;
+  delta_prepare_kernel<<<dim3(n_tokens, ceil_div(2 * kv_heads + heads + 1, 4)), 256, 0, (hipStream_t)stream>>>(
+      in, in_stride, (const elem_t*)w, taps, state, state_stride, copy_elems, tail_at, positions, seq_rows, beta_at, decay_at, a_log,
+      a_log_is_f32, dt_bias, dt_bias_is_f32, u, terms, heads, kv_heads, N, P, q_scale);
+  AXK_LAUNCH_CHECK("delta_prepare");
+  return 0;
+}
+
+extern "C" int axk_delta_scan(const float* u, const float* terms, float* state, long state_stride, long copy_elems, long tail_at,
+                              const int32_t* spans, int n_spans, const int32_t* positions, const int32_t* seq_rows,
+                              const float* conv_in, long conv_in_stride, float* y, int heads, int kv_heads, int N, int P, int taps,
+                              void* stream) {
+  AXK_REQUIRE(n_spans >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && N > 0 && N <= 256 && P > 0 && taps >= 1,
+              "delta_scan: bad sizes spans=%d heads=%d kv heads=%d keys=%d (at most 256) values=%d taps=%d", n_spans, heads, kv_heads,
+              N, P, taps);
+  const long channels = 2L * kv_heads * N + (long)heads * P;
+  AXK_REQUIRE(tail_at >= (long)heads * N * P && copy_elems >= tail_at + (taps - 1) * channels && state_stride >= 2 * copy_elems &&
+              conv_in_stride >= channels,
+              "delta_scan: a state row of %ld floats does not hold two copies of %ld (%d x %d x %d, then %d x %ld from %ld)", state_stride,
+              copy_elems, heads, N, P, taps - 1, channels, tail_at);
+  AXK_REQUIRE((spans != nullptr || seq_rows != nullptr) && positions != nullptr, "delta_scan: neither spans nor slots, or no positions");
+  if (n_spans == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  const bool vec = N % 4 == 0 && channels % 4 == 0 && copy_elems % 4 == 0 && state_stride % 4 == 0 && ((uintptr_t)u & 15) == 0 &&
+                   ((uintptr_t)state & 15) == 0;
+#define DELTA_ARGS u, terms, state, state_stride, copy_elems, tail_at, spans, positions, seq_rows, conv_in, conv_in_stride, y, heads, \
+                   kv_heads, N, P, taps
+#define DELTA_LAUNCH(LK, OWN)                                                                    \
+  {                                                                                              \
+    const dim3 grid(n_spans, heads, ceil_div(P, REC_THREADS / LK));                              \
+    if (vec) delta_scan_kernel<LK, OWN, true><<<grid, REC_THREADS, 0, s>>>(DELTA_ARGS);          \
+    else delta_scan_kernel<LK, OWN, false><<<grid, REC_THREADS, 0, s>>>(DELTA_ARGS);             \
+  }
+  REC_BY_ROWS(N, DELTA_LAUNCH)
+#undef DELTA_LAUNCH
+#undef DELTA_ARGS
+  AXK_LAUNCH_CHECK("delta_scan");
+  return 0;
+}
+
+extern "C" int axk_head_norm_gate(const float* y, const float* gate, long gate_stride, const void* gain, int gain_is_f32,
+                                  int gain_per_head, float eps, void* out, int n_tokens, int heads, int P, void* stream) {
+  AXK_REQUIRE(n_tokens >= 0 && heads > 0 && P > 0 && gate_stride >= (long)heads * P,
+              "head_norm_gate: bad sizes T=%d heads=%d values=%d gate rows of %ld", n_tokens, heads, P, gate_stride);
+  if (n_tokens == 0) return 0;
+  const long items = (long)n_tokens * heads;
+  head_norm_gate_kernel<<<(unsigned)((items + 3) / 4), 256, 0, (hipStream_t)stream>>>(y, gate, gate_stride, gain, gain_is_f32,
+                                                                                     gain_per_head, eps, (elem_t*)out, items, heads, P);
+  AXK_LAUNCH_CHECK("head_norm_gate");
+  return 0;
+}

@@ -318,6 +318,92 @@ extern "C" int axk_layernorm(const float* x, const int32_t* rows, const void* ga
   return 0;
 }
 
+// ---------------------------------------------------------------------------- dynamic tanh
+// A norm without statistics: n(x) = tanh(alpha x) w + b, element by element, alpha one number a norm.
+// tanh_norm: out[r] = n(x[rows[r]]) in the compute dtype.  tanh_norm_add: x[r] += n(y[r]) and, if asked for,
+// next[r] = n'(the new x[r]) in the compute dtype, the norm that the sum goes into.  Four elements a thread where the
+// width is a multiple of 4 (VEC).
+__device__ inline float tanh_norm1(float x, float alpha, const void* w, int w_is_f32, const void* b, int b_is_f32, int i) {
+  return fmaf(tanhf(alpha * x), load_vec(w, w_is_f32, i), load_vec(b, b_is_f32, i));
+}
+
+template <bool VEC>
+__global__ void __launch_bounds__(NORM_THREADS)
+tanh_norm_kernel(const float* __restrict__ x, const int32_t* __restrict__ rows, float alpha, const void* __restrict__ w, int w_is_f32,
+                 const void* __restrict__ b, int b_is_f32, elem_t* __restrict__ out, int dim) {
+  const int r = blockIdx.x;
+  const float* src = x + (size_t)(rows ? rows[r] : r) * dim;
+  elem_t* dst = out + (size_t)r * dim;
+  if (VEC) {
+    const int e = 4 * (blockIdx.y * NORM_THREADS + threadIdx.x);
+    if (e >= dim) return;
+    const float4 v = *reinterpret_cast<const float4*>(src + e);
+    store4(dst + e, tanh_norm1(v.x, alpha, w, w_is_f32, b, b_is_f32, e), tanh_norm1(v.y, alpha, w, w_is_f32, b, b_is_f32, e + 1),
+           tanh_norm1(v.z, alpha, w, w_is_f32, b, b_is_f32, e + 2), tanh_norm1(v.w, alpha, w, w_is_f32, b, b_is_f32, e + 3));
+    return;
+  }
+  for (int i = threadIdx.x; i < dim; i += NORM_THREADS) dst[i] = from_float(tanh_norm1(src[i], alpha, w, w_is_f32, b, b_is_f32, i));
+}
+
+template <bool VEC>
+__global__ void __launch_bounds__(NORM_THREADS)
+tanh_norm_add_kernel(const float* __restrict__ y, float alpha, const void* __restrict__ w, int w_is_f32, const void* __restrict__ b,
+                     int b_is_f32, float* __restrict__ x, elem_t* __restrict__ next, float next_alpha, const void* __restrict__ next_w,
+                     int next_w_is_f32, const void* __restrict__ next_b, int next_b_is_f32, int dim) {
+  const size_t at = (size_t)blockIdx.x * dim;
+  if (VEC) {
+    const int e = 4 * (blockIdx.y * NORM_THREADS + threadIdx.x);
+    if (e >= dim) return;
+    const float4 v = *reinterpret_cast<const float4*>(y + at + e);
+    float4 s = *reinterpret_cast<const float4*>(x + at + e);
+    s.x += tanh_norm1(v.x, alpha, w, w_is_f32, b, b_is_f32, e);
+    s.y += tanh_norm1(v.y, alpha, w, w_is_f32, b, b_is_f32, e + 1);
+    s.z += tanh_norm1(v.z, alpha, w, w_is_f32, b, b_is_f32, e + 2);
+    s.w += tanh_norm1(v.w, alpha, w, w_is_f32, b, b_is_f32, e + 3);
+    *reinterpret_cast<float4*>(x + at + e) = s;
+    if (next)
+      store4(next + at + e, tanh_norm1(s.x, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, e),
+             tanh_norm1(s.y, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, e + 1),
+             tanh_norm1(s.z, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, e + 2),
+             tanh_norm1(s.w, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, e + 3));
+    return;
+  }
+  for (int i = threadIdx.x; i < dim; i += NORM_THREADS) {
+    const float s = x[at + i] + tanh_norm1(y[at + i], alpha, w, w_is_f32, b, b_is_f32, i);
+    x[at + i] = s;
+    if (next) next[at + i] = from_float(tanh_norm1(s, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, i));
+  }
+}
+
+extern "C" int axk_tanh_norm(const float* x, const int32_t* rows, float alpha, const void* w, int w_is_f32, const void* b, int b_is_f32,
+                             void* out, int n_rows, int dim, void* stream) {
+  AXK_REQUIRE(n_rows >= 0 && dim > 0, "tanh_norm: bad sizes rows=%d dim=%d", n_rows, dim);
+  if (n_rows == 0) return 0;
+  if (dim % 4 == 0 && ((uintptr_t)x & 15) == 0 && ((uintptr_t)out & 15) == 0)
+    tanh_norm_kernel<true><<<dim3(n_rows, ceil_div(dim, 4 * NORM_THREADS)), NORM_THREADS, 0, (hipStream_t)stream>>>(
+        x, rows, alpha, w, w_is_f32, b, b_is_f32, (elem_t*)out, dim);
+  else
+    tanh_norm_kernel<false><<<n_rows, NORM_THREADS, 0, (hipStream_t)stream>>>(x, rows, alpha, w, w_is_f32, b, b_is_f32, (elem_t*)out, dim);
+  AXK_LAUNCH_CHECK("tanh_norm");
+  return 0;
+}
+
+extern "C" int axk_tanh_norm_add(const float* y, float alpha, const void* w, int w_is_f32, const void* b, int b_is_f32, float* x,
+                                 void* next, float next_alpha, const void* next_w, int next_w_is_f32, const void* next_b,
+                                 int next_b_is_f32, int n_rows, int dim, void* stream) {
+  AXK_REQUIRE(n_rows >= 0 && dim > 0, "tanh_norm_add: bad sizes rows=%d dim=%d", n_rows, dim);
+  AXK_REQUIRE(next == nullptr || (next_w != nullptr && next_b != nullptr), "tanh_norm_add: rows of the next norm without its vectors");
+  if (n_rows == 0) return 0;
+#define TN_ARGS y, alpha, w, w_is_f32, b, b_is_f32, x, (elem_t*)next, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, dim
+  if (dim % 4 == 0 && ((uintptr_t)x & 15) == 0 && ((uintptr_t)y & 15) == 0 && ((uintptr_t)next & 15) == 0)
+    tanh_norm_add_kernel<true><<<dim3(n_rows, ceil_div(dim, 4 * NORM_THREADS)), NORM_THREADS, 0, (hipStream_t)stream>>>(TN_ARGS);
+  else
+    tanh_norm_add_kernel<false><<<n_rows, NORM_THREADS, 0, (hipStream_t)stream>>>(TN_ARGS);
+#undef TN_ARGS
+  AXK_LAUNCH_CHECK("tanh_norm_add");
+  return 0;
+}
+
 // ---------------------------------------------------------------------------- a norm behind the sum
 // x[r, :] = norm(alpha x[r, :] + y[r, :]) * gain, the norm an RMS norm (kind 0) or a layer norm (kind 1,
 // as layernorm_kernel), and rounded[r, :] = the new x[r, :] in the compute dtype if asked for (what the
@@ -462,7 +548,7 @@ extern "C" int axk_concat_round(const float* a, int wa, const float* b, int wb, 
 
 // ---------------------------------------------------------------------------- activations
 // In place.  kind 0: the tanh form of GELU, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)));
-// kind 1: the exact GELU, 0.5 z (1 + erf(z / sqrt 2)).
+// kind 1: the exact GELU, 0.5 z (1 + erf(z / sqrt 2)); kind 2: the square of relu, max(z, 0)^2.
 __global__ void activation_kernel(elem_t* __restrict__ v, long n, int kind) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= n) return;
@@ -471,12 +557,17 @@ __global__ void activation_kernel(elem_t* __restrict__ v, long n, int kind) {
     v[i] = from_float((0.5f * z) * (1.0f + erff(z * 0.7071067811865476f)));
     return;
   }
+  if (kind == 2) {
+    const float p = fmaxf(z, 0.0f);
+    v[i] = from_float(p * p);
+    return;
+  }
   const float inner = 0.7978845608028654f * (z + 0.044715f * ((z * z) * z));
   v[i] = from_float((0.5f * z) * (1.0f + tanhf(inner)));
 }
 
 extern "C" int axk_activation(void* v, long n, int kind, void* stream) {
-  AXK_REQUIRE(kind == 0 || kind == 1, "activation: kind %d is not known (0: gelu, tanh form; 1: gelu, exact)", kind);
+  AXK_REQUIRE(kind >= 0 && kind <= 2, "activation: kind %d is not known (0: gelu, tanh form; 1: gelu, exact; 2: relu squared)", kind);
   if (n <= 0) return 0;
   activation_kernel<<<(unsigned)((n + 255) / 256), 256, 0, (hipStream_t)stream>>>((elem_t*)v, n, kind);
   AXK_LAUNCH_CHECK("activation");

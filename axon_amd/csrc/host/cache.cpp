@@ -24,7 +24,7 @@ struct Group {
   std::vector<int> free_list;              // LIFO; page 0 handed out first
   std::vector<uint8_t> live;               // per page: held by a slot
   std::vector<std::vector<int>> pages;     // per slot: logical page -> physical, -1 once trimmed
-  std::vector<int> first_live;             // per slot: first logical page not yet trimmed
+  std::vector<int> first_live;             // per slot: first logical page behind the trimmed ones (the kept first pages aside)
 };
 
 struct Cache {
@@ -66,8 +66,8 @@ void give_page(Group& g, int page) {
 
 extern "C" {
 
-void* axh_cache_create(int n_groups, const int* n_pages, const int* page_size, const int* window, int max_seqs,
-                       int max_pages_per_seq, long shuffle_seed) {
+void* axh_cache_create(int n_groups, const int* n_pages, const int* page_size, const int* window, const int* keep,
+                       int max_seqs, int max_pages_per_seq, long shuffle_seed) {
   if (n_groups < 0 || max_seqs < 1 || max_pages_per_seq < 1) return nullptr;
   Cache* c = new Cache();
   c->max_seqs = max_seqs;
@@ -78,12 +78,12 @@ void* axh_cache_create(int n_groups, const int* n_pages, const int* page_size, c
   c->shuffle = shuffle_seed >= 0;
   c->rng = (uint64_t)shuffle_seed;
   for (int i = 0; i < n_groups; ++i) {
-    if (n_pages[i] < 1 || page_size[i] < 1 || window[i] < 0) {
+    if (n_pages[i] < 1 || page_size[i] < 1 || window[i] < 0 || keep[i] < 0) {
       delete c;
       return nullptr;
     }
     Group g;
-    g.geo = GroupGeometry{n_pages[i], page_size[i], window[i]};
+    g.geo = GroupGeometry{n_pages[i], page_size[i], window[i], keep[i]};
     for (int p = n_pages[i] - 1; p >= 0; --p) g.free_list.push_back(p);
     g.live.assign(n_pages[i], 0);
     g.pages.resize(max_seqs);
@@ -211,14 +211,14 @@ int axh_cache_reserve_many(void* h, int n, const int* slots, const long* n_token
 }
 
 // After a step: `n_cached` tokens are in the cache.  Windowed groups give back the pages the
-// window has passed.  Returns the pages freed.
+// window has passed, but for those of the first positions that stay readable.  Returns the pages freed.
 int axh_cache_trim(void* h, int slot, long n_cached) {
   Cache& c = *(Cache*)h;
   if (slot < 0 || slot >= c.max_seqs || !c.open[slot]) return -1;
   int freed = 0;
   for (Group& g : c.groups) {
     const int upto = std::min(first_needed_page(g.geo, n_cached), (int)g.pages[slot].size());
-    for (int i = g.first_live[slot]; i < upto; ++i) {
+    for (int i = std::max(g.first_live[slot], kept_pages(g.geo)); i < upto; ++i) {
       if (g.pages[slot][i] >= 0) {
         give_page(g, g.pages[slot][i]);
         g.pages[slot][i] = -1;

@@ -8,6 +8,7 @@ struct GroupGeometry {
   int n_pages;    // pages in the group's pool
   int page_size;  // positions in one page
   int window;     // 0: every position is kept; w > 0: a token reads the last w positions only
+  int keep;       // under a window: the first `keep` positions stay readable as well
 };
 
 // Pages that cover positions [0, n_tokens).
@@ -23,9 +24,13 @@ static inline int first_needed_page(const GroupGeometry& g, long n_cached) {
   return (int)(lo / g.page_size);
 }
 
+// The pages at a request's start that a window never gives back.
+static inline int kept_pages(const GroupGeometry& g) { return (int)(((long)g.keep + g.page_size - 1) / g.page_size); }
+
 // Pages a request holds in this group after `n_cached` tokens (and trimming).
 static inline int pages_held(const GroupGeometry& g, long n_cached) {
-  return pages_covering(g, n_cached) - std::min(first_needed_page(g, n_cached), pages_covering(g, n_cached));
+  const int all = pages_covering(g, n_cached);
+  return all - std::max(0, std::min(first_needed_page(g, n_cached), all) - kept_pages(g));
 }
 
 // New pages needed to go from n_cached to n_after tokens (pages are trimmed only after a step).

@@ -95,11 +95,11 @@ void preempt(Scheduler& s, Request& v, std::vector<long>& free, long& budget, st
 
 extern "C" {
 
-void* axh_sched_create(int n_groups, const int* n_pages, const int* page_size, const int* window,
+void* axh_sched_create(int n_groups, const int* n_pages, const int* page_size, const int* window, const int* keep,
                        int max_batch_tokens, int max_seqs, long max_seq_len) {
   if (n_groups < 0 || max_batch_tokens < 1 || max_seqs < 1 || max_seq_len < 1) return nullptr;
   Scheduler* s = new Scheduler();
-  for (int i = 0; i < n_groups; ++i) s->groups.push_back(GroupGeometry{n_pages[i], page_size[i], window[i]});
+  for (int i = 0; i < n_groups; ++i) s->groups.push_back(GroupGeometry{n_pages[i], page_size[i], window[i], keep[i]});
   s->max_batch_tokens = max_batch_tokens;
   s->max_seqs = max_seqs;
   s->max_seq_len = max_seq_len;

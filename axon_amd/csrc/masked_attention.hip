@@ -1,12 +1,14 @@
 // Grouped-query attention with the variations a configuration may ask for, each a parameter:
 //   * one or two score maps a head (two: differential attention, o = rms(a_1 - lambda a_2) c over one
 //     set of values), keys of `dim` and values of `vdim` elements, `heads` query heads over `kv_heads`;
-//   * a per-head RMS norm of queries and keys with a gain, rotation of the leading dims in either
+//   * an RMS norm of queries and keys with a gain, per head or over all heads at once, rotation of the leading dims in either
 //     pairing (places (2i, 2i + 1) or (i, i + n / 2)) with cos and sin scaled by a factor;
-//   * what a position sees: every earlier position, the last `size` positions (a sliding window), or
-//     the earlier positions of its own chunk of `size` (chunks counted from position 0);
+//   * what a position sees: every earlier position, the last `size` positions (a sliding window) and,
+//     if asked for, the first `keep` ones, or the earlier positions of its own chunk of `size` (chunks
+//     counted from position 0);
 //   * scores bent by cap tanh(s / cap);
-//   * a sink in the softmax: a key of a given score that has no value (its weight only enters the sum);
+//   * a sink in the softmax: a key of a given score, one number or one a head, that has no value (its
+//     weight only enters the sum);
 //   * a query temperature by position, q (1 + coef ln(floor((p + 1) / every) + 1));
 //   * a gate sigmoid(g) on the concatenated heads, a number an element or a number a head.
 //
@@ -28,18 +30,26 @@ __device__ inline int first_seen(int pos, int mask_kind, int mask_size) {
   return 0;
 }
 
+// A range of positions in blocks of 64 with the kept first positions in front: the blocks that hold kept
+// positions before block lo_block, then lo_block, lo_block + 1, ...  kept: how many there are in front.
+__device__ inline int kept_blocks(int keep, int lo_block) { return min((keep + 63) / 64, lo_block); }
+__device__ inline int nth_block(int i, int kept, int lo_block) { return i < kept ? i : lo_block + i - kept; }
+
 // One block per token (or several side by side, each with its share of the units), a wave a unit (one map of one head) at a time.  proj [T, stride] float32 holds
 // the projections' results: n_q units of `dim` from q_at, n_k units from k_at, and v_width values from
 // v_at (v_at may equal k_at: the values are the keys as projected).  Units are RMS-normed with a gain
 // shared by all units (if given), their first rot dims rotated by the step's table [T, rot / 2, 2]
 // (sin, cos), and stored: queries into q_out [T, n_q dim], keys and values into the token's page.
+// norm_rows: the norm's mean goes over all of a token's query units (and over all its key units) at once,
+// and the gain holds a number for every one of these dims.
 __global__ void __launch_bounds__(256)
 heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int n_q, int k_at, int n_k, int v_at, int v_width,
                      int dim, const void* __restrict__ q_gain, int q_gain_is_f32, const void* __restrict__ k_gain,
                      int k_gain_is_f32, float eps, int rot, int neighbours, float magnitude, const float* __restrict__ table,
                      const int32_t* __restrict__ positions, const int32_t* __restrict__ seq_rows,
                      const int32_t* __restrict__ block_table, int table_stride, elem_t* __restrict__ cache, int page_size,
-                     elem_t* __restrict__ q_out, int write_kv, float q_temp_coef, int q_temp_every) {
+                     elem_t* __restrict__ q_out, int write_kv, float q_temp_coef, int q_temp_every, int norm_rows) {
+  __shared__ float row_sums[2][256 / AXON_WAVE];
   const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   // a query's temperature by its position: 1 + coef ln(floor((p + 1) / every) + 1), or 1
   const float q_temp = q_temp_every > 0 ? 1.0f + q_temp_coef * logf((float)((positions[t] + 1) / q_temp_every + 1)) : 1.0f;
@@ -55,6 +65,17 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
     page_base = cache + (long)page * page_size * (kw + v_width);
     in_page = pos % page_size;
   }
+  float q_inv = 1.0f, k_inv = 1.0f;
+  if (norm_rows) {
+    float ss = 0.0f;
+    for (int i = threadIdx.x; i < n_q * dim; i += 256) ss = fmaf(row[q_at + i], row[q_at + i], ss);
+    q_inv = 1.0f / sqrtf(block_sum_256(ss, row_sums[0]) / (float)(n_q * dim) + eps);
+    if (write_kv) {
+      ss = 0.0f;
+      for (int i = threadIdx.x; i < kw; i += 256) ss = fmaf(row[k_at + i], row[k_at + i], ss);
+      k_inv = 1.0f / sqrtf(block_sum_256(ss, row_sums[1]) / (float)kw + eps);
+    }
+  }
   const int n_units = n_q + (write_kv ? n_k : 0);
   for (int u = blockIdx.y * 4 + wave; u < n_units; u += 4 * gridDim.y) {
     const bool is_q = u < n_q;
@@ -63,8 +84,9 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
     const void* gain = is_q ? q_gain : k_gain;
     const int gain_is_f32 = is_q ? q_gain_is_f32 : k_gain_is_f32;
     const float temp = is_q ? q_temp : 1.0f;
-    float inv = 1.0f;
-    if (gain != nullptr) {
+    const int gain_at = norm_rows ? (is_q ? u : u - n_q) * dim : 0;
+    float inv = is_q ? q_inv : k_inv;
+    if (gain != nullptr && !norm_rows) {
       float ss = 0.0f;
       for (int i = lane; i < dim; i += 64) ss = fmaf(src[i], src[i], ss);
       inv = 1.0f / sqrtf(wave_sum(ss) / (float)dim + eps);
@@ -73,8 +95,8 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
       const int ia = neighbours ? 2 * i : i, ib = neighbours ? 2 * i + 1 : i + half;
       float a = src[ia], b = src[ib];
       if (gain != nullptr) {
-        a = (a * inv) * load_vec(gain, gain_is_f32, ia);
-        b = (b * inv) * load_vec(gain, gain_is_f32, ib);
+        a = (a * inv) * load_vec(gain, gain_is_f32, gain_at + ia);
+        b = (b * inv) * load_vec(gain, gain_is_f32, gain_at + ib);
       }
       const float s = tab[2 * i] * magnitude, c = tab[2 * i + 1] * magnitude;
       dst[ia] = from_float(__fsub_rn(__fmul_rn(a, c), __fmul_rn(b, s)) * temp);
@@ -82,7 +104,7 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
     }
     for (int i = rot + lane; i < dim; i += 64) {
       float a = src[i];
-      if (gain != nullptr) a = (a * inv) * load_vec(gain, gain_is_f32, i);
+      if (gain != nullptr) a = (a * inv) * load_vec(gain, gain_is_f32, gain_at + i);
       dst[i] = from_float(a * temp);
     }
   }
@@ -103,7 +125,8 @@ masked_attention_kernel(const elem_t* __restrict__ q, const elem_t* __restrict__
                         int table_stride, const int32_t* __restrict__ positions, const int32_t* __restrict__ seq_rows,
                         const float* __restrict__ gate, long gate_stride, elem_t* __restrict__ out, int n_tokens, int heads,
                         int kv_heads, int maps, int dim, int vdim, int page_size, int mask_kind, int mask_size, float scale,
-                        float softcap, float lambda, float out_scale, float eps, float sink, int gate_per_head) {
+                        float softcap, float lambda, float out_scale, float eps, float sink, int gate_per_head, int keep,
+                        const float* __restrict__ sinks) {
   extern __shared__ float smem[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const long item = (long)blockIdx.x * MA_WAVES + wave;
@@ -131,9 +154,11 @@ masked_attention_kernel(const elem_t* __restrict__ q, const elem_t* __restrict__
     for (int i = 0; i < MA_OWN; ++i) acc[i] = 0.0f;
     float m = -INFINITY, l = 0.0f;
     const float* qm = qs + mp * dim;
-    for (int b = lo / 64; b <= pos / 64; ++b) {
+    const int lo_block = lo / 64, kept = kept_blocks(keep, lo_block), n_blocks = kept + pos / 64 - lo_block + 1;
+    for (int n = 0; n < n_blocks; ++n) {
+      const int b = nth_block(n, kept, lo_block);
       const int p = b * 64 + lane;
-      const bool seen = p >= lo && p <= pos;
+      const bool seen = (p >= lo || p < keep) && p <= pos;
       float s = -INFINITY;
       if (seen) {
         const elem_t* key = cache + (long)pages[p / page_size] * page_elems + (long)(p % page_size) * kw + (g * maps + mp) * dim;
@@ -149,8 +174,10 @@ masked_attention_kernel(const elem_t* __restrict__ q, const elem_t* __restrict__
       m = m_new;
 #pragma unroll
       for (int i = 0; i < MA_OWN; ++i) acc[i] *= fold;
-      const int j_lo = max(lo, b * 64) - b * 64, j_hi = min(pos, b * 64 + 63) - b * 64;
-      for (int j = j_lo; j <= j_hi; ++j) {
+      // kept positions first, then those from lo on (where the kept ones reach lo: one run of positions)
+      const int j_kept = min(min(keep, lo) - b * 64, 64), j_lo = max(lo, b * 64) - b * 64, j_hi = min(pos, b * 64 + 63) - b * 64;
+      for (int j = j_kept > 0 ? 0 : j_lo; j <= j_hi; ++j) {
+        if (j >= j_kept && j < j_lo) { j = j_lo - 1; continue; }
         const float wj = __shfl(w, j, 64);
         const int pj = b * 64 + j;
         const elem_t* val = cache + (long)pages[pj / page_size] * page_elems + (long)page_size * kw +
@@ -162,6 +189,7 @@ masked_attention_kernel(const elem_t* __restrict__ q, const elem_t* __restrict__
         }
       }
     }
+    if (sinks) sink = sinks[h];
     if (sink > -INFINITY) l += expf(sink - m);       // a key of this score that has no value
     const float inv = 1.0f / l;
 #pragma unroll
@@ -245,7 +273,7 @@ struct MaState {
 // sees every position of the block (no mask to apply).  The running maximum is kept in units of log2 e.
 template <int MAPS, int DT, int KC, class PTR, class QF>
 __device__ inline void ma_block(MaState<MAPS, DT>& st, PTR kbase, int kstride, PTR vbase, int vstride,
-                                QF qfrag, int p0, int my_lo, int my_pos, bool full, int dim, int dt_n, float scale, float softcap,
+                                QF qfrag, int p0, int my_lo, int my_pos, int keep, bool full, int dim, int dt_n, float scale, float softcap,
                                 int j, int g) {
   const int kc = (dim + 31) / 32;
   // the bend's constants: scale 2 log2(e) / c into the exponential; c log2(e) and twice that out of it
@@ -289,7 +317,7 @@ __device__ inline void ma_block(MaState<MAPS, DT>& st, PTR kbase, int kstride, P
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int p = p0 + 16 * pt + 4 * g + i;
-          s[pt][i] = (p >= my_lo && p <= my_pos) ? s[pt][i] : -INFINITY;
+          s[pt][i] = ((p >= my_lo || p < keep) && p <= my_pos) ? s[pt][i] : -INFINITY;
         }
     }
     float mx = -INFINITY;
@@ -414,7 +442,8 @@ masked_attention_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restr
                              const float* __restrict__ gate, long gate_stride, bf16_t* __restrict__ out,
                              const int32_t* __restrict__ tiles, int heads, int kv_heads, int dim, int vdim, int page_size,
                              int mask_kind, int mask_size, float scale, float softcap, float lambda, float out_scale, float eps,
-                             float* __restrict__ partial, int n_chunks, float sink_log2, int gate_per_head) {
+                             float* __restrict__ partial, int n_chunks, float sink_log2, int gate_per_head, int keep,
+                             const float* __restrict__ sinks) {
   constexpr int QMAP = KC * 32, QROW = MAPS * QMAP + 8;      // rows 16 bytes longer than their chunks: 16 rows, 16 banks apart
   __shared__ __align__(16) bf16_t qs[16 * QROW];
   const int lane = threadIdx.x, j = lane & 15, g = lane >> 4;
@@ -446,10 +475,12 @@ masked_attention_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restr
   __syncthreads();
   const int my_tok = n == 1 ? t0 : t0 + j, my_head = n == 1 ? h0 + j : h0;
   const bool my_col = j < ncols;
+  if (sinks) sink_log2 = my_col ? sinks[my_head] * 1.4426950408889634f : -INFINITY;
   const int my_pos = my_col ? positions[my_tok] : -1;
   const int my_lo = my_col ? first_seen(my_pos, mask_kind, mask_size) : 0;
   const int pos_first = positions[t0], pos_last = pos_first + n - 1;
   const int lo_first = first_seen(pos_first, mask_kind, mask_size), lo_last = first_seen(pos_last, mask_kind, mask_size);
+  const int lo_block = lo_first / 64, kept = kept_blocks(keep, lo_block), n_blocks = kept + pos_last / 64 - lo_block + 1;
   const int32_t* pages = block_table + (long)seq_rows[t0] * table_stride;
   const int kw = kv_heads * MAPS * dim, dt_n = vdim / 16;
   const long page_elems = (long)page_size * (kw + kv_heads * vdim);
@@ -459,14 +490,15 @@ masked_attention_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restr
   st.clear();
   const bool split = partial != nullptr && n == 1;
   if (!split && blockIdx.z > 0) return;
-  const int b_first = split ? lo_first / 64 + (int)blockIdx.z : lo_first / 64;
-  const int b_last = split ? min(b_first, pos_last / 64) : pos_last / 64;
-  for (int b = b_first; b <= b_last; ++b) {
+  const int n_first = split ? (int)blockIdx.z : 0, n_end = split ? min(n_first + 1, n_blocks) : n_blocks;
+  for (int nb = n_first; nb < n_end; ++nb) {
+    const int b = nth_block(nb, kept, lo_block);
     const int p0 = b * 64, in0 = p0 % page_size;
     const bf16_t* page = cache + (long)pages[p0 / page_size] * page_elems;
     ma_block<MAPS, DT, KC, const bf16_t*>(st, page + (long)in0 * kw + (long)gk * MAPS * dim + 8 * g, kw,
                            page + (long)page_size * kw + (long)gk * vdim * page_size + in0 + 4 * g, page_size, qfrag, p0, my_lo,
-                           my_pos, ncols == 16 && p0 >= lo_last && p0 + 63 <= pos_first, dim, dt_n, scale, softcap, j, g);
+                           my_pos, keep, ncols == 16 && (p0 >= lo_last || p0 + 63 < keep) && p0 + 63 <= pos_first, dim, dt_n, scale,
+                           softcap, j, g);
   }
   if (split) {
     if (!my_col) return;
@@ -498,10 +530,12 @@ template <int MAPS>
 __global__ void __launch_bounds__(64)
 masked_attention_fold_kernel(const float* __restrict__ partial, int n_chunks, const int32_t* __restrict__ tiles,
                              const float* __restrict__ gate, long gate_stride, bf16_t* __restrict__ out, int heads, int vdim,
-                             float lambda, float out_scale, float eps, float sink_log2, int gate_per_head) {
+                             float lambda, float out_scale, float eps, float sink_log2, int gate_per_head,
+                             const float* __restrict__ sinks) {
   const int t = tiles ? tiles[2 * blockIdx.x] : (int)blockIdx.x, n = tiles ? tiles[2 * blockIdx.x + 1] : 1;
   if (n != 1) return;
   const int h = blockIdx.y, lane = threadIdx.x;
+  if (sinks) sink_log2 = sinks[h] * 1.4426950408889634f;
   float o[MA_OWN];
 #pragma unroll
   for (int i = 0; i < MA_OWN; ++i) o[i] = 0.0f;
@@ -581,7 +615,8 @@ masked_attention_staged_kernel(const bf16_t* __restrict__ q, const bf16_t* __res
                                const int32_t* __restrict__ seq_rows, const float* __restrict__ gate, long gate_stride,
                                bf16_t* __restrict__ out, const int32_t* __restrict__ tiles, int heads, int kv_heads, int dim,
                                int vdim, int page_size, int mask_kind, int mask_size, float scale, float softcap, float lambda,
-                               float out_scale, float eps, float sink_log2, int gate_per_head) {
+                               float out_scale, float eps, float sink_log2, int gate_per_head, int keep,
+                               const float* __restrict__ sinks) {
   extern __shared__ __align__(16) bf16_t stage[];       // keys [64][MAPS dim + 8], then values [vdim][64 + 8]
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, j = lane & 15, g = lane >> 4;
   const int grp = heads / kv_heads, hb_n = (grp + MAS_WAVES - 1) / MAS_WAVES;
@@ -602,6 +637,7 @@ masked_attention_staged_kernel(const bf16_t* __restrict__ q, const bf16_t* __res
   }
   const int my_tok = n == 1 ? t0 : t0 + j, my_head = n == 1 ? h0 + j : h0;
   const bool my_col = active && j < ncols;
+  if (sinks) sink_log2 = my_col ? sinks[my_head] * 1.4426950408889634f : -INFINITY;
   const int qw = MAPS * dim;
   uint4 qf[MAPS][KC];
 #pragma unroll
@@ -655,9 +691,9 @@ masked_attention_staged_kernel(const bf16_t* __restrict__ q, const bf16_t* __res
   // the 16 bytes behind each staged key row are read with the last chunk of a map whose dims are no multiple of 32
   // (against a zero query operand): they hold zeros, never what LDS happened to hold
   if (threadIdx.x < 64) ma_store16(ks + threadIdx.x * krow + qw, make_uint4(0u, 0u, 0u, 0u));
-  const int b_last = pos_last / 64;
-  fetch(lo_first / 64);
-  for (int b = lo_first / 64; b <= b_last; ++b) {
+  const int lo_block = lo_first / 64, kept = kept_blocks(keep, lo_block), n_blocks = kept + pos_last / 64 - lo_block + 1;
+  fetch(nth_block(0, kept, lo_block));
+  for (int nb = 0; nb < n_blocks; ++nb) {
     __syncthreads();                                    // the block before has been read
 #pragma unroll
     for (int i = 0; i < KP; ++i)
@@ -666,11 +702,12 @@ masked_attention_staged_kernel(const bf16_t* __restrict__ q, const bf16_t* __res
     for (int i = 0; i < VP; ++i)
       if (v_from[i] >= 0) ma_store16(vs + v_to[i], vreg[i]);
     __syncthreads();
-    if (b < b_last) fetch(b + 1);
-    const int p0 = b * 64;
+    if (nb + 1 < n_blocks) fetch(nth_block(nb + 1, kept, lo_block));
+    const int p0 = nth_block(nb, kept, lo_block) * 64;
     if (active)
       ma_block<MAPS, DT, KC, ma_lds_cptr>(st, ks + 8 * g, krow, vs + 4 * g, vrow, qfrag, p0, my_lo, my_pos,
-                             ncols == 16 && p0 >= lo_last && p0 + 63 <= pos_first, dim, dt_n, scale, softcap, j, g);
+                             keep, ncols == 16 && (p0 >= lo_last || p0 + 63 < keep) && p0 + 63 <= pos_first, dim, dt_n, scale, softcap,
+                             j, g);
   }
   if (active)
     ma_finish<MAPS, DT>(st, my_col, my_tok, my_head, heads, vdim, dt_n, gate, gate_stride, out, lambda, out_scale, eps, g, sink_log2,
@@ -679,9 +716,9 @@ masked_attention_staged_kernel(const bf16_t* __restrict__ q, const bf16_t* __res
 
 // Blocks of positions a single token can touch under its mask (0: no bound known).  Without a window or chunks
 // the bound is the step's: `span`, the positions its longest row sees.
-static int masked_chunks(int mask_kind, int mask_size, int span) {
+static int masked_chunks(int mask_kind, int mask_size, int keep, int span) {
   if (mask_kind == MASK_CAUSAL) return span > 0 ? (span + 63) / 64 : 0;
-  return (mask_size + 62) / 64 + 1;
+  return (int)(((long)mask_size + 62) / 64 + 1 + ((long)keep + 63) / 64);
 }
 
 template <int MAPS, int DT, int KC>
@@ -689,7 +726,8 @@ static int launch_masked_mfma(const void* q, const void* cache, const int32_t* b
                               const int32_t* positions, const int32_t* seq_rows, const float* gate, long gate_stride, void* out,
                               const int32_t* tiles, int n_tiles, int heads, int kv_heads, int dim, int vdim, int page_size,
                               int mask_kind, int mask_size, float scale, float softcap, float lambda, float out_scale, float eps,
-                              float* partial, int span, float sink_log2, int gate_per_head, hipStream_t stream) {
+                              float* partial, int span, float sink_log2, int gate_per_head, int keep, const float* sinks,
+                              hipStream_t stream) {
   const int grp = heads / kv_heads;
   const size_t lds = ((size_t)64 * (MAPS * dim + 8) + (size_t)vdim * (64 + 8)) * sizeof(bf16_t);
   if (tiles != nullptr && partial == nullptr && KC <= 4 && DT <= 8 && lds <= 64 * 1024) {
@@ -707,18 +745,18 @@ static int launch_masked_mfma(const void* q, const void* cache, const int32_t* b
         <<<dim3(n_tiles, kv_heads * ((grp + MAS_WAVES - 1) / MAS_WAVES)), MAS_WAVES * 64, lds, stream>>>(
             (const bf16_t*)q, (const bf16_t*)cache, block_table, table_stride, positions, seq_rows, gate, gate_stride,
             (bf16_t*)out, tiles, heads, kv_heads, dim, vdim, page_size, mask_kind, mask_size, scale, softcap, lambda, out_scale, eps,
-            sink_log2, gate_per_head);
+            sink_log2, gate_per_head, keep, sinks);
     return 0;
   }
-  const int n_chunks = partial ? masked_chunks(mask_kind, mask_size, span) : 1;
+  const int n_chunks = partial ? masked_chunks(mask_kind, mask_size, keep, span) : 1;
   masked_attention_mfma_kernel<MAPS, DT, KC><<<dim3(n_tiles, heads, n_chunks), 64, 0, stream>>>(
       (const bf16_t*)q, (const bf16_t*)cache, block_table, table_stride, positions, seq_rows, gate, gate_stride, (bf16_t*)out, tiles,
       heads, kv_heads, dim, vdim, page_size, mask_kind, mask_size, scale, softcap, lambda, out_scale, eps, partial, n_chunks,
-      sink_log2, gate_per_head);
+      sink_log2, gate_per_head, keep, sinks);
   if (partial)
     masked_attention_fold_kernel<MAPS><<<dim3(n_tiles, heads), 64, 0, stream>>>(partial, n_chunks, tiles, gate, gate_stride,
                                                                               (bf16_t*)out, heads, vdim, lambda, out_scale, eps,
-                                                                              sink_log2, gate_per_head);
+                                                                              sink_log2, gate_per_head, sinks);
   return 0;
 }
 #endif
@@ -729,20 +767,21 @@ extern "C" int axk_heads_prepare(const float* proj, long stride, int q_at, int n
                                  int dim, const void* q_gain, int q_gain_is_f32, const void* k_gain, int k_gain_is_f32, float eps,
                                  int rot, int neighbours, float magnitude, const float* table, const int32_t* positions,
                                  const int32_t* seq_rows, const int32_t* block_table, int table_stride, void* cache, int page_size,
-                                 void* q_out, int n_tokens, int write_kv, float q_temp_coef, int q_temp_every, void* stream) {
+                                 void* q_out, int n_tokens, int write_kv, float q_temp_coef, int q_temp_every, int norm_rows, void* stream) {
   AXK_REQUIRE(n_tokens >= 0 && n_q > 0 && n_k > 0 && dim > 0 && v_width > 0 && page_size > 0,
               "heads_prepare: bad sizes T=%d q units=%d k units=%d dim=%d values=%d page=%d", n_tokens, n_q, n_k, dim, v_width,
               page_size);
   AXK_REQUIRE(rot >= 0 && rot <= dim && rot % 2 == 0, "heads_prepare: %d rotated dims of %d", rot, dim);
-  AXK_REQUIRE(q_at >= 0 && k_at >= 0 && v_at >= 0 && q_at + (long)n_q * dim <= stride && k_at + (long)n_k * dim <= stride &&
-              v_at + (long)v_width <= stride, "heads_prepare: the parts do not fit rows of %ld", stride);
+  AXK_REQUIRE(q_at >= 0 && q_at + (long)n_q * dim <= stride &&
+              (!write_kv || (k_at >= 0 && v_at >= 0 && k_at + (long)n_k * dim <= stride && v_at + (long)v_width <= stride)), "heads_prepare: the parts do not fit rows of %ld", stride);
+  AXK_REQUIRE(!norm_rows || (q_gain != nullptr && (!write_kv || k_gain != nullptr)), "heads_prepare: a norm over all rows without its gains");
   if (n_tokens == 0) return 0;
   // few tokens: a token's units side by side in several blocks
   const int per_token = n_tokens >= 1024 ? 1 : min((n_q + n_k + 3) / 4, 16);
   heads_prepare_kernel<<<dim3(n_tokens, per_token), 256, 0, (hipStream_t)stream>>>(
       proj, stride, q_at, n_q, k_at, n_k, v_at, v_width, dim, q_gain, q_gain_is_f32, k_gain, k_gain_is_f32, eps, rot, neighbours,
       magnitude, table, positions, seq_rows, block_table, table_stride, (elem_t*)cache, page_size, (elem_t*)q_out, write_kv, q_temp_coef,
-      q_temp_every);
+      q_temp_every, norm_rows);
   AXK_LAUNCH_CHECK("heads_prepare");
   return 0;
 }
@@ -761,10 +800,10 @@ extern "C" int axk_masked_attention_uses_mfma(int heads, int kv_heads, int maps,
 // positions, what the step's longest row sees, make); the floats of the workspace that takes (0: a wave walks its
 // token's blocks itself).
 extern "C" long axk_masked_attention_workspace(int n_tokens, int heads, int kv_heads, int maps, int dim, int vdim, int page_size,
-                                               int mask_kind, int mask_size, int span) {
+                                               int mask_kind, int mask_size, int keep, int span) {
 #if AXON_BF16
   if (!axk_masked_attention_uses_mfma(heads, kv_heads, maps, dim, vdim, page_size)) return 0;
-  const int chunks = masked_chunks(mask_kind, mask_size, span);
+  const int chunks = masked_chunks(mask_kind, mask_size, keep, span);
   if (chunks < 3 || (long)n_tokens * kv_heads >= 512) return 0;
   return (long)n_tokens * heads * chunks * maps * (vdim + 2);
 #else
@@ -777,7 +816,7 @@ extern "C" int axk_masked_attention(const void* q, const void* cache, const int3
                                     void* out, int n_tokens, int heads, int kv_heads, int maps, int dim, int vdim, int page_size,
                                     int mask_kind, int mask_size, float scale, float softcap, float lambda, float out_scale,
                                     float eps, const int32_t* tiles, int n_tiles, float* partial, long partial_floats,
-                                    float sink, int gate_per_head, int span, void* stream) {
+                                    float sink, const float* sinks, int gate_per_head, int keep, int span, void* stream) {
   AXK_REQUIRE(n_tokens >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && vdim > 0 && page_size > 0,
               "masked_attention: bad sizes T=%d heads=%d kv heads=%d dim=%d vdim=%d page=%d", n_tokens, heads, kv_heads, dim, vdim,
               page_size);
@@ -785,6 +824,7 @@ extern "C" int axk_masked_attention(const void* q, const void* cache, const int3
   AXK_REQUIRE(vdim <= 64 * MA_OWN, "masked_attention: values of %d dims (at most %d)", vdim, 64 * MA_OWN);
   AXK_REQUIRE(mask_kind == MASK_CAUSAL || ((mask_kind == MASK_WINDOW || mask_kind == MASK_CHUNK) && mask_size > 0),
               "masked_attention: mask kind %d of size %d", mask_kind, mask_size);
+  AXK_REQUIRE(keep >= 0 && (keep == 0 || mask_kind == MASK_WINDOW), "masked_attention: %d kept positions under mask kind %d", keep, mask_kind);
   AXK_REQUIRE((long)maps * dim * MA_WAVES * 4 <= 64 * 1024, "masked_attention: queries of %d dims do not fit LDS", maps * dim);
   if (n_tokens == 0) return 0;
 #if AXON_BF16
@@ -792,14 +832,15 @@ extern "C" int axk_masked_attention(const void* q, const void* cache, const int3
       ((uintptr_t)cache & 15) == 0 && ((uintptr_t)out & 7) == 0) {
     AXK_REQUIRE(tiles == nullptr || n_tiles > 0, "masked_attention: a list of %d tiles", n_tiles);
     const int nt = tiles ? n_tiles : n_tokens;
-    const long need = axk_masked_attention_workspace(n_tokens, heads, kv_heads, maps, dim, vdim, page_size, mask_kind, mask_size, span);
+    const long need = axk_masked_attention_workspace(n_tokens, heads, kv_heads, maps, dim, vdim, page_size, mask_kind, mask_size, keep, span);
     AXK_REQUIRE(partial == nullptr || partial_floats >= need, "masked_attention: a workspace of %ld floats, %ld needed",
                 partial_floats, need);
     if (need == 0) partial = nullptr;
 #define MA_LAUNCH(MAPS, DT, KC)                                                                                                 \
   rc = launch_masked_mfma<MAPS, DT, KC>(q, cache, block_table, table_stride, positions, seq_rows, gate, gate_stride, out, tiles, nt, \
                                    heads, kv_heads, dim, vdim, page_size, mask_kind, mask_size, scale, softcap, lambda,        \
-                                   out_scale, eps, partial, span, sink * 1.4426950408889634f, gate_per_head, (hipStream_t)stream)
+                                   out_scale, eps, partial, span, sink * 1.4426950408889634f, gate_per_head, keep, sinks,     \
+                                   (hipStream_t)stream)
     int rc = 0;
     // register tiles by the sizes: chunks of 32 key dims (2, 4 or 8), tiles of 16 value dims (4, 8 or 16)
 #define MA_BY_DIM(MAPS, DT)                                                                  \
@@ -824,7 +865,7 @@ extern "C" int axk_masked_attention(const void* q, const void* cache, const int3
   masked_attention_kernel<<<(unsigned)((items + MA_WAVES - 1) / MA_WAVES), MA_WAVES * 64, lds, (hipStream_t)stream>>>(
       (const elem_t*)q, (const elem_t*)cache, block_table, table_stride, positions, seq_rows, gate, gate_stride, (elem_t*)out,
       n_tokens, heads, kv_heads, maps, dim, vdim, page_size, mask_kind, mask_size, scale, softcap, lambda, out_scale, eps, sink,
-      gate_per_head);
+      gate_per_head, keep, sinks);
   AXK_LAUNCH_CHECK("masked_attention");
   return 0;
 }

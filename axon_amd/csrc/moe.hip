@@ -70,7 +70,7 @@ __global__ void route_topk_wave_kernel(const float* __restrict__ logits, int n_t
   if (lane < top) weights[(long)t * top + lane] = mine / sum;
 }
 
-// Scores that do not compete: s_e = sigmoid(z_e); the choice is made by s_e + correction_e (if given),
+// Scores of every expert: s_e = sigmoid(z_e), which do not compete, or (SOFTMAX) the softmax over all of them; the choice is made by s_e + correction_e (if given),
 // the weights come from s_e alone.  The experts form `groups` equal groups of neighbours; a group's
 // score is the sum of its two largest choice scores (of its one, if it has one expert), only experts
 // of the `keep` best groups can be chosen (of equal groups the lower), and among those the `top`
@@ -78,6 +78,7 @@ __global__ void route_topk_wave_kernel(const float* __restrict__ logits, int n_t
 // added in the order chosen, + 1e-20) * scale, or without `normalize` the score itself times scale.  Rows of
 // logits are logits_stride apart (further columns may hold other products of the same input).  A wave per token: lane l holds experts l, l + 64, ...
 // (up to 1,024) and, for the groups' scores, walks group l (up to 64 groups).
+template <bool SOFTMAX>
 __global__ void route_scored_wave_kernel(const float* __restrict__ logits, long logits_stride, const float* __restrict__ correction,
                                          int n_tokens, int n_experts, int top, int groups, int keep, float scale, int normalize,
                                          int32_t* __restrict__ experts, float* __restrict__ weights) {
@@ -85,12 +86,22 @@ __global__ void route_scored_wave_kernel(const float* __restrict__ logits, long 
   if (t >= n_tokens) return;
   const float* z = logits + (long)t * logits_stride;
   const int size = n_experts / groups;
+  float z_most = 0.0f, z_share = 1.0f;
+  if (SOFTMAX) {
+    z_most = -INFINITY;
+    for (int e = lane; e < n_experts; e += 64) z_most = fmaxf(z_most, z[e]);
+    z_most = wave_max(z_most);
+    float total = 0.0f;
+    for (int e = lane; e < n_experts; e += 64) total += expf(z[e] - z_most);
+    z_share = 1.0f / wave_sum(total);
+  }
+  auto score = [&](int e) { return SOFTMAX ? expf(z[e] - z_most) * z_share : 1.0f / (1.0f + expf(-z[e])); };
   unsigned long long kept = ~0ull;
   if (groups > 1) {
     float first = -INFINITY, second = -INFINITY;
     if (lane < groups)
       for (int e = lane * size; e < (lane + 1) * size; ++e) {
-        const float c = 1.0f / (1.0f + expf(-z[e])) + (correction ? correction[e] : 0.0f);
+        const float c = score(e) + (correction ? correction[e] : 0.0f);
         if (c > first) { second = first; first = c; }
         else if (c > second) second = c;
       }
@@ -107,7 +118,7 @@ __global__ void route_scored_wave_kernel(const float* __restrict__ logits, long 
   for (int i = 0; i < 16; ++i) {
     const int e = lane + 64 * i;
     choice[i] = -INFINITY;
-    if (e < n_experts && (kept >> (e / size) & 1)) choice[i] = 1.0f / (1.0f + expf(-z[e])) + (correction ? correction[e] : 0.0f);
+    if (e < n_experts && (kept >> (e / size) & 1)) choice[i] = score(e) + (correction ? correction[e] : 0.0f);
   }
   unsigned taken = 0;
   float sum = 0.0f, mine = 0.0f;                     // lane k keeps the k-th score
@@ -126,7 +137,7 @@ __global__ void route_scored_wave_kernel(const float* __restrict__ logits, long 
       if (other_at != 0x7fffffff && (at == 0x7fffffff || other > best || (other == best && other_at < at))) { best = other; at = other_at; }
     }
     if ((at & 63) == lane) taken |= 1u << (at >> 6);
-    const float s = 1.0f / (1.0f + expf(-z[at]));
+    const float s = score(at);
     sum += s;
     if (lane == k % 64) { mine = s; experts[(long)t * top + k] = at; }
   }
@@ -136,7 +147,8 @@ __global__ void route_scored_wave_kernel(const float* __restrict__ logits, long 
 // One block.  pairs p = t top + k in expert order -> sorted [n_pairs], with the token of each
 // (sorted_tokens); tiles [.][3] = (expert, first place in sorted, count <= tile_rows), *n_tiles of them.
 // Which place a pair gets inside its expert's stretch is not fixed (atomic counters); no result
-// depends on it: every row of a product is a chain of its own.
+// depends on it: every row of a product is a chain of its own.  Pairs whose expert is n_experts or more (an
+// identity, which has no matrices) are not listed.
 __global__ void __launch_bounds__(1024)
 route_sort_kernel(const int32_t* __restrict__ experts, int n_pairs, int n_experts, int top, int32_t* __restrict__ sorted,
                   int32_t* __restrict__ sorted_tokens, int32_t* __restrict__ tiles, int32_t* __restrict__ n_tiles,
@@ -145,7 +157,8 @@ route_sort_kernel(const int32_t* __restrict__ experts, int n_pairs, int n_expert
   int* next = counts + n_experts;
   for (int e = threadIdx.x; e < n_experts; e += blockDim.x) counts[e] = 0;
   __syncthreads();
-  for (int p = threadIdx.x; p < n_pairs; p += blockDim.x) atomicAdd(&counts[experts[p]], 1);
+  for (int p = threadIdx.x; p < n_pairs; p += blockDim.x)
+    if (experts[p] < n_experts) atomicAdd(&counts[experts[p]], 1);
   __syncthreads();
   if (threadIdx.x == 0) {
     int at = 0, tile = 0;
@@ -164,6 +177,7 @@ route_sort_kernel(const int32_t* __restrict__ experts, int n_pairs, int n_expert
   }
   __syncthreads();
   for (int p = threadIdx.x; p < n_pairs; p += blockDim.x) {
+    if (experts[p] >= n_experts) continue;
     const int place = atomicAdd(&next[experts[p]], 1);
     sorted[place] = p;
     sorted_tokens[place] = p / top;
@@ -173,17 +187,21 @@ route_sort_kernel(const int32_t* __restrict__ experts, int n_pairs, int n_expert
 
 // y[t, :] (+)= sum_k weights[t, k] rows[row of pair t top + k, :], k ascending; a pair's row is the pair
 // itself, or place_of[pair]; without weights the rows are added as they are.  extra (or null): a further
-// row a token, added last, times sigmoid(extra_gate[t extra_gate_stride]) if a gate is given.
+// row a token, added last, times sigmoid(extra_gate[t extra_gate_stride]) if a gate is given.  input (or null): a pair
+// whose expert (experts[pair]) is n_experts or more is an identity, its row is input[t, :].
 __global__ void route_combine_kernel(const float* __restrict__ rows, const float* __restrict__ weights, float* __restrict__ y,
                                      int top, int width, int accumulate, const int32_t* __restrict__ place_of,
-                                     const float* __restrict__ extra, const float* __restrict__ extra_gate, long extra_gate_stride) {
+                                     const float* __restrict__ extra, const float* __restrict__ extra_gate, long extra_gate_stride,
+                                     const int32_t* __restrict__ experts, int n_experts, const elem_t* __restrict__ input,
+                                     long input_stride) {
   const int t = blockIdx.y;
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   if (c >= width) return;
   float acc = accumulate ? y[(long)t * width + c] : 0.0f;
   for (int k = 0; k < top; ++k) {
     const long pair = (long)t * top + k;
-    const float row = rows[(place_of ? (long)place_of[pair] : pair) * width + c];
+    const float row = input && experts[pair] >= n_experts ? to_float(input[(long)t * input_stride + c])
+                                                          : rows[(place_of ? (long)place_of[pair] : pair) * width + c];
     acc = weights ? fmaf(weights[pair], row, acc) : acc + row;
   }
   if (extra) {
@@ -219,7 +237,7 @@ extern "C" int axk_route_topk(const float* logits, int n_tokens, int n_experts, 
 }
 
 extern "C" int axk_route_scored(const float* logits, long logits_stride, const float* correction, int n_tokens, int n_experts,
-                                int top, int groups, int keep, float scale, int normalize, int32_t* experts, float* weights,
+                                int top, int groups, int keep, float scale, int normalize, int softmax, int32_t* experts, float* weights,
                                 void* stream) {
   AXK_REQUIRE(logits_stride >= n_experts, "route_scored: rows of %ld logits for %d experts", logits_stride, n_experts);
   AXK_REQUIRE(n_tokens >= 0 && n_experts > 0 && n_experts <= 1024 && top > 0 && top <= 64,
@@ -228,8 +246,9 @@ extern "C" int axk_route_scored(const float* logits, long logits_stride, const f
               (long)keep * (n_experts / groups) >= top,
               "route_scored: %d of %d groups of %d experts for %d a token", keep, groups, n_experts / (groups > 0 ? groups : 1), top);
   if (n_tokens == 0) return 0;
-  route_scored_wave_kernel<<<ceil_div(n_tokens, 4), 256, 0, (hipStream_t)stream>>>(logits, logits_stride, correction, n_tokens, n_experts, top,
-                                                                                  groups, keep, scale, normalize, experts, weights);
+  auto kernel = softmax ? route_scored_wave_kernel<true> : route_scored_wave_kernel<false>;
+  kernel<<<ceil_div(n_tokens, 4), 256, 0, (hipStream_t)stream>>>(logits, logits_stride, correction, n_tokens, n_experts, top, groups,
+                                                                 keep, scale, normalize, experts, weights);
   AXK_LAUNCH_CHECK("route_scored");
   return 0;
 }
@@ -259,13 +278,16 @@ extern "C" int axk_route_sort(const int32_t* experts, int n_pairs, int n_experts
 
 extern "C" int axk_route_combine(const float* rows, const float* weights, float* y, int n_tokens, int top, int width,
                                  int accumulate, const int32_t* place_of, const float* extra, const float* extra_gate,
-                                 long extra_gate_stride, void* stream) {
+                                 long extra_gate_stride, const int32_t* experts, int n_experts, const void* input, long input_stride,
+                                 void* stream) {
   AXK_REQUIRE(n_tokens >= 0 && top > 0 && width > 0 && n_tokens <= 65535, "route_combine: T=%d top=%d width=%d", n_tokens, top,
               width);
+  AXK_REQUIRE(input == nullptr || (experts != nullptr && input_stride >= width), "route_combine: identities need the chosen experts and rows of %d", width);
   if (n_tokens == 0) return 0;
   dim3 grid(ceil_div(width, 256), n_tokens);
   route_combine_kernel<<<grid, 256, 0, (hipStream_t)stream>>>(rows, weights, y, top, width, accumulate, place_of, extra,
-                                                              extra_gate, extra_gate_stride);
+                                                              extra_gate, extra_gate_stride, experts, n_experts,
+                                                              (const elem_t*)input, input_stride);
   AXK_LAUNCH_CHECK("route_combine");
   return 0;
 }

@@ -13,7 +13,8 @@ from .runtime import Runtime
 
 def read_model_config(model_dir: str, checkpoint: Optional[Checkpoint] = None) -> ModelConfig:
     """config.json through the registry.  A configuration that does not know its vocabulary yet
-    names the tensor that does (`ModelConfig.vocab_tensor`)."""
+    names the tensor that does (`ModelConfig.vocab_tensor`); sizes that only a tensor's shape gives
+    are read from there (`ModelConfig.size_tensors`)."""
     config = config_from_dict(read_config_json(model_dir))
     name = config.vocab_tensor()
     if name is not None:
@@ -22,6 +23,10 @@ def read_model_config(model_dir: str, checkpoint: Optional[Checkpoint] = None) -
             from ..weights import WeightError
             raise WeightError([name], [], [])
         config = config.with_vocab(ck.shape(name)[0])
+    names = config.size_tensors()
+    if names:
+        ck = checkpoint or Checkpoint(model_dir)
+        config = config.with_sizes({n: ck.shape(n) for n in names if n in ck})
     return config
 
 

@@ -13,7 +13,7 @@ from __future__ import annotations
 import ctypes
 from ctypes import c_int, c_long
 from dataclasses import dataclass
-from typing import List, Sequence, Tuple
+from typing import List, Optional, Sequence, Tuple
 
 from ..cache.manager import host_lib
 
@@ -32,13 +32,13 @@ class Planned:
 
 class Scheduler:
     def __init__(self, n_pages: Sequence[int], page_size: Sequence[int], window: Sequence[int],
-                 max_batch_tokens: int, max_seqs: int, max_seq_len: int):
+                 max_batch_tokens: int, max_seqs: int, max_seq_len: int, keep: Optional[Sequence[int]] = None):
         self.lib = host_lib()
         n = len(n_pages)
         self.n_groups = n
         arr = lambda v: (c_int * max(n, 1))(*v)
-        self._h = self.lib.axh_sched_create(n, arr(n_pages), arr(page_size), arr(window), max_batch_tokens, max_seqs,
-                                            max_seq_len)
+        self._h = self.lib.axh_sched_create(n, arr(n_pages), arr(page_size), arr(window), arr(keep or [0] * n),
+                                            max_batch_tokens, max_seqs, max_seq_len)
         if not self._h:
             raise SchedulerError("bad scheduler settings")
         self.cap = max(max_seqs, 1) * 2 + 8
@@ -52,7 +52,7 @@ class Scheduler:
     def for_cache(cls, cache, max_batch_tokens: int) -> "Scheduler":
         plans = cache.plans
         return cls([p.n_pages for p in plans], [p.page_size for p in plans], [p.spec.window for p in plans],
-                   max_batch_tokens, cache.max_seqs, cache.max_seq_len)
+                   max_batch_tokens, cache.max_seqs, cache.max_seq_len, [p.spec.keep for p in plans])
 
     def __del__(self):
         try:

@@ -83,10 +83,14 @@ _SIGNATURES = {
                          c_void_p, c_void_p, c_long, c_int, c_void_p, c_int, c_float, c_float, c_float, c_void_p, c_void_p, c_int, c_int,
                          c_int, c_int, c_int, c_int, c_void_p],
     "axk_route_topk": [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p],
-    "axk_route_scored": [c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p, c_void_p],
+    "axk_route_scored": [c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_void_p, c_void_p],
     "axk_route_max_tiles": [c_int, c_int, c_int],
     "axk_route_sort": [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p],
-    "axk_route_combine": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_long, c_void_p],
+    "axk_route_combine": [c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_int,
+                          c_void_p, c_long, c_void_p],
+    "axk_tanh_norm": [c_void_p, c_void_p, c_float, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p],
+    "axk_tanh_norm_add": [c_void_p, c_float, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_float, c_void_p, c_int, c_void_p,
+                          c_int, c_int, c_int, c_void_p],
     "axk_gather_rows": [c_void_p, c_long, c_void_p, c_void_p, c_int, c_int, c_void_p],
     "axk_causal_conv": [c_void_p, c_long, c_void_p, c_void_p, c_int, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int,
                         c_int, c_void_p],
@@ -98,6 +102,16 @@ _SIGNATURES = {
                              c_void_p, c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_void_p,
                              c_void_p, c_void_p, c_void_p],
     "axk_gated_group_norm": [c_void_p, c_void_p, c_long, c_void_p, c_int, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
+    "axk_token_shift": [c_void_p, c_void_p, c_int, c_void_p, c_long, c_long, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p],
+    "axk_time_mix_decay": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p],
+    "axk_wkv_scan": [c_void_p, c_long, c_long, c_long, c_long, c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_int,
+                     c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_void_p,
+                     c_void_p, c_void_p, c_void_p],
+    "axk_delta_prepare": [c_void_p, c_long, c_void_p, c_int, c_void_p, c_long, c_long, c_long, c_void_p, c_void_p, c_int, c_int,
+                          c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p],
+    "axk_delta_scan": [c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_long,
+                       c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "axk_head_norm_gate": [c_void_p, c_void_p, c_long, c_void_p, c_int, c_int, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
     "axk_latent_prepare": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_int,
                            c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p],
     "axk_latent_query_rope": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
@@ -110,11 +124,11 @@ _SIGNATURES = {
     "axk_add_scaled": [c_void_p, c_void_p, c_float, c_long, c_void_p],
     "axk_heads_prepare": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_float,
                           c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int,
-                          c_int, c_float, c_int, c_void_p],
+                          c_int, c_float, c_int, c_int, c_void_p],
     "axk_masked_attention_uses_mfma": [c_int, c_int, c_int, c_int, c_int, c_int],
     "axk_masked_attention": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_int, c_int,
                              c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_float, c_float,
-                             c_void_p, c_int, c_void_p, c_long, c_float, c_int, c_int, c_void_p],
+                             c_void_p, c_int, c_void_p, c_long, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
     "axk_concat_round": [c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_void_p],
     "axk_fill_i32": [c_void_p, c_int, c_int, c_void_p],
     "axk_fill_f32": [c_void_p, c_float, c_int, c_void_p],
@@ -167,7 +181,7 @@ class Kernels:
         self.lib.axk_attention_decode_workspace.restype = ctypes.c_long
         self.lib.axk_latent_attention_workspace.argtypes = [c_int, c_int, c_int, c_int, c_int, c_int, c_int]
         self.lib.axk_latent_attention_workspace.restype = ctypes.c_long
-        self.lib.axk_masked_attention_workspace.argtypes = [c_int] * 10
+        self.lib.axk_masked_attention_workspace.argtypes = [c_int] * 11
         self.lib.axk_masked_attention_workspace.restype = ctypes.c_long
         self.lib.axk_packed_elems.argtypes = [c_int, c_int]
         self.lib.axk_packed_elems.restype = ctypes.c_long
@@ -228,7 +242,8 @@ class Kernels:
     # what launches kernels: wrapped while a step is profiled
     _LAUNCHING = ("embed", "rmsnorm", "rope_table", "rope_kv_write", "gemm_qkv_rope", "attention", "attention_prefill",
                   "attention_decode", "gemm", "gemm_normed_glu", "gemm_normed_qkv_rope", "swiglu", "argmax", "topk",
-                  "fill_i32", "fill_f32", "call", "norm_add", "round_rows", "activation", "clamped_glu", "grouped_gemm",
+                  "fill_i32", "fill_f32", "call", "norm_add", "tanh_norm", "tanh_norm_add", "token_shift", "time_mix_decay", "wkv_scan", "delta_prepare", "delta_scan",
+                  "head_norm_gate", "round_rows", "activation", "clamped_glu", "grouped_gemm",
                   "route_topk", "route_sort", "route_combine", "gather_rows", "causal_conv", "gated_scan", "latent_prepare",
                   "latent_query_rope", "latent_attention", "heads_prepare", "masked_attention", "concat_round", "scale_rows",
                   "add_scaled", "state_conv", "state_space_scan", "gated_group_norm", "route_scored", "sum_norm", "layernorm",
@@ -689,6 +704,38 @@ class Kernels:
                                           _ptr(x), _ptr(rounded), x.shape[0], x.shape[1], _stream()))
         return x
 
+    def tanh_norm(self, x: torch.Tensor, norm, out: torch.Tensor, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """out = tanh(alpha x) w + b of float32 rows (`rows`: which of them); norm = (alpha, w, b)."""
+        self._f32(x, "tanh_norm x"); self._elem(out, "tanh_norm out")
+        alpha, w, b = norm
+        n = x.shape[0]
+        if rows is not None:
+            self._i32(rows, "tanh_norm rows")
+            n = rows.numel()
+        if x.dim() != 2 or out.shape != (n, x.shape[1]) or not out.is_contiguous() or w.numel() != x.shape[1] or b.numel() != x.shape[1]:
+            raise KernelError(f"tanh_norm: x {tuple(x.shape)}, out {tuple(out.shape)}, vectors of {w.numel()} and {b.numel()}")
+        self._check(self.lib.axk_tanh_norm(_ptr(x), _ptr(rows), float(alpha), _ptr(w), self._vec_flag(w, "tanh_norm w"), _ptr(b),
+                                           self._vec_flag(b, "tanh_norm b"), _ptr(out), n, x.shape[1], _stream()))
+        return out
+
+    def tanh_norm_add(self, y: torch.Tensor, norm, x: torch.Tensor, following=None) -> torch.Tensor:
+        """x += tanh(alpha y) w + b, norm = (alpha, w, b); `following` = ((alpha, w, b), values): values also gets
+        that norm of the new x in the compute dtype."""
+        self._f32(y, "tanh_norm_add y"); self._f32(x, "tanh_norm_add x")
+        next_norm, values = following if following is not None else ((0.0, None, None), None)
+        if y.shape != x.shape or y.dim() != 2 or any(v is not None and v.numel() != x.shape[1] for v in (*norm[1:], *next_norm[1:])):
+            raise KernelError(f"tanh_norm_add: y {tuple(y.shape)}, x {tuple(x.shape)}, or vectors of another width")
+        if values is not None:
+            self._elem(values, "tanh_norm_add values")
+            if values.shape != x.shape or not values.is_contiguous():
+                raise KernelError(f"tanh_norm_add: values {tuple(values.shape)} are not {tuple(x.shape)} contiguous")
+        flag = lambda v: self._vec_flag(v, "tanh_norm_add vector")
+        self._check(self.lib.axk_tanh_norm_add(
+            _ptr(y), float(norm[0]), _ptr(norm[1]), flag(norm[1]), _ptr(norm[2]), flag(norm[2]), _ptr(x), _ptr(values),
+            float(next_norm[0]), _ptr(next_norm[1]), flag(next_norm[1]), _ptr(next_norm[2]), flag(next_norm[2]), x.shape[0],
+            x.shape[1], _stream()))
+        return x
+
     NORM_KINDS = {"rms": 0, "layer": 1}
 
     def sum_norm(self, y: torch.Tensor, alpha: float, gain: torch.Tensor, eps: float, kind: str, x: torch.Tensor,
@@ -749,7 +796,7 @@ class Kernels:
         self._check(self.lib.axk_round_rows(_ptr(x), _ptr(out), x.numel(), _stream()))
         return out
 
-    ACTIVATIONS = {"gelu_tanh": 0, "gelu_erf": 1}
+    ACTIVATIONS = {"gelu_tanh": 0, "gelu_erf": 1, "relu_squared": 2}
 
     def activation(self, v: torch.Tensor, kind: str = "gelu_tanh") -> torch.Tensor:
         self._elem(v, "activation")
@@ -841,8 +888,9 @@ class Kernels:
         self._check(self.lib.axk_route_topk(_ptr(logits), T, E, top, _ptr(experts), _ptr(weights), _stream()))
 
     def route_scored(self, logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int, keep: int, scale: float,
-                     experts: torch.Tensor, weights: torch.Tensor, normalize: bool = True, n_experts: Optional[int] = None) -> None:
-        """Sigmoid scores, the choice by score + correction among the `keep` best of `groups` groups of
+                     experts: torch.Tensor, weights: torch.Tensor, normalize: bool = True, n_experts: Optional[int] = None,
+                     softmax: bool = False) -> None:
+        """Sigmoid scores (with `softmax`: the softmax over all experts), the choice by score + correction among the `keep` best of `groups` groups of
         neighbouring experts, weights the chosen scores over their sum (without `normalize`: the scores
         themselves), times scale (axk_route_scored).  `n_experts`: the leading columns of `logits` that
         are router logits (all, unless given)."""
@@ -859,7 +907,7 @@ class Kernels:
             if correction.numel() != E:
                 raise KernelError(f"route_scored: a correction of {correction.numel()} for {E} experts")
         self._check(self.lib.axk_route_scored(_ptr(logits), logits.stride(0), _ptr(correction), T, E, top, int(groups), int(keep),
-                                              float(scale), 1 if normalize else 0, _ptr(experts), _ptr(weights), _stream()))
+                                              float(scale), 1 if normalize else 0, 1 if softmax else 0, _ptr(experts), _ptr(weights), _stream()))
 
     def route_max_tiles(self, n_pairs: int, n_experts: int, tile_rows: int = 16) -> int:
         return int(self.lib.axk_route_max_tiles(n_pairs, n_experts, tile_rows))
@@ -887,10 +935,11 @@ class Kernels:
 
     def route_combine(self, rows: torch.Tensor, weights: Optional[torch.Tensor], y: torch.Tensor, accumulate: bool = False,
                       place_of: Optional[torch.Tensor] = None, top: Optional[int] = None, extra: Optional[torch.Tensor] = None,
-                      extra_gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                      extra_gate: Optional[torch.Tensor] = None, identity=None) -> torch.Tensor:
         """y[t] (+)= sum_k weights[t, k] rows[t top + k] (weights None: all 1, `top` then says how many rows a
         token) + extra[t] sigmoid(extra_gate[t]) (extra: float32 like y; extra_gate: a float32 column, one logit a
-        token, rows may be strided; None: no gate)."""
+        token, rows may be strided; None: no gate).  `identity` = (chosen experts int32 [T, top], n, input [T, width] in
+        the compute dtype): the row of a pair whose expert is n or more is its token's row of the input."""
         self._f32(rows, "expert rows"); self._f32(y, "combine y")
         if place_of is not None:
             self._i32(place_of, "combine place_of")
@@ -914,8 +963,14 @@ class Kernels:
                 gate_stride = extra_gate.stride(0)
         elif extra_gate is not None:
             raise KernelError("route_combine: a gate without the rows it gates")
+        chosen, n_listed, given = identity if identity is not None else (None, 0, None)
+        if identity is not None:
+            self._i32(chosen, "combine experts"); self._elem(given, "combine input")
+            if chosen.numel() != T * top or given.shape != y.shape or given.stride(1) != 1:
+                raise KernelError(f"route_combine: experts {tuple(chosen.shape)}, input {tuple(given.shape)} for y {tuple(y.shape)}")
         self._check(self.lib.axk_route_combine(_ptr(rows), _ptr(weights), _ptr(y), T, top, y.shape[1], 1 if accumulate else 0,
-                                               _ptr(place_of), _ptr(extra), _ptr(extra_gate), gate_stride, _stream()))
+                                               _ptr(place_of), _ptr(extra), _ptr(extra_gate), gate_stride, _ptr(chosen), int(n_listed), _ptr(given),
+                                               0 if given is None else given.stride(0), _stream()))
         return y
 
     # ------------------------------------------------------------------ convolution and recurrence with per-request state
@@ -1040,6 +1095,118 @@ class Kernels:
                                                   float(eps), _ptr(out), T, W, int(parts), _stream()))
         return out
 
+    # ------------------------------------------------------------------ time mixing and the delta rule, with per-request state
+    def _state_rows(self, state, seq_rows, positions, T, what) -> None:
+        self._f32(state, what + " state"); self._i32(seq_rows, "seq_rows"); self._i32(positions, "positions")
+        if state.dim() != 2 or seq_rows.numel() != T or positions.numel() != T:
+            raise KernelError(f"{what}: state {tuple(state.shape)}, {seq_rows.numel()} slots for {T} tokens")
+
+    def token_shift(self, h, mu, state, copy_elems: int, tail_at: int, positions, seq_rows, out) -> torch.Tensor:
+        """out[s, t] = h[t] + (h'[t] - h[t]) mu[s], h' the request's row before, from the float32 state rows where the
+        step does not hold it (see csrc/time_mix.hip): h [T, W] and out [n, T, W] in the compute dtype, mu float32 [n, W]."""
+        self._elem(h, "token_shift h"); self._elem(out, "token_shift out"); self._f32(mu, "token_shift mu")
+        T, W = h.shape
+        self._state_rows(state, seq_rows, positions, T, "token_shift")
+        if not h.is_contiguous() or mu.dim() != 2 or mu.shape[1] != W or out.shape != (mu.shape[0], T, W) or not out.is_contiguous():
+            raise KernelError(f"token_shift: h {tuple(h.shape)}, mu {tuple(mu.shape)}, out {tuple(out.shape)}")
+        self._check(self.lib.axk_token_shift(_ptr(h), _ptr(mu), mu.shape[0], _ptr(state), state.stride(0), int(copy_elems), int(tail_at),
+                                             _ptr(positions), _ptr(seq_rows), _ptr(out), T, W, _stream()))
+        return out
+
+    def time_mix_decay(self, low, w2, w0, w) -> torch.Tensor:
+        """w[t, c] = exp(-exp(w0[c] + sum_k w2[c, k] tanh(low[t, k]))): low [T, rank] and w [T, channels] float32, w2
+        [channels, rank] in the compute dtype."""
+        self._f32(low, "decay low"); self._elem(w2, "decay w2"); self._f32(w, "decay w")
+        T, C = w.shape
+        if low.dim() != 2 or low.shape[0] != T or w2.shape != (C, low.shape[1]) or not w2.is_contiguous() or w0.numel() != C:
+            raise KernelError(f"time_mix_decay: low {tuple(low.shape)}, w2 {tuple(w2.shape)}, w {tuple(w.shape)}")
+        self._check(self.lib.axk_time_mix_decay(_ptr(low), _ptr(w2), _ptr(w0), self._vec_flag(w0, "decay w0"), _ptr(w), T, C,
+                                                low.shape[1], _stream()))
+        return w
+
+    def wkv_scan(self, rows, r_at: int, k_at: int, v_at: int, w, u, state, copy_elems: int, tail_at: int, spans, positions, seq_rows,
+                 h_in, y, heads: int, keys: int, values: int, segments=None) -> torch.Tensor:
+        """The decayed state of time mixing over each request's tokens (see csrc/time_mix.hip): rows float32 [T, .] with r
+        and k of heads keys columns and v of heads values; w [T, heads keys], u [heads, keys], y [T, heads values] float32;
+        spans int32 [n, 3] = (slot, first token, tokens) or None (each token a request of its own in slot seq_rows[t]); h_in
+        [T, W]: the mixer's input, whose last row a request is kept.  `segments` as in `state_space_scan`."""
+        for t, what in ((w, "wkv w"), (u, "wkv u"), (y, "wkv y")):
+            self._f32(t, what)
+        self._f32_rows(rows, "wkv rows"); self._elem(h_in, "wkv h_in")
+        T = rows.shape[0]
+        self._state_rows(state, seq_rows, positions, T, "wkv_scan")
+        if w.shape != (T, heads * keys) or u.numel() != heads * keys or y.shape != (T, heads * values) or h_in.shape[0] != T \
+                or not h_in.is_contiguous():
+            raise KernelError(f"wkv_scan: w {tuple(w.shape)}, u {tuple(u.shape)}, y {tuple(y.shape)}, h_in {tuple(h_in.shape)}")
+        n = T
+        if spans is not None:
+            self._i32(spans, "scan spans")
+            n = spans.shape[0]
+        segs = spans5 = ends = decays = rc = None
+        n_segs = longest = 0
+        if segments is not None:
+            segs, spans5, longest = segments
+            self._i32(segs, "scan segments"); self._i32(spans5, "scan requests")
+            n_segs = segs.shape[0]
+            if spans is None or segs.dim() != 2 or segs.shape[1] != 4 or spans5.shape != (n, 5):
+                raise KernelError(f"wkv_scan: segments {tuple(segs.shape)} of requests {tuple(spans5.shape)} for {n} requests")
+            take = lambda *shape: torch.empty(shape, dtype=torch.float32, device=y.device)
+            ends, decays, rc = take(n_segs, heads, values, keys), take(n_segs, heads, keys), take(T, heads * keys)
+        self._check(self.lib.axk_wkv_scan(
+            _ptr(rows), rows.stride(0), int(r_at), int(k_at), int(v_at), _ptr(w), _ptr(u), _ptr(state), state.stride(0), int(copy_elems),
+            int(tail_at), _ptr(spans), n, _ptr(positions), _ptr(seq_rows), _ptr(h_in), h_in.shape[1], _ptr(y), heads, keys, values,
+            _ptr(segs), n_segs, int(longest), _ptr(spans5), _ptr(ends), _ptr(decays), _ptr(rc), _stream()))
+        return y
+
+    def delta_prepare(self, rows, w, state, copy_elems: int, tail_at: int, positions, seq_rows, beta_at: int, decay_at: int, a_log,
+                      dt_bias, u, terms, heads: int, kv_heads: int, keys: int, values: int, q_scale: float) -> None:
+        """The delta rule's operands from the projections' float32 rows [T, .]: the channels [q | k | v] convolved
+        (w [channels, taps] in the compute dtype), through silu, queries and keys of length 1 a head, into u [T, channels];
+        terms [T, heads, 2] = (g, beta) (see csrc/delta_rule.hip)."""
+        self._f32_rows(rows, "delta rows"); self._elem(w, "delta conv"); self._f32(u, "delta u"); self._f32(terms, "delta terms")
+        T, C = u.shape
+        self._state_rows(state, seq_rows, positions, T, "delta_prepare")
+        if C != 2 * kv_heads * keys + heads * values or rows.shape[0] != T or w.dim() != 2 or w.shape[0] != C or not w.is_contiguous() \
+                or terms.shape != (T, heads, 2) or a_log.numel() != heads or dt_bias.numel() != heads:
+            raise KernelError(f"delta_prepare: rows {tuple(rows.shape)}, conv {tuple(w.shape)}, u {tuple(u.shape)}, terms {tuple(terms.shape)}")
+        self._check(self.lib.axk_delta_prepare(
+            _ptr(rows), rows.stride(0), _ptr(w), w.shape[1], _ptr(state), state.stride(0), int(copy_elems), int(tail_at), _ptr(positions),
+            _ptr(seq_rows), int(beta_at), int(decay_at), _ptr(a_log), self._vec_flag(a_log, "A_log"), _ptr(dt_bias),
+            self._vec_flag(dt_bias, "dt bias"), _ptr(u), _ptr(terms), T, heads, kv_heads, keys, values, float(q_scale), _stream()))
+
+    def delta_scan(self, u, terms, state, copy_elems: int, tail_at: int, spans, positions, seq_rows, conv_in, y, heads: int,
+                   kv_heads: int, keys: int, values: int, taps: int) -> torch.Tensor:
+        """The gated delta rule over each request's tokens (see csrc/delta_rule.hip): u [T, channels] and terms [T, heads, 2]
+        float32; spans int32 [n, 3] or None as in the other scans; conv_in: the convolutions' inputs (float32, rows may be
+        strided), kept for the next step; y [T, heads values] float32."""
+        for t, what in ((u, "delta u"), (terms, "delta terms"), (y, "delta y")):
+            self._f32(t, what)
+        self._f32_rows(conv_in, "delta conv_in")
+        T, C = u.shape
+        self._state_rows(state, seq_rows, positions, T, "delta_scan")
+        if C != 2 * kv_heads * keys + heads * values or terms.shape != (T, heads, 2) or y.shape != (T, heads * values) \
+                or conv_in.shape[0] != T or conv_in.shape[1] < C:
+            raise KernelError(f"delta_scan: u {tuple(u.shape)}, terms {tuple(terms.shape)}, y {tuple(y.shape)}, conv_in {tuple(conv_in.shape)}")
+        n = T
+        if spans is not None:
+            self._i32(spans, "scan spans")
+            n = spans.shape[0]
+        self._check(self.lib.axk_delta_scan(
+            _ptr(u), _ptr(terms), _ptr(state), state.stride(0), int(copy_elems), int(tail_at), _ptr(spans), n, _ptr(positions),
+            _ptr(seq_rows), _ptr(conv_in), conv_in.stride(0), _ptr(y), heads, kv_heads, keys, values, int(taps), _stream()))
+        return y
+
+    def head_norm_gate(self, y, gate, gain, eps: float, out, heads: int) -> torch.Tensor:
+        """out = (y / sqrt(mean y^2 + eps)) gain silu(gate), the mean over each of `heads` equal parts of a row: y float32
+        [T, W], gate float32 [T, W] (rows may be strided), gain of a part's width (shared) or of W, out in the compute dtype."""
+        self._f32(y, "head norm y"); self._f32_rows(gate, "head norm gate"); self._elem(out, "head norm out")
+        T, W = y.shape
+        if W % heads or gate.shape != (T, W) or out.shape != (T, W) or not out.is_contiguous() or gain.numel() not in (W, W // heads):
+            raise KernelError(f"head_norm_gate: y {tuple(y.shape)}, gate {tuple(gate.shape)}, a gain of {gain.numel()}, {heads} heads")
+        self._check(self.lib.axk_head_norm_gate(_ptr(y), _ptr(gate), gate.stride(0), _ptr(gain), self._vec_flag(gain, "head norm gain"),
+                                                1 if gain.numel() == W else 0, float(eps), _ptr(out), T, heads, W // heads, _stream()))
+        return out
+
     # ------------------------------------------------------------------ attention over a latent cache
     def latent_prepare(self, fused, q_at, q_rank, kv_at, rank, rot, rot_dims, q_gain, kv_gain, eps, table, positions, seq_rows,
                        block_table, cache, page_size, cq, write_kv=True, neighbours=False, magnitude=1.0) -> None:
@@ -1105,9 +1272,11 @@ class Kernels:
             raise KernelError(f"{what}: cache {tuple(cache.shape)} is not [pages, 1, {page_size}, {row}]")
 
     def heads_prepare(self, proj, q_at, n_q, k_at, n_k, v_at, v_width, dim, q_gain, k_gain, eps, rot, neighbours, magnitude,
-                      table, positions, seq_rows, block_table, cache, page_size, q_out, write_kv=True, q_temp=None) -> None:
+                      table, positions, seq_rows, block_table, cache, page_size, q_out, write_kv=True, q_temp=None,
+                      norm_rows=False) -> None:
         """The projections' float32 rows into queries (q_out) and the page's keys and values: see
-        axk_heads_prepare in csrc/api.h.  `q_temp` = (coef, every): a query's temperature by its position."""
+        axk_heads_prepare in csrc/api.h.  `q_temp` = (coef, every): a query's temperature by its position.
+        `norm_rows`: the norm goes over all query (all key) units of a token at once."""
         self._f32(proj, "heads proj"); self._f32(table, "rope table"); self._i32(positions, "positions")
         self._i32(seq_rows, "seq_rows"); self._i32(block_table, "block_table"); self._elem(q_out, "heads q_out")
         T = positions.numel()
@@ -1116,24 +1285,26 @@ class Kernels:
         self._check_heads_cache(cache, page_size, n_k * dim + v_width, "heads_prepare")
         if q_out.shape != (T, n_q * dim) or not q_out.is_contiguous():
             raise KernelError(f"heads_prepare: q_out {tuple(q_out.shape)} is not [{T}, {n_q * dim}]")
-        for gain in (q_gain, k_gain):
-            if gain is not None and gain.numel() != dim:
-                raise KernelError(f"heads_prepare: a gain of {gain.numel()} for units of {dim}")
+        for gain, units in ((q_gain, n_q), (k_gain, n_k)):
+            if gain is not None and gain.numel() != (units * dim if norm_rows else dim):
+                raise KernelError(f"heads_prepare: a gain of {gain.numel()} for {units} units of {dim}")
         self._check(self.lib.axk_heads_prepare(
             _ptr(proj), proj.stride(0), q_at, n_q, k_at, n_k, v_at, v_width, dim, _ptr(q_gain), self._vec_flag(q_gain, "q gain"),
             _ptr(k_gain), self._vec_flag(k_gain, "k gain"), float(eps), rot, 1 if neighbours else 0, float(magnitude), _ptr(table),
             _ptr(positions), _ptr(seq_rows), _ptr(block_table), block_table.shape[-1], _ptr(cache), page_size, _ptr(q_out), T,
-            1 if write_kv else 0, float(q_temp[0]) if q_temp else 0.0, int(q_temp[1]) if q_temp else 0, _stream()))
+            1 if write_kv else 0, float(q_temp[0]) if q_temp else 0.0, int(q_temp[1]) if q_temp else 0, 1 if norm_rows else 0,
+            _stream()))
 
     def masked_attention_uses_mfma(self, heads, kv_heads, maps, dim, vdim, page_size) -> bool:
         return bool(self.lib.axk_masked_attention_uses_mfma(heads, kv_heads, maps, dim, vdim, page_size))
 
     def masked_attention(self, q, cache, block_table, positions, seq_rows, out, heads, kv_heads, maps, dim, vdim, page_size,
                          mask, mask_size, scale, softcap=0.0, lam=0.0, out_scale=1.0, eps=0.0, gate=None, tiles=None,
-                         sink=None, gate_per_head=False, span=0) -> torch.Tensor:
+                         sink=None, gate_per_head=False, span=0, keep=0) -> torch.Tensor:
         """q [T, heads maps dim] -> out [T, heads vdim] (compute dtype): see axk_masked_attention in csrc/api.h.
         `gate`: float32 rows (a view whose rows may be strided) of heads vdim gate logits (of heads logits with
-        `gate_per_head`), or None.  `sink`: the score of a key without a value in every softmax, or None.  `span`
+        `gate_per_head`), or None.  `sink`: the score of a key without a value in every softmax (a number, or
+        float32 [heads]: one a head), or None.  `keep` (window masks): the first positions that stay visible.  `span`
         (causal masks): the positions the step's longest row sees, so that a step of few tokens can run a token's
         blocks of positions side by side; 0: a wave walks them."""
         self._elem(q, "attention q"); self._elem(out, "attention out")
@@ -1156,13 +1327,19 @@ class Kernels:
             self._i32(tiles, "attention tiles")
             n_tiles = tiles.shape[0]
         need = int(self.lib.axk_masked_attention_workspace(T, heads, kv_heads, maps, dim, vdim, page_size, self.MASKS[mask],
-                                                           int(mask_size), int(span)))
+                                                           int(mask_size), int(keep), int(span)))
+        sinks = sink if isinstance(sink, torch.Tensor) else None
+        if sinks is not None:
+            self._f32(sinks, "attention sinks")
+            if sinks.numel() != heads:
+                raise KernelError(f"masked_attention: {sinks.numel()} sinks for {heads} heads")
         partial = torch.empty(need, dtype=torch.float32, device=out.device) if need else None
         self._check(self.lib.axk_masked_attention(
             _ptr(q), _ptr(cache), _ptr(block_table), block_table.shape[-1], _ptr(positions), _ptr(seq_rows), _ptr(gate),
             gate_stride, _ptr(out), T, heads, kv_heads, maps, dim, vdim, page_size, self.MASKS[mask], int(mask_size), float(scale),
             float(softcap), float(lam), float(out_scale), float(eps), _ptr(tiles), n_tiles, _ptr(partial), need,
-            float("-inf") if sink is None else float(sink), 1 if gate_per_head else 0, int(span), _stream()))
+            float("-inf") if sink is None or sinks is not None else float(sink), _ptr(sinks), 1 if gate_per_head else 0, int(keep),
+            int(span), _stream()))
         return out
 
     def fill_i32(self, dst: torch.Tensor, value: int) -> None:

@@ -63,19 +63,29 @@ class DecoderModel:
         group_of_key: Dict[Tuple, int] = {}
         specs, counts = [], []
         where: Dict[int, Tuple[int, int]] = {}      # cache id -> (group, index in group)
-        writer_spec: Dict[int, object] = {}
+        needs: Dict[int, object] = {}               # cache id -> what its writer and its readers need of it
         for run in self.order:                      # first the runs that store
             cs = self.blocks[run.layer].mixer.cache_spec()
             if cs is None or not run.writes_cache:
                 continue
-            if run.cache in where:
+            if run.cache in needs:
                 raise ConfigError(f"two runs store into cache {run.cache}")
+            needs[run.cache] = cs
+        for run in self.order:                      # then those that only read
+            cs = self.blocks[run.layer].mixer.cache_spec()
+            if cs is None or run.writes_cache:
+                continue
+            if run.cache not in needs:
+                raise ConfigError(f"a run of layer {run.layer} reads cache {run.cache}, which no run stores")
+            if needs[run.cache].shape_key() != cs.shape_key():
+                raise ConfigError(f"layer {run.layer} cannot read cache {run.cache}: its shape differs")
+            needs[run.cache] = needs[run.cache].widened(cs)
+        for cache, cs in needs.items():
             g = group_of_key.setdefault(cs.group_key(), len(specs))
             if g == len(specs):
                 specs.append(cs)
                 counts.append(0)
-            where[run.cache] = (g, counts[g])
-            writer_spec[run.cache] = cs
+            where[cache] = (g, counts[g])
             counts[g] += 1
         bindings, state_elems = [], []
         for run in self.order:
@@ -83,10 +93,6 @@ class DecoderModel:
             cs, ss = mixer.cache_spec(), mixer.state_spec()
             b = CacheBinding(writes=run.writes_cache)
             if cs is not None:
-                if run.cache not in where:
-                    raise ConfigError(f"a run of layer {run.layer} reads cache {run.cache}, which no run stores")
-                if writer_spec[run.cache].group_key() != cs.group_key():
-                    raise ConfigError(f"layer {run.layer} cannot read cache {run.cache}: its shape differs")
                 b.group, b.index = where[run.cache]
             if ss is not None:
                 b.state_index = len(state_elems)

@@ -19,7 +19,7 @@ configuration then names it in a `PartSpec`.
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from typing import Any, Callable, Dict, List, Optional, Sequence, Tuple
 
 from ..config.base import ConfigError, PartSpec
@@ -40,16 +40,28 @@ class TensorDecl:
 class CacheSpec:
     """Paged per-token storage a mixer wants for one run: `entries` arrays (keys and values:
     2) of `heads` x `head_dim` elements per position.  `window` > 0: only the last `window`
-    positions are ever read, so earlier pages can be given back.  `dtype`: the element type of
+    positions are ever read, so earlier pages can be given back, but for those of the first `keep`
+    positions, which stay readable.  A run that reads another run's cache says what it reads of it with
+    a spec of its own: the cache then keeps what any of its readers needs.  `dtype`: the element type of
     the pages ("float32", "bfloat16", "int8", ...); None: the engine's compute dtype."""
     entries: int
     heads: int
     head_dim: int
     window: int = 0
     dtype: Optional[str] = None
+    keep: int = 0
+
+    def shape_key(self):
+        return (self.entries, self.heads, self.head_dim, self.dtype)
 
     def group_key(self):
-        return (self.entries, self.heads, self.head_dim, self.window, self.dtype)
+        return self.shape_key() + (self.window, self.keep)
+
+    def widened(self, other: "CacheSpec") -> "CacheSpec":
+        """Storage of this shape that keeps what this spec and `other` read."""
+        if self.window == 0 or other.window == 0:
+            return replace(self, window=0, keep=0)
+        return replace(self, window=max(self.window, other.window), keep=max(self.keep, other.keep))
 
 
 @dataclass(frozen=True)

@@ -234,7 +234,58 @@ class ParallelBlock(Block):
             self.feed_forward.forward(ctx, h, x)
 
 
+class SandwichNormBlock(Block):
+    """x += norm1b(mixer(norm1(x))); x += norm2b(feed_forward(norm2(x))): a norm on each sublayer's input and one on its
+    output (a layer may have no feed-forward, and then no second pair).  The outer norm and the sum are one 32-bit pass
+    over the sublayer's 32-bit output (`Norm.add_to`: RMS norms and TanhNorm); where the norm that reads the sum is a
+    TanhNorm that pass writes it too, the next block's first norm included."""
+    graph_safe = True
+    norm_names = ("norm1", "norm1b", "norm2", "norm2b")
+
+    def __init__(self, norm_factory, mixer, feed_forward, prefix):
+        super().__init__(norm_factory, mixer, feed_forward, prefix)
+        names = self.norm_names if feed_forward is not None else self.norm_names[:2]
+        self.norms = [norm_factory(name) for name in names]
+        for norm in self.norms[1::2]:
+            if not hasattr(norm, "add_to"):
+                raise ConfigError(f"a norm on a sublayer's output adds it into the stream ({type(norm).__name__} cannot)")
+
+    def parts(self):
+        return [p for p in (*self.norms, self.mixer, self.feed_forward) if p is not None]
+
+    def tensors(self) -> List[TensorDecl]:
+        return [d for p in self.parts() for d in p.tensors()]
+
+    def load(self, store, rt) -> None:
+        for part in self.parts():
+            part.load(store, rt)
+
+    def first_norm(self):
+        return self.norms[0]
+
+    @staticmethod
+    def following_of(ctx, part, norm, n_rows: int):
+        """The norm behind a sum as work for the pass that makes the sum, whatever part's output it adds."""
+        return norm.following_values(ctx, n_rows) if hasattr(norm, "following_values") else None
+
+    _run = staticmethod(SublayerNormBlock._run)
+
+    def forward(self, ctx, binding: CacheBinding, x, normed=None, following=None) -> None:
+        h = normed if normed is not None else self.norms[0].forward(ctx, x)
+        y = ctx.ws.take(tuple(x.shape), torch.float32)
+        self._run(self.mixer, ctx, y, binding, h)
+        if self.feed_forward is None:
+            self.norms[1].add_to(ctx, y, x, following)
+            return
+        second = self.following_of(ctx, None, self.norms[2], x.shape[0])
+        self.norms[1].add_to(ctx, y, x, second)
+        h = second.values if second is not None else self.norms[2].forward(ctx, x)
+        self._run(self.feed_forward, ctx, y, h)
+        self.norms[3].add_to(ctx, y, x, following)
+
+
 register_block("prenorm", PreNormBlock)
+register_block("sandwich_norm", SandwichNormBlock)
 register_block("parallel", ParallelBlock)
 register_block("prenorm_short_names", ShortNamedPreNormBlock)
 register_block("sublayer_norm", SublayerNormBlock)

@@ -1,0 +1,93 @@
+"""The gated delta rule (the linear attention of Gated-DeltaNet-like models), with its state in the cache manager's
+state slots.
+
+From the input h one product gives [q | k | v | beta | decay | gate]: q and k of kv_heads x dim, v and the gate of
+heads x vdim, the others a number a head; head a uses query and key head a // (heads / kv_heads).  q, k and v pass a
+causal convolution of `conv` taps per channel (no bias), then silu; q and k become vectors of length 1 a head,
+x / sqrt(sum(x^2) + 1e-6), q also times dim^(-1/2).  With beta = sigmoid(.) and
+g = exp(-exp(A_log) softplus(. + dt_bias)), per head
+
+    S <- g S,  u = beta (v - S^T k),  S <- S + k u^T,  o = S^T q          (S: dim x vdim, zero at first)
+
+and the output is W_o (o / sqrt(mean(o^2) + eps) head by head, times a gain of vdim shared by the heads, times
+silu(gate)).  The product's rows, the convolutions' results, the step sizes, the state and the norm are 32-bit; a
+request's state row holds S and the convolutions' last conv - 1 inputs, twice: the state behind position p in copy
+p & 1, so that a decoding step reads one copy and writes the other and may be run again with the same result.
+
+Parameters: `hidden_size`, `heads`, `kv_heads`, `dim`, `vdim`, `conv`, `eps`, `names` (the tensors' names under the
+prefix: scope "mix.", q, k, v, b, a, g, A_log, dt_bias, norm, o; a convolution is the name + ".conv").
+`forward(..., accumulate=False)` stores the 32-bit output instead of adding it.
+"""
+from __future__ import annotations
+
+from typing import List
+
+import torch
+
+from ..config.base import ConfigError
+from ..kernels import MODE_ADD_F32, MODE_STORE_F32
+from .base import CacheBinding, Mixer, StateSpec, TensorDecl, register_mixer
+from .recurrent import step_spans
+
+
+class GatedDeltaRule(Mixer):
+    graph_safe = True
+    stores_output = True
+
+    def __init__(self, params, prefix=""):
+        super().__init__(params, prefix)
+        p = params
+        self.hidden, self.heads, self.kv_heads = int(p["hidden_size"]), int(p["heads"]), int(p["kv_heads"])
+        self.dim, self.vdim, self.taps, self.eps = int(p["dim"]), int(p["vdim"]), int(p["conv"]), float(p["eps"])
+        if self.kv_heads < 1 or self.heads % self.kv_heads:
+            raise ConfigError(f"{self.heads} heads are not a multiple of {self.kv_heads} query/key heads")
+        if not 1 <= self.dim <= 256:
+            raise ConfigError(f"the delta rule with keys of {self.dim} dims: the scan's kernel takes 1 to 256")
+        if self.taps < 1:
+            raise ConfigError(f"a convolution of {self.taps} taps")
+        self.qk, self.inner = self.kv_heads * self.dim, self.heads * self.vdim
+        self.channels = 2 * self.qk + self.inner                   # what the convolutions see: q, k, v
+        self.beta_at, self.decay_at = self.channels, self.channels + self.heads
+        self.gate_at = self.channels + 2 * self.heads
+        self.tail_at = self.inner * self.dim                       # a copy of the state: S, then the kept inputs
+        self.copy_elems = -(-(self.tail_at + (self.taps - 1) * self.channels) // 4) * 4
+        names = p.get("names", {})
+        base = prefix + names.get("scope", "mix.")
+        self.n = {k: base + names.get(k, k) for k in ("q", "k", "v", "b", "a", "g", "A_log", "dt_bias", "norm", "o")}
+
+    def tensors(self) -> List[TensorDecl]:
+        n, W = self.n, self.hidden
+        widths = {"q": self.qk, "k": self.qk, "v": self.inner, "b": self.heads, "a": self.heads, "g": self.inner}
+        return ([TensorDecl(n[k], (rows, W)) for k, rows in widths.items()]
+                + [TensorDecl(n[k] + ".conv", (widths[k], self.taps)) for k in ("q", "k", "v")]
+                + [TensorDecl(n["A_log"], (self.heads,), "bias"), TensorDecl(n["dt_bias"], (self.heads,), "bias"),
+                   TensorDecl(n["norm"], (self.vdim,), "gain"), TensorDecl(n["o"], (W, self.inner))])
+
+    def state_spec(self) -> StateSpec:
+        return StateSpec(2 * self.copy_elems)
+
+    def load(self, store, rt) -> None:
+        n = self.n
+        self.w_in = rt.k.prepare_weight(store.fused_matrix([n[k] for k in ("q", "k", "v", "b", "a", "g")]))
+        self.conv_w = store.fused_matrix([n[k] + ".conv" for k in ("q", "k", "v")])
+        self.a_log, self.dt_bias, self.gain = store.vector(n["A_log"]), store.vector(n["dt_bias"]), store.vector(n["norm"])
+        self.w_o = rt.k.prepare_weight(store.matrix(n["o"]))
+        store.forget(n["o"])
+
+    def forward(self, ctx, binding: CacheBinding, h, out, accumulate: bool = True) -> None:
+        k, T, f32 = ctx.rt.k, h.shape[0], torch.float32
+        state = ctx.cache.state(binding.state_index)
+        rows = ctx.ws.take((T, self.gate_at + self.inner), f32)
+        k.gemm(h, self.w_in, rows, None, MODE_STORE_F32)
+        u, terms = ctx.ws.take((T, self.channels), f32), ctx.ws.take((T, self.heads, 2), f32)
+        k.delta_prepare(rows, self.conv_w, state, self.copy_elems, self.tail_at, ctx.positions, ctx.seq_rows, self.beta_at, self.decay_at,
+                        self.a_log, self.dt_bias, u, terms, self.heads, self.kv_heads, self.dim, self.vdim, self.dim ** -0.5)
+        y = ctx.ws.take((T, self.inner), f32)
+        k.delta_scan(u, terms, state, self.copy_elems, self.tail_at, step_spans(ctx), ctx.positions, ctx.seq_rows, rows, y, self.heads,
+                     self.kv_heads, self.dim, self.vdim, self.taps)
+        gated = ctx.ws.take((T, self.inner), ctx.rt.dtype)
+        k.head_norm_gate(y, rows[:, self.gate_at:], self.gain, self.eps, gated, self.heads)
+        k.gemm(gated, self.w_o, out, None, MODE_ADD_F32 if accumulate else MODE_STORE_F32)
+
+
+register_mixer("gated_delta_rule", GatedDeltaRule)

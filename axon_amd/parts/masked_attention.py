@@ -10,29 +10,36 @@ i // (heads / kv_heads).  What a configuration may turn on, each on its own:
   `dim`), and rms(o) = o / sqrt(mean(o^2) + eps) over the head's `vdim` outputs, no gain;
 * `values` = "keys": there is no Wv, the values are the keys as projected (before norm and
   rotation), so `vdim` = `dim`; "projected": v = Wv h (+ bv) of `vdim` a kv head;
-* `qk_norm`: per head, q and k go through an RMS norm over `dim` with a gain of `dim` shared by
-  all heads (`q.norm`, `k.norm`), before the rotation;
+* `qk_norm`: q and k go through an RMS norm with a gain (`q.norm`, `k.norm`), before the rotation:
+  per head over `dim` with a gain of `dim` shared by all heads (true, or "heads"), or over all rows
+  of q (of k) at once with a gain for every one of them ("rows");
 * `position`: a rotary encoding (its `pairing`, scaling and magnitude are the encoding's own);
-* `mask`: {"kind": "causal"}, {"kind": "window", "size": n} (position i sees 0 <= i - j < n) or
+* `mask`: {"kind": "causal"}, {"kind": "window", "size": n, "keep": m} (position i sees 0 <= i - j < n,
+  and every j <= i below `keep`, 0 unless given) or
   {"kind": "chunk", "size": n} (j <= i in the same chunk, floor(i / n) = floor(j / n), counted
   from position 0 of the request);
 * `softcap` c > 0: score <- c tanh(score / c), after the scale;
-* `sink` (a number): every softmax has one more key of that score, which has no value:
-  p_j = exp(s_j) / (exp(sink) + sum exp(s_j')); 0 adds one to the denominator;
+* `sink`: every softmax has one more key of that score, which has no value:
+  p_j = exp(s_j) / (exp(sink) + sum exp(s_j')); a number (0 adds one to the denominator), or "heads": the
+  tensor `sink` of one score a head;
 * `q_temp` = {"coef": c, "every": n}: the query at position p is multiplied by
   1 + c ln(floor((p + 1) / n) + 1), in 32-bit, behind norm and rotation;
 * `gate`: the concatenated heads are multiplied by sigmoid(Wg h) before the output projection, a number
-  an element (true, or "elements": Wg has heads vdim rows) or a number a head ("heads": Wg has heads rows).
+  an element (true, or "elements": Wg has heads vdim rows) or a number a head ("heads": Wg has heads rows);
+* `out_bias`: the output projection adds a bias (`o.b`);
+* `reads_cache`: there are no keys and values of its own: the run reads another run's cache (with its own
+  queries, mask and scale), as that run's keys left norm and rotation.
 
 All projections of h are one product into 32-bit rows; one kernel norms, rotates and stores
 (queries for the attention kernel, keys and values into the request's page, whose row holds a
 position's keys of all kv heads and maps and, position-contiguous, its values); one kernel does
 the attention of all maps, their combination, the norm and the gate; the output projection adds
-into the residual stream.  With a window or chunks only the last `size` positions are ever read,
+into the residual stream.  With a window or chunks only the last `size` positions (and the kept ones) are ever read,
 so the cache manager may take back earlier pages.
 
 Parameters: `hidden_size`, `heads`, `kv_heads`, `dim`, `vdim`, `maps`, `diff`, `values`, `bias`,
-`qk_norm`, `eps`, `scale`, `softcap`, `sink`, `q_temp`, `mask`, `gate`, `position` (a PartSpec), `names`.
+`out_bias`, `qk_norm`, `eps`, `scale`, `softcap`, `sink`, `q_temp`, `mask`, `gate`, `reads_cache`, `position` (a
+PartSpec), `names`.
 `forward(..., accumulate=False)` stores the 32-bit output instead of adding it (for a part that combines
 several mixers' outputs itself).
 """
@@ -95,7 +102,12 @@ class MaskedAttention(Mixer):
         if p.get("gate") not in (None, False, True, "elements", "heads"):
             raise ConfigError(f"gate {p.get('gate')!r} is not known (elements, heads)")
         self.gate_per_head = p.get("gate") == "heads"
-        self.sink = None if p.get("sink") is None else float(p["sink"])
+        self.sink_per_head = p.get("sink") == "heads"
+        self.sink = None if p.get("sink") is None or self.sink_per_head else float(p["sink"])
+        self.norm_rows = p.get("qk_norm") == "rows"
+        if p.get("qk_norm") not in (None, False, True, "heads", "rows"):
+            raise ConfigError(f"qk_norm {p.get('qk_norm')!r} is not known (heads, rows)")
+        self.out_bias, self.reads_cache = bool(p.get("out_bias", False)), bool(p.get("reads_cache", False))
         temp = p.get("q_temp")
         self.q_temp = None if not temp else (float(temp["coef"]), int(temp["every"]))
         if self.q_temp is not None and self.q_temp[1] < 1:
@@ -103,7 +115,7 @@ class MaskedAttention(Mixer):
         self.eps, self.scale = float(p.get("eps", 0.0)), float(p["scale"])
         self.softcap, self.diff = float(p.get("softcap") or 0.0), float(p.get("diff", 0.0))
         mask = p.get("mask") or {"kind": "causal"}
-        self.mask, self.mask_size = mask.get("kind", "causal"), int(mask.get("size", 0))
+        self.mask, self.mask_size, self.keep = mask.get("kind", "causal"), int(mask.get("size", 0)), int(mask.get("keep", 0))
         if self.heads % self.kv_heads:
             raise ConfigError(f"{self.heads} query heads are not a multiple of {self.kv_heads} key/value heads")
         if self.maps not in (1, 2):
@@ -114,6 +126,8 @@ class MaskedAttention(Mixer):
             raise ConfigError(f"values that are the keys have their size: vdim {self.vdim}, keys of {self.maps * self.dim}")
         if self.mask not in ("causal", "window", "chunk") or (self.mask != "causal" and self.mask_size < 1):
             raise ConfigError(f"mask {mask!r} is not causal, a window or chunks of a size")
+        if self.keep < 0 or (self.keep > 0 and self.mask != "window"):
+            raise ConfigError(f"mask {mask!r}: first positions are kept under a window")
         if self.vdim > 512:
             raise ConfigError(f"values of {self.vdim} dims are more than the attention kernel's 512")
         self.position = build_part("position", p["position"]) if p.get("position") is not None else None
@@ -122,7 +136,7 @@ class MaskedAttention(Mixer):
             raise ConfigError(f"{self.rot} rotated dims in keys of {self.dim}")
         names = p.get("names", {})
         base = prefix + names.get("scope", "mix.")
-        self.n = {k: base + names.get(k, k) for k in ("q", "k", "v", "g", "o", "lq1", "lk1", "lq2", "lk2")}
+        self.n = {k: base + names.get(k, k) for k in ("q", "k", "v", "g", "o", "sink", "lq1", "lk1", "lq2", "lk2")}
         self.n_q, self.n_k = self.heads * self.maps, self.kv_heads * self.maps
         self.q_width, self.k_width, self.v_width = self.n_q * self.dim, self.n_k * self.dim, self.kv_heads * self.vdim
         self.o_width = self.heads * self.vdim
@@ -130,14 +144,17 @@ class MaskedAttention(Mixer):
         self.k_at = self.q_width
         self.v_at = self.k_at if self.values == "keys" else self.k_at + self.k_width
         self.g_at = self.k_at + self.k_width + (0 if self.values == "keys" else self.v_width)
+        if self.reads_cache:
+            self.g_at = self.k_at
         self.g_width = 0 if not self.gate else self.heads if self.gate_per_head else self.o_width
         self.proj_width = self.g_at + self.g_width
         self.lam = 0.0
-        self.q_gain = self.k_gain = self.b_proj = None
+        self.q_gain = self.k_gain = self.b_proj = self.b_o = self.sinks = None
 
     # ------------------------------------------------------------------ declarations
     def _projections(self) -> List[str]:
-        return ["q", "k"] + (["v"] if self.values == "projected" else []) + (["g"] if self.gate else [])
+        own = [] if self.reads_cache else ["k"] + (["v"] if self.values == "projected" else [])
+        return ["q"] + own + (["g"] if self.gate else [])
 
     def tensors(self) -> List[TensorDecl]:
         n = self.n
@@ -146,15 +163,23 @@ class MaskedAttention(Mixer):
         if self.bias:
             t += [TensorDecl(n[k] + ".b", (rows[k],), "bias") for k in self._projections() if k != "g"]
         if self.qk_norm:
-            t += [TensorDecl(n["q"] + ".norm", (self.dim,), "gain"), TensorDecl(n["k"] + ".norm", (self.dim,), "gain")]
+            widths = {"q": self.q_width, "k": self.k_width}
+            t += [TensorDecl(n[k] + ".norm", (widths[k] if self.norm_rows else self.dim,), "gain") for k in self._normed()]
+        if self.sink_per_head:
+            t.append(TensorDecl(n["sink"], (self.heads,), "bias"))
         if self.maps == 2:
             t += [TensorDecl(n[k], (self.dim,), "bias") for k in ("lq1", "lk1", "lq2", "lk2")]
         t.append(TensorDecl(n["o"], (self.hidden, self.o_width)))
+        if self.out_bias:
+            t.append(TensorDecl(n["o"] + ".b", (self.hidden,), "bias"))
         return t
+
+    def _normed(self) -> List[str]:
+        return ["q"] if self.reads_cache else ["q", "k"]
 
     def cache_spec(self) -> Optional[CacheSpec]:
         return CacheSpec(entries=1, heads=1, head_dim=self.k_width + self.v_width,
-                         window=self.mask_size if self.mask != "causal" else 0)
+                         window=self.mask_size if self.mask != "causal" else 0, keep=self.keep)
 
     def load(self, store, rt) -> None:
         n = self.n
@@ -164,13 +189,18 @@ class MaskedAttention(Mixer):
             parts = [store.vector(n[k] + ".b").float() if k != "g" else torch.zeros(self.g_width, device=rt.device) for k in names]
             self.b_proj = torch.cat(parts).contiguous()
         if self.qk_norm:
-            self.q_gain, self.k_gain = store.vector(n["q"] + ".norm"), store.vector(n["k"] + ".norm")
+            self.q_gain = store.vector(n["q"] + ".norm")
+            self.k_gain = None if self.reads_cache else store.vector(n["k"] + ".norm")
+        if self.sink_per_head:
+            self.sinks = store.vector(n["sink"]).float().contiguous()
         if self.maps == 2:
             lq1, lk1, lq2, lk2 = (store.vector(n[k]).float() for k in ("lq1", "lk1", "lq2", "lk2"))
             # one number a layer, in 32-bit, once
             self.lam = float((torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum())).item()) + self.diff
         self.w_o = rt.k.prepare_weight(store.matrix(n["o"]))
         store.forget(n["o"])
+        if self.out_bias:
+            self.b_o = store.vector(n["o"] + ".b")
         if self.position is not None:
             self.position.load(store, rt)
 
@@ -201,7 +231,7 @@ class MaskedAttention(Mixer):
         q = ctx.ws.take((T, self.q_width), ctx.rt.dtype)
         k.heads_prepare(proj, 0, self.n_q, self.k_at, self.n_k, self.v_at, self.v_width, self.dim, self.q_gain, self.k_gain,
                         self.eps, self.rot, neighbours, magnitude, table, ctx.positions, ctx.seq_rows, group.block_table, cache,
-                        group.page_size, q, binding.writes, q_temp=self.q_temp)
+                        group.page_size, q, binding.writes and not self.reads_cache, q_temp=self.q_temp, norm_rows=self.norm_rows)
         att = ctx.ws.take((T, self.o_width), ctx.rt.dtype)
         tiles = None
         if k.masked_attention_uses_mfma(self.heads, self.kv_heads, self.maps, self.dim, self.vdim, group.page_size):
@@ -212,11 +242,11 @@ class MaskedAttention(Mixer):
         k.masked_attention(q, cache, group.block_table, ctx.positions, ctx.seq_rows, att, self.heads, self.kv_heads, self.maps,
                            self.dim, self.vdim, group.page_size, self.mask, self.mask_size, self.scale, self.softcap, self.lam,
                            1.0 - self.diff, self.eps, gate=proj[:, self.g_at:] if self.gate else None, tiles=tiles,
-                           sink=self.sink, gate_per_head=self.gate_per_head, span=span)
+                           sink=self.sinks if self.sink_per_head else self.sink, gate_per_head=self.gate_per_head, span=span, keep=self.keep)
         if not accumulate:          # the output itself, for a part that sums and norms on its own
-            k.gemm(att, self.w_o, residual, None, MODE_STORE_F32)
+            k.gemm(att, self.w_o, residual, self.b_o, MODE_STORE_F32)
             return
-        k.gemm(att, self.w_o, residual, None, MODE_ADD_F32,
+        k.gemm(att, self.w_o, residual, self.b_o, MODE_ADD_F32,
                following_norm=None if following is None else following.as_argument())
 
 

@@ -3,7 +3,9 @@ expert, if any, sees every token.  Two routers: "softmax" (the default): the lar
 the softmax over those logits alone; "sigmoid": scores s = sigmoid(logits) that do not compete, the
 choice made by s + a stored correction among the experts of the `keep` best of `groups` equal groups of
 neighbours (a group's score: the sum of its two largest choice scores), weighted by s over the sum of
-the chosen s, times `scale` (with `normalize` false: the chosen s themselves, times `scale`).  A weight
+the chosen s, times `scale` (with `normalize` false: the chosen s themselves, times `scale`); "softmax_all":
+the same with s the softmax over all logits.  With `identity` n, the router ranks n outputs more, behind
+the experts', which stand for the token's row itself (times its weight) and have no tensors.  A weight
 multiplies its expert's output, or with `weight_on` = "input" the expert's input: sum_e expert_e(w_e h),
 which differs since an expert is not linear (the products being linear, the factor is applied to their sums
 in 32-bit, before the unit).
@@ -18,8 +20,8 @@ through LDS: the same chains and bits as the tiles of 16 of a short step.
 
 Parameters: `hidden_size`, `experts`, `top`, `ff`, `limit` (None: no clamps), `alpha` (default 1.702),
 `shift` (default 1: the unit is g sigmoid(alpha g) (u + shift); no clamps, alpha 1 and shift 0 make it
-silu(gate) up), `router` (None, or {"scores": "sigmoid", "correction": bool, "groups", "keep", "scale",
-"normalize"}), `weight_on` ("output", the default, or "input"), `shared` (None, or {"ff", "limit"}: the clamped
+silu(gate) up), `router` (None, or {"scores": "sigmoid" or "softmax_all", "correction": bool, "groups", "keep",
+"scale", "normalize"}), `identity` (default 0), `weight_on` ("output", the default, or "input"), `shared` (None, or {"ff", "limit"}: the clamped
 unit; {"ff", "unit": "gated"}: silu(gate) up without clamps; with "gate": name, the shared expert's output is
 multiplied by sigmoid(w . h), w the tensor [1, hidden] of that name in the shared expert's scope, whose logit
 is one more row of the router's product), `names` (scope "mlp.", router, correction, expert "e{}.", shared
@@ -47,15 +49,18 @@ class RoutedExperts(FeedForward):
         self.hidden, self.n_experts, self.top = int(p["hidden_size"]), int(p["experts"]), int(p["top"])
         self.ff, self.alpha, self.shift = int(p["ff"]), float(p.get("alpha", 1.702)), float(p.get("shift", 1.0))
         self.limit = math.inf if p.get("limit") is None else float(p["limit"])
-        if not 1 <= self.top <= self.n_experts:
-            raise ConfigError(f"{self.top} of {self.n_experts} experts a token")
+        self.identity = int(p.get("identity", 0))
+        self.n_ranked = self.n_experts + self.identity         # what the router chooses among
+        if self.identity < 0 or not 1 <= self.top <= self.n_ranked:
+            raise ConfigError(f"{self.top} of {self.n_ranked} experts a token")
         names = p.get("names", {})
         self.base = prefix + names.get("scope", "mlp.")
         self.router_name = self.base + names.get("router", "router")
         router = dict(p.get("router") or {})
         self.scores = router.get("scores", "softmax")
-        if self.scores not in ("softmax", "sigmoid"):
-            raise ConfigError(f"a router with '{self.scores}' scores is not known (softmax, sigmoid)")
+        if self.scores not in ("softmax", "sigmoid", "softmax_all"):
+            raise ConfigError(f"a router with '{self.scores}' scores is not known (softmax, sigmoid, softmax_all)")
+        self.scored = self.scores != "softmax"                 # every expert has a score of its own
         self.groups, self.keep = int(router.get("groups", 1)), int(router.get("keep", 1))
         self.route_scale = float(router.get("scale", 1.0))
         self.normalize = bool(router.get("normalize", True))
@@ -64,15 +69,17 @@ class RoutedExperts(FeedForward):
             raise ConfigError(f"a router's weight on '{self.weight_on}' is not known (output, input)")
         self.correction_name = self.base + names.get("correction", "correction") if router.get("correction") else None
         self.correction = None
-        if self.scores == "sigmoid":
-            if self.n_experts > 1024 or self.top > 64 or self.groups > 64:
-                raise ConfigError(f"the sigmoid router takes up to 1024 experts in up to 64 groups and up to 64 a token, "
-                                  f"not {self.top} of {self.n_experts} in {self.groups}")
-            if self.groups < 1 or self.n_experts % self.groups or not 1 <= self.keep <= self.groups \
-                    or self.keep * (self.n_experts // self.groups) < self.top:
-                raise ConfigError(f"{self.keep} of {self.groups} groups of {self.n_experts} experts cannot give {self.top} a token")
-        elif router:
-            raise ConfigError("groups, a correction and a scale belong to the router with sigmoid scores")
+        if self.scored:
+            if self.n_ranked > 1024 or self.top > 64 or self.groups > 64:
+                raise ConfigError(f"the router of scores takes up to 1024 experts in up to 64 groups and up to 64 a token, "
+                                  f"not {self.top} of {self.n_ranked} in {self.groups}")
+            if self.groups < 1 or self.n_ranked % self.groups or not 1 <= self.keep <= self.groups \
+                    or self.keep * (self.n_ranked // self.groups) < self.top:
+                raise ConfigError(f"{self.keep} of {self.groups} groups of {self.n_ranked} experts cannot give {self.top} a token")
+        elif router or self.identity:
+            raise ConfigError("groups, a correction, a scale and identities belong to the routers whose experts have scores")
+        if self.identity and self.weight_on == "input":
+            raise ConfigError("an identity has no input of its own: its weight is on the output")
         self.expert_scope = names.get("expert", "e{}.")
         self.shared = None
         self.shared_gate_name = None
@@ -90,17 +97,17 @@ class RoutedExperts(FeedForward):
             else:
                 raise ConfigError(f"a shared expert's unit '{sh.get('unit')}' is not known (clamped, gated)")
             if sh.get("gate"):
-                if self.scores != "sigmoid":
-                    raise ConfigError("a gate on the shared expert comes with the router of sigmoid scores (its logit is a row of that product)")
+                if not self.scored:
+                    raise ConfigError("a gate on the shared expert comes with the routers of scores (its logit is a row of that product)")
                 self.shared_gate_name = prefix + scope + str(sh["gate"])
 
     def _expert(self, e: int, which: str) -> str:
         return self.base + self.expert_scope.format(e) + which
 
     def tensors(self) -> List[TensorDecl]:
-        t = [TensorDecl(self.router_name, (self.n_experts, self.hidden))]
+        t = [TensorDecl(self.router_name, (self.n_ranked, self.hidden))]
         if self.correction_name is not None:
-            t.append(TensorDecl(self.correction_name, (self.n_experts,), "bias"))
+            t.append(TensorDecl(self.correction_name, (self.n_ranked,), "bias"))
         for e in range(self.n_experts):
             t += [TensorDecl(self._expert(e, "gate"), (self.ff, self.hidden)), TensorDecl(self._expert(e, "up"), (self.ff, self.hidden)),
                   TensorDecl(self._expert(e, "down"), (self.hidden, self.ff))]
@@ -129,15 +136,18 @@ class RoutedExperts(FeedForward):
             self.shared.load(store, rt)
 
     def forward(self, ctx, h, out, accumulate: bool = True) -> None:
-        k, T, E, top = ctx.rt.k, h.shape[0], self.n_experts, self.top
+        k, T, E, R, top = ctx.rt.k, h.shape[0], self.n_experts, self.n_ranked, self.top
         i32 = torch.int32
         gated_shared = self.shared_gate_name is not None
-        logits = ctx.ws.take((T, E + 1 if gated_shared else E), torch.float32)
+        logits = ctx.ws.take((T, R + 1 if gated_shared else R), torch.float32)
         k.gemm(h, self.w_router, logits, None, MODE_STORE_F32)
         chosen, weights = ctx.ws.take((T, top), i32), ctx.ws.take((T, top), torch.float32)
-        if self.scores == "sigmoid" and (gated_shared or not self.normalize):
+        if self.scores == "softmax_all":
             k.route_scored(logits, self.correction, top, self.groups, self.keep, self.route_scale, chosen, weights,
-                           normalize=self.normalize, n_experts=E)
+                           normalize=self.normalize, n_experts=R, softmax=True)
+        elif self.scores == "sigmoid" and (gated_shared or not self.normalize):
+            k.route_scored(logits, self.correction, top, self.groups, self.keep, self.route_scale, chosen, weights,
+                           normalize=self.normalize, n_experts=R)
         elif self.scores == "sigmoid":
             k.route_scored(logits, self.correction, top, self.groups, self.keep, self.route_scale, chosen, weights)
         else:
@@ -156,12 +166,14 @@ class RoutedExperts(FeedForward):
         rows = ctx.ws.take((P, self.hidden), torch.float32)
         k.grouped_gemm(act, self.w_down, rows, x_group_stride=0, out_group_stride=0,
                        routed=(tiles, n_tiles, max_tiles, pairs, pairs, tile_rows), rows=P)
+        identity = (chosen, E, h) if self.identity else None
         if gated_shared:
             extra = ctx.ws.take((T, self.hidden), torch.float32)
             self.shared.forward(ctx, h, extra, accumulate=False)
-            k.route_combine(rows, None if on_input else weights, out, accumulate, top=top, extra=extra, extra_gate=logits[:, E:])
+            k.route_combine(rows, None if on_input else weights, out, accumulate, top=top, extra=extra, extra_gate=logits[:, R:],
+                            identity=identity)
             return
-        k.route_combine(rows, None if on_input else weights, out, accumulate, top=top)
+        k.route_combine(rows, None if on_input else weights, out, accumulate, top=top, identity=identity)
         if self.shared is not None:
             self.shared.forward(ctx, h, out)
 

@@ -8,6 +8,7 @@ Parameters: `head_dim`, `rotary_dim` (the leading dims that rotate; the whole he
 default, or "neighbours", (2i, 2i + 1); the table is the same, the mixer's kernel applies it) and
 `scaling`, a change of the frequencies for contexts longer than a model was trained on:
 
+* {"kind": "linear", factor}: every frequency is divided by `factor`;
 * {"kind": "stretch", factor, low, high, original}: by wavelength l = 2 pi / f against the
   original context: f is kept where l < original / high, divided by `factor` where
   l > original / low, and between the two blended with s = (original / l - low) / (high - low)
@@ -44,8 +45,8 @@ class RotaryEncoding(PositionEncoding):
         self.magnitude = 1.0
         if self.scaling is not None:
             kind = self.scaling.get("kind")
-            if kind not in ("stretch", "ramp"):
-                raise ConfigError(f"rotary scaling '{kind}' is not known (stretch, ramp)")
+            if kind not in ("linear", "stretch", "ramp"):
+                raise ConfigError(f"rotary scaling '{kind}' is not known (linear, stretch, ramp)")
             if kind == "ramp":
                 self.magnitude = 0.1 * math.log(float(self.scaling["factor"])) + 1.0
         self.key = None
@@ -55,7 +56,9 @@ class RotaryEncoding(PositionEncoding):
         n, dims = self.rotary_dim // 2, self.rotary_dim
         f = [self.theta ** (-2.0 * i / dims) for i in range(n)]
         sc = self.scaling
-        if sc is not None and sc["kind"] == "stretch":
+        if sc is not None and sc["kind"] == "linear":
+            f = [fi / float(sc["factor"]) for fi in f]
+        elif sc is not None and sc["kind"] == "stretch":
             factor, low, high, original = (float(sc[k]) for k in ("factor", "low", "high", "original"))
             for i, fi in enumerate(f):
                 wavelength = 2.0 * math.pi / fi
