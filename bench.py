@@ -168,6 +168,24 @@ def _zugutar_sizes(width, heads, kv_heads, ss_heads, groups, experts, top, exper
             "loop": {"start": 2, "stop": 3, "times": 2}, "logit_scale": 0.25, "norm": {"eps": 1e-6}, "vocab": 32000, "width": width}
 
 
+# --design lilunex: four layers: time mixing with a dense feed-forward (1.5 times the gated one's width: the same weights
+# a token), windowed attention beside kept first tokens with experts and identities, the gated delta rule with the same
+# experts, and attention that reads the second layer's keys, dense.  Beside it the closest design the engine has, Zugutar
+# (a state-space scan, attention with a sink, as many experts of the same width), and the dense decoder of equal width.
+def _lilunex_sizes(width, heads, kv_heads, wkv_heads, delta_heads, window, experts, identity, top, expert_ff, shared_ff, dense_ff):
+    mixer = {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+             "mask": {"size": window, "keep_first": 4}, "rot": {"base": 10000.0, "dims": 128, "scaling": {"factor": 8.0}}}
+    moe = {"kind": "moe", "router": {"experts": experts, "identity": identity, "top": top}, "expert": {"ff": expert_ff},
+           "shared": {"ff": shared_ff}}
+    dense = {"kind": "dense", "ff": dense_ff * 3 // 2}
+    return {"architecture": "Lilunex", "embedding": {"scale": width ** 0.5}, "norm": {"eps": 1e-5}, "vocab": 32000, "width": width,
+            "layers": [{"type": "wkv", "mixer": {"heads": wkv_heads, "dim": 64}, "mlp": dense},
+                       {"type": "attention", "mixer": mixer, "mlp": moe},
+                       {"type": "delta", "mixer": {"heads": delta_heads, "kv_heads": delta_heads // 2, "dim": 128, "vdim": 128, "conv": 4},
+                        "mlp": moe},
+                       {"type": "attention", "mixer": dict(mixer, kv_from=1), "mlp": dense}]}
+
+
 # design -> size -> the models measured side by side, the design's own first
 DESIGN_SIZES = {
     "pikesun": {
@@ -186,6 +204,11 @@ DESIGN_SIZES = {
                  ("pikesun", _pikesun_sizes(2048, 2560, 10, 16, 768, 32, 4, 704, 1408, 5632, 1024)), ("qwen2", _qwen_sizes(2048, 16, 2, 5632))],
         "4096": [("zugutar", _zugutar_sizes(4096, 32, 8, 64, 8, 64, 6, 1408, 2816)),
                  ("pikesun", _pikesun_sizes(4096, 5120, 20, 32, 1536, 64, 6, 1408, 2816, 11008, 2048)), ("qwen2", _qwen_sizes(4096, 32, 8, 11008))]},
+    "lilunex": {
+        "2048": [("lilunex", _lilunex_sizes(2048, 16, 2, 32, 32, 1024, 32, 8, 4, 704, 1408, 5632)),
+                 ("zugutar", _zugutar_sizes(2048, 16, 2, 32, 2, 32, 4, 704, 1408)), ("qwen2", _qwen_sizes(2048, 16, 2, 5632))],
+        "4096": [("lilunex", _lilunex_sizes(4096, 32, 8, 64, 64, 2048, 64, 16, 6, 1408, 2816, 11008)),
+                 ("zugutar", _zugutar_sizes(4096, 32, 8, 64, 8, 64, 6, 1408, 2816)), ("qwen2", _qwen_sizes(4096, 32, 8, 11008))]},
 }
 
 
@@ -250,7 +273,7 @@ def design(args, torch) -> int:
 
 def main() -> int:
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", default="", choices=["", "pikesun", "figalorn", "napizen", "zugutar"], help="instead of the headline benchmark: prefill and "
+    ap.add_argument("--design", default="", choices=["", *DESIGN_SIZES], help="instead of the headline benchmark: prefill and "
                     "decoding of this design at sizes that resemble real models' layers, beside the dense decoder of equal size")
     ap.add_argument("--design-size", default="", help="with --design: only this size (2048 or 4096)")
     ap.add_argument("--gpus", type=int, default=1)
