@@ -373,6 +373,16 @@ int axk_delta_prepare(const float* in, long in_stride, const void* w, int taps, 
 int axk_delta_scan(const float* u, const float* terms, float* state, long state_stride, long copy_elems, long tail_at,
                    const int32_t* spans, int n_spans, const int32_t* positions, const int32_t* seq_rows, const float* conv_in,
                    long conv_in_stride, float* y, int heads, int kv_heads, int N, int P, int taps, void* stream);
+// axk_delta_chunked (where axk_delta_chunked_ok says 1): the same for long stretches, in chunks of up to 64 tokens on the
+// 32-bit matrix cores (sums in another order, by rounding): chunks [n_chunks][2] = (first token, tokens), spans5 [n_spans][5]
+// = (slot, first token, tokens, first chunk, chunks), a request's chunks in order and full but the last;
+// work: axk_delta_chunked_workspace floats.
+int axk_delta_chunked_ok(int kv_heads, int heads, int N, int P);
+long axk_delta_chunked_workspace(int n_chunks, int heads, int N, int P);
+int axk_delta_chunked(const float* u, const float* terms, float* state, long state_stride, long copy_elems, long tail_at,
+                      const int32_t* chunks, int n_chunks, const int32_t* spans5, int n_spans, const int32_t* positions,
+                      const float* conv_in, long conv_in_stride, float* y, int heads, int kv_heads, int N, int P, int taps,
+                      float* work, long work_floats, void* stream);
 int axk_head_norm_gate(const float* y, const float* gate, long gate_stride, const void* gain, int gain_is_f32, int gain_per_head,
                        float eps, void* out, int n_tokens, int heads, int P, void* stream);
 

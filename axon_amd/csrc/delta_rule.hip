@@ -68,6 +68,19 @@ delta_prepare_kernel(const float* __restrict__ in, long in_stride, const elem_t*
     if (lane + 64 * j < size) dst[c0 + lane + 64 * j] = v[j] * inv;
 }
 
+// The convolutions' last taps - 1 inputs: of (what was kept, this step's inputs) the last taps - 1; place i takes what
+// lies `count` places later (where both copies are one: read before it is written, ascending).  The channels are shared
+// out over a request's threads, this being the one numbered `me` of `all`.
+__device__ inline void keep_conv_inputs(const float* __restrict__ kept_from, float* kept, const float* __restrict__ conv_in,
+                                        long conv_in_stride, int first, int count, int channels, int taps, int me, int all) {
+  for (int c = me; c < channels; c += all)
+    for (int i = 0; i < taps - 1; ++i) {
+      const int at = i + count;
+      kept[(long)i * channels + c] = at < taps - 1 ? kept_from[(long)at * channels + c]
+                                                   : conv_in[(long)(first + at - (taps - 1)) * conv_in_stride + c];
+    }
+}
+
 // The walk.  grid (requests of the step, heads, blocks of value dims); LK lanes share a value dim, OWN rows of the
 // state a lane.  With a = S^T k and b = S^T q of the state as the token finds it, u = beta (v - g a) and the read-out
 // behind the token's write is o = g b + (k . q) u: both sums leave for the lanes' permutations together.  The operands
@@ -143,17 +156,234 @@ delta_scan_kernel(const float* __restrict__ u, const float* __restrict__ terms, 
     work(odd, t + AHEAD);
   }
   if (has_p) rec_store<OWN, VEC>(to + s_at, S, n0, N);
-  if (blockIdx.y != 0 || blockIdx.z != 0) return;
-  // the convolutions' last taps - 1 inputs: of (what was kept, this step's inputs) the last taps - 1; place i takes
-  // what lies `count` places later (where both copies are one: read before it is written, ascending)
-  float* kept = to + tail_at;
-  const float* kept_from = from + tail_at;
-  for (int c = threadIdx.x; c < channels; c += REC_THREADS)
-    for (int i = 0; i < taps - 1; ++i) {
-      const int at = i + s.count;
-      kept[(long)i * channels + c] = at < taps - 1 ? kept_from[(long)at * channels + c]
-                                                   : conv_in[(long)(s.first + at - (taps - 1)) * conv_in_stride + c];
+  keep_conv_inputs(from + tail_at, to + tail_at, conv_in, conv_in_stride, s.first, s.count, channels, taps,
+                   (blockIdx.y * gridDim.z + blockIdx.z) * REC_THREADS + threadIdx.x, gridDim.y * gridDim.z * REC_THREADS);
+}
+
+// Long stretches in chunks of 64 tokens, on the 32-bit matrix cores.  Inside a chunk that finds the state S, with
+// b_i the product of the chunk's g up to token i, D_ij = g_(j+1) ... g_i and A_ij = beta_i D_ij (k_i . k_j) for j < i,
+// the tokens' corrections solve a unit lower triangular system that the state enters linearly:
+//   (I + A) U = diag(beta) V - diag(beta b) K S,     U = U' - W S,
+//   O = diag(b) Q S + M U,  M_ij = D_ij (q_i . k_j) for j <= i,     S <- b_last S + (diag(D_last) K)^T U.
+// The first kernel makes U', W, M and the scaled transposed keys of every (chunk, head) side by side: the products
+// k_i . k_j and q_i . k_j by MFMA, the products of decays one multiplication after the other (never a quotient, so a
+// decay of 0 is nothing special), the two right-hand sides by forward substitution, a column a thread with its 64 rows
+// in registers.  The second walks a request's chunks per (head, sixteen value dims).  The sums of a token are those of
+// the walk token by token in another order.
+// Layouts of a (chunk, head), item = chunk heads + head: U' [64][P], W [64][N], kt [N][64], M [64][64] (its upper tiles
+// are not written), b [64].  Rows beyond the chunk's tokens have g 1 and beta 0: they change nothing.
+#define DC 64
+typedef __attribute__((ext_vector_type(4))) float dc_f32x4;
+__device__ inline dc_f32x4 dc_load(const float* p) { return *reinterpret_cast<const dc_f32x4*>(p); }
+// four chained products over sixteen k: lane l holds rows l % 16 at k = 4 (l / 16) .. + 3 of either operand
+__device__ inline dc_f32x4 dc_mfma(dc_f32x4 a, dc_f32x4 b, dc_f32x4 c) {
+#pragma unroll
+  for (int j = 0; j < 4; ++j) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], b[j], c, 0, 0, 0);
+  return c;
+}
+
+template <int NT>
+__global__ void __launch_bounds__(256)
+delta_chunk_terms_kernel(const float* __restrict__ u, const float* __restrict__ terms, const int32_t* __restrict__ chunks, int heads,
+                         int kv_heads, int P, float* __restrict__ up, float* __restrict__ w, float* __restrict__ kt,
+                         float* __restrict__ m, float* __restrict__ b) {
+  constexpr int N = 16 * NT, ROW = DC + 4;
+  __shared__ float D[DC][DC + 1];
+  __shared__ __align__(16) float A[DC][ROW];
+  __shared__ float gs[DC], betas[DC], bs[DC];
+  const int h = blockIdx.x, kh = h / (heads / kv_heads), first = chunks[2 * blockIdx.y], count = chunks[2 * blockIdx.y + 1];
+  const long item = (long)blockIdx.y * heads + h;
+  const int channels = 2 * kv_heads * N + heads * P;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 15, g4 = lane >> 4;
+  if (tid < DC) {
+    gs[tid] = tid < count ? terms[((long)(first + tid) * heads + h) * 2] : 1.0f;
+    betas[tid] = tid < count ? terms[((long)(first + tid) * heads + h) * 2 + 1] : 0.0f;
+  }
+  __syncthreads();
+  if (tid < DC) {
+    float d = 1.0f;
+    D[tid][tid] = 1.0f;
+    for (int i = tid + 1; i < DC; ++i) { d *= gs[i]; D[i][tid] = d; }
+  } else if (tid == DC) {
+    float d = 1.0f;
+    for (int i = 0; i < DC; ++i) { d *= gs[i]; bs[i] = d; b[item * DC + i] = d; }
+  }
+  const float* keys = u + (long)(kv_heads + kh) * N;
+  const float* mine = u + (long)(first + min(16 * wave + r, count - 1)) * channels + (long)kh * N + 4 * g4;
+  dc_f32x4 qf[NT], kf[NT];
+#pragma unroll
+  for (int c = 0; c < NT; ++c) { qf[c] = dc_load(mine + 16 * c); kf[c] = dc_load(mine + (long)kv_heads * N + 16 * c); }
+  __syncthreads();
+  for (int jt = 0; jt <= wave; ++jt) {
+    const float* other = keys + (long)(first + min(16 * jt + r, count - 1)) * channels + 4 * g4;
+    dc_f32x4 kk = {0.0f, 0.0f, 0.0f, 0.0f}, qk = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+    for (int c = 0; c < NT; ++c) {
+      const dc_f32x4 o = dc_load(other + 16 * c);
+      kk = dc_mfma(kf[c], o, kk);
+      qk = dc_mfma(qf[c], o, qk);
     }
+    const int j = 16 * jt + r;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = 16 * wave + 4 * g4 + e;
+      A[i][j] = j < i ? (betas[i] * D[i][j]) * kk[e] : 0.0f;
+      m[(item * DC + i) * DC + j] = j <= i ? D[i][j] * qk[e] : 0.0f;
+    }
+  }
+  __syncthreads();
+  const int cols = P + N;
+  for (int col = tid; col < cols; col += 256) {
+    float X[DC];
+    const bool is_v = col < P;
+    const float* src = u + (is_v ? 2L * kv_heads * N + (long)h * P + col : (long)(kv_heads + kh) * N + col - P);
+#pragma unroll
+    for (int i = 0; i < DC; ++i) X[i] = src[(long)(first + min(i, count - 1)) * channels];
+    if (!is_v) {
+      float* dst = kt + (item * N + col - P) * DC;
+#pragma unroll
+      for (int i = 0; i < DC; i += 4)
+        *reinterpret_cast<dc_f32x4*>(dst + i) = dc_f32x4{X[i] * D[DC - 1][i], X[i + 1] * D[DC - 1][i + 1], X[i + 2] * D[DC - 1][i + 2],
+                                                         X[i + 3] * D[DC - 1][i + 3]};
+    }
+#pragma unroll
+    for (int i = 0; i < DC; ++i) X[i] *= is_v ? betas[i] : betas[i] * bs[i];
+#pragma unroll
+    for (int i = 1; i < DC; ++i) {
+      float x = X[i];
+#pragma unroll
+      for (int j = 0; j < i; j += 4) {
+        const dc_f32x4 a = dc_load(&A[i][j]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (j + e < i) x = fmaf(-a[e], X[j + e], x);
+      }
+      X[i] = x;
+      __builtin_amdgcn_sched_barrier(0);       // a row of A at a time in registers
+    }
+    float* dst = is_v ? up + item * DC * P + col : w + item * DC * N + col - P;
+    const int step = is_v ? P : N;
+#pragma unroll
+    for (int i = 0; i < DC; ++i) dst[(long)i * step] = X[i];
+  }
+}
+
+// grid (heads, P / 16, requests), four waves: a wave the sixteen tokens 16 wave .. of a chunk, and of the state the tiles
+// of sixteen rows wave, wave + 4 in its accumulators.  The state's slice and U travel between the waves through LDS, value
+// dim by value dim.  A chunk's operands are asked for while the chunk before is worked on.  spans5 [n][5] = (slot, first
+// token, tokens, first chunk, chunks).
+template <int NT>
+struct DeltaChunkOperands {
+  static constexpr int TILES = (NT + 3) / 4;
+  dc_f32x4 w[NT], q[NT], m[4], k[TILES][4];
+  float up[4], b[4], b_last;
+};
+
+template <int NT>
+__global__ void __launch_bounds__(256)
+delta_chunk_walk_kernel(const float* __restrict__ u, const float* __restrict__ up, const float* __restrict__ w,
+                        const float* __restrict__ kt, const float* __restrict__ m, const float* __restrict__ b,
+                        const int32_t* __restrict__ spans5, const int32_t* __restrict__ positions, float* __restrict__ state,
+                        long state_stride, long copy_elems, long tail_at, const float* __restrict__ conv_in, long conv_in_stride,
+                        float* __restrict__ y, int heads, int kv_heads, int P, int taps) {
+  typedef DeltaChunkOperands<NT> Ops;
+  constexpr int N = 16 * NT, TILES = Ops::TILES;
+  __shared__ __align__(16) float Sl[16][N + 4];
+  __shared__ __align__(16) float Ul[16][DC + 4];
+  const int h = blockIdx.x, kh = h / (heads / kv_heads), p0 = 16 * blockIdx.y;
+  const int32_t* span = spans5 + 5 * blockIdx.z;
+  const int slot = span[0], first = span[1], count = span[2], chunk0 = span[3], n_chunks = span[4];
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, g4 = lane >> 4;
+  const int start = positions[first], channels = 2 * kv_heads * N + heads * P;
+  const float* from = rec_copy_before(state, state_stride, copy_elems, slot, start);
+  float* to = rec_copy_behind(state, state_stride, copy_elems, slot, start + count - 1);
+  const long s_at = (long)h * N * P + (long)(p0 + r) * N + 4 * g4;
+  dc_f32x4 S[TILES];
+#pragma unroll
+  for (int tt = 0; tt < TILES; ++tt) {
+    const int tile = wave + 4 * tt;
+    if (tile < NT) {
+      S[tt] = dc_load(from + s_at + 16 * tile);
+      *reinterpret_cast<dc_f32x4*>(&Sl[r][16 * tile + 4 * g4]) = S[tt];
+    }
+  }
+  auto fetch = [&](Ops& o, int c) {
+    const long item = (long)(chunk0 + c) * heads + h;
+    const int t0 = first + DC * c, last = first + count - 1;
+    const float* wr = w + (item * DC + 16 * wave + r) * N + 4 * g4;
+    const float* qr = u + (long)min(t0 + 16 * wave + r, last) * channels + (long)kh * N + 4 * g4;
+#pragma unroll
+    for (int i = 0; i < NT; ++i) { o.w[i] = dc_load(wr + 16 * i); o.q[i] = dc_load(qr + 16 * i); }
+    const float* mr = m + (item * DC + 16 * wave + r) * DC + 4 * g4;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (i <= wave) o.m[i] = dc_load(mr + 16 * i);
+#pragma unroll
+    for (int tt = 0; tt < TILES; ++tt)
+      if (wave + 4 * tt < NT) {
+        const float* kr = kt + (item * N + 16 * (wave + 4 * tt) + r) * DC + 4 * g4;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o.k[tt][i] = dc_load(kr + 16 * i);
+      }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      o.up[e] = up[(item * DC + 16 * wave + 4 * g4 + e) * P + p0 + r];
+      o.b[e] = b[item * DC + 16 * wave + 4 * g4 + e];
+    }
+    o.b_last = b[item * DC + DC - 1];
+  };
+  auto work = [&](const Ops& o, int c) {
+    dc_f32x4 ws = {0.0f, 0.0f, 0.0f, 0.0f}, out = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      const dc_f32x4 s = dc_load(&Sl[r][16 * i + 4 * g4]);
+      ws = dc_mfma(o.w[i], s, ws);
+      out = dc_mfma(o.q[i], s, out);
+    }
+    dc_f32x4 mine;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { mine[e] = o.up[e] - ws[e]; out[e] *= o.b[e]; }
+    *reinterpret_cast<dc_f32x4*>(&Ul[r][16 * wave + 4 * g4]) = mine;
+    __syncthreads();                       // every wave's part of U is there, and every wave has read the state
+    dc_f32x4 all[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) all[i] = dc_load(&Ul[r][16 * i + 4 * g4]);
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (i <= wave) out = dc_mfma(o.m[i], all[i], out);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = DC * c + 16 * wave + 4 * g4 + e;
+      if (i < count) y[((long)(first + i) * heads + h) * P + p0 + r] = out[e];
+    }
+#pragma unroll
+    for (int tt = 0; tt < TILES; ++tt) {
+      const int tile = wave + 4 * tt;
+      if (tile < NT) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) S[tt][e] *= o.b_last;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) S[tt] = dc_mfma(o.k[tt][i], all[i], S[tt]);
+        *reinterpret_cast<dc_f32x4*>(&Sl[r][16 * tile + 4 * g4]) = S[tt];
+      }
+    }
+    __syncthreads();
+  };
+  Ops even, odd;
+  fetch(even, 0);
+  __syncthreads();
+  for (int c = 0; c < n_chunks; c += 2) {
+    if (c + 1 < n_chunks) fetch(odd, c + 1);
+    work(even, c);
+    if (c + 1 >= n_chunks) break;
+    if (c + 2 < n_chunks) fetch(even, c + 2);
+    work(odd, c + 1);
+  }
+#pragma unroll
+  for (int tt = 0; tt < TILES; ++tt)
+    if (wave + 4 * tt < NT) *reinterpret_cast<dc_f32x4*>(to + s_at + 16 * (wave + 4 * tt)) = S[tt];
+  keep_conv_inputs(from + tail_at, to + tail_at, conv_in, conv_in_stride, first, count, channels, taps,
+                   (blockIdx.x * gridDim.y + blockIdx.y) * 256 + threadIdx.x, gridDim.x * gridDim.y * 256);
 }
 
 // out[t, a] = (y[t, a] / sqrt(mean(y[t, a]^2) + eps)) gain silu(gate[t, a]) head by head; the gain holds P numbers
@@ -239,6 +469,53 @@ extern "C" int axk_delta_scan(const float* u, const float* terms, float* state, 
 #undef DELTA_LAUNCH
 #undef DELTA_ARGS
   AXK_LAUNCH_CHECK("delta_scan");
+  return 0;
+}
+
+// 1 where axk_delta_chunked takes these sizes.
+extern "C" int axk_delta_chunked_ok(int kv_heads, int heads, int N, int P) {
+  return (N == 32 || N == 64 || N == 96 || N == 128) && P % 16 == 0 && P / 16 <= 65535 && heads > 0 && kv_heads > 0;
+}
+
+// The floats of workspace that axk_delta_chunked wants for this many chunks.
+extern "C" long axk_delta_chunked_workspace(int n_chunks, int heads, int N, int P) {
+  return (long)n_chunks * heads * DC * (2L * N + P + DC + 1);
+}
+
+extern "C" int axk_delta_chunked(const float* u, const float* terms, float* state, long state_stride, long copy_elems, long tail_at,
+                                 const int32_t* chunks, int n_chunks, const int32_t* spans5, int n_spans, const int32_t* positions,
+                                 const float* conv_in, long conv_in_stride, float* y, int heads, int kv_heads, int N, int P, int taps,
+                                 float* work, long work_floats, void* stream) {
+  AXK_REQUIRE(n_spans >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && taps >= 1 && axk_delta_chunked_ok(kv_heads, heads, N, P),
+              "delta_chunked: bad sizes spans=%d heads=%d kv heads=%d keys=%d values=%d taps=%d", n_spans, heads, kv_heads, N, P, taps);
+  const long channels = 2L * kv_heads * N + (long)heads * P;
+  AXK_REQUIRE(tail_at >= (long)heads * N * P && copy_elems >= tail_at + (taps - 1) * channels && state_stride >= 2 * copy_elems &&
+              conv_in_stride >= channels,
+              "delta_chunked: a state row of %ld floats does not hold two copies of %ld (%d x %d x %d, then %d x %ld from %ld)",
+              state_stride, copy_elems, heads, N, P, taps - 1, channels, tail_at);
+  AXK_REQUIRE(copy_elems % 4 == 0 && state_stride % 4 == 0 && ((uintptr_t)u & 15) == 0 && ((uintptr_t)state & 15) == 0 &&
+              ((uintptr_t)work & 15) == 0, "delta_chunked: rows are not 16-byte aligned");
+  AXK_REQUIRE(n_chunks >= n_spans && n_chunks <= 65535 && n_spans <= 65535, "delta_chunked: %d chunks of %d requests", n_chunks, n_spans);
+  AXK_REQUIRE(work != nullptr && work_floats >= axk_delta_chunked_workspace(n_chunks, heads, N, P), "delta_chunked: a workspace of %ld floats",
+              work_floats);
+  if (n_spans == 0) return 0;
+  const long items = (long)n_chunks * heads;
+  float* up = work;
+  float* w = up + items * DC * P;
+  float* kt = w + items * DC * N;
+  float* m = kt + items * DC * N;
+  float* b = m + items * DC * DC;
+  hipStream_t s = (hipStream_t)stream;
+#define DC_LAUNCH(NT)                                                                                                            \
+  {                                                                                                                              \
+    delta_chunk_terms_kernel<NT><<<dim3(heads, n_chunks), 256, 0, s>>>(u, terms, chunks, heads, kv_heads, P, up, w, kt, m, b);   \
+    delta_chunk_walk_kernel<NT><<<dim3(heads, P / 16, n_spans), 256, 0, s>>>(u, up, w, kt, m, b, spans5, positions, state,       \
+                                                                            state_stride, copy_elems, tail_at, conv_in,          \
+                                                                            conv_in_stride, y, heads, kv_heads, P, taps);        \
+  }
+  if (N == 32) DC_LAUNCH(2) else if (N == 64) DC_LAUNCH(4) else if (N == 96) DC_LAUNCH(6) else DC_LAUNCH(8)
+#undef DC_LAUNCH
+  AXK_LAUNCH_CHECK("delta_chunked");
   return 0;
 }
 

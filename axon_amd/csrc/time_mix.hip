@@ -186,8 +186,9 @@ wkv_scan_kernel(const float* __restrict__ rows, long stride, long r_at, long k_a
     if (tells) rec_store<OWN, VEC>(decays + ((long)blockIdx.x * heads + h) * N, D, n0, N);
     return;
   }
-  if (blockIdx.y == 0 && blockIdx.z == 0)
-    for (int c = threadIdx.x; c < width; c += REC_THREADS) to[tail_at + c] = to_float(h_in[(long)(last - 1) * width + c]);
+  const int n_blocks = gridDim.y * gridDim.z;          // the last row, shared out over the request's blocks
+  for (int c = (blockIdx.y * gridDim.z + blockIdx.z) * REC_THREADS + threadIdx.x; c < width; c += n_blocks * REC_THREADS)
+    to[tail_at + c] = to_float(h_in[(long)(last - 1) * width + c]);
 }
 
 // Long stretches in segments: the walk above runs every segment of a request side by side, the first from the

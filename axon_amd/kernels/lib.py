@@ -111,6 +111,9 @@ _SIGNATURES = {
                           c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p],
     "axk_delta_scan": [c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_long,
                        c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
+    "axk_delta_chunked_ok": [c_int, c_int, c_int, c_int],
+    "axk_delta_chunked": [c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p,
+                          c_long, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_long, c_void_p],
     "axk_head_norm_gate": [c_void_p, c_void_p, c_long, c_void_p, c_int, c_int, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
     "axk_latent_prepare": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_int,
                            c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p],
@@ -183,6 +186,8 @@ class Kernels:
         self.lib.axk_latent_attention_workspace.restype = ctypes.c_long
         self.lib.axk_masked_attention_workspace.argtypes = [c_int] * 11
         self.lib.axk_masked_attention_workspace.restype = ctypes.c_long
+        self.lib.axk_delta_chunked_workspace.argtypes = [c_int] * 4
+        self.lib.axk_delta_chunked_workspace.restype = ctypes.c_long
         self.lib.axk_packed_elems.argtypes = [c_int, c_int]
         self.lib.axk_packed_elems.restype = ctypes.c_long
         self.lib.axk_gemm_workspace.argtypes = [c_int, c_int, c_int, c_int]
@@ -1175,10 +1180,12 @@ class Kernels:
             self._vec_flag(dt_bias, "dt bias"), _ptr(u), _ptr(terms), T, heads, kv_heads, keys, values, float(q_scale), _stream()))
 
     def delta_scan(self, u, terms, state, copy_elems: int, tail_at: int, spans, positions, seq_rows, conv_in, y, heads: int,
-                   kv_heads: int, keys: int, values: int, taps: int) -> torch.Tensor:
+                   kv_heads: int, keys: int, values: int, taps: int, chunks=None) -> torch.Tensor:
         """The gated delta rule over each request's tokens (see csrc/delta_rule.hip): u [T, channels] and terms [T, heads, 2]
         float32; spans int32 [n, 3] or None as in the other scans; conv_in: the convolutions' inputs (float32, rows may be
-        strided), kept for the next step; y [T, heads values] float32."""
+        strided), kept for the next step; y [T, heads values] float32.  `chunks` = (chunks int32 [n, 2]: first token, tokens;
+        spans5 int32 [m, 5]: slot, first token, tokens, first chunk, chunks): these requests' stretches run in chunks on the
+        matrix cores (`delta_chunked_ok`; sums in another order, by rounding), `spans` then names the others (it may be empty)."""
         for t, what in ((u, "delta u"), (terms, "delta terms"), (y, "delta y")):
             self._f32(t, what)
         self._f32_rows(conv_in, "delta conv_in")
@@ -1191,10 +1198,27 @@ class Kernels:
         if spans is not None:
             self._i32(spans, "scan spans")
             n = spans.shape[0]
+        if chunks is not None:
+            list_, spans5 = chunks
+            self._i32(list_, "delta chunks"); self._i32(spans5, "delta requests")
+            if spans is None or list_.dim() != 2 or list_.shape[1] != 2 or spans5.dim() != 2 or spans5.shape[1] != 5:
+                raise KernelError(f"delta_scan: chunks {tuple(list_.shape)} of requests {tuple(spans5.shape)}")
+            need = int(self.lib.axk_delta_chunked_workspace(list_.shape[0], heads, keys, values))
+            work = torch.empty(need, dtype=torch.float32, device=y.device)
+            self._check(self.lib.axk_delta_chunked(
+                _ptr(u), _ptr(terms), _ptr(state), state.stride(0), int(copy_elems), int(tail_at), _ptr(list_), list_.shape[0], _ptr(spans5),
+                spans5.shape[0], _ptr(positions), _ptr(conv_in), conv_in.stride(0), _ptr(y), heads, kv_heads, keys, values, int(taps),
+                _ptr(work), need, _stream()))
+            if n == 0:
+                return y
         self._check(self.lib.axk_delta_scan(
             _ptr(u), _ptr(terms), _ptr(state), state.stride(0), int(copy_elems), int(tail_at), _ptr(spans), n, _ptr(positions),
             _ptr(seq_rows), _ptr(conv_in), conv_in.stride(0), _ptr(y), heads, kv_heads, keys, values, int(taps), _stream()))
         return y
+
+    def delta_chunked_ok(self, kv_heads: int, heads: int, keys: int, values: int) -> bool:
+        """Whether `delta_scan` takes `chunks` at these sizes."""
+        return bool(self.lib.axk_delta_chunked_ok(kv_heads, heads, keys, values))
 
     def head_norm_gate(self, y, gate, gain, eps: float, out, heads: int) -> torch.Tensor:
         """out = (y / sqrt(mean y^2 + eps)) gain silu(gate), the mean over each of `heads` equal parts of a row: y float32

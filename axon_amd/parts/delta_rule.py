@@ -12,7 +12,8 @@ g = exp(-exp(A_log) softplus(. + dt_bias)), per head
 and the output is W_o (o / sqrt(mean(o^2) + eps) head by head, times a gain of vdim shared by the heads, times
 silu(gate)).  The product's rows, the convolutions' results, the step sizes, the state and the norm are 32-bit; a
 request's state row holds S and the convolutions' last conv - 1 inputs, twice: the state behind position p in copy
-p & 1, so that a decoding step reads one copy and writes the other and may be run again with the same result.
+p & 1, so that a decoding step reads one copy and writes the other and may be run again with the same result.  Long stretches of tokens run in chunks on the
+32-bit matrix cores where the sizes allow (`step_chunks`): the same sums in another order.
 
 Parameters: `hidden_size`, `heads`, `kv_heads`, `dim`, `vdim`, `conv`, `eps`, `names` (the tensors' names under the
 prefix: scope "mix.", q, k, v, b, a, g, A_log, dt_bias, norm, o; a convolution is the name + ".conv").
@@ -20,7 +21,7 @@ prefix: scope "mix.", q, k, v, b, a, g, A_log, dt_bias, norm, o; a convolution i
 """
 from __future__ import annotations
 
-from typing import List
+from typing import List, Optional, Tuple
 
 import torch
 
@@ -28,6 +29,30 @@ from ..config.base import ConfigError
 from ..kernels import MODE_ADD_F32, MODE_STORE_F32
 from .base import CacheBinding, Mixer, StateSpec, TensorDecl, register_mixer
 from .recurrent import step_spans
+
+
+CHUNK = 64             # tokens of a chunk of the matrix-core form
+LONG = 24              # a request's tokens of a step from which that form is used
+
+
+def step_chunks(ctx) -> Optional[Tuple]:
+    """The long stretches of a step in chunks, and the other requests: ((chunks int32 [n, 2] = (first token, tokens),
+    spans5 int32 [m, 5] = (slot, first token, tokens, first chunk, chunks)), spans int32 [k, 3] = (slot, first token,
+    tokens) of the rest) on the device, made once a step; None where no stretch is long."""
+    if ctx.decode_only or all(s.q_len < LONG for s in ctx.spans):
+        return None
+    made = ctx.shared.get("delta_rule_chunks")
+    if made is None:
+        chunks, spans5, rest = [], [], []
+        for s in ctx.spans:
+            if s.q_len < LONG:
+                rest.append([s.slot, s.q_start, s.q_len])
+                continue
+            spans5.append([s.slot, s.q_start, s.q_len, len(chunks), -(-s.q_len // CHUNK)])
+            chunks += [[s.q_start + at, min(CHUNK, s.q_len - at)] for at in range(0, s.q_len, CHUNK)]
+        put = lambda rows, width: torch.tensor(rows, dtype=torch.int32).view(-1, width).to(ctx.rt.device)
+        made = ctx.shared["delta_rule_chunks"] = ((put(chunks, 2), put(spans5, 5)), put(rest, 3))
+    return made
 
 
 class GatedDeltaRule(Mixer):
@@ -83,8 +108,10 @@ class GatedDeltaRule(Mixer):
         k.delta_prepare(rows, self.conv_w, state, self.copy_elems, self.tail_at, ctx.positions, ctx.seq_rows, self.beta_at, self.decay_at,
                         self.a_log, self.dt_bias, u, terms, self.heads, self.kv_heads, self.dim, self.vdim, self.dim ** -0.5)
         y = ctx.ws.take((T, self.inner), f32)
-        k.delta_scan(u, terms, state, self.copy_elems, self.tail_at, step_spans(ctx), ctx.positions, ctx.seq_rows, rows, y, self.heads,
-                     self.kv_heads, self.dim, self.vdim, self.taps)
+        long = step_chunks(ctx) if k.delta_chunked_ok(self.kv_heads, self.heads, self.dim, self.vdim) else None
+        chunks, spans = long if long is not None else (None, step_spans(ctx))
+        k.delta_scan(u, terms, state, self.copy_elems, self.tail_at, spans, ctx.positions, ctx.seq_rows, rows, y, self.heads,
+                     self.kv_heads, self.dim, self.vdim, self.taps, chunks=chunks)
         gated = ctx.ws.take((T, self.inner), ctx.rt.dtype)
         k.head_norm_gate(y, rows[:, self.gate_at:], self.gain, self.eps, gated, self.heads)
         k.gemm(gated, self.w_o, out, None, MODE_ADD_F32 if accumulate else MODE_STORE_F32)

@@ -405,7 +405,8 @@ def test_time_mixing_alone_in_portions(heads, dim, rank, width, dtype):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("heads,kv_heads,dim,vdim,conv", [(3, 1, 5, 7, 3), (4, 2, 64, 32, 4), (2, 2, 132, 24, 1), (1, 1, 16, 40, 5),
-                                                          (6, 3, 200, 16, 2), (8, 4, 128, 128, 4), (2, 1, 32, 72, 4), (4, 4, 6, 9, 2)])
+                                                          (6, 3, 200, 16, 2), (8, 4, 128, 128, 4), (2, 1, 32, 72, 4), (4, 4, 6, 9, 2),
+                                                          (3, 3, 96, 80, 3), (6, 2, 32, 16, 2)])
 def test_the_delta_rule_alone_in_portions(heads, kv_heads, dim, vdim, conv, dtype):
     """The walk with its state and the convolutions' kept inputs carried across cuts of every kind: whole, a token at a
     time from the first token on, portions that end inside the convolutions' reach."""
