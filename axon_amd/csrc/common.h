@@ -73,6 +73,15 @@ __device__ inline float load_vec(const void* p, int is_f32, int i) {
   return is_f32 ? ((const float*)p)[i] : bf16_to_float(((const bf16_t*)p)[i]);
 }
 
+// Four neighbouring numbers of such a vector in one load: i is a multiple of 4 and the vector aligned for it.
+__device__ inline float4 load_vec4(const void* p, int is_f32, int i) {
+  if (is_f32) return *reinterpret_cast<const float4*>((const float*)p + i);
+  const uint2 raw = *reinterpret_cast<const uint2*>((const bf16_t*)p + i);
+  union { uint32_t u; float f; } a, b, c, d;
+  a.u = raw.x << 16; b.u = raw.x & 0xffff0000u; c.u = raw.y << 16; d.u = raw.y & 0xffff0000u;
+  return make_float4(a.f, b.f, c.f, d.f);
+}
+
 // Four consecutive elements as floats: one 8- or 16-byte load where `vec` says the address is
 // aligned for it and all four exist, else the `valid` first ones singly and zeros behind them.
 __device__ inline void load4_guarded(const elem_t* __restrict__ p, int valid, bool vec, float out[4]) {

@@ -417,6 +417,105 @@ head_norm_gate_kernel(const float* __restrict__ y, const float* __restrict__ gat
     dst[i] = from_float(((src[i] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * rec_silu(g[i]));
 }
 
+// The same for heads of 4 LANES values (16 to 256): LANES lanes a head, four values each.
+template <int LANES>
+__global__ void __launch_bounds__(256)
+head_norm_gate_vec_kernel(const float* __restrict__ y, const float* __restrict__ gate, long gate_stride, const void* __restrict__ gain,
+                          int gain_is_f32, int gain_per_head, float eps, elem_t* __restrict__ out, long items, int heads) {
+  constexpr int P = 4 * LANES;
+  const long item = ((long)blockIdx.x * 256 + threadIdx.x) / LANES;
+  const int e = 4 * (threadIdx.x % LANES);
+  const bool active = item < items;
+  const long it = active ? item : items - 1;
+  const int h = (int)(it % heads);
+  const float4 v = *reinterpret_cast<const float4*>(y + it * P + e);
+  const float4 g = *reinterpret_cast<const float4*>(gate + it / heads * gate_stride + (long)h * P + e);
+  const float4 w = load_vec4(gain, gain_is_f32, (gain_per_head ? h * P : 0) + e);
+  float ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, v.w * v.w)));
+#pragma unroll
+  for (int off = LANES / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+  const float inv = 1.0f / sqrtf(ss / (float)P + eps);
+  if (!active) return;
+  const float o0 = ((v.x * inv) * w.x) * rec_silu(g.x), o1 = ((v.y * inv) * w.y) * rec_silu(g.y);
+  const float o2 = ((v.z * inv) * w.z) * rec_silu(g.z), o3 = ((v.w * inv) * w.w) * rec_silu(g.w);
+  elem_t* dst = out + it * P + e;
+#if AXON_BF16
+  *reinterpret_cast<uint2*>(dst) = make_uint2(pack2_bf16(o0, o1), pack2_bf16(o2, o3));
+#else
+  *reinterpret_cast<float4*>(dst) = make_float4(o0, o1, o2, o3);
+#endif
+}
+
+// delta_prepare for long steps and up to four taps: a wave a head of queries or keys or up to 256 value channels, over
+// DP_TOKENS tokens in a row, whose inputs and weights stay in registers.  The same sums as the kernel above.
+#define DP_TOKENS 8
+template <int TAPS>
+__global__ void __launch_bounds__(256)
+delta_prepare_run_kernel(const float* __restrict__ in, long in_stride, const elem_t* __restrict__ w, const float* __restrict__ state,
+                         long state_stride, long copy_elems, long tail_at, const int32_t* __restrict__ positions,
+                         const int32_t* __restrict__ seq_rows, int beta_at, int decay_at, const void* __restrict__ a_log,
+                         int a_log_is_f32, const void* __restrict__ dt_bias, int dt_bias_is_f32, float* __restrict__ u,
+                         float* __restrict__ terms, int n_tokens, int heads, int kv_heads, int N, int P, float q_scale) {
+  const int t0 = blockIdx.x * DP_TOKENS, t1 = min(t0 + DP_TOKENS, n_tokens), unit = blockIdx.y * 4 + (threadIdx.x >> 6),
+            lane = threadIdx.x & 63;
+  const int v_units = (heads * P + 255) / 256, channels = 2 * kv_heads * N + heads * P;
+  if (unit > 2 * kv_heads + v_units) return;
+  if (unit == 2 * kv_heads + v_units) {
+    for (int i = lane; i < heads * (t1 - t0); i += 64) {
+      const int t = t0 + i / heads, a = i % heads;
+      const float* row = in + (long)t * in_stride;
+      const float step = rec_softplus(row[decay_at + a] + load_vec(dt_bias, dt_bias_is_f32, a));
+      terms[((long)t * heads + a) * 2] = expf(-(expf(load_vec(a_log, a_log_is_f32, a)) * step));
+      terms[((long)t * heads + a) * 2 + 1] = rec_sigmoid(row[beta_at + a]);
+    }
+    return;
+  }
+  const bool is_v = unit >= 2 * kv_heads;
+  const int c0 = is_v ? 2 * kv_heads * N + 256 * (unit - 2 * kv_heads) : unit * N, size = is_v ? min(256, channels - c0) : N;
+  float wt[DP_KEPT][TAPS], past[DP_KEPT][TAPS];        // past[j][k]: the input k tokens before
+  int c[DP_KEPT];
+#pragma unroll
+  for (int j = 0; j < DP_KEPT; ++j) {
+    c[j] = c0 + min(lane + 64 * j, size - 1);
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) wt[j][k] = to_float(w[(long)c[j] * TAPS + k]);
+  }
+  int slot_before = -1;
+  for (int t = t0; t < t1; ++t) {
+    const int slot = seq_rows[t];
+    const float* row = in + (long)t * in_stride;
+    if (slot != slot_before) {
+      const int inside = rec_inside(seq_rows, t, TAPS - 1);
+      const float* kept = rec_copy_before(state, state_stride, copy_elems, slot, positions[t] - inside) + tail_at;
+#pragma unroll
+      for (int j = 0; j < DP_KEPT; ++j)
+#pragma unroll
+        for (int k = 1; k < TAPS; ++k)
+          past[j][k] = k <= inside ? row[c[j] - (long)k * in_stride] : kept[(long)(TAPS - 1 - (k - inside)) * channels + c[j]];
+      slot_before = slot;
+    }
+    float v[DP_KEPT], ss = 0.0f;
+#pragma unroll
+    for (int j = 0; j < DP_KEPT; ++j) {
+      v[j] = 0.0f;
+      if (64 * j >= size) continue;                    // the whole wave
+      past[j][0] = row[c[j]];
+      float acc = 0.0f;
+#pragma unroll
+      for (int k = 0; k < TAPS; ++k) acc = fmaf(wt[j][k], past[j][TAPS - 1 - k], acc);
+#pragma unroll
+      for (int k = TAPS - 1; k > 0; --k) past[j][k] = past[j][k - 1];
+      v[j] = lane + 64 * j < size ? rec_silu(acc) : 0.0f;
+      ss = fmaf(v[j], v[j], ss);
+    }
+    const float inv = is_v ? 1.0f : (1.0f / sqrtf(wave_sum(ss) + 1e-6f)) * (unit < kv_heads ? q_scale : 1.0f);
+    float* dst = u + (long)t * channels + c0;
+#pragma unroll
+    for (int j = 0; j < DP_KEPT; ++j)
+      if (lane + 64 * j < size) dst[lane + 64 * j] = v[j] * inv;
+  }
+}
+
 }  // namespace
 
 extern "C" int axk_delta_prepare(const float* in, long in_stride, const void* w, int taps, const float* state, long state_stride,
@@ -433,6 +532,17 @@ extern "C" int axk_delta_prepare(const float* in, long in_stride, const void* w,
               "delta_prepare: a state row of %ld floats does not hold two copies of %ld with %d x %ld kept inputs from %ld",
               state_stride, copy_elems, taps - 1, channels, tail_at);
   if (n_tokens == 0) return 0;
+  if (n_tokens >= 256 && taps <= 4) {
+    const dim3 grid(ceil_div(n_tokens, DP_TOKENS), ceil_div(2 * kv_heads + ceil_div(heads * P, 256) + 1, 4));
+#define DP_RUN(TAPS)                                                                                                            \
+  delta_prepare_run_kernel<TAPS><<<grid, 256, 0, (hipStream_t)stream>>>(in, in_stride, (const elem_t*)w, state, state_stride, \
+      copy_elems, tail_at, positions, seq_rows, beta_at, decay_at, a_log, a_log_is_f32, dt_bias, dt_bias_is_f32, u, terms,      \
+      n_tokens, heads, kv_heads, N, P, q_scale)
+    if (taps == 1) DP_RUN(1); else if (taps == 2) DP_RUN(2); else if (taps == 3) DP_RUN(3); else DP_RUN(4);
+#undef DP_RUN
+    AXK_LAUNCH_CHECK("delta_prepare");
+    return 0;
+  }
   delta_prepare_kernel<<<dim3(n_tokens, ceil_div(2 * kv_heads + heads + 1, 4)), 256, 0, (hipStream_t)stream>>>(
       in, in_stride, (const elem_t*)w, taps, state, state_stride, copy_elems, tail_at, positions, seq_rows, beta_at, decay_at, a_log,
       a_log_is_f32, dt_bias, dt_bias_is_f32, u, terms, heads, kv_heads, N, P, q_scale);
@@ -525,6 +635,16 @@ extern "C" int axk_head_norm_gate(const float* y, const float* gate, long gate_s
               "head_norm_gate: bad sizes T=%d heads=%d values=%d gate rows of %ld", n_tokens, heads, P, gate_stride);
   if (n_tokens == 0) return 0;
   const long items = (long)n_tokens * heads;
+  const bool vec = gate_stride % 4 == 0 && (((uintptr_t)y | (uintptr_t)gate | (uintptr_t)gain | (uintptr_t)out) & 15) == 0;
+#define HN_VEC(LANES)                                                                                                       \
+  if (vec && P == 4 * LANES) {                                                                                              \
+    head_norm_gate_vec_kernel<LANES><<<(unsigned)((items * LANES + 255) / 256), 256, 0, (hipStream_t)stream>>>(             \
+        y, gate, gate_stride, gain, gain_is_f32, gain_per_head, eps, (elem_t*)out, items, heads);                           \
+    AXK_LAUNCH_CHECK("head_norm_gate");                                                                                     \
+    return 0;                                                                                                               \
+  }
+  HN_VEC(4) HN_VEC(8) HN_VEC(16) HN_VEC(32) HN_VEC(64)
+#undef HN_VEC
   head_norm_gate_kernel<<<(unsigned)((items + 3) / 4), 256, 0, (hipStream_t)stream>>>(y, gate, gate_stride, gain, gain_is_f32,
                                                                                      gain_per_head, eps, (elem_t*)out, items, heads, P);
   AXK_LAUNCH_CHECK("head_norm_gate");

@@ -323,8 +323,11 @@ extern "C" int axk_layernorm(const float* x, const int32_t* rows, const void* ga
 // tanh_norm: out[r] = n(x[rows[r]]) in the compute dtype.  tanh_norm_add: x[r] += n(y[r]) and, if asked for,
 // next[r] = n'(the new x[r]) in the compute dtype, the norm that the sum goes into.  Four elements a thread where the
 // width is a multiple of 4 (VEC).
-__device__ inline float tanh_norm1(float x, float alpha, const void* w, int w_is_f32, const void* b, int b_is_f32, int i) {
-  return fmaf(tanhf(alpha * x), load_vec(w, w_is_f32, i), load_vec(b, b_is_f32, i));
+__device__ inline float tanh_norm1(float x, float alpha, float w, float b) { return fmaf(tanhf(alpha * x), w, b); }
+__device__ inline float4 tanh_norm4(float4 x, float alpha, const void* w, int w_is_f32, const void* b, int b_is_f32, int e) {
+  const float4 wv = load_vec4(w, w_is_f32, e), bv = load_vec4(b, b_is_f32, e);
+  return make_float4(tanh_norm1(x.x, alpha, wv.x, bv.x), tanh_norm1(x.y, alpha, wv.y, bv.y), tanh_norm1(x.z, alpha, wv.z, bv.z),
+                     tanh_norm1(x.w, alpha, wv.w, bv.w));
 }
 
 template <bool VEC>
@@ -337,12 +340,12 @@ tanh_norm_kernel(const float* __restrict__ x, const int32_t* __restrict__ rows, 
   if (VEC) {
     const int e = 4 * (blockIdx.y * NORM_THREADS + threadIdx.x);
     if (e >= dim) return;
-    const float4 v = *reinterpret_cast<const float4*>(src + e);
-    store4(dst + e, tanh_norm1(v.x, alpha, w, w_is_f32, b, b_is_f32, e), tanh_norm1(v.y, alpha, w, w_is_f32, b, b_is_f32, e + 1),
-           tanh_norm1(v.z, alpha, w, w_is_f32, b, b_is_f32, e + 2), tanh_norm1(v.w, alpha, w, w_is_f32, b, b_is_f32, e + 3));
+    const float4 v = tanh_norm4(*reinterpret_cast<const float4*>(src + e), alpha, w, w_is_f32, b, b_is_f32, e);
+    store4(dst + e, v.x, v.y, v.z, v.w);
     return;
   }
-  for (int i = threadIdx.x; i < dim; i += NORM_THREADS) dst[i] = from_float(tanh_norm1(src[i], alpha, w, w_is_f32, b, b_is_f32, i));
+  for (int i = threadIdx.x; i < dim; i += NORM_THREADS)
+    dst[i] = from_float(tanh_norm1(src[i], alpha, load_vec(w, w_is_f32, i), load_vec(b, b_is_f32, i)));
 }
 
 template <bool VEC>
@@ -354,24 +357,20 @@ tanh_norm_add_kernel(const float* __restrict__ y, float alpha, const void* __res
   if (VEC) {
     const int e = 4 * (blockIdx.y * NORM_THREADS + threadIdx.x);
     if (e >= dim) return;
-    const float4 v = *reinterpret_cast<const float4*>(y + at + e);
     float4 s = *reinterpret_cast<const float4*>(x + at + e);
-    s.x += tanh_norm1(v.x, alpha, w, w_is_f32, b, b_is_f32, e);
-    s.y += tanh_norm1(v.y, alpha, w, w_is_f32, b, b_is_f32, e + 1);
-    s.z += tanh_norm1(v.z, alpha, w, w_is_f32, b, b_is_f32, e + 2);
-    s.w += tanh_norm1(v.w, alpha, w, w_is_f32, b, b_is_f32, e + 3);
+    const float4 v = tanh_norm4(*reinterpret_cast<const float4*>(y + at + e), alpha, w, w_is_f32, b, b_is_f32, e);
+    s.x += v.x; s.y += v.y; s.z += v.z; s.w += v.w;
     *reinterpret_cast<float4*>(x + at + e) = s;
-    if (next)
-      store4(next + at + e, tanh_norm1(s.x, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, e),
-             tanh_norm1(s.y, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, e + 1),
-             tanh_norm1(s.z, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, e + 2),
-             tanh_norm1(s.w, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, e + 3));
+    if (next) {
+      const float4 n = tanh_norm4(s, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, e);
+      store4(next + at + e, n.x, n.y, n.z, n.w);
+    }
     return;
   }
   for (int i = threadIdx.x; i < dim; i += NORM_THREADS) {
-    const float s = x[at + i] + tanh_norm1(y[at + i], alpha, w, w_is_f32, b, b_is_f32, i);
+    const float s = x[at + i] + tanh_norm1(y[at + i], alpha, load_vec(w, w_is_f32, i), load_vec(b, b_is_f32, i));
     x[at + i] = s;
-    if (next) next[at + i] = from_float(tanh_norm1(s, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, i));
+    if (next) next[at + i] = from_float(tanh_norm1(s, next_alpha, load_vec(next_w, next_w_is_f32, i), load_vec(next_b, next_b_is_f32, i)));
   }
 }
 
@@ -379,7 +378,7 @@ extern "C" int axk_tanh_norm(const float* x, const int32_t* rows, float alpha, c
                              void* out, int n_rows, int dim, void* stream) {
   AXK_REQUIRE(n_rows >= 0 && dim > 0, "tanh_norm: bad sizes rows=%d dim=%d", n_rows, dim);
   if (n_rows == 0) return 0;
-  if (dim % 4 == 0 && ((uintptr_t)x & 15) == 0 && ((uintptr_t)out & 15) == 0)
+  if (dim % 4 == 0 && (((uintptr_t)x | (uintptr_t)out | (uintptr_t)w | (uintptr_t)b) & 15) == 0)
     tanh_norm_kernel<true><<<dim3(n_rows, ceil_div(dim, 4 * NORM_THREADS)), NORM_THREADS, 0, (hipStream_t)stream>>>(
         x, rows, alpha, w, w_is_f32, b, b_is_f32, (elem_t*)out, dim);
   else
@@ -395,7 +394,8 @@ extern "C" int axk_tanh_norm_add(const float* y, float alpha, const void* w, int
   AXK_REQUIRE(next == nullptr || (next_w != nullptr && next_b != nullptr), "tanh_norm_add: rows of the next norm without its vectors");
   if (n_rows == 0) return 0;
 #define TN_ARGS y, alpha, w, w_is_f32, b, b_is_f32, x, (elem_t*)next, next_alpha, next_w, next_w_is_f32, next_b, next_b_is_f32, dim
-  if (dim % 4 == 0 && ((uintptr_t)x & 15) == 0 && ((uintptr_t)y & 15) == 0 && ((uintptr_t)next & 15) == 0)
+  if (dim % 4 == 0 && (((uintptr_t)x | (uintptr_t)y | (uintptr_t)next | (uintptr_t)w | (uintptr_t)b | (uintptr_t)next_w |
+                        (uintptr_t)next_b) & 15) == 0)
     tanh_norm_add_kernel<true><<<dim3(n_rows, ceil_div(dim, 4 * NORM_THREADS)), NORM_THREADS, 0, (hipStream_t)stream>>>(TN_ARGS);
   else
     tanh_norm_add_kernel<false><<<n_rows, NORM_THREADS, 0, (hipStream_t)stream>>>(TN_ARGS);
@@ -549,27 +549,39 @@ extern "C" int axk_concat_round(const float* a, int wa, const float* b, int wb, 
 // ---------------------------------------------------------------------------- activations
 // In place.  kind 0: the tanh form of GELU, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)));
 // kind 1: the exact GELU, 0.5 z (1 + erf(z / sqrt 2)); kind 2: the square of relu, max(z, 0)^2.
-__global__ void activation_kernel(elem_t* __restrict__ v, long n, int kind) {
-  const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i >= n) return;
-  const float z = to_float(v[i]);
-  if (kind == 1) {
-    v[i] = from_float((0.5f * z) * (1.0f + erff(z * 0.7071067811865476f)));
-    return;
-  }
+__device__ inline float activation1(float z, int kind) {
+  if (kind == 1) return (0.5f * z) * (1.0f + erff(z * 0.7071067811865476f));
   if (kind == 2) {
     const float p = fmaxf(z, 0.0f);
-    v[i] = from_float(p * p);
-    return;
+    return p * p;
   }
   const float inner = 0.7978845608028654f * (z + 0.044715f * ((z * z) * z));
-  v[i] = from_float((0.5f * z) * (1.0f + tanhf(inner)));
+  return (0.5f * z) * (1.0f + tanhf(inner));
+}
+
+__global__ void activation_kernel(elem_t* __restrict__ v, long n, int kind) {
+  const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) v[i] = from_float(activation1(to_float(v[i]), kind));
+}
+
+// Four elements a thread.
+__global__ void activation_vec_kernel(elem_t* __restrict__ v, long n4, int kind) {
+  const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= n4) return;
+  float z[4];
+  load4_guarded(v + 4 * i, 4, true, z);
+#pragma unroll
+  for (int j = 0; j < 4; ++j) z[j] = activation1(z[j], kind);
+  store4(v + 4 * i, z[0], z[1], z[2], z[3]);
 }
 
 extern "C" int axk_activation(void* v, long n, int kind, void* stream) {
   AXK_REQUIRE(kind >= 0 && kind <= 2, "activation: kind %d is not known (0: gelu, tanh form; 1: gelu, exact; 2: relu squared)", kind);
   if (n <= 0) return 0;
-  activation_kernel<<<(unsigned)((n + 255) / 256), 256, 0, (hipStream_t)stream>>>((elem_t*)v, n, kind);
+  if (n % 4 == 0 && ((uintptr_t)v & 15) == 0)
+    activation_vec_kernel<<<(unsigned)((n / 4 + 255) / 256), 256, 0, (hipStream_t)stream>>>((elem_t*)v, n / 4, kind);
+  else
+    activation_kernel<<<(unsigned)((n + 255) / 256), 256, 0, (hipStream_t)stream>>>((elem_t*)v, n, kind);
   AXK_LAUNCH_CHECK("activation");
   return 0;
 }

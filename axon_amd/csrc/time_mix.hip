@@ -11,80 +11,124 @@
 
 namespace {
 
-// out[s, t] = h[t] + (h'[t] - h[t]) mu[s], s < n_mix: one read of the rows for all uses.
+// out[s, t] = h[t] + (h'[t] - h[t]) mu[s], s < n_mix: one read of the rows for all uses, four channels a thread over
+// `run` tokens in a row.
+__device__ inline void ts_store4(elem_t* dst, const float (&v)[4]) {
+#if AXON_BF16
+  *reinterpret_cast<uint2*>(dst) = make_uint2(pack2_bf16(v[0], v[1]), pack2_bf16(v[2], v[3]));
+#else
+  *reinterpret_cast<float4*>(dst) = make_float4(v[0], v[1], v[2], v[3]);
+#endif
+}
+
+template <int MIXES>        // how many uses, or 0: any number
 __global__ void __launch_bounds__(256)
 token_shift_kernel(const elem_t* __restrict__ h, const float* __restrict__ mu, int n_mix, const float* __restrict__ state,
                    long state_stride, long copy_elems, long tail_at, const int32_t* __restrict__ positions,
-                   const int32_t* __restrict__ seq_rows, elem_t* __restrict__ out, int n_tokens, int width) {
-  const int t = blockIdx.x, c = 4 * (blockIdx.y * 256 + threadIdx.x);
+                   const int32_t* __restrict__ seq_rows, elem_t* __restrict__ out, int n_tokens, int width, int run) {
+  const int t0 = blockIdx.x * run, t1 = min(t0 + run, n_tokens), c = 4 * (blockIdx.y * 256 + threadIdx.x);
   if (c >= width) return;
   const int valid = min(4, width - c);
   const bool vec = (width & 3) == 0;
-  const int slot = seq_rows[t];
-  float cur[4], prev[4];
-  load4_guarded(h + (long)t * width + c, valid, vec, cur);
-  if (t > 0 && seq_rows[t - 1] == slot) {
-    load4_guarded(h + (long)(t - 1) * width + c, valid, vec, prev);
-  } else {
-    const float* kept = rec_copy_before(state, state_stride, copy_elems, slot, positions[t]) + tail_at + c;
+  float m[MIXES > 0 ? MIXES : 1][4];
+  if (MIXES > 0) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) prev[i] = i < valid ? kept[i] : 0.0f;
+    for (int s = 0; s < MIXES; ++s)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) m[s][i] = i < valid ? mu[(long)s * width + c + i] : 0.0f;
   }
-  for (int s = 0; s < n_mix; ++s) {
-    const float* m = mu + (long)s * width + c;
-    elem_t* dst = out + ((long)s * n_tokens + t) * width + c;
-    elem_t v[4];
+  float prev[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  int slot_before = -1;
+  for (int t = t0; t < t1; ++t) {
+    const int slot = seq_rows[t];
+    if (slot != slot_before) {
+      if (t > 0 && seq_rows[t - 1] == slot) {
+        load4_guarded(h + (long)(t - 1) * width + c, valid, vec, prev);
+      } else {
+        const float* kept = rec_copy_before(state, state_stride, copy_elems, slot, positions[t]) + tail_at + c;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = from_float(i < valid ? fmaf(prev[i] - cur[i], m[i], cur[i]) : 0.0f);
-    if (vec) {
-#if AXON_BF16
-      *reinterpret_cast<uint2*>(dst) = make_uint2(v[0].bits | ((uint32_t)v[1].bits << 16), v[2].bits | ((uint32_t)v[3].bits << 16));
-#else
-      *reinterpret_cast<float4*>(dst) = make_float4(v[0], v[1], v[2], v[3]);
-#endif
-    } else {
-      for (int i = 0; i < valid; ++i) dst[i] = v[i];
+        for (int i = 0; i < 4; ++i) prev[i] = i < valid ? kept[i] : 0.0f;
+      }
+      slot_before = slot;
     }
+    float cur[4];
+    load4_guarded(h + (long)t * width + c, valid, vec, cur);
+    const int n = MIXES > 0 ? MIXES : n_mix;
+#pragma unroll
+    for (int s = 0; s < n; ++s) {
+      elem_t* dst = out + ((long)s * n_tokens + t) * width + c;
+      float v[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float share = MIXES > 0 ? m[MIXES > 0 ? s : 0][i] : i < valid ? mu[(long)s * width + c + i] : 0.0f;
+        v[i] = fmaf(prev[i] - cur[i], share, cur[i]);
+      }
+      if (vec) ts_store4(dst, v);
+      else
+        for (int i = 0; i < valid; ++i) dst[i] = from_float(v[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) prev[i] = cur[i];
   }
 }
 
-// w[t, c] = exp(-exp(w0[c] + sum_k W2[c, k] tanh(low[t, k]))), all in 32-bit: tiles of 16 tokens x 64 channels, the
-// rank in pieces of 64 through LDS, a chain in ascending k an output.
-#define TD_TOKENS 16
+// w[t, c] = exp(-exp(w0[c] + sum_k W2[c, k] tanh(low[t, k]))), all in 32-bit: tiles of 16 OWN tokens x 64 channels, a
+// thread OWN tokens x 4 channels, the rank in pieces of 64 through LDS, a chain in ascending k an output.
 #define TD_CHANNELS 64
 #define TD_RANK 64
+template <int OWN>
 __global__ void __launch_bounds__(256)
 time_mix_decay_kernel(const float* __restrict__ low, const elem_t* __restrict__ w2, const void* __restrict__ w0, int w0_is_f32,
                       float* __restrict__ w, int n_tokens, int channels, int rank) {
-  __shared__ float ts[TD_RANK][TD_TOKENS];
-  __shared__ float ws[TD_CHANNELS][TD_RANK + 1];
-  const int t0 = blockIdx.y * TD_TOKENS, c0 = blockIdx.x * TD_CHANNELS;
-  const int tx = threadIdx.x & 63, ty = threadIdx.x >> 6;
-  float acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  constexpr int TOKENS = 16 * OWN;
+  __shared__ __align__(16) float ts[TD_RANK][TOKENS + 4];
+  __shared__ __align__(16) float ws[TD_RANK][TD_CHANNELS + 4];
+  const int t0 = blockIdx.y * TOKENS, c0 = blockIdx.x * TD_CHANNELS;
+  const int tx = threadIdx.x & 15, ty = threadIdx.x >> 4;
+  float acc[OWN][4];
+#pragma unroll
+  for (int i = 0; i < OWN; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = 0.0f;
   for (int k0 = 0; k0 < rank; k0 += TD_RANK) {
     const int n = min(TD_RANK, rank - k0);
     __syncthreads();
-    for (int i = threadIdx.x; i < TD_TOKENS * TD_RANK; i += 256) {
-      const int t = i / TD_RANK, k = i % TD_RANK;
+#pragma unroll
+    for (int it = 0; it < TOKENS * TD_RANK / 256; ++it) {
+      const int i = it * 256 + threadIdx.x, t = i / TD_RANK, k = i % TD_RANK;
       ts[k][t] = k < n && t0 + t < n_tokens ? tanhf(low[(long)(t0 + t) * rank + k0 + k]) : 0.0f;
     }
-    for (int i = threadIdx.x; i < TD_CHANNELS * TD_RANK; i += 256) {
-      const int c = i / TD_RANK, k = i % TD_RANK;
-      ws[c][k] = k < n && c0 + c < channels ? to_float(w2[(long)(c0 + c) * rank + k0 + k]) : 0.0f;
+#pragma unroll
+    for (int it = 0; it < TD_CHANNELS * TD_RANK / 1024; ++it) {
+      const int i = it * 256 + threadIdx.x, c = i / (TD_RANK / 4), k = 4 * (i % (TD_RANK / 4));
+      float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+      if (k < n && c0 + c < channels) load4_guarded(w2 + (long)(c0 + c) * rank + k0 + k, n - k, (rank & 3) == 0, v);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) ws[k + j][c] = v[j];
     }
     __syncthreads();
-    for (int k = 0; k < n; ++k) {
-      const float x = ws[tx][k];
+#pragma unroll 8
+    for (int k = 0; k < TD_RANK; ++k) {              // behind the rank: zeros
+      const float4 x = *reinterpret_cast<const float4*>(&ws[k][4 * tx]);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) acc[i] = fmaf(ts[k][4 * ty + i], x, acc[i]);
+      for (int i = 0; i < OWN; ++i) {
+        const float a = ts[k][OWN * ty + i];
+        acc[i][0] = fmaf(a, x.x, acc[i][0]);
+        acc[i][1] = fmaf(a, x.y, acc[i][1]);
+        acc[i][2] = fmaf(a, x.z, acc[i][2]);
+        acc[i][3] = fmaf(a, x.w, acc[i][3]);
+      }
     }
   }
-  if (c0 + tx >= channels) return;
-  const float base = load_vec(w0, w0_is_f32, c0 + tx);
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    const int t = t0 + 4 * ty + i;
-    if (t < n_tokens) w[(long)t * channels + c0 + tx] = expf(-expf(acc[i] + base));
+  for (int i = 0; i < OWN; ++i) {
+    const int t = t0 + OWN * ty + i;
+    if (t >= n_tokens) continue;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int c = c0 + 4 * tx + j;
+      if (c < channels) w[(long)t * channels + c] = expf(-expf(acc[i][j] + load_vec(w0, w0_is_f32, c)));
+    }
   }
 }
 
@@ -282,8 +326,10 @@ extern "C" int axk_token_shift(const void* h, const float* mu, int n_mix, const 
               copy_elems, width, tail_at);
   AXK_REQUIRE(((uintptr_t)h & 15) == 0 && ((uintptr_t)out & 15) == 0, "token_shift: rows are not 16-byte aligned");
   if (n_tokens == 0) return 0;
-  token_shift_kernel<<<dim3(n_tokens, ceil_div(width, 1024)), 256, 0, (hipStream_t)stream>>>(
-      (const elem_t*)h, mu, n_mix, state, state_stride, copy_elems, tail_at, positions, seq_rows, (elem_t*)out, n_tokens, width);
+  const int run = n_tokens >= 512 ? 8 : 1;
+  auto kernel = n_mix == 5 ? token_shift_kernel<5> : token_shift_kernel<0>;
+  kernel<<<dim3(ceil_div(n_tokens, run), ceil_div(width, 1024)), 256, 0, (hipStream_t)stream>>>(
+      (const elem_t*)h, mu, n_mix, state, state_stride, copy_elems, tail_at, positions, seq_rows, (elem_t*)out, n_tokens, width, run);
   AXK_LAUNCH_CHECK("token_shift");
   return 0;
 }
@@ -291,10 +337,14 @@ extern "C" int axk_token_shift(const void* h, const float* mu, int n_mix, const 
 extern "C" int axk_time_mix_decay(const float* low, const void* w2, const void* w0, int w0_is_f32, float* w, int n_tokens,
                                   int channels, int rank, void* stream) {
   AXK_REQUIRE(n_tokens >= 0 && channels > 0 && rank > 0, "time_mix_decay: bad sizes T=%d channels=%d rank=%d", n_tokens, channels, rank);
-  AXK_REQUIRE(ceil_div(n_tokens, TD_TOKENS) <= 65535, "time_mix_decay: %d tokens in one step", n_tokens);
+  AXK_REQUIRE(n_tokens <= 65535 * 16 && ((uintptr_t)w2 & 15) == 0, "time_mix_decay: %d tokens in one step, or w2 is not aligned", n_tokens);
   if (n_tokens == 0) return 0;
-  time_mix_decay_kernel<<<dim3(ceil_div(channels, TD_CHANNELS), ceil_div(n_tokens, TD_TOKENS)), 256, 0, (hipStream_t)stream>>>(
-      low, (const elem_t*)w2, w0, w0_is_f32, w, n_tokens, channels, rank);
+  if (n_tokens >= 512)
+    time_mix_decay_kernel<4><<<dim3(ceil_div(channels, TD_CHANNELS), ceil_div(n_tokens, 64)), 256, 0, (hipStream_t)stream>>>(
+        low, (const elem_t*)w2, w0, w0_is_f32, w, n_tokens, channels, rank);
+  else
+    time_mix_decay_kernel<1><<<dim3(ceil_div(channels, TD_CHANNELS), ceil_div(n_tokens, 16)), 256, 0, (hipStream_t)stream>>>(
+        low, (const elem_t*)w2, w0, w0_is_f32, w, n_tokens, channels, rank);
   AXK_LAUNCH_CHECK("time_mix_decay");
   return 0;
 }

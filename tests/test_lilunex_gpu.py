@@ -214,14 +214,14 @@ def test_unequal_requests_side_by_side_with_pages_and_slots_used_again(folders, 
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("name", ["A", "B", "E"])
+@pytest.mark.parametrize("name", ["A", "B", "C", "E"])
 def test_long_stretches_run_the_scans_in_segments(folders, plain_logits, name, dtype):
     """Hundreds of tokens of a request in one step: the scans cut the stretch into pieces that run side by side; the
     state they leave is what later portions and decoded tokens go on from.  Beside a short request in the same step."""
-    n = 420
+    n = 720
     long, short = sequences(name, [n, 9], seed=5)
     page = MODELS[name]["page"]
-    eng = engine_for(folders(name), dtype, page, -(-n // page) + 4, max_seqs=2, max_seq_len=448, max_batch_tokens=512)
+    eng = engine_for(folders(name), dtype, page, -(-n // page) + 4, max_seqs=2, max_seq_len=768, max_batch_tokens=544)
     seen = []
     inner = eng.rt.k.wkv_scan
 
@@ -230,7 +230,7 @@ def test_long_stretches_run_the_scans_in_segments(folders, plain_logits, name, d
         return inner(*a, segments=segments, **kw)
     eng.rt.k.wkv_scan = logged
     try:
-        got, chose = run_schedule(eng, name, {"a": long, "b": short}, [[("a", 300), ("b", 4)], [("a", 1), ("b", 5)], [("a", 2)], [("a", 117)]])
+        got, chose = run_schedule(eng, name, {"a": long, "b": short}, [[("a", 530), ("b", 4)], [("a", 1), ("b", 5)], [("a", 2)], [("a", 187)]])
     finally:
         del eng.rt.k.wkv_scan
     assert any(k is not None and k > 2 for k in seen) and any(k is None for k in seen)
