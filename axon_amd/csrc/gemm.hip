@@ -1,11 +1,12 @@
 // Matrix products out = X [M, K] . W [N, K]^T with a bias / residual epilogue.
 //
-// The rule every variant keeps: the K-reduction of one output element is one chain in
+// The rule every variant keeps: the K-reduction of one output element is one order of additions in
 // ascending k that does not depend on M, on the tile shape or on what else is in the batch
 // (the reference states the rule for its own kernels: src/cuda/decode.cu:352-369,
 // src/cuda/prefill.cu:6-16).  Rows only ride along.
 //
-// gemm_fma: any M, N, K and strides, 32-bit FMA, one chain per output: the float32 build's
+// gemm_fma: any M, N, K and strides, 32-bit FMA, a chain per output and 32 k, whose sums are added in
+// ascending order (a third of the rounding of one chain over all k): the float32 build's
 // product (true 32-bit), and the bfloat16 build's fallback for shapes the MFMA kernels refuse.
 #include "api.h"
 #include "common.h"
@@ -13,6 +14,7 @@
 
 #define FMA_BN 64
 #define FMA_BK 16
+#define FMA_PART 32    // k of one chain
 #define FMA_THREADS 256
 
 // BM rows x 64 columns per block of 256 threads; thread (ty, tx) owns RM = BM / 16 rows and
@@ -30,13 +32,13 @@ gemm_fma_kernel(const elem_t* __restrict__ x, int x_stride, const elem_t* __rest
   const int tx = tid & 15, ty = tid >> 4;
   const int m0 = blockIdx.y * BM, n0 = blockIdx.x * FMA_BN;
 
-  float acc[RM][4], acc_up[GLU ? RM : 1][4];
+  float acc[RM][4], acc_up[GLU ? RM : 1][4], sum[RM][4], sum_up[GLU ? RM : 1][4];
 #pragma unroll
   for (int i = 0; i < RM; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-      acc[i][j] = 0.0f;
-      if (GLU) acc_up[i][j] = 0.0f;
+      acc[i][j] = sum[i][j] = 0.0f;
+      if (GLU) acc_up[i][j] = sum_up[i][j] = 0.0f;
     }
 
   // loader: each thread brings 4 consecutive k of one row, a step ahead of the products
@@ -79,6 +81,16 @@ gemm_fma_kernel(const elem_t* __restrict__ x, int x_stride, const elem_t* __rest
           for (int j = 0; j < 4; ++j) acc_up[i][j] = fmaf(a[i], b[j], acc_up[i][j]);
       }
     }
+    if ((k0 + FMA_BK) % FMA_PART == 0 || k0 + FMA_BK >= K) {
+#pragma unroll
+      for (int i = 0; i < RM; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          sum[i][j] += acc[i][j];
+          acc[i][j] = 0.0f;
+          if (GLU) { sum_up[i][j] += acc_up[i][j]; acc_up[i][j] = 0.0f; }
+        }
+    }
     __syncthreads();
   }
 
@@ -90,10 +102,10 @@ gemm_fma_kernel(const elem_t* __restrict__ x, int x_stride, const elem_t* __rest
     for (int j = 0; j < 4; ++j) {
       const int n = n0 + tx * 4 + j;
       if (n >= N) continue;
-      float v = acc[i][j];
+      float v = sum[i][j];
       if (bias) v += load_vec(bias, bias_is_f32, n);
       const size_t at = (size_t)m * out_stride + n;
-      if (GLU) ((elem_t*)out)[at] = from_float(swiglu1(v, acc_up[i][j]));
+      if (GLU) ((elem_t*)out)[at] = from_float(swiglu1(v, sum_up[i][j]));
       else if (mode == MODE_STORE) ((elem_t*)out)[at] = from_float(v);
       else if (mode == MODE_ADD_F32) ((float*)out)[at] += v;
       else ((float*)out)[at] = v;
@@ -104,7 +116,7 @@ gemm_fma_kernel(const elem_t* __restrict__ x, int x_stride, const elem_t* __rest
 // Up to 16 rows (a decoding step): 16 rows x 16 columns a block, one output a thread, K in steps
 // of 256 through LDS, the next step's loads in flight while this one is multiplied.  Such a
 // product only waits for W, so it wants many blocks with much in flight each (the tile above
-// gives N / 64 blocks with 4 KB each).  The chain of an output is the same: fmaf in ascending k.
+// gives N / 64 blocks with 4 KB each).  The chains of an output are the same.
 #define FEW_BK 256
 #define FEW_LD (FEW_BK + 4)   // rows 4 banks apart: the 16 rows a wave reads fall into all 64 banks
 template <bool GLU>
@@ -141,38 +153,43 @@ gemm_fma_few_rows_kernel(const elem_t* __restrict__ x, int x_stride, const elem_
     }
   };
 
-  float acc = 0.0f, acc_up = 0.0f;
+  float sum = 0.0f, sum_up = 0.0f;
   fetch(0);
   for (int k0 = 0; k0 < K; k0 += FEW_BK) {
     stage();
     __syncthreads();
     if (k0 + FEW_BK < K) fetch(k0 + FEW_BK);
-    const int k_end = min(FEW_BK, K - k0);   // beyond K the last group of four holds zeros
-#pragma unroll 4
-    for (int kk = 0; kk < k_end; kk += 4) {
-      const float4 a = *reinterpret_cast<const float4*>(&xs[ty][kk]);
-      const float4 b = *reinterpret_cast<const float4*>(&ws[tx][kk]);
-      acc = fmaf(a.x, b.x, acc);
-      acc = fmaf(a.y, b.y, acc);
-      acc = fmaf(a.z, b.z, acc);
-      acc = fmaf(a.w, b.w, acc);
-      if (GLU) {
-        const float4 u = *reinterpret_cast<const float4*>(&us[tx][kk]);
-        acc_up = fmaf(a.x, u.x, acc_up);
-        acc_up = fmaf(a.y, u.y, acc_up);
-        acc_up = fmaf(a.z, u.z, acc_up);
-        acc_up = fmaf(a.w, u.w, acc_up);
+    const int k_end = min(FEW_BK, K - k0);   // beyond K the stage holds zeros
+    for (int part = 0; part < k_end; part += FMA_PART) {
+      float acc = 0.0f, acc_up = 0.0f;
+#pragma unroll
+      for (int i = 0; i < FMA_PART; i += 4) {    // beyond K, too: zeros
+        const float4 a = *reinterpret_cast<const float4*>(&xs[ty][part + i]);
+        const float4 b = *reinterpret_cast<const float4*>(&ws[tx][part + i]);
+        acc = fmaf(a.x, b.x, acc);
+        acc = fmaf(a.y, b.y, acc);
+        acc = fmaf(a.z, b.z, acc);
+        acc = fmaf(a.w, b.w, acc);
+        if (GLU) {
+          const float4 u = *reinterpret_cast<const float4*>(&us[tx][part + i]);
+          acc_up = fmaf(a.x, u.x, acc_up);
+          acc_up = fmaf(a.y, u.y, acc_up);
+          acc_up = fmaf(a.z, u.z, acc_up);
+          acc_up = fmaf(a.w, u.w, acc_up);
+        }
       }
+      sum += acc;
+      sum_up += acc_up;
     }
     __syncthreads();
   }
 
   const int m = ty, n = n0 + tx;
   if (m >= M || n >= N) return;
-  float v = acc;
+  float v = sum;
   if (bias) v += load_vec(bias, bias_is_f32, n);
   const size_t at = (size_t)m * out_stride + n;
-  if (GLU) ((elem_t*)out)[at] = from_float(swiglu1(v, acc_up));
+  if (GLU) ((elem_t*)out)[at] = from_float(swiglu1(v, sum_up));
   else if (mode == MODE_STORE) ((elem_t*)out)[at] = from_float(v);
   else if (mode == MODE_ADD_F32) ((float*)out)[at] += v;
   else ((float*)out)[at] = v;
