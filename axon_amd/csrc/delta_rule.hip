@@ -170,23 +170,26 @@ delta_scan_kernel(const float* __restrict__ u, const float* __restrict__ terms, 
 // decay of 0 is nothing special), the two right-hand sides by forward substitution, a column a thread with its 64 rows
 // in registers.  The second walks a request's chunks per (head, sixteen value dims).  The sums of a token are those of
 // the walk token by token in another order.
-// Layouts of a (chunk, head), item = chunk heads + head: U' [64][P], W [64][N], kt [N][64], M [64][64] (its upper tiles
-// are not written), b [64].  Rows beyond the chunk's tokens have g 1 and beta 0: they change nothing.
+// Of a (chunk, head), item = chunk heads + head: U' [64][P] and b [64] row by row; W [64][N], M [64][64] (its upper tiles
+// are not written) and kt [N][64], and of a (chunk, query head) Q [64][N], as the walk's operands, tile of sixteen rows
+// by tile, sixteen columns by sixteen, in the order of a wave's lanes (dc_at): a load of four floats a lane then reads
+// 1 KB side by side.  Rows beyond the chunk's tokens have g 1 and beta 0: they change nothing.
 #define DC 64
 typedef __attribute__((ext_vector_type(4))) float dc_f32x4;
 __device__ inline dc_f32x4 dc_load(const float* p) { return *reinterpret_cast<const dc_f32x4*>(p); }
-// four chained products over sixteen k: lane l holds rows l % 16 at k = 4 (l / 16) .. + 3 of either operand
-__device__ inline dc_f32x4 dc_mfma(dc_f32x4 a, dc_f32x4 b, dc_f32x4 c) {
-#pragma unroll
-  for (int j = 0; j < 4; ++j) c = __builtin_amdgcn_mfma_f32_16x16x4f32(a[j], b[j], c, 0, 0, 0);
-  return c;
+// where a matrix of 16 cols16 columns keeps (row, col): lane l = row % 16 + 16 (col % 16 / 4) of block (row / 16, col / 16)
+__device__ inline long dc_at(int row, int col, int cols16) {
+  return ((long)(row / 16 * cols16 + col / 16) * 64 + row % 16 + 16 * (col % 16 / 4)) * 4 + col % 4;
 }
+// sixteen k of a product are four chained instructions: lane l holds rows l % 16 at k = 4 (l / 16) .. + 3 of either
+// operand, instruction j takes their j-th.  Independent chains run interleaved, so that none waits for itself.
+#define DC_MFMA(acc, a, b, j) acc = __builtin_amdgcn_mfma_f32_16x16x4f32((a)[j], (b)[j], acc, 0, 0, 0)
 
 template <int NT>
 __global__ void __launch_bounds__(256)
 delta_chunk_terms_kernel(const float* __restrict__ u, const float* __restrict__ terms, const int32_t* __restrict__ chunks, int heads,
                          int kv_heads, int P, float* __restrict__ up, float* __restrict__ w, float* __restrict__ kt,
-                         float* __restrict__ m, float* __restrict__ b) {
+                         float* __restrict__ m, float* __restrict__ q, float* __restrict__ b) {
   constexpr int N = 16 * NT, ROW = DC + 4;
   __shared__ float D[DC][DC + 1];
   __shared__ __align__(16) float A[DC][ROW];
@@ -213,6 +216,11 @@ delta_chunk_terms_kernel(const float* __restrict__ u, const float* __restrict__ 
   dc_f32x4 qf[NT], kf[NT];
 #pragma unroll
   for (int c = 0; c < NT; ++c) { qf[c] = dc_load(mine + 16 * c); kf[c] = dc_load(mine + (long)kv_heads * N + 16 * c); }
+  if (h % (heads / kv_heads) == 0) {
+    float* dst = q + ((long)blockIdx.y * kv_heads + kh) * DC * N;
+#pragma unroll
+    for (int c = 0; c < NT; ++c) *reinterpret_cast<dc_f32x4*>(dst + ((wave * NT + c) * 64 + lane) * 4) = qf[c];
+  }
   __syncthreads();
   for (int jt = 0; jt <= wave; ++jt) {
     const float* other = keys + (long)(first + min(16 * jt + r, count - 1)) * channels + 4 * g4;
@@ -220,15 +228,15 @@ delta_chunk_terms_kernel(const float* __restrict__ u, const float* __restrict__ 
 #pragma unroll
     for (int c = 0; c < NT; ++c) {
       const dc_f32x4 o = dc_load(other + 16 * c);
-      kk = dc_mfma(kf[c], o, kk);
-      qk = dc_mfma(qf[c], o, qk);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { DC_MFMA(kk, kf[c], o, j); DC_MFMA(qk, qf[c], o, j); }
     }
     const int j = 16 * jt + r;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int i = 16 * wave + 4 * g4 + e;
       A[i][j] = j < i ? (betas[i] * D[i][j]) * kk[e] : 0.0f;
-      m[(item * DC + i) * DC + j] = j <= i ? D[i][j] * qk[e] : 0.0f;
+      m[item * DC * DC + dc_at(i, j, DC / 16)] = j <= i ? D[i][j] * qk[e] : 0.0f;
     }
   }
   __syncthreads();
@@ -240,10 +248,10 @@ delta_chunk_terms_kernel(const float* __restrict__ u, const float* __restrict__ 
 #pragma unroll
     for (int i = 0; i < DC; ++i) X[i] = src[(long)(first + min(i, count - 1)) * channels];
     if (!is_v) {
-      float* dst = kt + (item * N + col - P) * DC;
+      float* dst = kt + item * N * DC;
 #pragma unroll
       for (int i = 0; i < DC; i += 4)
-        *reinterpret_cast<dc_f32x4*>(dst + i) = dc_f32x4{X[i] * D[DC - 1][i], X[i + 1] * D[DC - 1][i + 1], X[i + 2] * D[DC - 1][i + 2],
+        *reinterpret_cast<dc_f32x4*>(dst + dc_at(col - P, i, DC / 16)) = dc_f32x4{X[i] * D[DC - 1][i], X[i + 1] * D[DC - 1][i + 1], X[i + 2] * D[DC - 1][i + 2],
                                                          X[i + 3] * D[DC - 1][i + 3]};
     }
 #pragma unroll
@@ -261,10 +269,15 @@ delta_chunk_terms_kernel(const float* __restrict__ u, const float* __restrict__ 
       X[i] = x;
       __builtin_amdgcn_sched_barrier(0);       // a row of A at a time in registers
     }
-    float* dst = is_v ? up + item * DC * P + col : w + item * DC * N + col - P;
-    const int step = is_v ? P : N;
+    if (is_v) {
+      float* dst = up + item * DC * P + col;
 #pragma unroll
-    for (int i = 0; i < DC; ++i) dst[(long)i * step] = X[i];
+      for (int i = 0; i < DC; ++i) dst[(long)i * P] = X[i];
+    } else {
+      float* dst = w + item * DC * N;
+#pragma unroll
+      for (int i = 0; i < DC; ++i) dst[dc_at(i, col - P, NT)] = X[i];
+    }
   }
 }
 
@@ -281,7 +294,7 @@ struct DeltaChunkOperands {
 
 template <int NT>
 __global__ void __launch_bounds__(256)
-delta_chunk_walk_kernel(const float* __restrict__ u, const float* __restrict__ up, const float* __restrict__ w,
+delta_chunk_walk_kernel(const float* __restrict__ q, const float* __restrict__ up, const float* __restrict__ w,
                         const float* __restrict__ kt, const float* __restrict__ m, const float* __restrict__ b,
                         const int32_t* __restrict__ spans5, const int32_t* __restrict__ positions, float* __restrict__ state,
                         long state_stride, long copy_elems, long tail_at, const float* __restrict__ conv_in, long conv_in_stride,
@@ -301,6 +314,7 @@ delta_chunk_walk_kernel(const float* __restrict__ u, const float* __restrict__ u
   dc_f32x4 S[TILES];
 #pragma unroll
   for (int tt = 0; tt < TILES; ++tt) {
+    S[tt] = dc_f32x4{0.0f, 0.0f, 0.0f, 0.0f};
     const int tile = wave + 4 * tt;
     if (tile < NT) {
       S[tt] = dc_load(from + s_at + 16 * tile);
@@ -309,21 +323,20 @@ delta_chunk_walk_kernel(const float* __restrict__ u, const float* __restrict__ u
   }
   auto fetch = [&](Ops& o, int c) {
     const long item = (long)(chunk0 + c) * heads + h;
-    const int t0 = first + DC * c, last = first + count - 1;
-    const float* wr = w + (item * DC + 16 * wave + r) * N + 4 * g4;
-    const float* qr = u + (long)min(t0 + 16 * wave + r, last) * channels + (long)kh * N + 4 * g4;
+    const float* wr = w + item * DC * N + (wave * NT * 64 + lane) * 4;
+    const float* qr = q + ((long)(chunk0 + c) * kv_heads + kh) * DC * N + (wave * NT * 64 + lane) * 4;
 #pragma unroll
-    for (int i = 0; i < NT; ++i) { o.w[i] = dc_load(wr + 16 * i); o.q[i] = dc_load(qr + 16 * i); }
-    const float* mr = m + (item * DC + 16 * wave + r) * DC + 4 * g4;
+    for (int i = 0; i < NT; ++i) { o.w[i] = dc_load(wr + 256 * i); o.q[i] = dc_load(qr + 256 * i); }
+    const float* mr = m + item * DC * DC + (wave * 4 * 64 + lane) * 4;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      if (i <= wave) o.m[i] = dc_load(mr + 16 * i);
+      if (i <= wave) o.m[i] = dc_load(mr + 256 * i);
 #pragma unroll
     for (int tt = 0; tt < TILES; ++tt)
       if (wave + 4 * tt < NT) {
-        const float* kr = kt + (item * N + 16 * (wave + 4 * tt) + r) * DC + 4 * g4;
+        const float* kr = kt + item * N * DC + ((wave + 4 * tt) * 4 * 64 + lane) * 4;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o.k[tt][i] = dc_load(kr + 16 * i);
+        for (int i = 0; i < 4; ++i) o.k[tt][i] = dc_load(kr + 256 * i);
       }
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
@@ -333,40 +346,49 @@ delta_chunk_walk_kernel(const float* __restrict__ u, const float* __restrict__ u
     o.b_last = b[item * DC + DC - 1];
   };
   auto work = [&](const Ops& o, int c) {
-    dc_f32x4 ws = {0.0f, 0.0f, 0.0f, 0.0f}, out = {0.0f, 0.0f, 0.0f, 0.0f};
+    // two halves of the sum over the state's rows, two products: four chains
+    dc_f32x4 ws[2] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}}, qs[2] = {ws[0], ws[0]};
+    dc_f32x4 s[NT];
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const dc_f32x4 s = dc_load(&Sl[r][16 * i + 4 * g4]);
-      ws = dc_mfma(o.w[i], s, ws);
-      out = dc_mfma(o.q[i], s, out);
-    }
-    dc_f32x4 mine;
+    for (int i = 0; i < NT; ++i) s[i] = dc_load(&Sl[r][16 * i + 4 * g4]);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) { mine[e] = o.up[e] - ws[e]; out[e] *= o.b[e]; }
+    for (int i = 0; i < NT / 2; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        DC_MFMA(ws[0], o.w[i], s[i], j);
+        DC_MFMA(qs[0], o.q[i], s[i], j);
+        DC_MFMA(ws[1], o.w[NT / 2 + i], s[NT / 2 + i], j);
+        DC_MFMA(qs[1], o.q[NT / 2 + i], s[NT / 2 + i], j);
+      }
+    dc_f32x4 mine, out;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { mine[e] = o.up[e] - (ws[0][e] + ws[1][e]); out[e] = (qs[0][e] + qs[1][e]) * o.b[e]; }
     *reinterpret_cast<dc_f32x4*>(&Ul[r][16 * wave + 4 * g4]) = mine;
     __syncthreads();                       // every wave's part of U is there, and every wave has read the state
     dc_f32x4 all[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) all[i] = dc_load(&Ul[r][16 * i + 4 * g4]);
 #pragma unroll
+    for (int tt = 0; tt < TILES; ++tt)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) S[tt][e] *= o.b_last;
+#pragma unroll
     for (int i = 0; i < 4; ++i)
-      if (i <= wave) out = dc_mfma(o.m[i], all[i], out);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        if (i <= wave) DC_MFMA(out, o.m[i], all[i], j);
+#pragma unroll
+        for (int tt = 0; tt < TILES; ++tt)
+          if (wave + 4 * tt < NT) DC_MFMA(S[tt], o.k[tt][i], all[i], j);
+      }
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int i = DC * c + 16 * wave + 4 * g4 + e;
       if (i < count) y[((long)(first + i) * heads + h) * P + p0 + r] = out[e];
     }
 #pragma unroll
-    for (int tt = 0; tt < TILES; ++tt) {
-      const int tile = wave + 4 * tt;
-      if (tile < NT) {
-#pragma unroll
-        for (int e = 0; e < 4; ++e) S[tt][e] *= o.b_last;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) S[tt] = dc_mfma(o.k[tt][i], all[i], S[tt]);
-        *reinterpret_cast<dc_f32x4*>(&Sl[r][16 * tile + 4 * g4]) = S[tt];
-      }
-    }
+    for (int tt = 0; tt < TILES; ++tt)
+      if (wave + 4 * tt < NT) *reinterpret_cast<dc_f32x4*>(&Sl[r][16 * (wave + 4 * tt) + 4 * g4]) = S[tt];
     __syncthreads();
   };
   Ops even, odd;
@@ -589,7 +611,7 @@ extern "C" int axk_delta_chunked_ok(int kv_heads, int heads, int N, int P) {
 
 // The floats of workspace that axk_delta_chunked wants for this many chunks.
 extern "C" long axk_delta_chunked_workspace(int n_chunks, int heads, int N, int P) {
-  return (long)n_chunks * heads * DC * (2L * N + P + DC + 1);
+  return (long)n_chunks * heads * DC * (3L * N + P + DC + 1);
 }
 
 extern "C" int axk_delta_chunked(const float* u, const float* terms, float* state, long state_stride, long copy_elems, long tail_at,
@@ -614,12 +636,13 @@ extern "C" int axk_delta_chunked(const float* u, const float* terms, float* stat
   float* w = up + items * DC * P;
   float* kt = w + items * DC * N;
   float* m = kt + items * DC * N;
-  float* b = m + items * DC * DC;
+  float* q = m + items * DC * DC;
+  float* b = q + (long)n_chunks * kv_heads * DC * N;
   hipStream_t s = (hipStream_t)stream;
 #define DC_LAUNCH(NT)                                                                                                            \
   {                                                                                                                              \
-    delta_chunk_terms_kernel<NT><<<dim3(heads, n_chunks), 256, 0, s>>>(u, terms, chunks, heads, kv_heads, P, up, w, kt, m, b);   \
-    delta_chunk_walk_kernel<NT><<<dim3(heads, P / 16, n_spans), 256, 0, s>>>(u, up, w, kt, m, b, spans5, positions, state,       \
+    delta_chunk_terms_kernel<NT><<<dim3(heads, n_chunks), 256, 0, s>>>(u, terms, chunks, heads, kv_heads, P, up, w, kt, m, q, b);\
+    delta_chunk_walk_kernel<NT><<<dim3(heads, P / 16, n_spans), 256, 0, s>>>(q, up, w, kt, m, b, spans5, positions, state,       \
                                                                             state_stride, copy_elems, tail_at, conv_in,          \
                                                                             conv_in_stride, y, heads, kv_heads, P, taps);        \
   }
