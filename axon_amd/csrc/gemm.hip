@@ -162,7 +162,7 @@ gemm_fma_few_rows_kernel(const elem_t* __restrict__ x, int x_stride, const elem_
     const int k_end = min(FEW_BK, K - k0);   // beyond K the stage holds zeros
     for (int part = 0; part < k_end; part += FMA_PART) {
       float acc = 0.0f, acc_up = 0.0f;
-#pragma unroll
+#pragma unroll 4
       for (int i = 0; i < FMA_PART; i += 4) {    // beyond K, too: zeros
         const float4 a = *reinterpret_cast<const float4*>(&xs[ty][part + i]);
         const float4 b = *reinterpret_cast<const float4*>(&ws[tx][part + i]);
