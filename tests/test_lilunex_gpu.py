@@ -20,7 +20,7 @@ from axon_amd.parts import CacheBinding, build_part
 from axon_amd.weights import WeightStore
 from gpu_helpers import DTYPES, DictSource, PartHarness
 from helpers import ROOT, TraceBuilder, engine_for, run_trace, tolerance
-from lilunex_models import MODELS, att, config, delta, dense, draw_weights, layer, make, moe, wkv
+from lilunex_models import MODELS, att, config, delta, draw_weights, layer, make, moe, wkv
 from plain import lilunex_plain as P
 
 pytestmark = pytest.mark.gpu
