@@ -360,17 +360,21 @@ int axk_wkv_scan(const float* rows, long stride, long r_at, long k_at, long v_at
 // axk_delta_prepare: from the float32 rows of the projections (the channels first, the heads' logits of beta from
 // beta_at and of the decay from decay_at) u [T, channels], convolved, through silu, queries and keys of length 1 a head
 // (x / sqrt(sum x^2 + 1e-6)), queries times q_scale; terms [T, heads, 2] = (g, beta), g = exp(-exp(a_log) softplus(. +
-// dt_bias)), beta = sigmoid(.).  Reads the state only.
+// dt_bias)), beta = sigmoid(.); without a_log (null) g = 1.  Reads the state only.
+// axk_delta_low_rank: decays and gates of low rank in one launch, float32 (either may have 0 channels): decay[t, c] =
+// exp(-exp(a_log[c / head_dim]) softplus(w_decay[c] . rows[t, decay_at ..] + dt_bias[c])), gate[t, c] = w_gate[c] .
+// rows[t, gate_at ..]; the matrices elem [channels, rank].
 // axk_delta_scan: per request of the step (spans [n][3] = (slot, first token, tokens); null: each token a request of its
 // own in slot seq_rows[t]) and head, over its tokens in order, S = g S, c = beta (v - S^T k), S = S + k c^T, y = S^T q;
+// with decay (float32 [T, heads N], or null) a row n of S is decayed by a number of its own (terms' g is 1 then);
 // then the state row is brought up to date (S, and the convolutions' inputs from conv_in, rows conv_in_stride apart).
-// axk_head_norm_gate: out elem [T, heads P] = (y / sqrt(mean y^2 + eps)) gain silu(gate), the mean over a head's P; gain
-// of P numbers, or with gain_per_head of heads P.
+// axk_head_norm_gate: out elem [T, heads P] = (y / sqrt(mean y^2 + eps)) gain act(gate), the mean over a head's P; gain
+// of P numbers, or with gain_per_head of heads P; act 0: silu, 1: sigmoid.
 int axk_delta_prepare(const float* in, long in_stride, const void* w, int taps, const float* state, long state_stride,
                       long copy_elems, long tail_at, const int32_t* positions, const int32_t* seq_rows, int beta_at, int decay_at,
                       const void* a_log, int a_log_is_f32, const void* dt_bias, int dt_bias_is_f32, float* u, float* terms,
                       int n_tokens, int heads, int kv_heads, int N, int P, float q_scale, void* stream);
-int axk_delta_scan(const float* u, const float* terms, float* state, long state_stride, long copy_elems, long tail_at,
+int axk_delta_scan(const float* u, const float* terms, const float* decay, float* state, long state_stride, long copy_elems, long tail_at,
                    const int32_t* spans, int n_spans, const int32_t* positions, const int32_t* seq_rows, const float* conv_in,
                    long conv_in_stride, float* y, int heads, int kv_heads, int N, int P, int taps, void* stream);
 // axk_delta_chunked (where axk_delta_chunked_ok says 1): the same for long stretches, in chunks of up to 64 tokens on the
@@ -384,7 +388,43 @@ int axk_delta_chunked(const float* u, const float* terms, float* state, long sta
                       const float* conv_in, long conv_in_stride, float* y, int heads, int kv_heads, int N, int P, int taps,
                       float* work, long work_floats, void* stream);
 int axk_head_norm_gate(const float* y, const float* gate, long gate_stride, const void* gain, int gain_is_f32, int gain_per_head,
-                       float eps, void* out, int n_tokens, int heads, int P, void* stream);
+                       int act, float eps, void* out, int n_tokens, int heads, int P, void* stream);
+int axk_delta_low_rank(const float* rows, long stride, int decay_at, int decay_rank, const void* w_decay, const void* dt_bias,
+                       int dt_bias_is_f32, const void* a_log, int a_log_is_f32, int head_dim, float* decay, int decay_channels,
+                       int gate_at, int gate_rank, const void* w_gate, float* gate, int gate_channels, int n_tokens, void* stream);
+
+// Linear attention with a constant decay a head (csrc/linear_attention.hip).  A copy of the state row: the heads' states
+// [heads][P][N].  q, k [T, heads N] and v [T, heads P] are float32 columns of rows `stride` apart; decay float32 [heads].
+// axk_lightning_scan: per request of the step (spans, as above) and head, over its tokens in order, S = decay S + k v^T,
+// y = S^T q (silu: of silu(q), silu(k), silu(v)); then the state row is brought up to date.
+// axk_lightning_chunked (where axk_lightning_chunked_ok says 1): the same for long stretches in chunks of up to 64 tokens
+// (chunks, spans5 as in axk_delta_chunked; operands as they are: axk_silu_rows has been there), sums in another order, by
+// rounding; ends: n_chunks heads N P floats of workspace.
+// axk_silu_rows: silu in place over the first `columns` numbers of float32 rows.
+int axk_silu_rows(float* rows, long stride, int columns, int n_rows, void* stream);
+int axk_lightning_scan(const float* rows, long stride, int q_at, int k_at, int v_at, int silu, const float* decay, float* state,
+                       long state_stride, long copy_elems, const int32_t* spans, int n_spans, const int32_t* positions,
+                       const int32_t* seq_rows, float* y, int heads, int N, int P, void* stream);
+int axk_lightning_chunked_ok(int heads, int N, int P, long stride, int q_at, int k_at);
+int axk_lightning_chunked(const float* rows, long stride, int q_at, int k_at, int v_at, const float* decay, float* state,
+                          long state_stride, long copy_elems, const int32_t* chunks, int n_chunks, const int32_t* spans5, int n_spans,
+                          const int32_t* positions, float* y, int heads, int N, int P, float* ends, long ends_floats, void* stream);
+
+// Passes over the residual stream (csrc/stream.hip).  States: two copies, the one behind position p in copy p & 1.
+// axk_embed_pairs: x[t] = table[token] scale + pairs[(before mul_prev + token mul_cur) mod buckets] (elem [buckets + 1, dim];
+// the last row for a request's first token); state int32 [slots, 2]: the last token.
+// axk_scaled_sum: x += n0(y0) s0 + n1(y1) s1 (float32 rows; s float32 [dim]; y1 may be null; n(y) = y / sqrt(mean(y^2) +
+// norm_eps), or y where norm_eps < 0); h (or null) elem rows of the RMS norm of the new x, gain float32 [dim]; share (or
+// null; single tokens of different requests only): h moved towards the request's h before, which state [slots, 2 dim] keeps.
+// axk_shifted_norm: h = norm(x), out = h + (the request's h before - h) share, for any step.
+int axk_embed_pairs(const int32_t* tokens, const void* table, int packed, float scale, const void* pairs, int buckets, long mul_prev,
+                    long mul_cur, int32_t* state, const int32_t* positions, const int32_t* seq_rows, float* x, int n_tokens, int dim,
+                    int vocab, void* stream);
+int axk_scaled_sum(const float* y0, const float* s0, float norm_eps0, const float* y1, const float* s1, float norm_eps1, float* x,
+                   const float* gain, float eps, void* h, const float* share, float* state, long state_stride,
+                   const int32_t* positions, const int32_t* seq_rows, int n_tokens, int dim, void* stream);
+int axk_shifted_norm(const float* x, const float* gain, float eps, const float* share, float* state, long state_stride,
+                     const int32_t* positions, const int32_t* seq_rows, void* out, int n_tokens, int dim, void* stream);
 
 // Attention over a latent cache (csrc/latent_attention.hip); a page is [page_size][rank + rot] elem
 // (the latent and the rotated key part of each position), then [rank][page_size] (the latents again,
@@ -424,12 +464,18 @@ int axk_latent_attention(const float* q_full, const void* cache, const int32_t* 
 // values into the page (if write_kv).  q_temp_every > 0: a query at position p is multiplied by
 // 1 + q_temp_coef ln(floor((p + 1) / q_temp_every) + 1).  norm_rows: the norm goes over all query units (all key
 // units) of a token at once, its gains hold n_q dim (n_k dim) numbers.  Without write_kv the key and value columns
-// need not be there.
+// need not be there.  conv_w (elem [channels, taps], or null; the channels are the columns [q | k | v], side by side): the
+// projections pass a causal convolution over time first, the last column the current token's; a request's last
+// conv_taps - 1 projections are kept in its state row (two copies of conv_copy_elems floats, [taps - 1][channels], oldest
+// first, the one behind position p in copy p & 1).  conv_spans [n_spans][3] = (slot, first token, tokens), the step's
+// requests, or null: every token a request of its own.
 int axk_heads_prepare(const float* proj, long stride, int q_at, int n_q, int k_at, int n_k, int v_at, int v_width, int dim,
                       const void* q_gain, int q_gain_is_f32, const void* k_gain, int k_gain_is_f32, float eps, int rot,
                       int neighbours, float magnitude, const float* table, const int32_t* positions, const int32_t* seq_rows,
                       const int32_t* block_table, int table_stride, void* cache, int page_size, void* q_out, int n_tokens,
-                      int write_kv, float q_temp_coef, int q_temp_every, int norm_rows, void* stream);
+                      int write_kv, float q_temp_coef, int q_temp_every, int norm_rows, const void* conv_w, int conv_taps,
+                      float* conv_state, long conv_state_stride, long conv_copy_elems, const int32_t* conv_spans, int n_spans,
+                      void* stream);
 // axk_masked_attention: q elem [T, heads maps dim] -> out elem [T, heads vdim].  mask_kind 0: all earlier
 // positions; 1: the last mask_size positions and, whatever their distance, the first `keep`; 2: the earlier positions of the same chunk of mask_size.
 // softcap > 0: s <- softcap tanh(s / softcap).  maps 2: o = rms(a_1 - lambda a_2, eps) out_scale.  gate

@@ -18,6 +18,14 @@ namespace {
 // head (convolution, silu), or the token's step sizes, terms[t, a] = (g, beta) with
 // g = exp(-exp(A_log_a) softplus(decay_in_a + dt_bias_a)), beta = sigmoid(beta_in_a).  in [T, in_stride]: the
 // projections' rows, [q: kv_heads N | k: kv_heads N | v: heads P] first.
+// Without a_log (a decay a key channel, which comes from elsewhere) g is 1.
+__device__ inline float delta_decay(const float* __restrict__ row, int decay_at, const void* __restrict__ a_log, int a_log_is_f32,
+                                    const void* __restrict__ dt_bias, int dt_bias_is_f32, int a) {
+  if (a_log == nullptr) return 1.0f;
+  const float step = rec_softplus(row[decay_at + a] + load_vec(dt_bias, dt_bias_is_f32, a));
+  return expf(-(expf(load_vec(a_log, a_log_is_f32, a)) * step));
+}
+
 #define DP_KEPT 4        // channels of a query or key head a lane holds: N up to 256
 __global__ void __launch_bounds__(256)
 delta_prepare_kernel(const float* __restrict__ in, long in_stride, const elem_t* __restrict__ w, int taps,
@@ -30,8 +38,7 @@ delta_prepare_kernel(const float* __restrict__ in, long in_stride, const elem_t*
   if (unit > 2 * kv_heads + heads) return;
   if (unit == 2 * kv_heads + heads) {
     for (int a = lane; a < heads; a += 64) {
-      const float step = rec_softplus(row[decay_at + a] + load_vec(dt_bias, dt_bias_is_f32, a));
-      terms[((long)t * heads + a) * 2] = expf(-(expf(load_vec(a_log, a_log_is_f32, a)) * step));
+      terms[((long)t * heads + a) * 2] = delta_decay(row, decay_at, a_log, a_log_is_f32, dt_bias, dt_bias_is_f32, a);
       terms[((long)t * heads + a) * 2 + 1] = rec_sigmoid(row[beta_at + a]);
     }
     return;
@@ -84,21 +91,22 @@ __device__ inline void keep_conv_inputs(const float* __restrict__ kept_from, flo
 // The walk.  grid (requests of the step, heads, blocks of value dims); LK lanes share a value dim, OWN rows of the
 // state a lane.  With a = S^T k and b = S^T q of the state as the token finds it, u = beta (v - g a) and the read-out
 // behind the token's write is o = g b + (k . q) u: both sums leave for the lanes' permutations together.  The operands
-// of AHEAD tokens are asked for while those before them are worked on.
-template <int OWN, int AHEAD>
+// of AHEAD tokens are asked for while those before them are worked on.  CHANNEL: a decay a head and key channel, from
+// decay [T, heads N] (the state's rows are then decayed before the sums, and g is 1).
+template <int OWN, int AHEAD, bool CHANNEL>
 struct DeltaOperands {
-  float q[AHEAD][OWN], k[AHEAD][OWN], v[AHEAD], g[AHEAD], beta[AHEAD];
+  float q[AHEAD][OWN], k[AHEAD][OWN], v[AHEAD], g[AHEAD], beta[AHEAD], w[CHANNEL ? AHEAD : 1][OWN];
 };
 
-template <int LK, int OWN, bool VEC>
+template <int LK, int OWN, bool VEC, bool CHANNEL>
 __global__ void __launch_bounds__(REC_THREADS)
-delta_scan_kernel(const float* __restrict__ u, const float* __restrict__ terms, float* __restrict__ state, long state_stride,
+delta_scan_kernel(const float* __restrict__ u, const float* __restrict__ terms, const float* __restrict__ decay, float* __restrict__ state, long state_stride,
                   long copy_elems, long tail_at, const int32_t* __restrict__ spans, const int32_t* __restrict__ positions,
                   const int32_t* __restrict__ seq_rows, const float* __restrict__ conv_in, long conv_in_stride,
                   float* __restrict__ y, int heads, int kv_heads, int N, int P, int taps) {
   constexpr int AHEAD = OWN >= 16 ? 2 : 4;
   const RecStretch s = rec_stretch(nullptr, spans, seq_rows, blockIdx.x);
-  const int h = blockIdx.y, g = h / (heads / kv_heads), ns = threadIdx.x % LK, n0 = ns * OWN;
+  const int h = blockIdx.y, kh = h / (heads / kv_heads), ns = threadIdx.x % LK, n0 = ns * OWN;
   const int p = blockIdx.z * (REC_THREADS / LK) + threadIdx.x / LK;
   const bool has_p = p < P;
   const int start = positions[s.first];
@@ -112,8 +120,8 @@ delta_scan_kernel(const float* __restrict__ u, const float* __restrict__ terms, 
     for (int i = 0; i < OWN; ++i) S[i] = 0.0f;
   }
   const int channels = 2 * kv_heads * N + heads * P, last = s.first + s.count;
-  const long q_col = (long)g * N, k_col = (long)(kv_heads + g) * N, v_col = 2L * kv_heads * N + (long)h * P + (has_p ? p : 0);
-  typedef DeltaOperands<OWN, AHEAD> Ops;
+  const long q_col = (long)kh * N, k_col = (long)(kv_heads + kh) * N, v_col = 2L * kv_heads * N + (long)h * P + (has_p ? p : 0);
+  typedef DeltaOperands<OWN, AHEAD, CHANNEL> Ops;
   auto fetch = [&](Ops& o, int t0) {
 #pragma unroll
     for (int a = 0; a < AHEAD; ++a) {
@@ -121,6 +129,7 @@ delta_scan_kernel(const float* __restrict__ u, const float* __restrict__ terms, 
       const float* row = u + (long)t * channels;
       rec_load<OWN, VEC>(o.q[a], row + q_col, n0, N);
       rec_load<OWN, VEC>(o.k[a], row + k_col, n0, N);
+      if (CHANNEL) rec_load<OWN, VEC>(o.w[CHANNEL ? a : 0], decay + ((long)t * heads + h) * N, n0, N);
       o.v[a] = row[v_col];
       o.g[a] = terms[((long)t * heads + h) * 2];
       o.beta[a] = terms[((long)t * heads + h) * 2 + 1];
@@ -131,8 +140,10 @@ delta_scan_kernel(const float* __restrict__ u, const float* __restrict__ terms, 
     for (int a = 0; a < AHEAD; ++a) {
       if (t0 + a >= last) break;
       float sk = 0.0f, sq = 0.0f, kq = 0.0f;
+      const float g = CHANNEL ? 1.0f : o.g[a];
 #pragma unroll
       for (int i = 0; i < OWN; ++i) {
+        if (CHANNEL) S[i] *= o.w[CHANNEL ? a : 0][i];
         sk = fmaf(S[i], o.k[a][i], sk);
         sq = fmaf(S[i], o.q[a][i], sq);
         kq = fmaf(o.k[a][i], o.q[a][i], kq);
@@ -140,10 +151,10 @@ delta_scan_kernel(const float* __restrict__ u, const float* __restrict__ terms, 
       sk = rec_row_sum<LK>(sk);
       sq = rec_row_sum<LK>(sq);
       kq = rec_row_sum<LK>(kq);
-      const float c = o.beta[a] * (o.v[a] - o.g[a] * sk);
+      const float c = o.beta[a] * (o.v[a] - g * sk);
 #pragma unroll
-      for (int i = 0; i < OWN; ++i) S[i] = fmaf(o.k[a][i], c, o.g[a] * S[i]);
-      if (ns == 0 && has_p) y[((long)(t0 + a) * heads + h) * P + p] = fmaf(kq, c, o.g[a] * sq);
+      for (int i = 0; i < OWN; ++i) S[i] = fmaf(o.k[a][i], c, g * S[i]);
+      if (ns == 0 && has_p) y[((long)(t0 + a) * heads + h) * P + p] = fmaf(kq, c, g * sq);
     }
   };
   Ops even, odd;
@@ -408,12 +419,17 @@ delta_chunk_walk_kernel(const float* __restrict__ q, const float* __restrict__ u
                    (blockIdx.x * gridDim.y + blockIdx.y) * 256 + threadIdx.x, gridDim.x * gridDim.y * 256);
 }
 
-// out[t, a] = (y[t, a] / sqrt(mean(y[t, a]^2) + eps)) gain silu(gate[t, a]) head by head; the gain holds P numbers
-// shared by the heads, or one for every channel (gain_per_head).  A wave a (token, head).
+// out[t, a] = (y[t, a] / sqrt(mean(y[t, a]^2) + eps)) gain act(gate[t, a]) head by head, act silu or sigmoid (GATE); the
+// gain holds P numbers shared by the heads, or one for every channel (gain_per_head).  A wave a (token, head), or a block
+// for heads of many values.
+#define GATE_SILU 0
+#define GATE_SIGMOID 1
+__device__ inline float gate_act(float z, int kind) { return kind == GATE_SILU ? rec_silu(z) : rec_sigmoid(z); }
 #define HN_KEPT 4
 __global__ void __launch_bounds__(256)
 head_norm_gate_kernel(const float* __restrict__ y, const float* __restrict__ gate, long gate_stride, const void* __restrict__ gain,
-                      int gain_is_f32, int gain_per_head, float eps, elem_t* __restrict__ out, long items, int heads, int P) {
+                      int gain_is_f32, int gain_per_head, float eps, elem_t* __restrict__ out, long items, int heads, int P,
+                      int act) {
   const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (item >= items) return;
   const int lane = threadIdx.x & 63, h = (int)(item % heads);
@@ -433,17 +449,17 @@ head_norm_gate_kernel(const float* __restrict__ y, const float* __restrict__ gat
 #pragma unroll
   for (int j = 0; j < HN_KEPT; ++j) {
     const int i = lane + 64 * j;
-    if (i < P) dst[i] = from_float(((kept[j] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * rec_silu(g[i]));
+    if (i < P) dst[i] = from_float(((kept[j] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * gate_act(g[i], act));
   }
   for (int i = lane + 64 * HN_KEPT; i < P; i += 64)
-    dst[i] = from_float(((src[i] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * rec_silu(g[i]));
+    dst[i] = from_float(((src[i] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * gate_act(g[i], act));
 }
 
 // The same for heads of 4 LANES values (16 to 256): LANES lanes a head, four values each.
 template <int LANES>
 __global__ void __launch_bounds__(256)
 head_norm_gate_vec_kernel(const float* __restrict__ y, const float* __restrict__ gate, long gate_stride, const void* __restrict__ gain,
-                          int gain_is_f32, int gain_per_head, float eps, elem_t* __restrict__ out, long items, int heads) {
+                          int gain_is_f32, int gain_per_head, float eps, elem_t* __restrict__ out, long items, int heads, int act) {
   constexpr int P = 4 * LANES;
   const long item = ((long)blockIdx.x * 256 + threadIdx.x) / LANES;
   const int e = 4 * (threadIdx.x % LANES);
@@ -458,14 +474,42 @@ head_norm_gate_vec_kernel(const float* __restrict__ y, const float* __restrict__
   for (int off = LANES / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
   const float inv = 1.0f / sqrtf(ss / (float)P + eps);
   if (!active) return;
-  const float o0 = ((v.x * inv) * w.x) * rec_silu(g.x), o1 = ((v.y * inv) * w.y) * rec_silu(g.y);
-  const float o2 = ((v.z * inv) * w.z) * rec_silu(g.z), o3 = ((v.w * inv) * w.w) * rec_silu(g.w);
+  const float o0 = ((v.x * inv) * w.x) * gate_act(g.x, act), o1 = ((v.y * inv) * w.y) * gate_act(g.y, act);
+  const float o2 = ((v.z * inv) * w.z) * gate_act(g.z, act), o3 = ((v.w * inv) * w.w) * gate_act(g.w, act);
   elem_t* dst = out + it * P + e;
 #if AXON_BF16
   *reinterpret_cast<uint2*>(dst) = make_uint2(pack2_bf16(o0, o1), pack2_bf16(o2, o3));
 #else
   *reinterpret_cast<float4*>(dst) = make_float4(o0, o1, o2, o3);
 #endif
+}
+
+// The same for heads of many values (all channels of a row normed together, say): a block a (token, head).
+__global__ void __launch_bounds__(256)
+head_norm_gate_wide_kernel(const float* __restrict__ y, const float* __restrict__ gate, long gate_stride, const void* __restrict__ gain,
+                           int gain_is_f32, int gain_per_head, float eps, elem_t* __restrict__ out, int heads, int P, int act) {
+  __shared__ float partial[256 / AXON_WAVE];
+  const long item = blockIdx.x;
+  const int h = (int)(item % heads), gain_at = gain_per_head ? h * P : 0;
+  const float* src = y + item * P;
+  const float* g = gate + item / heads * gate_stride + (long)h * P;
+  elem_t* dst = out + item * P;
+  float kept[HN_KEPT], ss = 0.0f;
+#pragma unroll
+  for (int j = 0; j < HN_KEPT; ++j) {
+    const int i = threadIdx.x + 256 * j;
+    kept[j] = i < P ? src[i] : 0.0f;
+    ss = fmaf(kept[j], kept[j], ss);
+  }
+  for (int i = threadIdx.x + 256 * HN_KEPT; i < P; i += 256) ss = fmaf(src[i], src[i], ss);
+  const float inv = 1.0f / sqrtf(block_sum_256(ss, partial) / (float)P + eps);
+#pragma unroll
+  for (int j = 0; j < HN_KEPT; ++j) {
+    const int i = threadIdx.x + 256 * j;
+    if (i < P) dst[i] = from_float(((kept[j] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * gate_act(g[i], act));
+  }
+  for (int i = threadIdx.x + 256 * HN_KEPT; i < P; i += 256)
+    dst[i] = from_float(((src[i] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * gate_act(g[i], act));
 }
 
 // delta_prepare for long steps and up to four taps: a wave a head of queries or keys or up to 256 value channels, over
@@ -486,8 +530,7 @@ delta_prepare_run_kernel(const float* __restrict__ in, long in_stride, const ele
     for (int i = lane; i < heads * (t1 - t0); i += 64) {
       const int t = t0 + i / heads, a = i % heads;
       const float* row = in + (long)t * in_stride;
-      const float step = rec_softplus(row[decay_at + a] + load_vec(dt_bias, dt_bias_is_f32, a));
-      terms[((long)t * heads + a) * 2] = expf(-(expf(load_vec(a_log, a_log_is_f32, a)) * step));
+      terms[((long)t * heads + a) * 2] = delta_decay(row, decay_at, a_log, a_log_is_f32, dt_bias, dt_bias_is_f32, a);
       terms[((long)t * heads + a) * 2 + 1] = rec_sigmoid(row[beta_at + a]);
     }
     return;
@@ -548,7 +591,8 @@ extern "C" int axk_delta_prepare(const float* in, long in_stride, const void* w,
               "delta_prepare: bad sizes T=%d heads=%d kv heads=%d keys=%d (at most 256) values=%d taps=%d", n_tokens, heads, kv_heads,
               N, P, taps);
   const long channels = 2L * kv_heads * N + (long)heads * P;
-  AXK_REQUIRE(in_stride >= channels && beta_at >= 0 && decay_at >= 0 && beta_at + heads <= in_stride && decay_at + heads <= in_stride,
+  AXK_REQUIRE(in_stride >= channels && beta_at >= 0 && beta_at + heads <= in_stride &&
+              (a_log == nullptr || (decay_at >= 0 && decay_at + heads <= in_stride)),
               "delta_prepare: the parts do not fit rows of %ld", in_stride);
   AXK_REQUIRE(tail_at >= 0 && copy_elems >= tail_at + (taps - 1) * channels && state_stride >= 2 * copy_elems,
               "delta_prepare: a state row of %ld floats does not hold two copies of %ld with %d x %ld kept inputs from %ld",
@@ -572,7 +616,7 @@ extern "C" int axk_delta_prepare(const float* in, long in_stride, const void* w,
   return 0;
 }
 
-extern "C" int axk_delta_scan(const float* u, const float* terms, float* state, long state_stride, long copy_elems, long tail_at,
+extern "C" int axk_delta_scan(const float* u, const float* terms, const float* decay, float* state, long state_stride, long copy_elems, long tail_at,
                               const int32_t* spans, int n_spans, const int32_t* positions, const int32_t* seq_rows,
                               const float* conv_in, long conv_in_stride, float* y, int heads, int kv_heads, int N, int P, int taps,
                               void* stream) {
@@ -588,14 +632,17 @@ extern "C" int axk_delta_scan(const float* u, const float* terms, float* state, 
   if (n_spans == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   const bool vec = N % 4 == 0 && channels % 4 == 0 && copy_elems % 4 == 0 && state_stride % 4 == 0 && ((uintptr_t)u & 15) == 0 &&
-                   ((uintptr_t)state & 15) == 0;
-#define DELTA_ARGS u, terms, state, state_stride, copy_elems, tail_at, spans, positions, seq_rows, conv_in, conv_in_stride, y, heads, \
+                   ((uintptr_t)state & 15) == 0 && ((uintptr_t)decay & 15) == 0;
+#define DELTA_ARGS u, terms, decay, state, state_stride, copy_elems, tail_at, spans, positions, seq_rows, conv_in, conv_in_stride, y, heads, \
                    kv_heads, N, P, taps
 #define DELTA_LAUNCH(LK, OWN)                                                                    \
   {                                                                                              \
     const dim3 grid(n_spans, heads, ceil_div(P, REC_THREADS / LK));                              \
-    if (vec) delta_scan_kernel<LK, OWN, true><<<grid, REC_THREADS, 0, s>>>(DELTA_ARGS);          \
-    else delta_scan_kernel<LK, OWN, false><<<grid, REC_THREADS, 0, s>>>(DELTA_ARGS);             \
+    if (decay == nullptr) {                                                                      \
+      if (vec) delta_scan_kernel<LK, OWN, true, false><<<grid, REC_THREADS, 0, s>>>(DELTA_ARGS); \
+      else delta_scan_kernel<LK, OWN, false, false><<<grid, REC_THREADS, 0, s>>>(DELTA_ARGS);    \
+    } else if (vec) delta_scan_kernel<LK, OWN, true, true><<<grid, REC_THREADS, 0, s>>>(DELTA_ARGS); \
+    else delta_scan_kernel<LK, OWN, false, true><<<grid, REC_THREADS, 0, s>>>(DELTA_ARGS);       \
   }
   REC_BY_ROWS(N, DELTA_LAUNCH)
 #undef DELTA_LAUNCH
@@ -653,23 +700,30 @@ extern "C" int axk_delta_chunked(const float* u, const float* terms, float* stat
 }
 
 extern "C" int axk_head_norm_gate(const float* y, const float* gate, long gate_stride, const void* gain, int gain_is_f32,
-                                  int gain_per_head, float eps, void* out, int n_tokens, int heads, int P, void* stream) {
+                                  int gain_per_head, int act, float eps, void* out, int n_tokens, int heads, int P, void* stream) {
   AXK_REQUIRE(n_tokens >= 0 && heads > 0 && P > 0 && gate_stride >= (long)heads * P,
               "head_norm_gate: bad sizes T=%d heads=%d values=%d gate rows of %ld", n_tokens, heads, P, gate_stride);
+  AXK_REQUIRE(act == GATE_SILU || act == GATE_SIGMOID, "head_norm_gate: unknown gate %d", act);
   if (n_tokens == 0) return 0;
   const long items = (long)n_tokens * heads;
   const bool vec = gate_stride % 4 == 0 && (((uintptr_t)y | (uintptr_t)gate | (uintptr_t)gain | (uintptr_t)out) & 15) == 0;
 #define HN_VEC(LANES)                                                                                                       \
   if (vec && P == 4 * LANES) {                                                                                              \
     head_norm_gate_vec_kernel<LANES><<<(unsigned)((items * LANES + 255) / 256), 256, 0, (hipStream_t)stream>>>(             \
-        y, gate, gate_stride, gain, gain_is_f32, gain_per_head, eps, (elem_t*)out, items, heads);                           \
+        y, gate, gate_stride, gain, gain_is_f32, gain_per_head, eps, (elem_t*)out, items, heads, act);                         \
     AXK_LAUNCH_CHECK("head_norm_gate");                                                                                     \
     return 0;                                                                                                               \
   }
   HN_VEC(4) HN_VEC(8) HN_VEC(16) HN_VEC(32) HN_VEC(64)
 #undef HN_VEC
+  if (P > 512) {
+    head_norm_gate_wide_kernel<<<(unsigned)items, 256, 0, (hipStream_t)stream>>>(y, gate, gate_stride, gain, gain_is_f32, gain_per_head,
+                                                                                eps, (elem_t*)out, heads, P, act);
+    AXK_LAUNCH_CHECK("head_norm_gate");
+    return 0;
+  }
   head_norm_gate_kernel<<<(unsigned)((items + 3) / 4), 256, 0, (hipStream_t)stream>>>(y, gate, gate_stride, gain, gain_is_f32,
-                                                                                     gain_per_head, eps, (elem_t*)out, items, heads, P);
+                                                                                     gain_per_head, eps, (elem_t*)out, items, heads, P, act);
   AXK_LAUNCH_CHECK("head_norm_gate");
   return 0;
 }

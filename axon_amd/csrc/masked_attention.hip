@@ -10,6 +10,7 @@
 //   * a sink in the softmax: a key of a given score, one number or one a head, that has no value (its
 //     weight only enters the sum);
 //   * a query temperature by position, q (1 + coef ln(floor((p + 1) / every) + 1));
+//   * a short causal convolution over time on every channel of the projections, before everything else;
 //   * a gate sigmoid(g) on the concatenated heads, a number an element or a number a head.
 //
 // A page of the cache holds, for its positions, the key rows [page_size][kv_heads maps dim] and behind
@@ -18,7 +19,7 @@
 #include <math.h>
 
 #include "api.h"
-#include "common.h"
+#include "recurrence.h"
 
 namespace {
 
@@ -42,14 +43,47 @@ __device__ inline int nth_block(int i, int kept, int lo_block) { return i < kept
 // (sin, cos), and stored: queries into q_out [T, n_q dim], keys and values into the token's page.
 // norm_rows: the norm's mean goes over all of a token's query units (and over all its key units) at once,
 // and the gain holds a number for every one of these dims.
+//
+// CONV: what is normed, rotated and stored is sum_k w[c, k] (the projection taps - 1 - k tokens before)[c], the columns
+// q_at .. being the channels [q | k | v]; what a request's earlier steps left of its projections comes from its state row
+// (two copies of [taps - 1][channels], oldest first, the one behind position p in copy p & 1).  In a step of single tokens
+// (single) a channel's thread also writes the copy behind its token: it is the only one that reads or writes that channel.
+// Longer stretches may end in the copy they start from: there a launch of its own keeps the projections.
+struct HeadsConv {
+  const elem_t* w;           // [channels, taps]
+  int taps, channels, single;
+  float* state;
+  long state_stride, copy_elems;
+};
+
+__device__ inline const float* conv_kept(const HeadsConv& cv, const int32_t* seq_rows, const int32_t* positions, int t, int inside) {
+  return rec_copy_before(cv.state, cv.state_stride, cv.copy_elems, seq_rows[t], positions[t] - inside);
+}
+
+// row: the token's projections at channel 0.
+__device__ inline float conv_value(const HeadsConv& cv, const float* __restrict__ row, long stride, const float* kept, float* keep,
+                                   int inside, int c) {
+  float acc = 0.0f;
+  for (int k = 0; k < cv.taps; ++k) {
+    const int back = cv.taps - 1 - k;            // the projection `back` tokens before this one
+    const int at = cv.taps - 1 - (back - inside);
+    const float v = back <= inside ? row[c - (long)back * stride] : kept[(long)at * cv.channels + c];
+    acc = fmaf(to_float(cv.w[(long)c * cv.taps + k]), v, acc);
+    if (keep != nullptr && k > 0) keep[(long)(k - 1) * cv.channels + c] = v;
+  }
+  return acc;
+}
+
+template <bool CONV>
 __global__ void __launch_bounds__(256)
 heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int n_q, int k_at, int n_k, int v_at, int v_width,
                      int dim, const void* __restrict__ q_gain, int q_gain_is_f32, const void* __restrict__ k_gain,
                      int k_gain_is_f32, float eps, int rot, int neighbours, float magnitude, const float* __restrict__ table,
                      const int32_t* __restrict__ positions, const int32_t* __restrict__ seq_rows,
                      const int32_t* __restrict__ block_table, int table_stride, elem_t* __restrict__ cache, int page_size,
-                     elem_t* __restrict__ q_out, int write_kv, float q_temp_coef, int q_temp_every, int norm_rows) {
+                     elem_t* __restrict__ q_out, int write_kv, float q_temp_coef, int q_temp_every, int norm_rows, HeadsConv cv) {
   __shared__ float row_sums[2][256 / AXON_WAVE];
+  extern __shared__ float convolved[];         // CONV: a unit of `dim` a wave
   const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   // a query's temperature by its position: 1 + coef ln(floor((p + 1) / every) + 1), or 1
   const float q_temp = q_temp_every > 0 ? 1.0f + q_temp_coef * logf((float)((positions[t] + 1) / q_temp_every + 1)) : 1.0f;
@@ -64,6 +98,14 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
     const int page = block_table[(long)seq_rows[t] * table_stride + pos / page_size];
     page_base = cache + (long)page * page_size * (kw + v_width);
     in_page = pos % page_size;
+  }
+  int inside = 0;
+  const float* kept = nullptr;
+  float* keep = nullptr;
+  if (CONV) {
+    inside = rec_inside(seq_rows, t, cv.taps - 1);
+    kept = conv_kept(cv, seq_rows, positions, t, inside);
+    if (cv.single) keep = rec_copy_behind(cv.state, cv.state_stride, cv.copy_elems, seq_rows[t], positions[t]);
   }
   float q_inv = 1.0f, k_inv = 1.0f;
   if (norm_rows) {
@@ -86,6 +128,12 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
     const float temp = is_q ? q_temp : 1.0f;
     const int gain_at = norm_rows ? (is_q ? u : u - n_q) * dim : 0;
     float inv = is_q ? q_inv : k_inv;
+    if (CONV) {                                  // the wave's own corner of LDS: no other wave touches it
+      float* mine = convolved + wave * dim;
+      for (int i = lane; i < dim; i += 64) mine[i] = conv_value(cv, row + q_at, stride, kept, keep, inside, (int)(src - row) - q_at + i);
+      __builtin_amdgcn_wave_barrier();
+      src = mine;
+    }
     if (gain != nullptr && !norm_rows) {
       float ss = 0.0f;
       for (int i = lane; i < dim; i += 64) ss = fmaf(src[i], src[i], ss);
@@ -110,7 +158,27 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
   }
   if (!write_kv) return;
   elem_t* by_dim = page_base + (long)page_size * kw + in_page;
-  for (int i = blockIdx.y * 256 + threadIdx.x; i < v_width; i += 256 * gridDim.y) by_dim[(long)i * page_size] = from_float(row[v_at + i]);
+  for (int i = blockIdx.y * 256 + threadIdx.x; i < v_width; i += 256 * gridDim.y) {
+    const float v = CONV ? conv_value(cv, row + q_at, stride, kept, keep, inside, v_at - q_at + i) : row[v_at + i];
+    by_dim[(long)i * page_size] = from_float(v);
+  }
+}
+
+// A request's last taps - 1 projections, of (what was kept, this step's): place i takes what lies `count` places later
+// (where both copies are one: read before it is written, ascending).  grid (blocks of channels, requests).
+__global__ void __launch_bounds__(256)
+heads_keep_kernel(const float* __restrict__ proj, long stride, HeadsConv cv, const int32_t* __restrict__ spans,
+                  const int32_t* __restrict__ positions) {
+  const int slot = spans[3 * blockIdx.y], first = spans[3 * blockIdx.y + 1], count = spans[3 * blockIdx.y + 2];
+  const int c = blockIdx.x * 256 + threadIdx.x, start = positions[first];
+  if (c >= cv.channels) return;
+  const float* kept = rec_copy_before(cv.state, cv.state_stride, cv.copy_elems, slot, start);
+  float* keep = rec_copy_behind(cv.state, cv.state_stride, cv.copy_elems, slot, start + count - 1);
+  for (int i = 0; i < cv.taps - 1; ++i) {
+    const int at = i + count;
+    keep[(long)i * cv.channels + c] = at < cv.taps - 1 ? kept[(long)at * cv.channels + c]
+                                                       : proj[(long)(first + at - (cv.taps - 1)) * stride + c];
+  }
 }
 
 // One wave per (token, head), four waves a block; any sizes, both builds.  For each map: positions
@@ -767,7 +835,9 @@ extern "C" int axk_heads_prepare(const float* proj, long stride, int q_at, int n
                                  int dim, const void* q_gain, int q_gain_is_f32, const void* k_gain, int k_gain_is_f32, float eps,
                                  int rot, int neighbours, float magnitude, const float* table, const int32_t* positions,
                                  const int32_t* seq_rows, const int32_t* block_table, int table_stride, void* cache, int page_size,
-                                 void* q_out, int n_tokens, int write_kv, float q_temp_coef, int q_temp_every, int norm_rows, void* stream) {
+                                 void* q_out, int n_tokens, int write_kv, float q_temp_coef, int q_temp_every, int norm_rows, const void* conv_w,
+                                 int conv_taps, float* conv_state, long conv_state_stride, long conv_copy_elems, const int32_t* conv_spans,
+                                 int n_spans, void* stream) {
   AXK_REQUIRE(n_tokens >= 0 && n_q > 0 && n_k > 0 && dim > 0 && v_width > 0 && page_size > 0,
               "heads_prepare: bad sizes T=%d q units=%d k units=%d dim=%d values=%d page=%d", n_tokens, n_q, n_k, dim, v_width,
               page_size);
@@ -775,13 +845,33 @@ extern "C" int axk_heads_prepare(const float* proj, long stride, int q_at, int n
   AXK_REQUIRE(q_at >= 0 && q_at + (long)n_q * dim <= stride &&
               (!write_kv || (k_at >= 0 && v_at >= 0 && k_at + (long)n_k * dim <= stride && v_at + (long)v_width <= stride)), "heads_prepare: the parts do not fit rows of %ld", stride);
   AXK_REQUIRE(!norm_rows || (q_gain != nullptr && (!write_kv || k_gain != nullptr)), "heads_prepare: a norm over all rows without its gains");
+  HeadsConv cv = {};
+  if (conv_w != nullptr) {
+    cv = HeadsConv{(const elem_t*)conv_w, conv_taps, n_q * dim + n_k * dim + v_width, conv_spans == nullptr, conv_state, conv_state_stride,
+                   conv_copy_elems};
+    AXK_REQUIRE(conv_taps >= 1 && conv_state != nullptr && conv_copy_elems >= (long)(conv_taps - 1) * cv.channels &&
+                conv_state_stride >= 2 * conv_copy_elems,
+                "heads_prepare: a state row of %ld floats does not hold two copies of %ld with %d x %d kept projections", conv_state_stride,
+                conv_copy_elems, conv_taps - 1, cv.channels);
+    AXK_REQUIRE(k_at == q_at + n_q * dim && v_at == k_at + n_k * dim && write_kv && !norm_rows && n_spans >= 0 &&
+                4L * dim * (long)sizeof(float) <= 48 * 1024,
+                "heads_prepare: a convolution wants q, k and v side by side, all stored, normed head by head or not at all");
+  }
   if (n_tokens == 0) return 0;
   // few tokens: a token's units side by side in several blocks
   const int per_token = n_tokens >= 1024 ? 1 : min((n_q + n_k + 3) / 4, 16);
-  heads_prepare_kernel<<<dim3(n_tokens, per_token), 256, 0, (hipStream_t)stream>>>(
-      proj, stride, q_at, n_q, k_at, n_k, v_at, v_width, dim, q_gain, q_gain_is_f32, k_gain, k_gain_is_f32, eps, rot, neighbours,
-      magnitude, table, positions, seq_rows, block_table, table_stride, (elem_t*)cache, page_size, (elem_t*)q_out, write_kv, q_temp_coef,
-      q_temp_every, norm_rows);
+#define HEADS_ARGS proj, stride, q_at, n_q, k_at, n_k, v_at, v_width, dim, q_gain, q_gain_is_f32, k_gain, k_gain_is_f32, eps, rot, neighbours, \
+                   magnitude, table, positions, seq_rows, block_table, table_stride, (elem_t*)cache, page_size, (elem_t*)q_out, write_kv,      \
+                   q_temp_coef, q_temp_every, norm_rows, cv
+  if (conv_w == nullptr) {
+    heads_prepare_kernel<false><<<dim3(n_tokens, per_token), 256, 0, (hipStream_t)stream>>>(HEADS_ARGS);
+  } else {
+    heads_prepare_kernel<true><<<dim3(n_tokens, per_token), 256, 4 * dim * sizeof(float), (hipStream_t)stream>>>(HEADS_ARGS);
+    if (conv_spans != nullptr && conv_taps > 1 && n_spans > 0)
+      heads_keep_kernel<<<dim3(ceil_div(cv.channels, 256), n_spans), 256, 0, (hipStream_t)stream>>>(proj + q_at, stride, cv, conv_spans,
+                                                                                                   positions);
+  }
+#undef HEADS_ARGS
   AXK_LAUNCH_CHECK("heads_prepare");
   return 0;
 }

@@ -1,7 +1,8 @@
 // Time mixing with a state matrix a head, decayed per key channel (the time-mix block of RWKV-6-like models):
 //
 //   token shift   a mix of a token's row and the one before it, h + (h' - h) mu, for each of several uses
-//   decay         w = exp(-exp(w0 + W2 tanh(t))), t the low-rank projection of its mix
+//   decay         w = exp(-exp(w0 + W2 tanh(t))), t the low-rank projection of its mix (the kernel of the second product
+//                 also makes the delta rule's decays and gates of low rank)
 //   per head      o_t = (S_(t-1) + diag(u) k_t v_t^T)^T r_t,  S_t = diag(w_t) S_(t-1) + k_t v_t^T
 //
 // A copy of the state row (see recurrence.h) holds the heads' states [heads][P][N], then the request's last row
@@ -72,18 +73,43 @@ token_shift_kernel(const elem_t* __restrict__ h, const float* __restrict__ mu, i
   }
 }
 
-// w[t, c] = exp(-exp(w0[c] + sum_k W2[c, k] tanh(low[t, k]))), all in 32-bit: tiles of 16 OWN tokens x 64 channels, a
-// thread OWN tokens x 4 channels, the rank in pieces of 64 through LDS, a chain in ascending k an output.
+// The second half of low-rank products, out[t, c] = act(sum_k W[c, k] in(low[t, k])), all in 32-bit: tiles of 16 OWN tokens x
+// 64 channels, a thread OWN tokens x 4 channels, the rank in pieces of 64 through LDS, a chain in ascending k an output.
+// Up to two products of the same tokens share a launch (the first takes the first blocks of a row of the grid).
+enum { LR_TIME_MIX_DECAY = 0, LR_DELTA_DECAY = 1, LR_PLAIN = 2 };
+struct LowRank {
+  const float* low;          // rows of the first half's results
+  long low_stride;
+  const elem_t* w;           // [channels, rank]
+  int channels, rank, kind;
+  const void* bias;          // LR_TIME_MIX_DECAY, LR_DELTA_DECAY: [channels]
+  int bias_is_f32;
+  const void* a_log;         // LR_DELTA_DECAY: one a head of head_dim channels
+  int a_log_is_f32, head_dim;
+  float* out;                // [T, channels]
+};
+
+// in: tanh for LR_TIME_MIX_DECAY, else as it is.
+__device__ inline float low_rank_act(const LowRank& r, float v, int c) {
+  if (r.kind == LR_PLAIN) return v;
+  v += load_vec(r.bias, r.bias_is_f32, c);
+  if (r.kind == LR_TIME_MIX_DECAY) return expf(-expf(v));
+  return expf(-(expf(load_vec(r.a_log, r.a_log_is_f32, c / r.head_dim)) * rec_softplus(v)));
+}
+
 #define TD_CHANNELS 64
 #define TD_RANK 64
 template <int OWN>
 __global__ void __launch_bounds__(256)
-time_mix_decay_kernel(const float* __restrict__ low, const elem_t* __restrict__ w2, const void* __restrict__ w0, int w0_is_f32,
-                      float* __restrict__ w, int n_tokens, int channels, int rank) {
+low_rank_kernel(LowRank first, LowRank second, int n_tokens) {
   constexpr int TOKENS = 16 * OWN;
   __shared__ __align__(16) float ts[TD_RANK][TOKENS + 4];
   __shared__ __align__(16) float ws[TD_RANK][TD_CHANNELS + 4];
-  const int t0 = blockIdx.y * TOKENS, c0 = blockIdx.x * TD_CHANNELS;
+  const int first_blocks = (first.channels + TD_CHANNELS - 1) / TD_CHANNELS;
+  const bool is_first = (int)blockIdx.x < first_blocks;
+  const LowRank r = is_first ? first : second;
+  const int t0 = blockIdx.y * TOKENS, c0 = ((int)blockIdx.x - (is_first ? 0 : first_blocks)) * TD_CHANNELS;
+  const int rank = r.rank, channels = r.channels;
   const int tx = threadIdx.x & 15, ty = threadIdx.x >> 4;
   float acc[OWN][4];
 #pragma unroll
@@ -96,19 +122,22 @@ time_mix_decay_kernel(const float* __restrict__ low, const elem_t* __restrict__ 
 #pragma unroll
     for (int it = 0; it < TOKENS * TD_RANK / 256; ++it) {
       const int i = it * 256 + threadIdx.x, t = i / TD_RANK, k = i % TD_RANK;
-      ts[k][t] = k < n && t0 + t < n_tokens ? tanhf(low[(long)(t0 + t) * rank + k0 + k]) : 0.0f;
+      float v = k < n && t0 + t < n_tokens ? r.low[(long)(t0 + t) * r.low_stride + k0 + k] : 0.0f;
+      if (r.kind == LR_TIME_MIX_DECAY) v = tanhf(v);
+      ts[k][t] = v;
     }
 #pragma unroll
     for (int it = 0; it < TD_CHANNELS * TD_RANK / 1024; ++it) {
       const int i = it * 256 + threadIdx.x, c = i / (TD_RANK / 4), k = 4 * (i % (TD_RANK / 4));
       float v[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-      if (k < n && c0 + c < channels) load4_guarded(w2 + (long)(c0 + c) * rank + k0 + k, n - k, (rank & 3) == 0, v);
+      if (k < n && c0 + c < channels) load4_guarded(r.w + (long)(c0 + c) * rank + k0 + k, n - k, (rank & 3) == 0, v);
 #pragma unroll
       for (int j = 0; j < 4; ++j) ws[k + j][c] = v[j];
     }
     __syncthreads();
+    const int n_pad = (n + 7) & ~7;
 #pragma unroll 8
-    for (int k = 0; k < TD_RANK; ++k) {              // behind the rank: zeros
+    for (int k = 0; k < n_pad; ++k) {                // behind the rank: zeros
       const float4 x = *reinterpret_cast<const float4*>(&ws[k][4 * tx]);
 #pragma unroll
       for (int i = 0; i < OWN; ++i) {
@@ -127,9 +156,19 @@ time_mix_decay_kernel(const float* __restrict__ low, const elem_t* __restrict__ 
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int c = c0 + 4 * tx + j;
-      if (c < channels) w[(long)t * channels + c] = expf(-expf(acc[i][j] + load_vec(w0, w0_is_f32, c)));
+      if (c < channels) r.out[(long)t * channels + c] = low_rank_act(r, acc[i][j], c);
     }
   }
+}
+
+static int launch_low_rank(const LowRank& first, const LowRank& second, int n_tokens, hipStream_t stream, const char* name) {
+  const int blocks = ceil_div(first.channels, TD_CHANNELS) + (second.channels > 0 ? ceil_div(second.channels, TD_CHANNELS) : 0);
+  if (n_tokens >= 512)
+    low_rank_kernel<4><<<dim3(blocks, ceil_div(n_tokens, 64)), 256, 0, stream>>>(first, second, n_tokens);
+  else
+    low_rank_kernel<1><<<dim3(blocks, ceil_div(n_tokens, 16)), 256, 0, stream>>>(first, second, n_tokens);
+  AXK_LAUNCH_CHECK(name);
+  return 0;
 }
 
 // The walk.  grid (stretches, heads, blocks of value dims); LK lanes share VP value dims, OWN rows of the state a
@@ -339,14 +378,28 @@ extern "C" int axk_time_mix_decay(const float* low, const void* w2, const void* 
   AXK_REQUIRE(n_tokens >= 0 && channels > 0 && rank > 0, "time_mix_decay: bad sizes T=%d channels=%d rank=%d", n_tokens, channels, rank);
   AXK_REQUIRE(n_tokens <= 65535 * 16 && ((uintptr_t)w2 & 15) == 0, "time_mix_decay: %d tokens in one step, or w2 is not aligned", n_tokens);
   if (n_tokens == 0) return 0;
-  if (n_tokens >= 512)
-    time_mix_decay_kernel<4><<<dim3(ceil_div(channels, TD_CHANNELS), ceil_div(n_tokens, 64)), 256, 0, (hipStream_t)stream>>>(
-        low, (const elem_t*)w2, w0, w0_is_f32, w, n_tokens, channels, rank);
-  else
-    time_mix_decay_kernel<1><<<dim3(ceil_div(channels, TD_CHANNELS), ceil_div(n_tokens, 16)), 256, 0, (hipStream_t)stream>>>(
-        low, (const elem_t*)w2, w0, w0_is_f32, w, n_tokens, channels, rank);
-  AXK_LAUNCH_CHECK("time_mix_decay");
-  return 0;
+  const LowRank job = {low, rank, (const elem_t*)w2, channels, rank, LR_TIME_MIX_DECAY, w0, w0_is_f32, nullptr, 0, 1, w};
+  LowRank none = job;
+  none.channels = 0;
+  return launch_low_rank(job, none, n_tokens, (hipStream_t)stream, "time_mix_decay");
+}
+
+extern "C" int axk_delta_low_rank(const float* rows, long stride, int decay_at, int decay_rank, const void* w_decay, const void* dt_bias,
+                                  int dt_bias_is_f32, const void* a_log, int a_log_is_f32, int head_dim, float* decay,
+                                  int decay_channels, int gate_at, int gate_rank, const void* w_gate, float* gate, int gate_channels,
+                                  int n_tokens, void* stream) {
+  AXK_REQUIRE(n_tokens >= 0 && decay_channels >= 0 && gate_channels >= 0 && decay_channels + gate_channels > 0 &&
+              n_tokens <= 65535 * 16, "delta_low_rank: bad sizes T=%d channels=%d, %d", n_tokens, decay_channels, gate_channels);
+  AXK_REQUIRE(decay_channels == 0 || (decay_rank > 0 && decay_at >= 0 && decay_at + (long)decay_rank <= stride && head_dim > 0 &&
+                                      ((uintptr_t)w_decay & 15) == 0),
+              "delta_low_rank: decays of rank %d from column %d of %ld, heads of %d", decay_rank, decay_at, stride, head_dim);
+  AXK_REQUIRE(gate_channels == 0 || (gate_rank > 0 && gate_at >= 0 && gate_at + (long)gate_rank <= stride && ((uintptr_t)w_gate & 15) == 0),
+              "delta_low_rank: gates of rank %d from column %d of %ld", gate_rank, gate_at, stride);
+  if (n_tokens == 0) return 0;
+  const LowRank d = {rows + decay_at, stride, (const elem_t*)w_decay, decay_channels, decay_rank, LR_DELTA_DECAY, dt_bias, dt_bias_is_f32,
+                     a_log, a_log_is_f32, head_dim, decay};
+  const LowRank g = {rows + gate_at, stride, (const elem_t*)w_gate, gate_channels, gate_rank, LR_PLAIN, nullptr, 0, nullptr, 0, 1, gate};
+  return launch_low_rank(d, g, n_tokens, (hipStream_t)stream, "delta_low_rank");
 }
 
 extern "C" int axk_wkv_scan(const float* rows, long stride, long r_at, long k_at, long v_at, const float* w, const float* u,

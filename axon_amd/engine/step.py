@@ -81,6 +81,10 @@ class StepContext:
     def no_rotation(self) -> torch.Tensor:
         return torch.empty((self.n_tokens, 0, 2), dtype=torch.float32, device=self.rt.device)
 
+    def no_state(self) -> torch.Tensor:
+        """State rows that hold nothing, for kernels that take a state of any size."""
+        return self.ws.take((1, 4), torch.float32)
+
 
 class PendingPicks:
     """The greedy picks of a decoding step on their way to the host: the copy was queued behind

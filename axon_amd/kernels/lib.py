@@ -109,12 +109,25 @@ _SIGNATURES = {
                      c_void_p, c_void_p, c_void_p],
     "axk_delta_prepare": [c_void_p, c_long, c_void_p, c_int, c_void_p, c_long, c_long, c_long, c_void_p, c_void_p, c_int, c_int,
                           c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p],
-    "axk_delta_scan": [c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_long,
+    "axk_delta_scan": [c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_long,
                        c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "axk_delta_chunked_ok": [c_int, c_int, c_int, c_int],
     "axk_delta_chunked": [c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p,
                           c_long, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_long, c_void_p],
-    "axk_head_norm_gate": [c_void_p, c_void_p, c_long, c_void_p, c_int, c_int, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
+    "axk_delta_low_rank": [c_void_p, c_long, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int,
+                           c_void_p, c_void_p, c_int, c_int, c_void_p],
+    "axk_silu_rows": [c_void_p, c_long, c_int, c_int, c_void_p],
+    "axk_lightning_scan": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_long, c_long, c_void_p, c_int, c_void_p,
+                           c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
+    "axk_lightning_chunked_ok": [c_int, c_int, c_int, c_long, c_int, c_int],
+    "axk_lightning_chunked": [c_void_p, c_long, c_int, c_int, c_int, c_void_p, c_void_p, c_long, c_long, c_void_p, c_int, c_void_p, c_int,
+                              c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_long, c_void_p],
+    "axk_embed_pairs": [c_void_p, c_void_p, c_int, c_float, c_void_p, c_int, c_long, c_long, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                        c_int, c_int, c_void_p],
+    "axk_scaled_sum": [c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_void_p,
+                       c_long, c_void_p, c_void_p, c_int, c_int, c_void_p],
+    "axk_shifted_norm": [c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_long, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p],
+    "axk_head_norm_gate": [c_void_p, c_void_p, c_long, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
     "axk_latent_prepare": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_int,
                            c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p],
     "axk_latent_query_rope": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
@@ -127,7 +140,7 @@ _SIGNATURES = {
     "axk_add_scaled": [c_void_p, c_void_p, c_float, c_long, c_void_p],
     "axk_heads_prepare": [c_void_p, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_int, c_float,
                           c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_int,
-                          c_int, c_float, c_int, c_int, c_void_p],
+                          c_int, c_float, c_int, c_int, c_void_p, c_int, c_void_p, c_long, c_long, c_void_p, c_int, c_void_p],
     "axk_masked_attention_uses_mfma": [c_int, c_int, c_int, c_int, c_int, c_int],
     "axk_masked_attention": [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_long, c_void_p, c_int, c_int,
                              c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_float, c_float,
@@ -252,7 +265,7 @@ class Kernels:
                   "route_topk", "route_sort", "route_combine", "gather_rows", "causal_conv", "gated_scan", "latent_prepare",
                   "latent_query_rope", "latent_attention", "heads_prepare", "masked_attention", "concat_round", "scale_rows",
                   "add_scaled", "state_conv", "state_space_scan", "gated_group_norm", "route_scored", "sum_norm", "layernorm",
-                  "softcap")
+                  "softcap", "embed_pairs", "scaled_sum", "shifted_norm", "delta_low_rank", "silu_rows", "lightning_scan")
     _MATRIX_AT = {"gemm": 1, "gemm_qkv_rope": 1, "gemm_normed_glu": 3, "gemm_normed_qkv_rope": 3, "grouped_gemm": 1}   # which argument is W
 
     def set_launch_hook(self, hook) -> None:
@@ -1167,12 +1180,12 @@ class Kernels:
                       dt_bias, u, terms, heads: int, kv_heads: int, keys: int, values: int, q_scale: float) -> None:
         """The delta rule's operands from the projections' float32 rows [T, .]: the channels [q | k | v] convolved
         (w [channels, taps] in the compute dtype), through silu, queries and keys of length 1 a head, into u [T, channels];
-        terms [T, heads, 2] = (g, beta) (see csrc/delta_rule.hip)."""
+        terms [T, heads, 2] = (g, beta), g 1 without a_log (see csrc/delta_rule.hip)."""
         self._f32_rows(rows, "delta rows"); self._elem(w, "delta conv"); self._f32(u, "delta u"); self._f32(terms, "delta terms")
         T, C = u.shape
         self._state_rows(state, seq_rows, positions, T, "delta_prepare")
         if C != 2 * kv_heads * keys + heads * values or rows.shape[0] != T or w.dim() != 2 or w.shape[0] != C or not w.is_contiguous() \
-                or terms.shape != (T, heads, 2) or a_log.numel() != heads or dt_bias.numel() != heads:
+                or terms.shape != (T, heads, 2) or (a_log is not None and (a_log.numel() != heads or dt_bias.numel() != heads)):
             raise KernelError(f"delta_prepare: rows {tuple(rows.shape)}, conv {tuple(w.shape)}, u {tuple(u.shape)}, terms {tuple(terms.shape)}")
         self._check(self.lib.axk_delta_prepare(
             _ptr(rows), rows.stride(0), _ptr(w), w.shape[1], _ptr(state), state.stride(0), int(copy_elems), int(tail_at), _ptr(positions),
@@ -1180,12 +1193,13 @@ class Kernels:
             self._vec_flag(dt_bias, "dt bias"), _ptr(u), _ptr(terms), T, heads, kv_heads, keys, values, float(q_scale), _stream()))
 
     def delta_scan(self, u, terms, state, copy_elems: int, tail_at: int, spans, positions, seq_rows, conv_in, y, heads: int,
-                   kv_heads: int, keys: int, values: int, taps: int, chunks=None) -> torch.Tensor:
+                   kv_heads: int, keys: int, values: int, taps: int, chunks=None, decay=None) -> torch.Tensor:
         """The gated delta rule over each request's tokens (see csrc/delta_rule.hip): u [T, channels] and terms [T, heads, 2]
         float32; spans int32 [n, 3] or None as in the other scans; conv_in: the convolutions' inputs (float32, rows may be
         strided), kept for the next step; y [T, heads values] float32.  `chunks` = (chunks int32 [n, 2]: first token, tokens;
         spans5 int32 [m, 5]: slot, first token, tokens, first chunk, chunks): these requests' stretches run in chunks on the
-        matrix cores (`delta_chunked_ok`; sums in another order, by rounding), `spans` then names the others (it may be empty)."""
+        matrix cores (`delta_chunked_ok`; sums in another order, by rounding), `spans` then names the others (it may be empty).
+        `decay` float32 [T, heads keys]: a decay a head and key channel, in place of terms' g (which is 1 then)."""
         for t, what in ((u, "delta u"), (terms, "delta terms"), (y, "delta y")):
             self._f32(t, what)
         self._f32_rows(conv_in, "delta conv_in")
@@ -1194,6 +1208,10 @@ class Kernels:
         if C != 2 * kv_heads * keys + heads * values or terms.shape != (T, heads, 2) or y.shape != (T, heads * values) \
                 or conv_in.shape[0] != T or conv_in.shape[1] < C:
             raise KernelError(f"delta_scan: u {tuple(u.shape)}, terms {tuple(terms.shape)}, y {tuple(y.shape)}, conv_in {tuple(conv_in.shape)}")
+        if decay is not None:
+            self._f32(decay, "delta decay")
+            if decay.shape != (T, heads * keys):
+                raise KernelError(f"delta_scan: decays {tuple(decay.shape)} for {T} tokens of {heads} x {keys}")
         n = T
         if spans is not None:
             self._i32(spans, "scan spans")
@@ -1212,7 +1230,7 @@ class Kernels:
             if n == 0:
                 return y
         self._check(self.lib.axk_delta_scan(
-            _ptr(u), _ptr(terms), _ptr(state), state.stride(0), int(copy_elems), int(tail_at), _ptr(spans), n, _ptr(positions),
+            _ptr(u), _ptr(terms), _ptr(decay), _ptr(state), state.stride(0), int(copy_elems), int(tail_at), _ptr(spans), n, _ptr(positions),
             _ptr(seq_rows), _ptr(conv_in), conv_in.stride(0), _ptr(y), heads, kv_heads, keys, values, int(taps), _stream()))
         return y
 
@@ -1220,15 +1238,141 @@ class Kernels:
         """Whether `delta_scan` takes `chunks` at these sizes."""
         return bool(self.lib.axk_delta_chunked_ok(kv_heads, heads, keys, values))
 
-    def head_norm_gate(self, y, gate, gain, eps: float, out, heads: int) -> torch.Tensor:
-        """out = (y / sqrt(mean y^2 + eps)) gain silu(gate), the mean over each of `heads` equal parts of a row: y float32
+    def delta_low_rank(self, rows, decay=None, gate=None) -> None:
+        """Decays and gates of low rank, from columns of the projections' float32 rows [T, .]: decay = (first column, w
+        [heads keys, rank], dt_bias, a_log [heads], out float32 [T, heads keys]): exp(-exp(a_log) softplus(w . + dt_bias));
+        gate = (first column, w [channels, rank], out float32 [T, channels]): w . (see csrc/time_mix.hip)."""
+        self._f32_rows(rows, "low-rank rows")
+        T = rows.shape[0]
+        d_at, d_w, d_bias, a_log, d_out = decay if decay is not None else (0, None, None, None, None)
+        g_at, g_w, g_out = gate if gate is not None else (0, None, None)
+        for w, out, what in ((d_w, d_out, "decay"), (g_w, g_out, "gate")):
+            if w is None:
+                continue
+            self._elem(w, "low-rank " + what); self._f32(out, "low-rank " + what)
+            if w.dim() != 2 or not w.is_contiguous() or out.shape != (T, w.shape[0]):
+                raise KernelError(f"delta_low_rank: {what} {tuple(w.shape)} into {tuple(out.shape)}")
+        if d_w is not None and (d_bias.numel() != d_w.shape[0] or d_w.shape[0] % a_log.numel()):
+            raise KernelError(f"delta_low_rank: {d_bias.numel()} biases and {a_log.numel()} heads for {d_w.shape[0]} decays")
+        size = lambda w, i: 0 if w is None else w.shape[i]
+        self._check(self.lib.axk_delta_low_rank(
+            _ptr(rows), rows.stride(0), int(d_at), size(d_w, 1), _ptr(d_w), _ptr(d_bias), self._vec_flag(d_bias, "dt bias"), _ptr(a_log),
+            self._vec_flag(a_log, "A_log"), 1 if d_w is None else d_w.shape[0] // a_log.numel(), _ptr(d_out), size(d_w, 0), int(g_at),
+            size(g_w, 1), _ptr(g_w), _ptr(g_out), size(g_w, 0), T, _stream()))
+
+    GATES = {"silu": 0, "sigmoid": 1}
+
+    def head_norm_gate(self, y, gate, gain, eps: float, out, heads: int, act: str = "silu") -> torch.Tensor:
+        """out = (y / sqrt(mean y^2 + eps)) gain act(gate), the mean over each of `heads` equal parts of a row: y float32
         [T, W], gate float32 [T, W] (rows may be strided), gain of a part's width (shared) or of W, out in the compute dtype."""
         self._f32(y, "head norm y"); self._f32_rows(gate, "head norm gate"); self._elem(out, "head norm out")
         T, W = y.shape
         if W % heads or gate.shape != (T, W) or out.shape != (T, W) or not out.is_contiguous() or gain.numel() not in (W, W // heads):
             raise KernelError(f"head_norm_gate: y {tuple(y.shape)}, gate {tuple(gate.shape)}, a gain of {gain.numel()}, {heads} heads")
         self._check(self.lib.axk_head_norm_gate(_ptr(y), _ptr(gate), gate.stride(0), _ptr(gain), self._vec_flag(gain, "head norm gain"),
-                                                1 if gain.numel() == W else 0, float(eps), _ptr(out), T, heads, W // heads, _stream()))
+                                                1 if gain.numel() == W else 0, self.GATES[act], float(eps), _ptr(out), T, heads, W // heads,
+                                                _stream()))
+        return out
+
+    # ------------------------------------------------------------------ linear attention with a constant decay a head
+    def silu_rows(self, rows, columns: int) -> torch.Tensor:
+        """silu in place over the first `columns` numbers of float32 rows."""
+        self._f32_rows(rows, "silu rows")
+        self._check(self.lib.axk_silu_rows(_ptr(rows), rows.stride(0), int(columns), rows.shape[0], _stream()))
+        return rows
+
+    def lightning_chunked_ok(self, heads: int, keys: int, values: int, stride: int, q_at: int, k_at: int) -> bool:
+        """Whether `lightning_scan` takes `chunks` at these sizes."""
+        return bool(self.lib.axk_lightning_chunked_ok(heads, keys, values, int(stride), int(q_at), int(k_at)))
+
+    def lightning_scan(self, rows, q_at: int, k_at: int, v_at: int, silu: bool, decay, state, copy_elems: int, spans, positions, seq_rows,
+                       y, heads: int, keys: int, values: int, chunks=None) -> torch.Tensor:
+        """The decayed states of linear attention over each request's tokens (see csrc/linear_attention.hip): rows float32
+        [T, .] with q and k of heads keys columns and v of heads values; decay float32 [heads]; spans, chunks as in
+        `delta_scan`; y [T, heads values] float32.  `silu`: q, k and v are taken through silu on the way (not with `chunks`,
+        whose operands are read more than once: `silu_rows` first)."""
+        self._f32_rows(rows, "lightning rows"); self._f32(decay, "lightning decay"); self._f32(y, "lightning y")
+        T = rows.shape[0]
+        self._state_rows(state, seq_rows, positions, T, "lightning_scan")
+        if decay.numel() != heads or y.shape != (T, heads * values) or (silu and chunks is not None):
+            raise KernelError(f"lightning_scan: {decay.numel()} decays of {heads} heads, y {tuple(y.shape)}")
+        n = T
+        if spans is not None:
+            self._i32(spans, "scan spans")
+            n = spans.shape[0]
+        if chunks is not None:
+            list_, spans5 = chunks
+            self._i32(list_, "lightning chunks"); self._i32(spans5, "lightning requests")
+            if spans is None or list_.dim() != 2 or list_.shape[1] != 2 or spans5.dim() != 2 or spans5.shape[1] != 5:
+                raise KernelError(f"lightning_scan: chunks {tuple(list_.shape)} of requests {tuple(spans5.shape)}")
+            need = list_.shape[0] * heads * keys * values
+            ends = torch.empty(need, dtype=torch.float32, device=y.device)
+            self._check(self.lib.axk_lightning_chunked(
+                _ptr(rows), rows.stride(0), int(q_at), int(k_at), int(v_at), _ptr(decay), _ptr(state), state.stride(0), int(copy_elems),
+                _ptr(list_), list_.shape[0], _ptr(spans5), spans5.shape[0], _ptr(positions), _ptr(y), heads, keys, values, _ptr(ends), need,
+                _stream()))
+            if n == 0:
+                return y
+        self._check(self.lib.axk_lightning_scan(
+            _ptr(rows), rows.stride(0), int(q_at), int(k_at), int(v_at), 1 if silu else 0, _ptr(decay), _ptr(state), state.stride(0),
+            int(copy_elems), _ptr(spans), n, _ptr(positions), _ptr(seq_rows), _ptr(y), heads, keys, values, _stream()))
+        return y
+
+    # ------------------------------------------------------------------ passes over the residual stream
+    def embed_pairs(self, tokens, table, scale: float, pairs, mul_prev: int, mul_cur: int, state, positions, seq_rows, out) -> torch.Tensor:
+        """out[t] = table[token] scale + pairs[(the request's token before mul_prev + token mul_cur) mod buckets] (pairs
+        [buckets + 1, dim]: the last row for a request's first token); state int32 [slots, 2] (see csrc/stream.hip)."""
+        packed = isinstance(table, PackedMatrix)
+        self._i32(tokens, "embed tokens"); self._elem(table.data if packed else table, "embed table"); self._elem(pairs, "pairs")
+        self._f32(out, "embed out"); self._i32(state, "embed state"); self._i32(positions, "positions"); self._i32(seq_rows, "seq_rows")
+        vocab, dim = table.shape
+        T = tokens.numel()
+        if out.shape != (T, dim) or pairs.dim() != 2 or pairs.shape[1] != dim or pairs.shape[0] < 2 or not pairs.is_contiguous() \
+                or not (packed or table.is_contiguous()) or state.dim() != 2 or state.shape[1] != 2:
+            raise KernelError(f"embed_pairs: pairs {tuple(pairs.shape)}, out {tuple(out.shape)} for {T} tokens of width {dim}")
+        self._check(self.lib.axk_embed_pairs(
+            _ptr(tokens), _ptr(table), 1 if packed else 0, float(scale), _ptr(pairs), pairs.shape[0] - 1, int(mul_prev), int(mul_cur),
+            _ptr(state), _ptr(positions), _ptr(seq_rows), _ptr(out), T, dim, vocab, _stream()))
+        return out
+
+    def scaled_sum(self, terms, x, norm=None, shift=None) -> torch.Tensor:
+        """x += sum of n(y) scales over one or two terms (y float32 rows, scales float32 [dim], norm_eps or None): n(y) is
+        y / sqrt(mean(y^2) + norm_eps), or y.  `norm` = (gain float32 [dim], eps, out): also the RMS norm of the new rows;
+        `shift` = (share, state, positions, seq_rows), in steps of single tokens: moved towards the request's rows before."""
+        self._f32(x, "scaled_sum x")
+        T, W = x.shape
+        if not 1 <= len(terms) <= 2:
+            raise KernelError(f"scaled_sum: {len(terms)} outputs (one or two)")
+        args = []
+        for y, scales, norm_eps in list(terms) + [(None, None, None)] * (2 - len(terms)):
+            if y is not None:
+                self._f32(y, "scaled_sum y"); self._f32(scales, "scaled_sum scales")
+                if y.shape != (T, W) or scales.numel() != W:
+                    raise KernelError(f"scaled_sum: y {tuple(y.shape)}, {scales.numel()} scales for x {tuple(x.shape)}")
+            args += [_ptr(y), _ptr(scales), -1.0 if norm_eps is None else float(norm_eps)]
+        gain, eps, out = norm if norm is not None else (None, 0.0, None)
+        share, state, positions, seq_rows = shift if shift is not None else (None, None, None, None)
+        if norm is not None:
+            self._f32(gain, "scaled_sum gain"); self._elem(out, "scaled_sum out")
+            if gain.numel() != W or out.shape != (T, W) or not out.is_contiguous():
+                raise KernelError(f"scaled_sum: a gain of {gain.numel()}, out {tuple(out.shape)} for x {tuple(x.shape)}")
+        if shift is not None:
+            self._f32(share, "scaled_sum share"); self._state_rows(state, seq_rows, positions, T, "scaled_sum")
+        self._check(self.lib.axk_scaled_sum(*args, _ptr(x), _ptr(gain), float(eps), _ptr(out), _ptr(share), _ptr(state),
+                                            0 if state is None else state.stride(0), _ptr(positions), _ptr(seq_rows), T, W, _stream()))
+        return x
+
+    def shifted_norm(self, x, gain, eps: float, share, state, positions, seq_rows, out) -> torch.Tensor:
+        """out = h + (h' - h) share with h the RMS norm of x (gain float32 [dim]) and h' the request's h before, which the
+        float32 state rows [slots, 2 dim] keep from step to step (see csrc/stream.hip)."""
+        self._f32(x, "shifted_norm x"); self._f32(gain, "shifted_norm gain"); self._f32(share, "shifted_norm share")
+        self._elem(out, "shifted_norm out")
+        T, W = x.shape
+        self._state_rows(state, seq_rows, positions, T, "shifted_norm")
+        if gain.numel() != W or share.numel() != W or out.shape != (T, W) or not out.is_contiguous():
+            raise KernelError(f"shifted_norm: x {tuple(x.shape)}, gain {gain.numel()}, share {share.numel()}, out {tuple(out.shape)}")
+        self._check(self.lib.axk_shifted_norm(_ptr(x), _ptr(gain), float(eps), _ptr(share), _ptr(state), state.stride(0), _ptr(positions),
+                                              _ptr(seq_rows), _ptr(out), T, W, _stream()))
         return out
 
     # ------------------------------------------------------------------ attention over a latent cache
@@ -1297,10 +1441,12 @@ class Kernels:
 
     def heads_prepare(self, proj, q_at, n_q, k_at, n_k, v_at, v_width, dim, q_gain, k_gain, eps, rot, neighbours, magnitude,
                       table, positions, seq_rows, block_table, cache, page_size, q_out, write_kv=True, q_temp=None,
-                      norm_rows=False) -> None:
+                      norm_rows=False, conv=None) -> None:
         """The projections' float32 rows into queries (q_out) and the page's keys and values: see
         axk_heads_prepare in csrc/api.h.  `q_temp` = (coef, every): a query's temperature by its position.
-        `norm_rows`: the norm goes over all query (all key) units of a token at once."""
+        `norm_rows`: the norm goes over all query (all key) units of a token at once.  `conv` = (w [channels, taps] in the
+        compute dtype, state rows, copy_elems, spans): the projections pass a causal convolution first, what a request's
+        later steps need of them is kept in its state row; spans int32 [n, 3], or None in a step of single tokens."""
         self._f32(proj, "heads proj"); self._f32(table, "rope table"); self._i32(positions, "positions")
         self._i32(seq_rows, "seq_rows"); self._i32(block_table, "block_table"); self._elem(q_out, "heads q_out")
         T = positions.numel()
@@ -1312,12 +1458,23 @@ class Kernels:
         for gain, units in ((q_gain, n_q), (k_gain, n_k)):
             if gain is not None and gain.numel() != (units * dim if norm_rows else dim):
                 raise KernelError(f"heads_prepare: a gain of {gain.numel()} for {units} units of {dim}")
+        w = state = spans = None
+        copy_elems = 0
+        if conv is not None:
+            w, state, copy_elems, spans = conv
+            self._elem(w, "heads conv")
+            self._state_rows(state, seq_rows, positions, T, "heads_prepare")
+            if w.dim() != 2 or w.shape[0] != (n_q + n_k) * dim + v_width or not w.is_contiguous():
+                raise KernelError(f"heads_prepare: a convolution {tuple(w.shape)} of {(n_q + n_k) * dim + v_width} channels")
+            if spans is not None:
+                self._i32(spans, "conv spans")
         self._check(self.lib.axk_heads_prepare(
             _ptr(proj), proj.stride(0), q_at, n_q, k_at, n_k, v_at, v_width, dim, _ptr(q_gain), self._vec_flag(q_gain, "q gain"),
             _ptr(k_gain), self._vec_flag(k_gain, "k gain"), float(eps), rot, 1 if neighbours else 0, float(magnitude), _ptr(table),
             _ptr(positions), _ptr(seq_rows), _ptr(block_table), block_table.shape[-1], _ptr(cache), page_size, _ptr(q_out), T,
             1 if write_kv else 0, float(q_temp[0]) if q_temp else 0.0, int(q_temp[1]) if q_temp else 0, 1 if norm_rows else 0,
-            _stream()))
+            _ptr(w), 0 if w is None else w.shape[1], _ptr(state), 0 if state is None else state.stride(0), int(copy_elems), _ptr(spans),
+            0 if spans is None else spans.shape[0], _stream()))
 
     def masked_attention_uses_mfma(self, heads, kv_heads, maps, dim, vdim, page_size) -> bool:
         return bool(self.lib.axk_masked_attention_uses_mfma(heads, kv_heads, maps, dim, vdim, page_size))

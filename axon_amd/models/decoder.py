@@ -20,7 +20,7 @@ class CachePlan:
     group_specs: List
     group_layers: List[int]
     bindings: List[CacheBinding]
-    state_elems: List[int]
+    state_elems: List[tuple]
 
 
 class DecoderModel:
@@ -88,16 +88,26 @@ class DecoderModel:
             where[cache] = (g, counts[g])
             counts[g] += 1
         bindings, state_elems = [], []
+
+        def arena(spec) -> int:
+            state_elems.append((spec.elems, spec.dtype))
+            return len(state_elems) - 1
+
         for run in self.order:
-            mixer = self.blocks[run.layer].mixer
-            cs, ss = mixer.cache_spec(), mixer.state_spec()
+            block = self.blocks[run.layer]
+            mixer, own = block.mixer, block.state_spec()
+            cs = mixer.cache_spec()
             b = CacheBinding(writes=run.writes_cache)
             if cs is not None:
                 b.group, b.index = where[run.cache]
-            if ss is not None:
-                b.state_index = len(state_elems)
-                state_elems.append((ss.elems, ss.dtype))
+            states = [arena(ss) for ss in mixer.state_specs()]
+            if states:
+                b.state_index, b.more_states = states[0], tuple(states[1:])
+            if own is not None:
+                b.block_state = arena(own)
             bindings.append(b)
+        if self.embedding.state_spec() is not None:
+            self.embedding.state_index = arena(self.embedding.state_spec())
         return CachePlan(specs, counts, bindings, state_elems)
 
     def group_plans(self, page_size: int, pages_of_group) -> List[GroupPlan]:
@@ -148,7 +158,7 @@ class DecoderModel:
             following = None
             if i + 1 < end and self.order[i + 1].enter is None:     # a rewritten stream is normed by its own pass
                 after = self.blocks[self.order[i + 1].layer]
-                following = block.following_of(ctx, block.last_part(), after.first_norm(), x.shape[0])
+                following = block.following_of(ctx, block.last_part(), after.entry_norm(self.cache_plan.bindings[i + 1]), x.shape[0])
             if normed is None and following is None:
                 block.forward(ctx, binding, x)          # a block that knows nothing of this is called plainly
             else:

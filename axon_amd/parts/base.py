@@ -75,11 +75,20 @@ class StateSpec:
 @dataclass
 class CacheBinding:
     """What a run of a layer is given by the cache manager: its cache group and its index in
-    that group's storage, whether it stores what it computes, and its state arena."""
+    that group's storage, whether it stores what it computes, and its state arena (a mixer that is
+    put together from others may have several: `more_states`).  `block_state`: the arena of what
+    the arrangement itself carries from token to token."""
     group: int = -1
     index: int = -1
     writes: bool = True
     state_index: int = -1
+    more_states: Tuple[int, ...] = ()
+    block_state: int = -1
+
+    def with_states(self, first: int, count: int) -> "CacheBinding":
+        """This binding with `count` of its mixer's state arenas from the `first`-th on."""
+        some = ((self.state_index,) + self.more_states)[first:first + count]
+        return replace(self, state_index=some[0] if some else -1, more_states=tuple(some[1:]))
 
 
 class Part:
@@ -165,6 +174,12 @@ class Mixer(Part):
     def state_spec(self) -> Optional[StateSpec]:
         return None
 
+    def state_specs(self) -> List[StateSpec]:
+        """All the state this mixer wants for one run, an arena each (`CacheBinding.state_index`, then
+        `more_states`)."""
+        spec = self.state_spec()
+        return [] if spec is None else [spec]
+
     def max_context(self) -> Optional[int]:
         """The most positions of a request this mixer's kernels take (None: no limit of its own).
         The engine refuses a longer `max_seq_len` when it is built, not in the middle of a step."""
@@ -210,6 +225,24 @@ class Mixer(Part):
     def forward(self, ctx, binding: CacheBinding, h, residual) -> None:
         raise NotImplementedError
 
+    def output_terms(self) -> List["OutputTerm"]:
+        """How the outputs that `forward_apart` stores make this mixer's result (one output, as it is)."""
+        return [OutputTerm()]
+
+    def forward_apart(self, ctx, binding: CacheBinding, h, outs) -> None:
+        """The mixer's outputs, one a term, stored into `outs` (32-bit rows): for a block that sums them
+        itself.  The default serves every mixer that can store its output."""
+        self.forward(ctx, binding, h, outs[0], accumulate=False)
+
+
+@dataclass
+class OutputTerm:
+    """One of the outputs whose sum is a mixer's result: n(y) gain factor with n(y) = y, or
+    y / sqrt(mean(y^2) + norm_eps) over the width; gain None: 1."""
+    gain: Any = None
+    factor: float = 1.0
+    norm_eps: Optional[float] = None
+
 
 class FeedForward(Part):
     def finishes_following_norm(self, ctx) -> bool:
@@ -254,8 +287,17 @@ class Block(Part):
         """The norm this block starts with, if the block before may do its work; None: it may not."""
         return None
 
+    def entry_norm(self, binding: CacheBinding) -> Optional[Norm]:
+        """The same for a run of this block: a norm that carries state from token to token is bound to
+        the run's."""
+        return self.first_norm()
+
     def last_part(self):
         """The part whose product ends this block (it may finish the next block's first norm)."""
+        return None
+
+    def state_spec(self) -> Optional[StateSpec]:
+        """State of the arrangement's own (`CacheBinding.block_state`), beside the mixer's."""
         return None
 
     def forward(self, ctx, binding: CacheBinding, x, normed=None, following: Optional[FollowingNorm] = None) -> None:

@@ -11,7 +11,7 @@ from typing import List
 import torch
 
 from ..config.base import ConfigError
-from .base import ROUNDED_STREAM, Block, CacheBinding, TensorDecl, register_block
+from .base import ROUNDED_STREAM, Block, CacheBinding, Mixer, Norm, OutputTerm, StateSpec, TensorDecl, register_block
 
 # A norm behind a product whose kernel holds the finished rows anyway can be written by that
 # kernel, and a norm before a product of few rows can be worked out inside that product (the same
@@ -284,7 +284,135 @@ class SandwichNormBlock(Block):
         self.norms[3].add_to(ctx, y, x, following)
 
 
+class ShiftedNorm(Norm):
+    """A run's first norm with its token shift, bound to the state of that run (see `ScaledPreNormBlock`).  It offers itself to
+    no product."""
+
+    def __init__(self, block, state_index: int):
+        super().__init__({}, block.prefix)
+        self.norm, self.share, self.state_index = block.norm1, block.share, state_index
+
+    def arguments(self, ctx):
+        return self.share, ctx.cache.state(self.state_index), ctx.positions, ctx.seq_rows
+
+
+class FollowingSum:
+    """A norm handed to the block before: `values` get its rows in the pass that adds that block's last sublayer's output."""
+
+    def __init__(self, norm, shift, values):
+        self.norm, self.shift, self.values = norm, shift, values
+
+    def arguments(self):
+        return (self.norm.gain, self.norm.eps, self.values)
+
+
+class ScaledPreNormBlock(Block):
+    """x += m ls1 mixer(shift(norm1(x))); x += m ls2 feed_forward(norm2(x)): a layer scale (`layer_scale`: vectors `ls1`, `ls2`)
+    and the residual's factor m (`residual_mult`) on each sublayer's output, and (`token_shift`: the vector `shift`) what the
+    mixer reads moved towards the token before, h + (h' - h) shift with h' the previous token's h (zeros before the first), as
+    it was before it was moved.  A layer may have no feed-forward (it then has no norm2 and no ls2).
+
+    The outputs of a sublayer are stored as 32-bit rows and go into the stream in one 32-bit pass: a pair of mixers' two outputs
+    with their norms or factors, the layer scale and m, the sum, and the norm behind it (the next block's first norm included:
+    in steps of single tokens with its shift; else, since a shift reads the stream of the token before, that norm is a pass of
+    its own).  h' is per-request state: two rows, the one behind position p in copy p & 1.
+
+    The norms are RMS norms whose gains are kept 32-bit.  `residual_mult`, `layer_scale` and `token_shift` come with the norm's
+    parameters."""
+    graph_safe = True
+
+    def __init__(self, norm_factory, mixer, feed_forward, prefix):
+        super().__init__(norm_factory, mixer, feed_forward, prefix)
+        self.norm1 = norm_factory("norm1")
+        self.norm2 = norm_factory("norm2") if feed_forward is not None else None
+        if getattr(self.norm1, "kind", None) != "rms":
+            raise ConfigError("a norm with a token shift, or behind a scaled sum, is an RMS norm")
+        for part in (mixer, feed_forward):
+            if part is not None and not getattr(part, "stores_output", False) and getattr(type(part), "forward_apart", None) in (
+                    None, Mixer.forward_apart):
+                raise ConfigError(f"a sublayer whose output is scaled must be able to store it ({type(part).__name__} cannot)")
+        p = self.norm1.params
+        self.width, self.mult = int(p["size"]), float(p.get("residual_mult", 1.0))
+        self.shift, self.layer_scale = bool(p.get("token_shift", False)), bool(p.get("layer_scale", False))
+        self.share = None
+
+    def parts(self):
+        return [p for p in (self.norm1, self.mixer, self.norm2, self.feed_forward) if p is not None]
+
+    def _vectors(self):
+        scales = ["ls1"] + (["ls2"] if self.feed_forward is not None else []) if self.layer_scale else []
+        return (["shift"] if self.shift else []), scales
+
+    def tensors(self) -> List[TensorDecl]:
+        shift, scales = self._vectors()
+        return ([d for p in self.parts() for d in p.tensors()] + [TensorDecl(self.prefix + n, (self.width,), "bias") for n in shift]
+                + [TensorDecl(self.prefix + n, (self.width,), "gain") for n in scales])
+
+    def state_spec(self):
+        return StateSpec(2 * self.width) if self.shift else None
+
+    def load(self, store, rt) -> None:
+        for part in self.parts():
+            part.load(store, rt)
+        for norm in (self.norm1, self.norm2):
+            if norm is not None:
+                norm.gain = norm.gain.float().contiguous()
+        if self.shift:
+            self.share = store.vector(self.prefix + "shift").float().contiguous()
+
+        def scales_of(terms, name):
+            # what a term is multiplied by, column by column: its own gain and factor, the layer scale, m
+            ls = store.vector(self.prefix + name).float() if self.layer_scale else torch.ones(self.width, device=rt.device)
+            return [((ls * (t.factor * self.mult) if t.gain is None else t.gain.float() * ls * (t.factor * self.mult)).contiguous(), t.norm_eps)
+                    for t in terms]
+        self.mixer_terms = scales_of(self.mixer.output_terms(), "ls1")
+        self.ff_terms = scales_of([OutputTerm()], "ls2") if self.feed_forward is not None else None
+
+    def first_norm(self):
+        return self.norm1
+
+    def entry_norm(self, binding: CacheBinding):
+        return ShiftedNorm(self, binding.block_state) if self.shift else self.norm1
+
+    def last_part(self):
+        return self.feed_forward if self.feed_forward is not None else self.mixer
+
+    @staticmethod
+    def following_of(ctx, part, norm, n_rows: int):
+        """The norm behind a sum as work for the pass that makes the sum."""
+        if isinstance(norm, ShiftedNorm):
+            if not ctx.decode_only:
+                return None
+            return FollowingSum(norm.norm, norm.arguments(ctx), ctx.ws.take((n_rows, norm.norm.size), ctx.rt.dtype))
+        if getattr(norm, "kind", None) != "rms" or norm.gain is None or norm.gain.dtype != torch.float32:
+            return None
+        return FollowingSum(norm, None, ctx.ws.take((n_rows, norm.size), ctx.rt.dtype))
+
+    def _add(self, ctx, outs, terms, x, following) -> None:
+        ctx.rt.k.scaled_sum([(y, scales, eps) for y, (scales, eps) in zip(outs, terms)], x,
+                            norm=None if following is None else following.arguments(),
+                            shift=None if following is None else following.shift)
+
+    def forward(self, ctx, binding: CacheBinding, x, normed=None, following=None) -> None:
+        h = normed
+        if h is None and self.shift:
+            entry = self.entry_norm(binding)
+            h = ctx.rt.k.shifted_norm(x, self.norm1.gain, self.norm1.eps, *entry.arguments(ctx), ctx.ws.take(tuple(x.shape), ctx.rt.dtype))
+        elif h is None:
+            h = self.norm1.forward(ctx, x)
+        outs = [ctx.ws.take(tuple(x.shape), torch.float32) for _ in self.mixer_terms]
+        self.mixer.forward_apart(ctx, binding, h, outs)
+        if self.feed_forward is None:
+            self._add(ctx, outs, self.mixer_terms, x, following)
+            return
+        second = self.following_of(ctx, None, self.norm2, x.shape[0])
+        self._add(ctx, outs, self.mixer_terms, x, second)
+        self.feed_forward.forward(ctx, second.values, outs[0], accumulate=False)
+        self._add(ctx, outs[:1], self.ff_terms, x, following)
+
+
 register_block("prenorm", PreNormBlock)
+register_block("prenorm_scaled", ScaledPreNormBlock)
 register_block("sandwich_norm", SandwichNormBlock)
 register_block("parallel", ParallelBlock)
 register_block("prenorm_short_names", ShortNamedPreNormBlock)

@@ -7,16 +7,18 @@ are computed only at the rows asked for (src/model.rs:2647-2654).
 """
 from __future__ import annotations
 
-from typing import List
+from typing import List, Optional
 
 import torch
 
+from ..config.base import ConfigError
 from ..kernels import MODE_STORE_F32, PackedMatrix
-from .base import Part, TensorDecl, register_embedding, register_head
+from .base import Part, StateSpec, TensorDecl, register_embedding, register_head
 
 
 class TokenEmbedding(Part):
     graph_safe = True
+    state_index = -1             # the arena of `state_spec`, if there is one
     def __init__(self, params, prefix=""):
         super().__init__(params, prefix)
         self.vocab = int(params["vocab_size"])
@@ -27,6 +29,10 @@ class TokenEmbedding(Part):
 
     def tensors(self) -> List[TensorDecl]:
         return [TensorDecl(self.name, (self.vocab, self.hidden), "matrix")]
+
+    def state_spec(self) -> Optional[StateSpec]:
+        """What an embedding carries from token to token, if anything."""
+        return None
 
     def load(self, store, rt) -> None:
         self.table = store.matrix(self.name)
@@ -41,6 +47,38 @@ class TokenEmbedding(Part):
         if out is None:
             out = ctx.ws.take((ctx.n_tokens, self.hidden), torch.float32)
         return ctx.rt.k.embed(ctx.tokens, self.table, out, self.scale)
+
+
+class PairEmbedding(TokenEmbedding):
+    """A token's row times `scale`, plus the row (previous token * mul_prev + token * mul_cur) mod buckets of a table of
+    token pairs [buckets + 1, hidden]; a request's first token takes the table's last row.  The previous token is state: two
+    of them a request, the one behind position p in place p & 1.  Further parameters: `pairs` (tensor, buckets, mul_prev,
+    mul_cur)."""
+
+    def __init__(self, params, prefix=""):
+        super().__init__(params, prefix)
+        pairs = params["pairs"]
+        self.pairs_name, self.buckets = prefix + pairs["tensor"], int(pairs["buckets"])
+        self.mul_prev, self.mul_cur = int(pairs["mul_prev"]), int(pairs["mul_cur"])
+        if self.buckets < 1 or not (0 <= self.mul_prev < 1 << 31 and 0 <= self.mul_cur < 1 << 31):
+            raise ConfigError(f"token pairs in {self.buckets} buckets by {self.mul_prev} and {self.mul_cur}")
+        self.pairs = None
+
+    def tensors(self) -> List[TensorDecl]:
+        return super().tensors() + [TensorDecl(self.pairs_name, (self.buckets + 1, self.hidden))]
+
+    def state_spec(self) -> StateSpec:
+        return StateSpec(2, "int32")
+
+    def load(self, store, rt) -> None:
+        super().load(store, rt)
+        self.pairs = store.matrix(self.pairs_name)
+
+    def forward(self, ctx, out=None):
+        if out is None:
+            out = ctx.ws.take((ctx.n_tokens, self.hidden), torch.float32)
+        return ctx.rt.k.embed_pairs(ctx.tokens, self.table, self.scale, self.pairs, self.mul_prev, self.mul_cur,
+                                    ctx.cache.state(self.state_index), ctx.positions, ctx.seq_rows, out)
 
 
 class LMHead(Part):
@@ -90,4 +128,5 @@ class LMHead(Part):
 
 
 register_embedding("token_embedding", TokenEmbedding)
+register_embedding("pair_embedding", PairEmbedding)
 register_head("lm_head", LMHead)

@@ -12,7 +12,11 @@ i // (heads / kv_heads).  What a configuration may turn on, each on its own:
   rotation), so `vdim` = `dim`; "projected": v = Wv h (+ bv) of `vdim` a kv head;
 * `qk_norm`: q and k go through an RMS norm with a gain (`q.norm`, `k.norm`), before the rotation:
   per head over `dim` with a gain of `dim` shared by all heads (true, or "heads"), or over all rows
-  of q (of k) at once with a gain for every one of them ("rows");
+  of q (of k) at once with a gain for every one of them ("rows"); "plain": per head without a gain, which is the
+  same before the rotation and behind it (a rotation keeps a vector's length);
+* `conv` = taps: q, k and v first pass a causal convolution over time on every channel (no bias; `q.conv`, `k.conv`,
+  `v.conv`, the last column the current token's); a request's last taps - 1 projections are per-request state, twice: those
+  behind position p in copy p & 1, so that a decoding step reads one copy and writes the other;
 * `position`: a rotary encoding (its `pairing`, scaling and magnitude are the encoding's own);
 * `mask`: {"kind": "causal"}, {"kind": "window", "size": n, "keep": m} (position i sees 0 <= i - j < n,
   and every j <= i below `keep`, 0 unless given) or
@@ -38,7 +42,7 @@ into the residual stream.  With a window or chunks only the last `size` position
 so the cache manager may take back earlier pages.
 
 Parameters: `hidden_size`, `heads`, `kv_heads`, `dim`, `vdim`, `maps`, `diff`, `values`, `bias`,
-`out_bias`, `qk_norm`, `eps`, `scale`, `softcap`, `sink`, `q_temp`, `mask`, `gate`, `reads_cache`, `position` (a
+`out_bias`, `qk_norm`, `conv`, `eps`, `scale`, `softcap`, `sink`, `q_temp`, `mask`, `gate`, `reads_cache`, `position` (a
 PartSpec), `names`.
 `forward(..., accumulate=False)` stores the 32-bit output instead of adding it (for a part that combines
 several mixers' outputs itself).
@@ -51,7 +55,8 @@ import torch
 
 from ..config.base import ConfigError
 from ..kernels import MODE_ADD_F32, MODE_STORE_F32, PackedMatrix
-from .base import CacheBinding, CacheSpec, Mixer, TensorDecl, build_part, register_mixer
+from .base import CacheBinding, CacheSpec, Mixer, StateSpec, TensorDecl, build_part, register_mixer
+from .recurrent import step_spans
 
 TILE_TOKENS = 16        # tokens of one request a tile of the matrix-core kernel holds
 
@@ -105,8 +110,10 @@ class MaskedAttention(Mixer):
         self.sink_per_head = p.get("sink") == "heads"
         self.sink = None if p.get("sink") is None or self.sink_per_head else float(p["sink"])
         self.norm_rows = p.get("qk_norm") == "rows"
-        if p.get("qk_norm") not in (None, False, True, "heads", "rows"):
-            raise ConfigError(f"qk_norm {p.get('qk_norm')!r} is not known (heads, rows)")
+        if p.get("qk_norm") not in (None, False, True, "heads", "rows", "plain"):
+            raise ConfigError(f"qk_norm {p.get('qk_norm')!r} is not known (heads, rows, plain)")
+        self.norm_plain = p.get("qk_norm") == "plain"
+        self.taps = int(p.get("conv") or 0)
         self.out_bias, self.reads_cache = bool(p.get("out_bias", False)), bool(p.get("reads_cache", False))
         temp = p.get("q_temp")
         self.q_temp = None if not temp else (float(temp["coef"]), int(temp["every"]))
@@ -148,7 +155,12 @@ class MaskedAttention(Mixer):
             self.g_at = self.k_at
         self.g_width = 0 if not self.gate else self.heads if self.gate_per_head else self.o_width
         self.proj_width = self.g_at + self.g_width
+        if self.taps < 0 or (self.taps and (self.values == "keys" or self.reads_cache or self.norm_rows)):
+            raise ConfigError("a convolution before the attention wants queries, keys and values of its own, normed head by head or not at all")
+        self.channels = self.q_width + self.k_width + self.v_width           # what the convolution sees
+        self.copy_elems = -(-(self.taps - 1) * self.channels // 4) * 4 if self.taps else 0
         self.lam = 0.0
+        self.conv_w = None
         self.q_gain = self.k_gain = self.b_proj = self.b_o = self.sinks = None
 
     # ------------------------------------------------------------------ declarations
@@ -162,7 +174,9 @@ class MaskedAttention(Mixer):
         t = [TensorDecl(n[k], (rows[k], self.hidden)) for k in self._projections()]
         if self.bias:
             t += [TensorDecl(n[k] + ".b", (rows[k],), "bias") for k in self._projections() if k != "g"]
-        if self.qk_norm:
+        if self.taps:
+            t += [TensorDecl(n[k] + ".conv", (rows[k], self.taps)) for k in ("q", "k", "v")]
+        if self.qk_norm and not self.norm_plain:
             widths = {"q": self.q_width, "k": self.k_width}
             t += [TensorDecl(n[k] + ".norm", (widths[k] if self.norm_rows else self.dim,), "gain") for k in self._normed()]
         if self.sink_per_head:
@@ -181,14 +195,21 @@ class MaskedAttention(Mixer):
         return CacheSpec(entries=1, heads=1, head_dim=self.k_width + self.v_width,
                          window=self.mask_size if self.mask != "causal" else 0, keep=self.keep)
 
+    def state_spec(self) -> Optional[StateSpec]:
+        return StateSpec(2 * self.copy_elems) if self.taps > 1 else None
+
     def load(self, store, rt) -> None:
         n = self.n
         names = self._projections()
+        if self.taps:
+            self.conv_w = store.fused_matrix([n[k] + ".conv" for k in ("q", "k", "v")])
         self.w_proj = rt.k.prepare_weight(store.fused_matrix([n[k] for k in names]))
         if self.bias:
             parts = [store.vector(n[k] + ".b").float() if k != "g" else torch.zeros(self.g_width, device=rt.device) for k in names]
             self.b_proj = torch.cat(parts).contiguous()
-        if self.qk_norm:
+        if self.norm_plain:
+            self.q_gain = self.k_gain = torch.ones(self.dim, dtype=torch.float32, device=rt.device)
+        elif self.qk_norm:
             self.q_gain = store.vector(n["q"] + ".norm")
             self.k_gain = None if self.reads_cache else store.vector(n["k"] + ".norm")
         if self.sink_per_head:
@@ -229,9 +250,14 @@ class MaskedAttention(Mixer):
         else:
             table, neighbours, magnitude = ctx.no_rotation(), False, 1.0
         q = ctx.ws.take((T, self.q_width), ctx.rt.dtype)
+        conv = None
+        if self.taps:
+            state = ctx.cache.state(binding.state_index) if self.taps > 1 else ctx.no_state()
+            conv = (self.conv_w, state, self.copy_elems, step_spans(ctx))
         k.heads_prepare(proj, 0, self.n_q, self.k_at, self.n_k, self.v_at, self.v_width, self.dim, self.q_gain, self.k_gain,
                         self.eps, self.rot, neighbours, magnitude, table, ctx.positions, ctx.seq_rows, group.block_table, cache,
-                        group.page_size, q, binding.writes and not self.reads_cache, q_temp=self.q_temp, norm_rows=self.norm_rows)
+                        group.page_size, q, binding.writes and not self.reads_cache, q_temp=self.q_temp, norm_rows=self.norm_rows,
+                        conv=conv)
         att = ctx.ws.take((T, self.o_width), ctx.rt.dtype)
         tiles = None
         if k.masked_attention_uses_mfma(self.heads, self.kv_heads, self.maps, self.dim, self.vdim, group.page_size):

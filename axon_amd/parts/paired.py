@@ -1,14 +1,17 @@
-"""Two mixers side by side on the same input: out = mult (rms(left(h)) g_l + rms(right(h)) g_r).
+"""Two mixers side by side on the same input: the result is the sum of their outputs, each normed or scaled.
 
-Each side is a mixer of its own (a `PartSpec`), run on the same rows h; its 32-bit output is normed
-over the model width (an RMS norm with a plain gain and the layer's eps) and added into the residual
-stream times `mult` (a half: the mean of the two), the norm, the factor and the sum in one 32-bit pass a
-side.  One side may keep pages (a `CacheSpec`) and one may keep per-request state (a `StateSpec`): the
-run's binding serves both; two sides that both want pages, or both want state, are refused.
+Each side is a mixer of its own (a `PartSpec`), run on the same rows h.  `combine`:
 
-Parameters: `hidden_size`, `eps`, `left`, `right` (the sides' PartSpecs; their tensors lie under
-`<scope>left.` and `<scope>right.`), `mult` (default 0.5), `names` (scope "mix.", left_out "left.out",
-right_out "right.out": the gains of the two norms).
+* "normed": mult (rms(left(h)) g_l + rms(right(h)) g_r), an RMS norm over the model width with a plain gain and the
+  layer's eps a side, times `mult` (a half: the mean of the two);
+* "scaled": scales[0] left(h) + scales[1] right(h).
+
+Norm, factors and the sum into the residual stream are one 32-bit pass.  One side may keep pages (a `CacheSpec`); per-request
+state either side may have (the run's binding holds the left side's arenas, then the right side's).
+
+Parameters: `hidden_size`, `left`, `right` (the sides' PartSpecs; their tensors lie under
+`<scope>left.` and `<scope>right.`), `combine` (default "normed"), `eps` and `mult` (default 0.5) for "normed", `scales` for
+"scaled", `names` (scope "mix.", left_out "left.out", right_out "right.out": the gains of the two norms).
 """
 from __future__ import annotations
 
@@ -17,7 +20,7 @@ from typing import List, Optional
 import torch
 
 from ..config.base import ConfigError, PartSpec
-from .base import CacheBinding, CacheSpec, Mixer, StateSpec, TensorDecl, build_part, register_mixer
+from .base import CacheBinding, CacheSpec, Mixer, OutputTerm, StateSpec, TensorDecl, build_part, register_mixer
 
 
 class PairedMixers(Mixer):
@@ -25,7 +28,11 @@ class PairedMixers(Mixer):
     def __init__(self, params, prefix=""):
         super().__init__(params, prefix)
         p = params
-        self.hidden, self.eps, self.mult = int(p["hidden_size"]), float(p["eps"]), float(p.get("mult", 0.5))
+        self.hidden, self.eps, self.mult = int(p["hidden_size"]), float(p.get("eps", 0.0)), float(p.get("mult", 0.5))
+        self.combine = p.get("combine", "normed")
+        if self.combine not in ("normed", "scaled"):
+            raise ConfigError(f"a pair of mixers is not combined '{self.combine}' (normed, scaled)")
+        self.scales = [float(s) for s in p["scales"]] if self.combine == "scaled" else [1.0, 1.0]
         names = p.get("names", {})
         base = prefix + names.get("scope", "mix.")
         self.gain_names = [base + names.get("left_out", "left.out"), base + names.get("right_out", "right.out")]
@@ -34,8 +41,8 @@ class PairedMixers(Mixer):
         for side in self.sides:
             if not getattr(side, "stores_output", False):
                 raise ConfigError(f"a side of a pair of mixers must be able to store its output ({type(side).__name__} cannot)")
-        if sum(s.cache_spec() is not None for s in self.sides) > 1 or sum(s.state_spec() is not None for s in self.sides) > 1:
-            raise ConfigError("a pair of mixers shares one binding: one side may keep pages, one may keep state")
+        if sum(s.cache_spec() is not None for s in self.sides) > 1:
+            raise ConfigError("a pair of mixers shares one binding: one side may keep pages")
         self.graph_safe = all(getattr(s, "graph_safe", False) for s in self.sides)
         self.gains = [None, None]
 
@@ -50,8 +57,12 @@ class PairedMixers(Mixer):
     def cache_spec(self) -> Optional[CacheSpec]:
         return self._first("cache_spec")
 
+    def state_specs(self) -> List[StateSpec]:
+        return [spec for side in self.sides for spec in side.state_specs()]
+
     def state_spec(self) -> Optional[StateSpec]:
-        return self._first("state_spec")
+        specs = self.state_specs()
+        return specs[0] if specs else None
 
     def max_context(self) -> Optional[int]:
         limits = [m for m in (s.max_context() for s in self.sides) if m is not None]
@@ -71,18 +82,36 @@ class PairedMixers(Mixer):
 
     def tensors(self) -> List[TensorDecl]:
         t = [d for s in self.sides for d in s.tensors()]
-        return t + [TensorDecl(name, (self.hidden,), "gain") for name in self.gain_names]
+        return t + [TensorDecl(name, (self.hidden,), "gain") for name in self.gain_names] if self.combine == "normed" else t
 
     def load(self, store, rt) -> None:
         for s in self.sides:
             s.load(store, rt)
-        self.gains = [store.vector(name) for name in self.gain_names]
+        if self.combine == "normed":
+            self.gains = [store.vector(name) for name in self.gain_names]
+        else:
+            self.gains = [torch.full((self.hidden,), s, dtype=torch.float32, device=rt.device) for s in self.scales]
+
+    def output_terms(self) -> List[OutputTerm]:
+        if self.combine == "normed":
+            return [OutputTerm(gain, self.mult, self.eps) for gain in self.gains]
+        return [OutputTerm(None, s) for s in self.scales]
+
+    def forward_apart(self, ctx, binding: CacheBinding, h, outs) -> None:
+        at = 0
+        for side, out in zip(self.sides, outs):
+            n = len(side.state_specs())
+            side.forward(ctx, binding.with_states(at, n), h, out, accumulate=False)
+            at += n
 
     def forward(self, ctx, binding: CacheBinding, h, residual) -> None:
         k = ctx.rt.k
-        y = ctx.ws.take(tuple(residual.shape), torch.float32)
-        for side, gain in zip(self.sides, self.gains):
-            side.forward(ctx, binding, h, y, accumulate=False)
+        outs = [ctx.ws.take(tuple(residual.shape), torch.float32) for _ in self.sides]
+        self.forward_apart(ctx, binding, h, outs)
+        if self.combine == "scaled":
+            k.scaled_sum([(y, gain, None) for y, gain in zip(outs, self.gains)], residual)
+            return
+        for y, gain in zip(outs, self.gains):
             k.norm_add(y, gain, self.eps, self.mult, residual)
 
 
