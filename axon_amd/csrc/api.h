@@ -383,7 +383,7 @@ int axk_delta_scan(const float* u, const float* terms, const float* decay, float
 // work: axk_delta_chunked_workspace floats.
 int axk_delta_chunked_ok(int kv_heads, int heads, int N, int P);
 long axk_delta_chunked_workspace(int n_chunks, int heads, int N, int P);
-int axk_delta_chunked(const float* u, const float* terms, float* state, long state_stride, long copy_elems, long tail_at,
+int axk_delta_chunked(const float* u, const float* terms, const float* decay, float* state, long state_stride, long copy_elems, long tail_at,
                       const int32_t* chunks, int n_chunks, const int32_t* spans5, int n_spans, const int32_t* positions,
                       const float* conv_in, long conv_in_stride, float* y, int heads, int kv_heads, int N, int P, int taps,
                       float* work, long work_floats, void* stream);

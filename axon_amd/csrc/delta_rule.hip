@@ -292,18 +292,177 @@ delta_chunk_terms_kernel(const float* __restrict__ u, const float* __restrict__ 
   }
 }
 
+// The same with a decay a key channel: D_ij and b_i are vectors over the channels, (k_i . k_j) and (q_i . k_j) become sums of
+// k_in D_ijn k_jn.  Such a sum is a product of two rows once D_ij is cut at a place x between the tokens: (the decays of
+// x .. i) times (those of j + 1 .. x - 1), both products of factors up to 1, so nothing overflows and nothing is divided.
+// Two tokens are cut where their numbers first differ: with s the highest bit in which i and j differ, x is the start of i's
+// run of s tokens, and a token's factor at level s is the product from its run's start to itself where bit s is set in its
+// number (`pre`), else from behind itself to its run's end (`suf`).  So each level is one scaling of the rows and one
+// product, of which the pairs that belong to the level are taken: levels 1 to 8 inside a wave's sixteen tokens, 16 and 32
+// between waves.  Level by level pre and suf double their reach by the neighbouring run's whole product.
+// Of a (chunk, head) q holds diag(b_i) q_i and b the last token's b [N].
+template <int NT>
+__global__ void __launch_bounds__(256)
+delta_chunk_channel_terms_kernel(const float* __restrict__ u, const float* __restrict__ terms, const float* __restrict__ decay,
+                                 const int32_t* __restrict__ chunks, int heads, int kv_heads, int P, float* __restrict__ up,
+                                 float* __restrict__ w, float* __restrict__ kt, float* __restrict__ m, float* __restrict__ q,
+                                 float* __restrict__ b) {
+  constexpr int N = 16 * NT, ROW = DC + 4, KROW = N + 4;
+  __shared__ __align__(16) float Kl[DC][KROW];        // rows 0 .. 31: level 16 of waves 0 and 2; 32 .. 63: level 32 of waves 0 and 1
+  __shared__ __align__(16) float A[DC][ROW];
+  __shared__ __align__(16) float tot[4][N];
+  __shared__ float betas[DC];
+  const int h = blockIdx.x, kh = h / (heads / kv_heads), first = chunks[2 * blockIdx.y], count = chunks[2 * blockIdx.y + 1];
+  const long item = (long)blockIdx.y * heads + h;
+  const int channels = 2 * kv_heads * N + heads * P;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 15, g4 = lane >> 4, row = 16 * wave + r;
+  if (tid < DC) betas[tid] = tid < count ? terms[((long)(first + tid) * heads + h) * 2 + 1] : 0.0f;
+  const long t = first + min(row, count - 1);
+  const float* mine = u + t * channels + (long)kh * N + 4 * g4;
+  const float* mine_g = decay + (t * heads + h) * N + 4 * g4;
+  dc_f32x4 qf[NT], kf[NT], pre[NT], suf[NT];
+  float own = 0.0f;                                   // q_i . k_i, nothing decayed
+#pragma unroll
+  for (int c = 0; c < NT; ++c) {
+    qf[c] = dc_load(mine + 16 * c);
+    kf[c] = dc_load(mine + (long)kv_heads * N + 16 * c);
+    pre[c] = row < count ? dc_load(mine_g + 16 * c) : dc_f32x4{1.0f, 1.0f, 1.0f, 1.0f};
+    suf[c] = dc_f32x4{1.0f, 1.0f, 1.0f, 1.0f};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) own = fmaf(qf[c][j], kf[c][j], own);
+  }
+  own += __shfl_xor(own, 16, 64);
+  own += __shfl_xor(own, 32, 64);
+  dc_f32x4 kk = {0.0f, 0.0f, 0.0f, 0.0f}, qk = kk;
+#pragma unroll
+  for (int s = 1; s < 16; s <<= 1) {
+    const bool high = (r & s) != 0;
+    dc_f32x4 ks = {0.0f, 0.0f, 0.0f, 0.0f}, qs = ks;
+#pragma unroll
+    for (int c = 0; c < NT; ++c) {
+      const dc_f32x4 f = high ? pre[c] : suf[c], kd = kf[c] * f, qd = qf[c] * f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { DC_MFMA(ks, kd, kd, j); DC_MFMA(qs, qd, kd, j); }
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = 4 * g4 + e, x = i ^ r;            // row i, column r
+      if ((i & s) != 0 && (x & s) != 0 && x < 2 * s) { kk[e] = ks[e]; qk[e] = qs[e]; }
+    }
+    const int from = (lane & 48) | ((r ^ s) | (s - 1));        // the last token of the neighbouring run
+#pragma unroll
+    for (int c = 0; c < NT; ++c)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float whole = __shfl(pre[c][j], from, 64);
+        pre[c][j] *= high ? whole : 1.0f;
+        suf[c][j] *= high ? 1.0f : whole;
+      }
+  }
+  // pre and suf now reach over the wave's tokens
+  if (r == 15) {
+#pragma unroll
+    for (int c = 0; c < NT; ++c) *reinterpret_cast<dc_f32x4*>(&tot[wave][16 * c + 4 * g4]) = pre[c];
+  }
+  if ((wave & 1) == 0) {
+#pragma unroll
+    for (int c = 0; c < NT; ++c) *reinterpret_cast<dc_f32x4*>(&Kl[8 * wave + r][16 * c + 4 * g4]) = kf[c] * suf[c];
+  }
+  __syncthreads();
+  auto tile = [&](int jt, dc_f32x4 kd, dc_f32x4 qd) {          // rows of this wave, columns 16 jt ..
+    const int j = 16 * jt + r;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = 16 * wave + 4 * g4 + e;
+      A[i][j] = j < i ? betas[i] * kd[e] : 0.0f;
+      m[item * DC * DC + dc_at(i, j, DC / 16)] = j < i ? qd[e] : j == i ? own : 0.0f;
+    }
+  };
+  auto product = [&](int jt, const float (*rows)[KROW]) {      // rows: the columns' tokens, scaled; pre: this wave's factors
+    dc_f32x4 ks = {0.0f, 0.0f, 0.0f, 0.0f}, qs = ks;
+#pragma unroll
+    for (int c = 0; c < NT; ++c) {
+      const dc_f32x4 o = dc_load(&rows[r][16 * c + 4 * g4]), kd = kf[c] * pre[c], qd = qf[c] * pre[c];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) { DC_MFMA(ks, kd, o, j); DC_MFMA(qs, qd, o, j); }
+    }
+    tile(jt, ks, qs);
+  };
+  tile(wave, kk, qk);
+  if (wave & 1) product(wave - 1, &Kl[8 * (wave - 1)]);
+#pragma unroll
+  for (int c = 0; c < NT; ++c) {
+    const dc_f32x4 whole = dc_load(&tot[wave ^ 1][16 * c + 4 * g4]);
+    if (wave & 1) pre[c] *= whole; else suf[c] *= whole;
+    if (wave < 2) *reinterpret_cast<dc_f32x4*>(&Kl[32 + row][16 * c + 4 * g4]) = kf[c] * suf[c];
+  }
+  __syncthreads();
+  if (wave & 2) {
+    product(0, &Kl[32]);
+    product(1, &Kl[48]);
+  }
+#pragma unroll
+  for (int c = 0; c < NT; ++c) {
+    const int other = wave & 2 ? 0 : 2;
+    const dc_f32x4 whole = dc_load(&tot[other][16 * c + 4 * g4]) * dc_load(&tot[other + 1][16 * c + 4 * g4]);
+    if (wave & 2) pre[c] *= whole; else suf[c] *= whole;
+  }
+  __syncthreads();                                   // the scaled rows have been read
+  // now over the whole chunk: q and the last decays as the walk wants them, the keys transposed, and the right-hand side
+#pragma unroll
+  for (int c = 0; c < NT; ++c) {
+    *reinterpret_cast<dc_f32x4*>(q + item * DC * N + ((wave * NT + c) * 64 + lane) * 4) = qf[c] * pre[c];
+    *reinterpret_cast<dc_f32x4*>(&Kl[row][16 * c + 4 * g4]) = (kf[c] * pre[c]) * betas[row];
+    if (row == DC - 1) *reinterpret_cast<dc_f32x4*>(b + item * N + 16 * c + 4 * g4) = pre[c];
+    const dc_f32x4 kd = kf[c] * suf[c];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) kt[item * N * DC + dc_at(16 * c + 4 * g4 + j, row, DC / 16)] = kd[j];
+  }
+  __syncthreads();
+  const int cols = P + N;
+  for (int col = tid; col < cols; col += 256) {
+    float X[DC];
+    const bool is_v = col < P;
+    const float* src = u + 2L * kv_heads * N + (long)h * P + (is_v ? col : 0);
+#pragma unroll
+    for (int i = 0; i < DC; ++i) X[i] = is_v ? src[(long)(first + min(i, count - 1)) * channels] * betas[i] : Kl[i][is_v ? 0 : col - P];
+#pragma unroll
+    for (int i = 1; i < DC; ++i) {
+      float x = X[i];
+#pragma unroll
+      for (int j = 0; j < i; j += 4) {
+        const dc_f32x4 a = dc_load(&A[i][j]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (j + e < i) x = fmaf(-a[e], X[j + e], x);
+      }
+      X[i] = x;
+      __builtin_amdgcn_sched_barrier(0);       // a row of A at a time in registers
+    }
+    if (is_v) {
+      float* dst = up + item * DC * P + col;
+#pragma unroll
+      for (int i = 0; i < DC; ++i) dst[(long)i * P] = X[i];
+    } else {
+      float* dst = w + item * DC * N;
+#pragma unroll
+      for (int i = 0; i < DC; ++i) dst[dc_at(i, col - P, NT)] = X[i];
+    }
+  }
+}
+
 // grid (heads, P / 16, requests), four waves: a wave the sixteen tokens 16 wave .. of a chunk, and of the state the tiles
 // of sixteen rows wave, wave + 4 in its accumulators.  The state's slice and U travel between the waves through LDS, value
 // dim by value dim.  A chunk's operands are asked for while the chunk before is worked on.  spans5 [n][5] = (slot, first
-// token, tokens, first chunk, chunks).
+// token, tokens, first chunk, chunks).  CHANNEL: a decay a key channel (see the kernel above).
 template <int NT>
 struct DeltaChunkOperands {
   static constexpr int TILES = (NT + 3) / 4;
-  dc_f32x4 w[NT], q[NT], m[4], k[TILES][4];
+  dc_f32x4 w[NT], q[NT], m[4], k[TILES][4], b_rows[TILES];
   float up[4], b[4], b_last;
 };
 
-template <int NT>
+template <int NT, bool CHANNEL>
 __global__ void __launch_bounds__(256)
 delta_chunk_walk_kernel(const float* __restrict__ q, const float* __restrict__ up, const float* __restrict__ w,
                         const float* __restrict__ kt, const float* __restrict__ m, const float* __restrict__ b,
@@ -335,7 +494,7 @@ delta_chunk_walk_kernel(const float* __restrict__ q, const float* __restrict__ u
   auto fetch = [&](Ops& o, int c) {
     const long item = (long)(chunk0 + c) * heads + h;
     const float* wr = w + item * DC * N + (wave * NT * 64 + lane) * 4;
-    const float* qr = q + ((long)(chunk0 + c) * kv_heads + kh) * DC * N + (wave * NT * 64 + lane) * 4;
+    const float* qr = q + (CHANNEL ? item : (long)(chunk0 + c) * kv_heads + kh) * DC * N + (wave * NT * 64 + lane) * 4;
 #pragma unroll
     for (int i = 0; i < NT; ++i) { o.w[i] = dc_load(wr + 256 * i); o.q[i] = dc_load(qr + 256 * i); }
     const float* mr = m + item * DC * DC + (wave * 4 * 64 + lane) * 4;
@@ -348,13 +507,14 @@ delta_chunk_walk_kernel(const float* __restrict__ q, const float* __restrict__ u
         const float* kr = kt + item * N * DC + ((wave + 4 * tt) * 4 * 64 + lane) * 4;
 #pragma unroll
         for (int i = 0; i < 4; ++i) o.k[tt][i] = dc_load(kr + 256 * i);
+        if (CHANNEL) o.b_rows[tt] = dc_load(b + item * N + 16 * (wave + 4 * tt) + 4 * g4);
       }
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       o.up[e] = up[(item * DC + 16 * wave + 4 * g4 + e) * P + p0 + r];
-      o.b[e] = b[item * DC + 16 * wave + 4 * g4 + e];
+      if (!CHANNEL) o.b[e] = b[item * DC + 16 * wave + 4 * g4 + e];
     }
-    o.b_last = b[item * DC + DC - 1];
+    if (!CHANNEL) o.b_last = b[item * DC + DC - 1];
   };
   auto work = [&](const Ops& o, int c) {
     // two halves of the sum over the state's rows, two products: four chains
@@ -373,7 +533,10 @@ delta_chunk_walk_kernel(const float* __restrict__ q, const float* __restrict__ u
       }
     dc_f32x4 mine, out;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) { mine[e] = o.up[e] - (ws[0][e] + ws[1][e]); out[e] = (qs[0][e] + qs[1][e]) * o.b[e]; }
+    for (int e = 0; e < 4; ++e) {
+      mine[e] = o.up[e] - (ws[0][e] + ws[1][e]);
+      out[e] = (qs[0][e] + qs[1][e]) * (CHANNEL ? 1.0f : o.b[e]);
+    }
     *reinterpret_cast<dc_f32x4*>(&Ul[r][16 * wave + 4 * g4]) = mine;
     __syncthreads();                       // every wave's part of U is there, and every wave has read the state
     dc_f32x4 all[4];
@@ -382,7 +545,7 @@ delta_chunk_walk_kernel(const float* __restrict__ q, const float* __restrict__ u
 #pragma unroll
     for (int tt = 0; tt < TILES; ++tt)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) S[tt][e] *= o.b_last;
+      for (int e = 0; e < 4; ++e) S[tt][e] *= CHANNEL ? o.b_rows[tt][e] : o.b_last;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
@@ -658,10 +821,10 @@ extern "C" int axk_delta_chunked_ok(int kv_heads, int heads, int N, int P) {
 
 // The floats of workspace that axk_delta_chunked wants for this many chunks.
 extern "C" long axk_delta_chunked_workspace(int n_chunks, int heads, int N, int P) {
-  return (long)n_chunks * heads * DC * (3L * N + P + DC + 1);
+  return (long)n_chunks * heads * (DC * (3L * N + P + DC) + (N > DC ? N : DC));
 }
 
-extern "C" int axk_delta_chunked(const float* u, const float* terms, float* state, long state_stride, long copy_elems, long tail_at,
+extern "C" int axk_delta_chunked(const float* u, const float* terms, const float* decay, float* state, long state_stride, long copy_elems, long tail_at,
                                  const int32_t* chunks, int n_chunks, const int32_t* spans5, int n_spans, const int32_t* positions,
                                  const float* conv_in, long conv_in_stride, float* y, int heads, int kv_heads, int N, int P, int taps,
                                  float* work, long work_floats, void* stream) {
@@ -673,7 +836,7 @@ extern "C" int axk_delta_chunked(const float* u, const float* terms, float* stat
               "delta_chunked: a state row of %ld floats does not hold two copies of %ld (%d x %d x %d, then %d x %ld from %ld)",
               state_stride, copy_elems, heads, N, P, taps - 1, channels, tail_at);
   AXK_REQUIRE(copy_elems % 4 == 0 && state_stride % 4 == 0 && ((uintptr_t)u & 15) == 0 && ((uintptr_t)state & 15) == 0 &&
-              ((uintptr_t)work & 15) == 0, "delta_chunked: rows are not 16-byte aligned");
+              ((uintptr_t)work & 15) == 0 && ((uintptr_t)decay & 15) == 0, "delta_chunked: rows are not 16-byte aligned");
   AXK_REQUIRE(n_chunks >= n_spans && n_chunks <= 65535 && n_spans <= 65535, "delta_chunked: %d chunks of %d requests", n_chunks, n_spans);
   AXK_REQUIRE(work != nullptr && work_floats >= axk_delta_chunked_workspace(n_chunks, heads, N, P), "delta_chunked: a workspace of %ld floats",
               work_floats);
@@ -684,17 +847,23 @@ extern "C" int axk_delta_chunked(const float* u, const float* terms, float* stat
   float* kt = w + items * DC * N;
   float* m = kt + items * DC * N;
   float* q = m + items * DC * DC;
-  float* b = q + (long)n_chunks * kv_heads * DC * N;
+  float* b = q + (decay ? items : (long)n_chunks * kv_heads) * DC * N;
   hipStream_t s = (hipStream_t)stream;
+#define DC_WALK(NT, CHANNEL)                                                                                                    \
+  delta_chunk_walk_kernel<NT, CHANNEL><<<dim3(heads, P / 16, n_spans), 256, 0, s>>>(                                            \
+      q, up, w, kt, m, b, spans5, positions, state, state_stride, copy_elems, tail_at, conv_in, conv_in_stride, y, heads, kv_heads, P, taps)
 #define DC_LAUNCH(NT)                                                                                                            \
-  {                                                                                                                              \
+  if (decay == nullptr) {                                                                                                        \
     delta_chunk_terms_kernel<NT><<<dim3(heads, n_chunks), 256, 0, s>>>(u, terms, chunks, heads, kv_heads, P, up, w, kt, m, q, b);\
-    delta_chunk_walk_kernel<NT><<<dim3(heads, P / 16, n_spans), 256, 0, s>>>(q, up, w, kt, m, b, spans5, positions, state,       \
-                                                                            state_stride, copy_elems, tail_at, conv_in,          \
-                                                                            conv_in_stride, y, heads, kv_heads, P, taps);        \
+    DC_WALK(NT, false);                                                                                                          \
+  } else {                                                                                                                       \
+    delta_chunk_channel_terms_kernel<NT><<<dim3(heads, n_chunks), 256, 0, s>>>(u, terms, decay, chunks, heads, kv_heads, P, up, w, kt, m, \
+                                                                              q, b);                                             \
+    DC_WALK(NT, true);                                                                                                           \
   }
-  if (N == 32) DC_LAUNCH(2) else if (N == 64) DC_LAUNCH(4) else if (N == 96) DC_LAUNCH(6) else DC_LAUNCH(8)
+  if (N == 32) { DC_LAUNCH(2) } else if (N == 64) { DC_LAUNCH(4) } else if (N == 96) { DC_LAUNCH(6) } else { DC_LAUNCH(8) }
 #undef DC_LAUNCH
+#undef DC_WALK
   AXK_LAUNCH_CHECK("delta_chunked");
   return 0;
 }

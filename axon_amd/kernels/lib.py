@@ -112,7 +112,7 @@ _SIGNATURES = {
     "axk_delta_scan": [c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_long,
                        c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "axk_delta_chunked_ok": [c_int, c_int, c_int, c_int],
-    "axk_delta_chunked": [c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p,
+    "axk_delta_chunked": [c_void_p, c_void_p, c_void_p, c_void_p, c_long, c_long, c_long, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p,
                           c_long, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p, c_long, c_void_p],
     "axk_delta_low_rank": [c_void_p, c_long, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_int,
                            c_void_p, c_void_p, c_int, c_int, c_void_p],
@@ -1224,7 +1224,7 @@ class Kernels:
             need = int(self.lib.axk_delta_chunked_workspace(list_.shape[0], heads, keys, values))
             work = torch.empty(need, dtype=torch.float32, device=y.device)
             self._check(self.lib.axk_delta_chunked(
-                _ptr(u), _ptr(terms), _ptr(state), state.stride(0), int(copy_elems), int(tail_at), _ptr(list_), list_.shape[0], _ptr(spans5),
+                _ptr(u), _ptr(terms), _ptr(decay), _ptr(state), state.stride(0), int(copy_elems), int(tail_at), _ptr(list_), list_.shape[0], _ptr(spans5),
                 spans5.shape[0], _ptr(positions), _ptr(conv_in), conv_in.stride(0), _ptr(y), heads, kv_heads, keys, values, int(taps),
                 _ptr(work), need, _stream()))
             if n == 0:

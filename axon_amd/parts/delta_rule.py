@@ -132,7 +132,7 @@ class GatedDeltaRule(Mixer):
             k.delta_low_rank(rows, decay=(self.decay_at, self.w_decay, self.dt_bias, self.a_log, decay) if self.decay_rank else None,
                              gate=(self.gate_at, self.w_gate, gate) if self.gate_rank else None)
         y = ctx.ws.take((T, self.inner), f32)
-        long = step_chunks(ctx) if decay is None and k.delta_chunked_ok(self.kv_heads, self.heads, self.dim, self.vdim) else None
+        long = step_chunks(ctx) if k.delta_chunked_ok(self.kv_heads, self.heads, self.dim, self.vdim) else None
         chunks, spans = long if long is not None else (None, step_spans(ctx))
         k.delta_scan(u, terms, state, self.copy_elems, self.tail_at, spans, ctx.positions, ctx.seq_rows, rows, y, self.heads,
                      self.kv_heads, self.dim, self.vdim, self.taps, chunks=chunks, decay=decay)
