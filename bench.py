@@ -186,6 +186,28 @@ def _lilunex_sizes(width, heads, kv_heads, wkv_heads, delta_heads, window, exper
                        {"type": "attention", "mixer": dict(mixer, kv_from=1), "mlp": dense}]}
 
 
+# --design bafavik: four layer runs: a pair of mixers run twice over (attention behind short convolutions with values of twice
+# the keys' size beside the delta rule with a decay a key channel), a pair of attention with queries and keys of unit size beside
+# linear attention with a constant decay a head, and differential attention in chunks; every layer with a dense feed-forward (1.5
+# times the gated one's width).  Beside it the closest designs the engine has, Lilunex (the delta rule, a decayed state, windowed
+# attention) and Zugutar (a pair of attention and a state-space scan), and the dense decoder of equal width.
+def _bafavik_sizes(width, heads, kv_heads, state_heads, chunk, dense_ff):
+    att = lambda h, kv, dim, vdim, **more: {"heads": h, "kv_heads": kv, "dim": dim, "vdim": vdim, "scale": dim ** -0.5, **more}
+    rot = {"base": 10000.0, "dims": 64}
+    mlp = {"kind": "dense", "ff": dense_ff * 3 // 2}
+    decay = [1.0 - 2.0 ** -(4 + 6 * i / state_heads) for i in range(state_heads)]
+    pair_2 = {"type": "parallel_2", "mixer": {
+        "left": att(heads // 2, kv_heads, 128, 256, conv=4, rot=rot),
+        "right": {"heads": state_heads, "kv_heads": state_heads, "dim": 128, "vdim": 128, "conv": 4}}}
+    pair = {"type": "parallel", "mixer": {
+        "left": att(heads, kv_heads, 128, 128, rot=rot), "right": {"heads": state_heads, "dim": 128, "vdim": 128, "decay": decay},
+        "left_scale": 0.7, "right_scale": 0.7}}
+    diff = {"type": "attention", "mixer": att(heads // 2, max(kv_heads // 2, 1), 64, 128, diff=0.3, mask={"size": chunk})}
+    return {"architecture": "Bafavik", "embedding": {"scale": 1.0, "bigram": {"buckets": 32003, "mul_prev": 8191, "mul_cur": 127}},
+            "layers": [dict(pair_2, mlp=mlp), dict(pair, mlp=mlp), dict(diff, mlp=mlp)], "loop": {"start": 0, "stop": 1, "times": 2},
+            "residual_mult": 0.5, "logit_scale": 1.0, "norm": {"eps": 1e-6}, "vocab": 32000, "width": width}
+
+
 # design -> size -> the models measured side by side, the design's own first
 DESIGN_SIZES = {
     "pikesun": {
@@ -208,6 +230,13 @@ DESIGN_SIZES = {
         "2048": [("lilunex", _lilunex_sizes(2048, 16, 2, 32, 32, 1024, 32, 8, 4, 704, 1408, 5632)),
                  ("zugutar", _zugutar_sizes(2048, 16, 2, 32, 2, 32, 4, 704, 1408)), ("qwen2", _qwen_sizes(2048, 16, 2, 5632))],
         "4096": [("lilunex", _lilunex_sizes(4096, 32, 8, 64, 64, 2048, 64, 16, 6, 1408, 2816, 11008)),
+                 ("zugutar", _zugutar_sizes(4096, 32, 8, 64, 8, 64, 6, 1408, 2816)), ("qwen2", _qwen_sizes(4096, 32, 8, 11008))]},
+    "bafavik": {
+        "2048": [("bafavik", _bafavik_sizes(2048, 16, 2, 16, 1536, 5632)),
+                 ("lilunex", _lilunex_sizes(2048, 16, 2, 32, 32, 1024, 32, 8, 4, 704, 1408, 5632)),
+                 ("zugutar", _zugutar_sizes(2048, 16, 2, 32, 2, 32, 4, 704, 1408)), ("qwen2", _qwen_sizes(2048, 16, 2, 5632))],
+        "4096": [("bafavik", _bafavik_sizes(4096, 32, 8, 32, 8192, 11008)),
+                 ("lilunex", _lilunex_sizes(4096, 32, 8, 64, 64, 2048, 64, 16, 6, 1408, 2816, 11008)),
                  ("zugutar", _zugutar_sizes(4096, 32, 8, 64, 8, 64, 6, 1408, 2816)), ("qwen2", _qwen_sizes(4096, 32, 8, 11008))]},
 }
 
