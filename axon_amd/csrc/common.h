@@ -224,7 +224,14 @@ void axk_set_error(const char* fmt, ...);
 static inline int ceil_div(int a, int b) { return (a + b - 1) / b; }
 
 // Epilogues of a matrix product (see axk_gemm).
-enum { MODE_STORE = 0, MODE_ADD_F32 = 1, MODE_STORE_F32 = 2, MODE_SWIGLU = 3 };
+enum { MODE_STORE = 0, MODE_ADD_F32 = 1, MODE_STORE_F32 = 2, MODE_SWIGLU = 3, MODE_RELU_SQUARED = 4 };
+
+// What MODE_STORE and MODE_RELU_SQUARED store of a finished sum (in the compute dtype).
+__host__ __device__ inline bool mode_stores_elem(int mode) { return mode == MODE_STORE || mode == MODE_RELU_SQUARED; }
+__device__ inline float mode_value(float v, int mode) {
+  const float r = fmaxf(v, 0.0f);
+  return mode == MODE_RELU_SQUARED ? r * r : v;
+}
 
 // act = (g / (1 + exp(-g))) * u: divide, then multiply (src/vmath.rs:128-132;
 // src/cuda/prefill.cu:109-123).

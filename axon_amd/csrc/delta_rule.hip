@@ -301,8 +301,20 @@ delta_chunk_terms_kernel(const float* __restrict__ u, const float* __restrict__ 
 // product, of which the pairs that belong to the level are taken: levels 1 to 8 inside a wave's sixteen tokens, 16 and 32
 // between waves.  Level by level pre and suf double their reach by the neighbouring run's whole product.
 // Of a (chunk, head) q holds diag(b_i) q_i and b the last token's b [N].
+// Of sixteen lanes in runs of s: the value that the neighbouring run's last lane holds, by lane permutations.
+__device__ inline float dc_neighbour_run(float v, int s, bool second_quad) {
+#define DC_DPP(val, ctrl) __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, val), ctrl, 0xf, 0xf, false))
+  if (s == 1) return DC_DPP(v, 0xb1);                        // quad_perm [1, 0, 3, 2]
+  if (s == 2) return DC_DPP(v, 0x5f);                        // quad_perm [3, 3, 1, 1]
+  const float last = DC_DPP(v, 0xff);                        // of a lane's own four: quad_perm [3, 3, 3, 3]
+  const float other = DC_DPP(last, 0x141);                   // of the other four of its eight: row_half_mirror
+  if (s == 4) return other;
+  return DC_DPP(second_quad ? last : other, 0x140);          // of the other eight: row_mirror
+#undef DC_DPP
+}
+
 template <int NT>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, 2)        // two waves a SIMD: 256 registers each
 delta_chunk_channel_terms_kernel(const float* __restrict__ u, const float* __restrict__ terms, const float* __restrict__ decay,
                                  const int32_t* __restrict__ chunks, int heads, int kv_heads, int P, float* __restrict__ up,
                                  float* __restrict__ w, float* __restrict__ kt, float* __restrict__ m, float* __restrict__ q,
@@ -349,12 +361,11 @@ delta_chunk_channel_terms_kernel(const float* __restrict__ u, const float* __res
       const int i = 4 * g4 + e, x = i ^ r;            // row i, column r
       if ((i & s) != 0 && (x & s) != 0 && x < 2 * s) { kk[e] = ks[e]; qk[e] = qs[e]; }
     }
-    const int from = (lane & 48) | ((r ^ s) | (s - 1));        // the last token of the neighbouring run
 #pragma unroll
     for (int c = 0; c < NT; ++c)
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        const float whole = __shfl(pre[c][j], from, 64);
+        const float whole = dc_neighbour_run(pre[c][j], s, (r & 4) != 0);
         pre[c][j] *= high ? whole : 1.0f;
         suf[c][j] *= high ? 1.0f : whole;
       }
@@ -647,7 +658,9 @@ head_norm_gate_vec_kernel(const float* __restrict__ y, const float* __restrict__
 #endif
 }
 
-// The same for heads of many values (all channels of a row normed together, say): a block a (token, head).
+// The same for heads of many values (all channels of a row normed together, say): a block a (token, head), G values a thread
+// at a time, the first HN_KEPT of these and their gates kept in registers.
+template <int G>
 __global__ void __launch_bounds__(256)
 head_norm_gate_wide_kernel(const float* __restrict__ y, const float* __restrict__ gate, long gate_stride, const void* __restrict__ gain,
                            int gain_is_f32, int gain_per_head, float eps, elem_t* __restrict__ out, int heads, int P, int act) {
@@ -657,22 +670,53 @@ head_norm_gate_wide_kernel(const float* __restrict__ y, const float* __restrict_
   const float* src = y + item * P;
   const float* g = gate + item / heads * gate_stride + (long)h * P;
   elem_t* dst = out + item * P;
-  float kept[HN_KEPT], ss = 0.0f;
+  auto load = [&](const float* p, float (&v)[G]) {
+    if (G == 4) {
+      const float4 q = *reinterpret_cast<const float4*>(p);
+      v[0] = q.x; v[1 % G] = q.y; v[2 % G] = q.z; v[3 % G] = q.w;
+    } else {
+      v[0] = p[0];
+    }
+  };
+  float kept[HN_KEPT][G], gates[HN_KEPT][G], ss = 0.0f;
 #pragma unroll
   for (int j = 0; j < HN_KEPT; ++j) {
-    const int i = threadIdx.x + 256 * j;
-    kept[j] = i < P ? src[i] : 0.0f;
-    ss = fmaf(kept[j], kept[j], ss);
+    const int i = G * (threadIdx.x + 256 * j);
+    if (i >= P) break;
+    load(src + i, kept[j]);
+    load(g + i, gates[j]);
+#pragma unroll
+    for (int e = 0; e < G; ++e) ss = fmaf(kept[j][e], kept[j][e], ss);
   }
-  for (int i = threadIdx.x + 256 * HN_KEPT; i < P; i += 256) ss = fmaf(src[i], src[i], ss);
+  for (int i = G * (threadIdx.x + 256 * HN_KEPT); i < P; i += G * 256) {
+    float v[G];
+    load(src + i, v);
+#pragma unroll
+    for (int e = 0; e < G; ++e) ss = fmaf(v[e], v[e], ss);
+  }
   const float inv = 1.0f / sqrtf(block_sum_256(ss, partial) / (float)P + eps);
+  auto store = [&](int i, const float (&v)[G], const float (&z)[G]) {
+    float o[G];
+#pragma unroll
+    for (int e = 0; e < G; ++e) o[e] = ((v[e] * inv) * load_vec(gain, gain_is_f32, gain_at + i + e)) * gate_act(z[e], act);
+#if AXON_BF16
+    if (G == 4) *reinterpret_cast<uint2*>(dst + i) = make_uint2(pack2_bf16(o[0], o[1 % G]), pack2_bf16(o[2 % G], o[3 % G]));
+#else
+    if (G == 4) *reinterpret_cast<float4*>(dst + i) = make_float4(o[0], o[1 % G], o[2 % G], o[3 % G]);
+#endif
+    else dst[i] = from_float(o[0]);
+  };
 #pragma unroll
   for (int j = 0; j < HN_KEPT; ++j) {
-    const int i = threadIdx.x + 256 * j;
-    if (i < P) dst[i] = from_float(((kept[j] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * gate_act(g[i], act));
+    const int i = G * (threadIdx.x + 256 * j);
+    if (i < P) store(i, kept[j], gates[j]);
   }
-  for (int i = threadIdx.x + 256 * HN_KEPT; i < P; i += 256)
-    dst[i] = from_float(((src[i] * inv) * load_vec(gain, gain_is_f32, gain_at + i)) * gate_act(g[i], act));
+  for (int i = G * (threadIdx.x + 256 * HN_KEPT); i < P; i += G * 256) {
+    float v[G], z[G];
+    load(src + i, v);
+    load(g + i, z);
+    store(i, v, z);
+  }
 }
 
 // delta_prepare for long steps and up to four taps: a wave a head of queries or keys or up to 256 value channels, over
@@ -886,8 +930,9 @@ extern "C" int axk_head_norm_gate(const float* y, const float* gate, long gate_s
   HN_VEC(4) HN_VEC(8) HN_VEC(16) HN_VEC(32) HN_VEC(64)
 #undef HN_VEC
   if (P > 512) {
-    head_norm_gate_wide_kernel<<<(unsigned)items, 256, 0, (hipStream_t)stream>>>(y, gate, gate_stride, gain, gain_is_f32, gain_per_head,
-                                                                                eps, (elem_t*)out, heads, P, act);
+    auto kernel = vec && P % 4 == 0 ? head_norm_gate_wide_kernel<4> : head_norm_gate_wide_kernel<1>;
+    kernel<<<(unsigned)items, 256, 0, (hipStream_t)stream>>>(y, gate, gate_stride, gain, gain_is_f32, gain_per_head, eps, (elem_t*)out,
+                                                             heads, P, act);
     AXK_LAUNCH_CHECK("head_norm_gate");
     return 0;
   }

@@ -106,7 +106,7 @@ gemm_fma_kernel(const elem_t* __restrict__ x, int x_stride, const elem_t* __rest
       if (bias) v += load_vec(bias, bias_is_f32, n);
       const size_t at = (size_t)m * out_stride + n;
       if (GLU) ((elem_t*)out)[at] = from_float(swiglu1(v, sum_up[i][j]));
-      else if (mode == MODE_STORE) ((elem_t*)out)[at] = from_float(v);
+      else if (mode_stores_elem(mode)) ((elem_t*)out)[at] = from_float(mode_value(v, mode));
       else if (mode == MODE_ADD_F32) ((float*)out)[at] += v;
       else ((float*)out)[at] = v;
     }
@@ -190,7 +190,7 @@ gemm_fma_few_rows_kernel(const elem_t* __restrict__ x, int x_stride, const elem_
   if (bias) v += load_vec(bias, bias_is_f32, n);
   const size_t at = (size_t)m * out_stride + n;
   if (GLU) ((elem_t*)out)[at] = from_float(swiglu1(v, sum_up));
-  else if (mode == MODE_STORE) ((elem_t*)out)[at] = from_float(v);
+  else if (mode_stores_elem(mode)) ((elem_t*)out)[at] = from_float(mode_value(v, mode));
   else if (mode == MODE_ADD_F32) ((float*)out)[at] += v;
   else ((float*)out)[at] = v;
 }
@@ -249,7 +249,7 @@ static int gemm_checked(const void* x, int x_stride, const void* w, int w_packed
   AXK_REQUIRE(m >= 0 && n > 0 && k > 0, "gemm: bad sizes M=%d N=%d K=%d", m, n, k);
   AXK_REQUIRE(x_stride >= k && out_stride >= n, "gemm: strides x=%d (K=%d) out=%d (N=%d) too small", x_stride, k,
               out_stride, n);
-  AXK_REQUIRE(mode >= 0 && mode <= 3, "gemm: unknown mode %d", mode);
+  AXK_REQUIRE(mode >= 0 && mode <= MODE_RELU_SQUARED, "gemm: unknown mode %d", mode);
   AXK_REQUIRE(mode != MODE_SWIGLU || bias == nullptr, "gemm: the gated epilogue takes no bias");
   AXK_REQUIRE(ceil_div(m, 16) <= 65535, "gemm: M=%d is more rows than one launch takes", m);
   if (m == 0) return 0;

@@ -311,7 +311,7 @@ gemm_tile_kernel(const bf16_t* __restrict__ x, int x_stride, const bf16_t* __res
         if (m >= M) continue;
         const float v = acc[i][j][e] + bv;
         const size_t at = (size_t)m * out_stride + n;
-        if (mode == MODE_STORE) reinterpret_cast<bf16_t*>(out)[at] = float_to_bf16(v);
+        if (mode_stores_elem(mode)) reinterpret_cast<bf16_t*>(out)[at] = float_to_bf16(mode_value(v, mode));
         else if (mode == MODE_ADD_F32) reinterpret_cast<float*>(out)[at] += v;
         else reinterpret_cast<float*>(out)[at] = v;
       }
@@ -333,7 +333,7 @@ gemm_split_reduce_any_kernel(const float* __restrict__ partial, int splits, int 
   for (int z = 1; z < splits; ++z) v += partial[(size_t)z * plane + idx];
   if (bias) v += load_vec(bias, bias_is_f32, n);
   const size_t at = (size_t)m * out_stride + n;
-  if (mode == MODE_STORE) reinterpret_cast<bf16_t*>(out)[at] = float_to_bf16(v);
+  if (mode_stores_elem(mode)) reinterpret_cast<bf16_t*>(out)[at] = float_to_bf16(mode_value(v, mode));
   else if (mode == MODE_ADD_F32) reinterpret_cast<float*>(out)[at] += v;
   else reinterpret_cast<float*>(out)[at] = v;
 }
@@ -382,7 +382,7 @@ gemm_split_reduce_kernel(const float* __restrict__ partial, int splits, int M, i
 #pragma unroll
   for (int e = 0; e < 4; ++e) {
     if (bias) v[e] += load_vec(bias, bias_is_f32, n + e);
-    if (mode == MODE_STORE) reinterpret_cast<bf16_t*>(out)[at + e] = float_to_bf16(v[e]);
+    if (mode_stores_elem(mode)) reinterpret_cast<bf16_t*>(out)[at + e] = float_to_bf16(mode_value(v[e], mode));
     else if (mode == MODE_ADD_F32) reinterpret_cast<float*>(out)[at + e] += v[e];
     else reinterpret_cast<float*>(out)[at + e] = v[e];
   }
@@ -818,8 +818,10 @@ __device__ inline void rows_epilogue(Summed summed, int share, int unit, int lan
     }
     const size_t at = (size_t)m * out_stride + n;
     const bool whole = n + 3 < N && out_stride % 4 == 0;
-    if (mode == MODE_STORE) {
+    if (mode_stores_elem(mode)) {
       bf16_t* dst = reinterpret_cast<bf16_t*>(out) + at;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = mode_value(v[e], mode);
       if (whole && ((uintptr_t)out & 7) == 0) {
         uint2 pk;
         pk.x = pack2_bf16(v[0], v[1]);
@@ -1694,7 +1696,7 @@ static int gemm_mfma_dispatch(const bf16_t* x, int x_stride, const bf16_t* w, co
     return gemm_mfma_pass(x, x_stride, w, bias, bias_is_f32, out, out_stride, m, n, k, mode, stream, segs, norm,
                           (float*)workspace, rope_after);
   // in passes: every operand that has a row per row of X moves on with it
-  const size_t out_elem = mode == MODE_STORE || mode == MODE_SWIGLU ? sizeof(bf16_t) : sizeof(float);
+  const size_t out_elem = mode_stores_elem(mode) || mode == MODE_SWIGLU ? sizeof(bf16_t) : sizeof(float);
   for (int m0 = 0; m0 < m; m0 += pass) {
     const int rows = m - m0 < pass ? m - m0 : pass;
     SplitNorm norm_at;

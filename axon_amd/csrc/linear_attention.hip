@@ -121,40 +121,64 @@ __device__ inline void lc_powers(float* powers, float d, int tid) {
   }
 }
 
-// grid (heads, chunks, row tiles of 64 keys): a wave sixteen rows n of the state, all value dims.
+// grid (heads, chunks, row tiles of 64 keys): a wave sixteen rows n of the state, all value dims, two tiles of them at a time
+// (two chains), the next two asked for while these are multiplied.
 __global__ void __launch_bounds__(256)
 lightning_ends_kernel(const float* __restrict__ rows, long stride, int k_at, int v_at, const float* __restrict__ decay,
                       const int32_t* __restrict__ chunks, float* __restrict__ ends, int heads, int N, int P) {
   __shared__ float powers[LC + 1];
   const int h = blockIdx.x, first = chunks[2 * blockIdx.y], count = chunks[2 * blockIdx.y + 1];
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 15, g4 = lane >> 4;
+  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, r = lane & 15, g4 = lane >> 4;
   lc_powers(powers, decay[h], tid);
   __syncthreads();
   const int n0 = 64 * blockIdx.z + 16 * wave;
   if (n0 >= N) return;
   lc_f32x4 k[LC / 16];
   const float* vcol = rows + v_at + (long)h * P + r;
-  long at[LC / 16][4];
+  int at[LC / 16][4];
 #pragma unroll
   for (int c = 0; c < LC / 16; ++c)
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int j = 16 * c + 4 * g4 + e;
-      at[c][e] = (long)(first + min(j, count - 1)) * stride;
-      k[c][e] = j < count ? rows[at[c][e] + k_at + (long)h * N + n0 + r] * powers[count - 1 - j] : 0.0f;
+      at[c][e] = first + min(j, count - 1);
+      k[c][e] = j < count ? rows[at[c][e] * stride + k_at + (long)h * N + n0 + r] * powers[count - 1 - j] : 0.0f;
     }
   float* dst = ends + ((long)blockIdx.y * heads + h) * N * P + n0 + 4 * g4;
-  for (int p0 = 0; p0 < P; p0 += 16) {
-    lc_f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f}, v[LC / 16];
+  lc_f32x4 even[2][LC / 16], odd[2][LC / 16];
+  auto fetch = [&](lc_f32x4 (&v)[2][LC / 16], int p0) {
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+      if (p0 + 16 * i < P) {
+#pragma unroll
+        for (int c = 0; c < LC / 16; ++c)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[i][c][e] = vcol[at[c][e] * stride + p0 + 16 * i];
+      }
+  };
+  auto work = [&](const lc_f32x4 (&v)[2][LC / 16], int p0) {
+    lc_f32x4 acc[2] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}};
 #pragma unroll
     for (int c = 0; c < LC / 16; ++c)
 #pragma unroll
-      for (int e = 0; e < 4; ++e) v[c][e] = vcol[at[c][e] + p0];
+      for (int j = 0; j < 4; ++j)
 #pragma unroll
-    for (int c = 0; c < LC / 16; ++c)
+        for (int i = 0; i < 2; ++i) LC_MFMA(acc[i], k[c], v[i][c], j);
 #pragma unroll
-      for (int j = 0; j < 4; ++j) LC_MFMA(acc, k[c], v[c], j);
-    *reinterpret_cast<lc_f32x4*>(dst + (long)(p0 + r) * N) = acc;
+    for (int i = 0; i < 2; ++i)
+      if (p0 + 16 * i < P) *reinterpret_cast<lc_f32x4*>(dst + (long)(p0 + 16 * i + r) * N) = acc[i];
+  };
+#pragma unroll
+  for (int i = 0; i < 2; ++i)                      // a tile beyond P holds zeros, then whatever was last there: not stored
+#pragma unroll
+    for (int c = 0; c < LC / 16; ++c) even[i][c] = odd[i][c] = lc_f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  fetch(even, 0);
+  for (int p0 = 0; p0 < P; p0 += 64) {
+    if (p0 + 32 < P) fetch(odd, p0 + 32);
+    work(even, p0);
+    if (p0 + 32 >= P) break;
+    if (p0 + 64 < P) fetch(even, p0 + 64);
+    work(odd, p0 + 32);
   }
 }
 
@@ -191,47 +215,72 @@ lightning_fold_kernel(float* __restrict__ ends, const float* __restrict__ decay,
 // grid (heads, chunks, blocks of VT tiles of sixteen value dims): a wave the sixteen tokens 16 wave .. of the chunk.  The
 // products k_j . q_i are made transposed (rows j, column i), which is how the weighted sum over j wants its first operand.
 #define LC_VT 4
+struct LcOperands {
+  lc_f32x4 q, k[LC / 16], s[LC_VT];
+};
+
 __global__ void __launch_bounds__(256)
 lightning_outputs_kernel(const float* __restrict__ rows, long stride, int q_at, int k_at, int v_at, const float* __restrict__ decay,
                          const int32_t* __restrict__ chunks, const float* __restrict__ states, float* __restrict__ y, int heads, int N,
                          int P) {
   __shared__ float powers[LC + 1];
   const int h = blockIdx.x, first = chunks[2 * blockIdx.y], count = chunks[2 * blockIdx.y + 1];
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, r = lane & 15, g4 = lane >> 4;
+  const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, r = lane & 15, g4 = lane >> 4;
   lc_powers(powers, decay[h], tid);
   __syncthreads();
   if (16 * wave >= count) return;
   const int nt = N / 16, p_first = 16 * LC_VT * blockIdx.z, tiles = min(LC_VT, (P - p_first) / 16);
   const float* q = rows + (long)(first + min(16 * wave + r, count - 1)) * stride + q_at + (long)h * N + 4 * g4;
-  const float* k = rows + k_at + (long)h * N + 4 * g4;
   const float* I = states + (((long)blockIdx.y * heads + h) * P + p_first + r) * N + 4 * g4;
+  const float* k[LC / 16];
+#pragma unroll
+  for (int c = 0; c < LC / 16; ++c) k[c] = rows + (long)(first + min(16 * c + r, count - 1)) * stride + k_at + (long)h * N + 4 * g4;
   lc_f32x4 m[LC / 16], out[LC_VT];
 #pragma unroll
   for (int c = 0; c < LC / 16; ++c) m[c] = lc_f32x4{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
   for (int v = 0; v < LC_VT; ++v) out[v] = lc_f32x4{0.0f, 0.0f, 0.0f, 0.0f};
-  long k_row[LC / 16];
-#pragma unroll
-  for (int c = 0; c < LC / 16; ++c) k_row[c] = (long)(first + min(16 * c + r, count - 1)) * stride;
-  for (int t = 0; t < nt; ++t) {
-    const lc_f32x4 qf = lc_load(q + 16 * t);
-    lc_f32x4 kf[LC / 16], sf[LC_VT];
+  auto fetch = [&](LcOperands& o, int t) {
+    o.q = lc_load(q + 16 * t);
 #pragma unroll
     for (int c = 0; c < LC / 16; ++c)
-      if (c <= wave) kf[c] = lc_load(k + k_row[c] + 16 * t);
+      if (c <= wave) o.k[c] = lc_load(k[c] + 16 * t);
 #pragma unroll
     for (int v = 0; v < LC_VT; ++v)
-      if (v < tiles) sf[v] = lc_load(I + (long)16 * v * N + 16 * t);
+      if (v < tiles) o.s[v] = lc_load(I + (long)16 * v * N + 16 * t);
+  };
+  auto work = [&](const LcOperands& o) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
 #pragma unroll
       for (int c = 0; c < LC / 16; ++c)
-        if (c <= wave) LC_MFMA(m[c], kf[c], qf, j);
+        if (c <= wave) LC_MFMA(m[c], o.k[c], o.q, j);
 #pragma unroll
       for (int v = 0; v < LC_VT; ++v)
-        if (v < tiles) LC_MFMA(out[v], qf, sf[v], j);
+        if (v < tiles) LC_MFMA(out[v], o.q, o.s[v], j);
     }
+  };
+  LcOperands even, odd;
+  fetch(even, 0);
+  for (int t = 0; t < nt; t += 2) {
+    if (t + 1 < nt) fetch(odd, t + 1);
+    work(even);
+    if (t + 1 >= nt) break;
+    if (t + 2 < nt) fetch(even, t + 2);
+    work(odd);
   }
+  // the values of the chunk's tokens 16 c .., as the weighted sum's second operand
+  lc_f32x4 v0[LC_VT], v1[LC_VT];
+  auto values = [&](lc_f32x4 (&vf)[LC_VT], int c) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float* vrow = rows + (long)(first + min(16 * c + 4 * g4 + e, count - 1)) * stride + v_at + (long)h * P + p_first + r;
+#pragma unroll
+      for (int v = 0; v < LC_VT; ++v)
+        if (v < tiles) vf[v][e] = vrow[16 * v];
+    }
+  };
+  values(v0, 0);
   // the state's share of token i is decayed i + 1 times; the result's lane holds rows 4 g4 + e, the products' column r
 #pragma unroll
   for (int v = 0; v < LC_VT; ++v)
@@ -241,21 +290,18 @@ lightning_outputs_kernel(const float* __restrict__ rows, long stride, int q_at, 
 #pragma unroll
   for (int c = 0; c < LC / 16; ++c)
     if (c <= wave) {
-      lc_f32x4 vf[LC_VT];
+      lc_f32x4 (&now)[LC_VT] = c % 2 ? v1 : v0;
+      if (c + 1 < LC / 16 && c + 1 <= wave) values(c % 2 ? v0 : v1, c + 1);
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int j = 16 * c + 4 * g4 + e;
         m[c][e] = j <= i ? m[c][e] * powers[max(i - j, 0)] : 0.0f;
-        const float* vrow = rows + (long)(first + min(j, count - 1)) * stride + v_at + (long)h * P + p_first + r;
-#pragma unroll
-        for (int v = 0; v < LC_VT; ++v)
-          if (v < tiles) vf[v][e] = vrow[16 * v];
       }
 #pragma unroll
       for (int j = 0; j < 4; ++j)
 #pragma unroll
         for (int v = 0; v < LC_VT; ++v)
-          if (v < tiles) LC_MFMA(out[v], m[c], vf[v], j);
+          if (v < tiles) LC_MFMA(out[v], m[c], now[v], j);
     }
 #pragma unroll
   for (int v = 0; v < LC_VT; ++v)

@@ -44,7 +44,7 @@ __device__ inline int nth_block(int i, int kept, int lo_block) { return i < kept
 // norm_rows: the norm's mean goes over all of a token's query units (and over all its key units) at once,
 // and the gain holds a number for every one of these dims.
 //
-// CONV: what is normed, rotated and stored is sum_k w[c, k] (the projection taps - 1 - k tokens before)[c], the columns
+// TAPS != 0 (the taps of a convolution, -1: more than four): what is normed, rotated and stored is sum_k w[c, k] (the projection taps - 1 - k tokens before)[c], the columns
 // q_at .. being the channels [q | k | v]; what a request's earlier steps left of its projections comes from its state row
 // (two copies of [taps - 1][channels], oldest first, the one behind position p in copy p & 1).  In a step of single tokens
 // (single) a channel's thread also writes the copy behind its token: it is the only one that reads or writes that channel.
@@ -61,20 +61,35 @@ __device__ inline const float* conv_kept(const HeadsConv& cv, const int32_t* seq
 }
 
 // row: the token's projections at channel 0.
+template <int TAPS>
 __device__ inline float conv_value(const HeadsConv& cv, const float* __restrict__ row, long stride, const float* kept, float* keep,
                                    int inside, int c) {
+  const int taps = TAPS > 0 ? TAPS : cv.taps;
+  auto input = [&](int k) {                      // the projection `back` tokens before this one
+    const int back = taps - 1 - k, at = taps - 1 - (back - inside);
+    return back <= inside ? row[c - (long)back * stride] : kept[(long)at * cv.channels + c];
+  };
   float acc = 0.0f;
-  for (int k = 0; k < cv.taps; ++k) {
-    const int back = cv.taps - 1 - k;            // the projection `back` tokens before this one
-    const int at = cv.taps - 1 - (back - inside);
-    const float v = back <= inside ? row[c - (long)back * stride] : kept[(long)at * cv.channels + c];
-    acc = fmaf(to_float(cv.w[(long)c * cv.taps + k]), v, acc);
+  if (TAPS > 0) {
+    float v[TAPS > 0 ? TAPS : 1], w[TAPS > 0 ? TAPS : 1];
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) { v[k] = input(k); w[k] = to_float(cv.w[(long)c * TAPS + k]); }
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) {
+      acc = fmaf(w[k], v[k], acc);
+      if (keep != nullptr && k > 0) keep[(long)(k - 1) * cv.channels + c] = v[k];
+    }
+    return acc;
+  }
+  for (int k = 0; k < taps; ++k) {
+    const float v = input(k);
+    acc = fmaf(to_float(cv.w[(long)c * taps + k]), v, acc);
     if (keep != nullptr && k > 0) keep[(long)(k - 1) * cv.channels + c] = v;
   }
   return acc;
 }
 
-template <bool CONV>
+template <int TAPS>
 __global__ void __launch_bounds__(256)
 heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int n_q, int k_at, int n_k, int v_at, int v_width,
                      int dim, const void* __restrict__ q_gain, int q_gain_is_f32, const void* __restrict__ k_gain,
@@ -82,6 +97,7 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
                      const int32_t* __restrict__ positions, const int32_t* __restrict__ seq_rows,
                      const int32_t* __restrict__ block_table, int table_stride, elem_t* __restrict__ cache, int page_size,
                      elem_t* __restrict__ q_out, int write_kv, float q_temp_coef, int q_temp_every, int norm_rows, HeadsConv cv) {
+  constexpr bool CONV = TAPS != 0;
   __shared__ float row_sums[2][256 / AXON_WAVE];
   extern __shared__ float convolved[];         // CONV: a unit of `dim` a wave
   const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -103,7 +119,7 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
   const float* kept = nullptr;
   float* keep = nullptr;
   if (CONV) {
-    inside = rec_inside(seq_rows, t, cv.taps - 1);
+    if (!cv.single) inside = rec_inside(seq_rows, t, cv.taps - 1);
     kept = conv_kept(cv, seq_rows, positions, t, inside);
     if (cv.single) keep = rec_copy_behind(cv.state, cv.state_stride, cv.copy_elems, seq_rows[t], positions[t]);
   }
@@ -130,7 +146,7 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
     float inv = is_q ? q_inv : k_inv;
     if (CONV) {                                  // the wave's own corner of LDS: no other wave touches it
       float* mine = convolved + wave * dim;
-      for (int i = lane; i < dim; i += 64) mine[i] = conv_value(cv, row + q_at, stride, kept, keep, inside, (int)(src - row) - q_at + i);
+      for (int i = lane; i < dim; i += 64) mine[i] = conv_value<TAPS>(cv, row + q_at, stride, kept, keep, inside, (int)(src - row) - q_at + i);
       __builtin_amdgcn_wave_barrier();
       src = mine;
     }
@@ -159,7 +175,7 @@ heads_prepare_kernel(const float* __restrict__ proj, long stride, int q_at, int 
   if (!write_kv) return;
   elem_t* by_dim = page_base + (long)page_size * kw + in_page;
   for (int i = blockIdx.y * 256 + threadIdx.x; i < v_width; i += 256 * gridDim.y) {
-    const float v = CONV ? conv_value(cv, row + q_at, stride, kept, keep, inside, v_at - q_at + i) : row[v_at + i];
+    const float v = CONV ? conv_value<TAPS>(cv, row + q_at, stride, kept, keep, inside, v_at - q_at + i) : row[v_at + i];
     by_dim[(long)i * page_size] = from_float(v);
   }
 }
@@ -798,7 +814,7 @@ static int launch_masked_mfma(const void* q, const void* cache, const int32_t* b
                               hipStream_t stream) {
   const int grp = heads / kv_heads;
   const size_t lds = ((size_t)64 * (MAPS * dim + 8) + (size_t)vdim * (64 + 8)) * sizeof(bf16_t);
-  if (tiles != nullptr && partial == nullptr && KC <= 4 && DT <= 8 && lds <= 64 * 1024) {
+  if (tiles != nullptr && partial == nullptr && KC <= 4 && DT <= 16 && lds <= 64 * 1024) {
     static bool configured = false;
     if (!configured && lds > 48 * 1024) {
       hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&masked_attention_staged_kernel<MAPS, DT, KC>),
@@ -864,9 +880,11 @@ extern "C" int axk_heads_prepare(const float* proj, long stride, int q_at, int n
                    magnitude, table, positions, seq_rows, block_table, table_stride, (elem_t*)cache, page_size, (elem_t*)q_out, write_kv,      \
                    q_temp_coef, q_temp_every, norm_rows, cv
   if (conv_w == nullptr) {
-    heads_prepare_kernel<false><<<dim3(n_tokens, per_token), 256, 0, (hipStream_t)stream>>>(HEADS_ARGS);
+    heads_prepare_kernel<0><<<dim3(n_tokens, per_token), 256, 0, (hipStream_t)stream>>>(HEADS_ARGS);
   } else {
-    heads_prepare_kernel<true><<<dim3(n_tokens, per_token), 256, 4 * dim * sizeof(float), (hipStream_t)stream>>>(HEADS_ARGS);
+    auto kernel = conv_taps == 1 ? heads_prepare_kernel<1> : conv_taps == 2 ? heads_prepare_kernel<2>
+                  : conv_taps == 3 ? heads_prepare_kernel<3> : conv_taps == 4 ? heads_prepare_kernel<4> : heads_prepare_kernel<-1>;
+    kernel<<<dim3(n_tokens, per_token), 256, 4 * dim * sizeof(float), (hipStream_t)stream>>>(HEADS_ARGS);
     if (conv_spans != nullptr && conv_taps > 1 && n_spans > 0)
       heads_keep_kernel<<<dim3(ceil_div(cv.channels, 256), n_spans), 256, 0, (hipStream_t)stream>>>(proj + q_at, stride, cv, conv_spans,
                                                                                                    positions);

@@ -255,7 +255,7 @@ extern "C" int axk_shifted_norm(const float* x, const float* gain, float eps, co
   if (n_tokens == 0) return 0;
   const bool vec = dim % 4 == 0 && state_stride % 4 == 0 &&
                    (((uintptr_t)x | (uintptr_t)gain | (uintptr_t)share | (uintptr_t)state | (uintptr_t)out) & 15) == 0;
-  const int run = n_tokens >= 1024 ? 4 : 1;
+  const int run = n_tokens >= 4096 ? 4 : 1;       // a row's sum is worked out again by the block behind it: from L2
   auto kernel = vec ? shifted_norm_kernel<4> : shifted_norm_kernel<1>;
   kernel<<<ceil_div(n_tokens, run), ST_THREADS, 0, (hipStream_t)stream>>>(x, gain, eps, share, state, state_stride, positions, seq_rows,
                                                                           (elem_t*)out, n_tokens, dim, run);

@@ -161,9 +161,133 @@ low_rank_kernel(LowRank first, LowRank second, int n_tokens) {
   }
 }
 
+// The same for up to 16 tokens (a decoding step): 64 channels a block, a lane a channel with 64 of its rank in registers, the
+// tokens shared out between the four waves.
+#define LF_TOKENS 16
+__global__ void __launch_bounds__(256)
+low_rank_few_kernel(LowRank first, LowRank second, int n_tokens) {
+  __shared__ __align__(16) float ts[LF_TOKENS][TD_RANK];
+  const int first_blocks = (first.channels + TD_CHANNELS - 1) / TD_CHANNELS;
+  const bool is_first = (int)blockIdx.x < first_blocks;
+  const LowRank r = is_first ? first : second;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int c = ((int)blockIdx.x - (is_first ? 0 : first_blocks)) * TD_CHANNELS + lane;
+  const elem_t* w = r.w + (long)min(c, r.channels - 1) * r.rank;
+  const bool vec = (r.rank & 3) == 0;
+  float acc[LF_TOKENS / 4] = {0.0f, 0.0f, 0.0f, 0.0f};
+  for (int k0 = 0; k0 < r.rank; k0 += TD_RANK) {
+    const int n = min(TD_RANK, r.rank - k0);
+    float x[TD_RANK / 4][4];
+#pragma unroll
+    for (int i = 0; i < TD_RANK / 4; ++i) load4_guarded(w + k0 + 4 * i, max(0, min(4, n - 4 * i)), vec, x[i]);
+    __syncthreads();
+    for (int i = threadIdx.x; i < n_tokens * TD_RANK; i += 256) {
+      const int t = i / TD_RANK, k = i % TD_RANK;
+      float v = k < n ? r.low[(long)t * r.low_stride + k0 + k] : 0.0f;
+      if (r.kind == LR_TIME_MIX_DECAY) v = tanhf(v);
+      ts[t][k] = v;
+    }
+    __syncthreads();
+#pragma unroll 1
+    for (int j = 0; j < LF_TOKENS / 4; ++j) {
+      const int t = wave + 4 * j;
+      if (t >= n_tokens) break;
+      float part[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+      for (int i = 0; i < TD_RANK / 4; ++i) {
+        const float4 a = *reinterpret_cast<const float4*>(&ts[t][4 * i]);
+        part[0] = fmaf(a.x, x[i][0], part[0]);
+        part[1] = fmaf(a.y, x[i][1], part[1]);
+        part[2] = fmaf(a.z, x[i][2], part[2]);
+        part[3] = fmaf(a.w, x[i][3], part[3]);
+      }
+      const float sum = (part[0] + part[1]) + (part[2] + part[3]);
+#pragma unroll
+      for (int i = 0; i < LF_TOKENS / 4; ++i)
+        if (i == j) acc[i] += sum;
+    }
+  }
+  if (c >= r.channels) return;
+#pragma unroll 1
+  for (int j = 0; j < LF_TOKENS / 4; ++j) {
+    const int t = wave + 4 * j;
+    if (t >= n_tokens) break;
+    float v = acc[0];
+#pragma unroll
+    for (int i = 1; i < LF_TOKENS / 4; ++i)
+      if (i == j) v = acc[i];
+    r.out[(long)t * r.channels + c] = low_rank_act(r, v, c);
+  }
+}
+
+// The same for many tokens on the 32-bit matrix cores (no tanh on the way in; ranks of whole sixteens): a wave 16 channels x 64
+// tokens, rows of W as the first operand, so that a lane holds four neighbouring channels of a token.
+typedef __attribute__((ext_vector_type(4))) float lr_f32x4;
+__global__ void __launch_bounds__(256)
+low_rank_mfma_kernel(LowRank first, LowRank second, int n_tokens) {
+  const int first_blocks = (first.channels + TD_CHANNELS - 1) / TD_CHANNELS;
+  const bool is_first = (int)blockIdx.x < first_blocks;
+  const LowRank r = is_first ? first : second;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, col = lane & 15, g4 = lane >> 4;
+  const int c0 = ((int)blockIdx.x - (is_first ? 0 : first_blocks)) * TD_CHANNELS + 16 * wave, t0 = 64 * blockIdx.y;
+  if (c0 >= r.channels) return;
+  const elem_t* w = r.w + (long)min(c0 + col, r.channels - 1) * r.rank + 4 * g4;
+  const float* low[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) low[i] = r.low + (long)min(t0 + 16 * i + col, n_tokens - 1) * r.low_stride + 4 * g4;
+  lr_f32x4 acc[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) acc[i] = lr_f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  for (int k = 0; k < r.rank; k += 32) {
+    float a[2][4];
+    lr_f32x4 b[2][4];
+#pragma unroll
+    for (int s = 0; s < 2; ++s)
+      if (k + 16 * s < r.rank) {
+        load4_guarded(w + k + 16 * s, 4, true, a[s]);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) b[s][i] = *reinterpret_cast<const lr_f32x4*>(low[i] + k + 16 * s);
+      }
+#pragma unroll
+    for (int s = 0; s < 2; ++s)
+      if (k + 16 * s < r.rank)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[s][j], b[s][i][j], acc[i], 0, 0, 0);
+  }
+  const int c = c0 + 4 * g4;
+  const bool whole = c + 3 < r.channels && (r.channels & 3) == 0;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int t = t0 + 16 * i + col;
+    if (t >= n_tokens) continue;
+    float* dst = r.out + (long)t * r.channels + c;
+    if (whole) {
+      lr_f32x4 v;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = low_rank_act(r, acc[i][e], c + e);
+      *reinterpret_cast<lr_f32x4*>(dst) = v;
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (c + e < r.channels) dst[e] = low_rank_act(r, acc[i][e], c + e);
+    }
+  }
+}
+
+static bool low_rank_mfma_ok(const LowRank& r) {
+  return r.channels == 0 || (r.kind != LR_TIME_MIX_DECAY && r.rank % 16 == 0 && r.low_stride % 4 == 0 && ((uintptr_t)r.low & 15) == 0 &&
+                             ((uintptr_t)r.out & 15) == 0);
+}
+
 static int launch_low_rank(const LowRank& first, const LowRank& second, int n_tokens, hipStream_t stream, const char* name) {
   const int blocks = ceil_div(first.channels, TD_CHANNELS) + (second.channels > 0 ? ceil_div(second.channels, TD_CHANNELS) : 0);
-  if (n_tokens >= 512)
+  if (n_tokens <= LF_TOKENS)
+    low_rank_few_kernel<<<blocks, 256, 0, stream>>>(first, second, n_tokens);
+  else if (low_rank_mfma_ok(first) && low_rank_mfma_ok(second) && ceil_div(n_tokens, 64) <= 65535)
+    low_rank_mfma_kernel<<<dim3(blocks, ceil_div(n_tokens, 64)), 256, 0, stream>>>(first, second, n_tokens);
+  else if (n_tokens >= 512)
     low_rank_kernel<4><<<dim3(blocks, ceil_div(n_tokens, 64)), 256, 0, stream>>>(first, second, n_tokens);
   else
     low_rank_kernel<1><<<dim3(blocks, ceil_div(n_tokens, 16)), 256, 0, stream>>>(first, second, n_tokens);

@@ -16,7 +16,7 @@ import torch
 
 from . import build
 
-MODE_STORE, MODE_ADD_F32, MODE_STORE_F32, MODE_SWIGLU = 0, 1, 2, 3
+MODE_STORE, MODE_ADD_F32, MODE_STORE_F32, MODE_SWIGLU, MODE_RELU_SQUARED = 0, 1, 2, 3, 4
 
 
 class KernelError(RuntimeError):
@@ -629,6 +629,7 @@ class Kernels:
         """out = epilogue(x . w^T + bias); x [M, K] (rows may be strided), w [N, K] contiguous or
         a PackedMatrix (the matrix-core kernels; a row-major w goes to the 32-bit FMA kernel).
         MODE_SWIGLU: w is [2 N, K], gate rows then up rows; out [M, N] = silu(x gate^T) * (x up^T).
+        MODE_RELU_SQUARED: out = max(. , 0)^2 in the compute dtype.
 
         `following_norm` = (gain, values [M, N], eps) with MODE_ADD_F32, where `gemm_then_norm_ok`:
         the kernel that finishes the product also writes the RMS norm of the new rows,
@@ -645,7 +646,7 @@ class Kernels:
             raise KernelError(f"gemm: x {tuple(x.shape)} w {tuple(w.shape)} do not multiply, or are not row-major")
         if out.shape != (M, N) or not out.is_cuda:
             raise KernelError(f"gemm: out {tuple(out.shape)} is not [{M}, {N}]")
-        want = self.dtype if mode in (MODE_STORE, MODE_SWIGLU) else torch.float32
+        want = self.dtype if mode in (MODE_STORE, MODE_SWIGLU, MODE_RELU_SQUARED) else torch.float32
         if out.dtype != want:
             raise KernelError(f"gemm: mode {mode} writes {want}, out is {out.dtype}")
         if bias is not None and bias.numel() != N:
@@ -1447,7 +1448,7 @@ class Kernels:
         `norm_rows`: the norm goes over all query (all key) units of a token at once.  `conv` = (w [channels, taps] in the
         compute dtype, state rows, copy_elems, spans): the projections pass a causal convolution first, what a request's
         later steps need of them is kept in its state row; spans int32 [n, 3], or None in a step of single tokens."""
-        self._f32(proj, "heads proj"); self._f32(table, "rope table"); self._i32(positions, "positions")
+        self._f32_rows(proj, "heads proj"); self._f32(table, "rope table"); self._i32(positions, "positions")
         self._i32(seq_rows, "seq_rows"); self._i32(block_table, "block_table"); self._elem(q_out, "heads q_out")
         T = positions.numel()
         if proj.dim() != 2 or proj.shape[0] != T or (rot and table.shape != (T, rot // 2, 2)) or seq_rows.numel() != T:

@@ -225,6 +225,12 @@ class Mixer(Part):
     def forward(self, ctx, binding: CacheBinding, h, residual) -> None:
         raise NotImplementedError
 
+    def input_projections(self) -> Optional[List[Tuple[str, int, Optional[str]]]]:
+        """The projections of `h` that `forward` starts with, in the order of their columns: (tensor, rows, bias tensor or
+        None), if `forward` also takes their float32 rows ready made (`rows=`, which may lie apart; `load(..., own_input=False)`
+        then leaves their matrices alone).  For a part that runs several mixers on one `h`.  None: it does not."""
+        return None
+
     def output_terms(self) -> List["OutputTerm"]:
         """How the outputs that `forward_apart` stores make this mixer's result (one output, as it is)."""
         return [OutputTerm()]

@@ -105,9 +105,15 @@ class GatedDeltaRule(Mixer):
     def state_spec(self) -> StateSpec:
         return StateSpec(2 * self.copy_elems)
 
-    def load(self, store, rt) -> None:
+    def input_projections(self):
+        widths = {"q": self.qk, "k": self.qk, "v": self.inner, "b": self.heads, "a": self.heads, "a1": self.decay_rank, "g": self.inner,
+                  "g1": self.gate_rank}
+        return [(self.n[k], widths[k], None) for k in self.first]
+
+    def load(self, store, rt, own_input: bool = True) -> None:
         n = self.n
-        self.w_in = rt.k.prepare_weight(store.fused_matrix([n[k] for k in self.first]))
+        if own_input:
+            self.w_in = rt.k.prepare_weight(store.fused_matrix([n[k] for k in self.first]))
         self.w_decay = store.matrix(n["a2"]) if self.decay_rank else None
         self.w_gate = store.matrix(n["g2"]) if self.gate_rank else None
         self.conv_w = store.fused_matrix([n[k] + ".conv" for k in ("q", "k", "v")])
@@ -115,15 +121,16 @@ class GatedDeltaRule(Mixer):
         self.w_o = rt.k.prepare_weight(store.matrix(n["o"]))
         store.forget(n["o"])
 
-    def forward(self, ctx, binding: CacheBinding, h, out, accumulate: bool = True) -> None:
+    def forward(self, ctx, binding: CacheBinding, h, out, accumulate: bool = True, rows=None) -> None:
         k, T, f32 = ctx.rt.k, h.shape[0], torch.float32
         state = ctx.cache.state(binding.state_index)
-        rows = ctx.ws.take((T, self.rows_width), f32)
-        k.gemm(h, self.w_in, rows, None, MODE_STORE_F32)
+        if rows is None:
+            rows = ctx.ws.take((T, self.rows_width), f32)
+            k.gemm(h, self.w_in, rows, None, MODE_STORE_F32)
         u, terms = ctx.ws.take((T, self.channels), f32), ctx.ws.take((T, self.heads, 2), f32)
         k.delta_prepare(rows, self.conv_w, state, self.copy_elems, self.tail_at, ctx.positions, ctx.seq_rows, self.beta_at, self.decay_at,
                         None if self.decay_rank else self.a_log, None if self.decay_rank else self.dt_bias, u, terms, self.heads, self.kv_heads, self.dim, self.vdim, self.dim ** -0.5)
-        decay, gate = None, rows[:, self.gate_at:]
+        decay, gate = None, rows[:, self.gate_at:self.rows_width]
         if self.decay_rank:
             decay = ctx.ws.take((T, self.heads * self.dim), f32)
         if self.gate_rank:

@@ -56,28 +56,35 @@ class LightningAttention(Mixer):
     def state_spec(self) -> StateSpec:
         return StateSpec(2 * self.copy_elems)
 
-    def load(self, store, rt) -> None:
+    def input_projections(self):
+        widths = {"q": self.qk, "k": self.qk, "v": self.inner, "g": self.inner}
+        return [(self.n[k], rows, None) for k, rows in widths.items()]
+
+    def load(self, store, rt, own_input: bool = True) -> None:
         n = self.n
-        self.w_in = rt.k.prepare_weight(store.fused_matrix([n[k] for k in ("q", "k", "v", "g")]))
+        if own_input:
+            self.w_in = rt.k.prepare_weight(store.fused_matrix([n[k] for k in ("q", "k", "v", "g")]))
         self.gain = store.vector(n["norm"])
         self.decay = torch.tensor(self.decays, dtype=torch.float32, device=rt.device)
         self.w_o = rt.k.prepare_weight(store.matrix(n["o"]))
         store.forget(n["o"])
 
-    def forward(self, ctx, binding: CacheBinding, h, out, accumulate: bool = True) -> None:
+    def forward(self, ctx, binding: CacheBinding, h, out, accumulate: bool = True, rows=None) -> None:
         k, T, f32 = ctx.rt.k, h.shape[0], torch.float32
         state = ctx.cache.state(binding.state_index)
-        rows = ctx.ws.take((T, self.gate_at + self.inner), f32)
-        k.gemm(h, self.w_in, rows, None, MODE_STORE_F32)
+        if rows is None:
+            rows = ctx.ws.take((T, self.gate_at + self.inner), f32)
+            k.gemm(h, self.w_in, rows, None, MODE_STORE_F32)
         y = ctx.ws.take((T, self.inner), f32)
-        long = step_chunks(ctx) if k.lightning_chunked_ok(self.heads, self.dim, self.vdim, rows.stride(0), 0, self.qk) else None
+        chunks_ok = rows.data_ptr() % 16 == 0 and k.lightning_chunked_ok(self.heads, self.dim, self.vdim, rows.stride(0), 0, self.qk)
+        long = step_chunks(ctx) if chunks_ok else None
         chunks, spans = long if long is not None else (None, step_spans(ctx))
         if chunks is not None:
             k.silu_rows(rows, self.gate_at)
         k.lightning_scan(rows, 0, self.qk, 2 * self.qk, chunks is None, self.decay, state, self.copy_elems, spans, ctx.positions,
                          ctx.seq_rows, y, self.heads, self.dim, self.vdim, chunks=chunks)
         gated = ctx.ws.take((T, self.inner), ctx.rt.dtype)
-        k.head_norm_gate(y, rows[:, self.gate_at:], self.gain, self.eps, gated, 1, act="sigmoid")
+        k.head_norm_gate(y, rows[:, self.gate_at:self.gate_at + self.inner], self.gain, self.eps, gated, 1, act="sigmoid")
         k.gemm(gated, self.w_o, out, None, MODE_ADD_F32 if accumulate else MODE_STORE_F32)
 
 

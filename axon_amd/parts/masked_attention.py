@@ -58,6 +58,16 @@ from ..kernels import MODE_ADD_F32, MODE_STORE_F32, PackedMatrix
 from .base import CacheBinding, CacheSpec, Mixer, StateSpec, TensorDecl, build_part, register_mixer
 from .recurrent import step_spans
 
+def load_projections(projections, store, rt):
+    """One matrix for projections as `Mixer.input_projections` lists them, and their bias (float32, zeros where a projection
+    has none; None if none has one)."""
+    weight = rt.k.prepare_weight(store.fused_matrix([name for name, _, _ in projections]))
+    if all(bias is None for _, _, bias in projections):
+        return weight, None
+    parts = [store.vector(bias).float() if bias is not None else torch.zeros(rows, device=rt.device) for _, rows, bias in projections]
+    return weight, torch.cat(parts).contiguous()
+
+
 TILE_TOKENS = 16        # tokens of one request a tile of the matrix-core kernel holds
 
 
@@ -198,15 +208,16 @@ class MaskedAttention(Mixer):
     def state_spec(self) -> Optional[StateSpec]:
         return StateSpec(2 * self.copy_elems) if self.taps > 1 else None
 
-    def load(self, store, rt) -> None:
+    def input_projections(self):
+        rows = {"q": self.q_width, "k": self.k_width, "v": self.v_width, "g": self.g_width}
+        return [(self.n[k], rows[k], self.n[k] + ".b" if self.bias and k != "g" else None) for k in self._projections()]
+
+    def load(self, store, rt, own_input: bool = True) -> None:
         n = self.n
-        names = self._projections()
         if self.taps:
             self.conv_w = store.fused_matrix([n[k] + ".conv" for k in ("q", "k", "v")])
-        self.w_proj = rt.k.prepare_weight(store.fused_matrix([n[k] for k in names]))
-        if self.bias:
-            parts = [store.vector(n[k] + ".b").float() if k != "g" else torch.zeros(self.g_width, device=rt.device) for k in names]
-            self.b_proj = torch.cat(parts).contiguous()
+        if own_input:
+            self.w_proj, self.b_proj = load_projections(self.input_projections(), store, rt)
         if self.norm_plain:
             self.q_gain = self.k_gain = torch.ones(self.dim, dtype=torch.float32, device=rt.device)
         elif self.qk_norm:
@@ -239,12 +250,14 @@ class MaskedAttention(Mixer):
         """In steps of many rows the output projection's last kernel also writes the norm behind it."""
         return isinstance(self.w_o, PackedMatrix) and ctx.rt.k.gemm_then_norm_ok(ctx.n_tokens, self.hidden, self.o_width)
 
-    def forward(self, ctx, binding: CacheBinding, h, residual, following=None, accumulate: bool = True) -> None:
+    def forward(self, ctx, binding: CacheBinding, h, residual, following=None, accumulate: bool = True, rows=None) -> None:
         k, T = ctx.rt.k, h.shape[0]
         group = ctx.cache.group(binding.group)
         (cache,) = group.layer(binding.index)
-        proj = ctx.ws.take((T, self.proj_width), torch.float32)
-        k.gemm(h, self.w_proj, proj, self.b_proj, MODE_STORE_F32)
+        proj = rows
+        if proj is None:
+            proj = ctx.ws.take((T, self.proj_width), torch.float32)
+            k.gemm(h, self.w_proj, proj, self.b_proj, MODE_STORE_F32)
         if self.position is not None:
             table, neighbours, magnitude = self.position.tables(ctx), self.position.pairing == "neighbours", self.position.magnitude
         else:
@@ -267,7 +280,7 @@ class MaskedAttention(Mixer):
             span = ctx.decode_shapes.get("masked_attention_span", 0) if ctx.decode_only else max(s.start_pos + s.q_len for s in ctx.spans)
         k.masked_attention(q, cache, group.block_table, ctx.positions, ctx.seq_rows, att, self.heads, self.kv_heads, self.maps,
                            self.dim, self.vdim, group.page_size, self.mask, self.mask_size, self.scale, self.softcap, self.lam,
-                           1.0 - self.diff, self.eps, gate=proj[:, self.g_at:] if self.gate else None, tiles=tiles,
+                           1.0 - self.diff, self.eps, gate=proj[:, self.g_at:self.proj_width] if self.gate else None, tiles=tiles,
                            sink=self.sinks if self.sink_per_head else self.sink, gate_per_head=self.gate_per_head, span=span, keep=self.keep)
         if not accumulate:          # the output itself, for a part that sums and norms on its own
             k.gemm(att, self.w_o, residual, self.b_o, MODE_STORE_F32)

@@ -10,7 +10,7 @@ from __future__ import annotations
 from typing import List
 
 from ..config.base import ConfigError
-from ..kernels import MODE_ADD_F32, MODE_STORE, MODE_STORE_F32, MODE_SWIGLU, PackedMatrix
+from ..kernels import MODE_ADD_F32, MODE_RELU_SQUARED, MODE_STORE, MODE_STORE_F32, MODE_SWIGLU, PackedMatrix
 from .base import FeedForward, PrecedingNorm, TensorDecl, register_feed_forward
 
 
@@ -95,8 +95,11 @@ class DenseMLP(FeedForward):
     def forward(self, ctx, h, out, following=None, accumulate: bool = True) -> None:
         k = ctx.rt.k
         act = ctx.ws.take((h.shape[0], self.ff), ctx.rt.dtype)
-        k.gemm(h, self.w_up, act, None, MODE_STORE)
-        k.activation(act, self.activation)
+        if self.activation == "relu_squared":                   # in the product's epilogue
+            k.gemm(h, self.w_up, act, None, MODE_RELU_SQUARED)
+        else:
+            k.gemm(h, self.w_up, act, None, MODE_STORE)
+            k.activation(act, self.activation)
         if following is not None and accumulate:
             k.gemm(act, self.w_down, out, None, MODE_ADD_F32, following_norm=following.as_argument())
         else:

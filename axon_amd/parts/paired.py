@@ -6,7 +6,8 @@ Each side is a mixer of its own (a `PartSpec`), run on the same rows h.  `combin
   layer's eps a side, times `mult` (a half: the mean of the two);
 * "scaled": scales[0] left(h) + scales[1] right(h).
 
-Norm, factors and the sum into the residual stream are one 32-bit pass.  One side may keep pages (a `CacheSpec`); per-request
+Where both sides take their projections of h ready made, one product makes them for both.  Norm, factors and the sum into the
+residual stream are one 32-bit pass.  One side may keep pages (a `CacheSpec`); per-request
 state either side may have (the run's binding holds the left side's arenas, then the right side's).
 
 Parameters: `hidden_size`, `left`, `right` (the sides' PartSpecs; their tensors lie under
@@ -20,7 +21,9 @@ from typing import List, Optional
 import torch
 
 from ..config.base import ConfigError, PartSpec
+from ..kernels import MODE_STORE_F32
 from .base import CacheBinding, CacheSpec, Mixer, OutputTerm, StateSpec, TensorDecl, build_part, register_mixer
+from .masked_attention import load_projections
 
 
 class PairedMixers(Mixer):
@@ -45,6 +48,9 @@ class PairedMixers(Mixer):
             raise ConfigError("a pair of mixers shares one binding: one side may keep pages")
         self.graph_safe = all(getattr(s, "graph_safe", False) for s in self.sides)
         self.gains = [None, None]
+        projections = [s.input_projections() for s in self.sides]
+        self.projections = None if any(p is None for p in projections) else projections
+        self.w_in = self.b_in = None
 
     # what the engine asks a mixer is answered by the side that it concerns
     def _first(self, method: str, *args):
@@ -85,8 +91,13 @@ class PairedMixers(Mixer):
         return t + [TensorDecl(name, (self.hidden,), "gain") for name in self.gain_names] if self.combine == "normed" else t
 
     def load(self, store, rt) -> None:
+        if self.projections is not None:
+            self.w_in, self.b_in = load_projections([p for side in self.projections for p in side], store, rt)
         for s in self.sides:
-            s.load(store, rt)
+            if self.projections is not None:
+                s.load(store, rt, own_input=False)
+            else:
+                s.load(store, rt)
         if self.combine == "normed":
             self.gains = [store.vector(name) for name in self.gain_names]
         else:
@@ -98,10 +109,15 @@ class PairedMixers(Mixer):
         return [OutputTerm(None, s) for s in self.scales]
 
     def forward_apart(self, ctx, binding: CacheBinding, h, outs) -> None:
-        at = 0
-        for side, out in zip(self.sides, outs):
+        at, parts = 0, [{}, {}]
+        if self.projections is not None:
+            left, right = (sum(rows for _, rows, _ in side) for side in self.projections)
+            rows = ctx.ws.take((h.shape[0], left + right), torch.float32)
+            ctx.rt.k.gemm(h, self.w_in, rows, self.b_in, MODE_STORE_F32)
+            parts = [{"rows": rows[:, :left]}, {"rows": rows[:, left:]}]
+        for side, out, ready in zip(self.sides, outs, parts):
             n = len(side.state_specs())
-            side.forward(ctx, binding.with_states(at, n), h, out, accumulate=False)
+            side.forward(ctx, binding.with_states(at, n), h, out, accumulate=False, **ready)
             at += n
 
     def forward(self, ctx, binding: CacheBinding, h, residual) -> None:

@@ -394,7 +394,7 @@ def weights_of(cfg, seed, ranks=None, scope="l0.mix."):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("h_n,dim,vdim", [(3, 5, 7), (2, 64, 32), (1, 132, 24), (4, 16, 16), (2, 256, 48), (8, 128, 128), (2, 48, 80),
-                                          (1, 1, 1), (3, 200, 9), (2, 112, 272)])
+                                          (1, 1, 1), (3, 200, 9), (2, 112, 272), (1, 8, 515)])
 def test_linear_attention_alone_in_portions(h_n, dim, vdim, dtype):
     """The walk (and, where the sizes allow, the chunks) with its state carried across cuts of every kind: whole, a token at a
     time from the first token on, portions down to one token.  Decays from none left to none lost."""
@@ -834,3 +834,18 @@ def test_wrong_shapes_are_refused():
         rt.k.heads_prepare(z(2, 24), 0, 1, 8, 1, 16, 8, 8, None, None, 0.0, 0, False, 1.0, z(2, 0, 2), i(2), i(2), i(1, 1),
                            z(1, 1, 8, 16), 8, z(2, 8), conv=(z(24, 3), z(1, 64), 32, None))      # a state too small for two rows of 24, twice
     build_part("mixer", PartSpec("lightning_attention", dict(hidden_size=8, heads=1, dim=4, vdim=4, decay=[0.5], eps=1e-5)))
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("m,n,k", [(3, 64, 64), (16, 40, 128), (40, 192, 256), (100, 130, 64), (300, 128, 2048), (700, 512, 4096), (33, 17, 30)])
+def test_a_product_whose_squared_relu_is_its_epilogue(m, n, k, dtype):
+    from axon_amd.kernels import MODE_RELU_SQUARED, MODE_STORE_F32
+    rt = Runtime(dtype)
+    g = torch.Generator().manual_seed(m)
+    x, w = torch.randn(m, k, generator=g).to(rt.dtype).cuda(), (torch.randn(n, k, generator=g) * k ** -0.5).to(rt.dtype).cuda()
+    for matrix in (rt.k.prepare_weight(w), w):
+        got = rt.k.gemm(x, matrix, torch.empty(m, n, dtype=rt.dtype, device="cuda"), None, MODE_RELU_SQUARED)
+        sums = rt.k.gemm(x, matrix, torch.empty(m, n, device="cuda"), None, MODE_STORE_F32)
+        assert torch.equal(got, (torch.relu(sums) ** 2).to(rt.dtype))          # of the unrounded sums, rounded once
+    want = torch.relu(x.double() @ w.double().T) ** 2
+    assert float((got.double() - want).abs().max()) <= (2e-5 if dtype == "float32" else 2e-2) * float(want.abs().max())
