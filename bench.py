@@ -203,7 +203,7 @@ def _bafavik_sizes(width, heads, kv_heads, state_heads, chunk, dense_ff):
         "left": att(heads, kv_heads, 128, 128, rot=rot), "right": {"heads": state_heads, "dim": 128, "vdim": 128, "decay": decay},
         "left_scale": 0.7, "right_scale": 0.7}}
     diff = {"type": "attention", "mixer": att(heads // 2, max(kv_heads // 2, 1), 64, 128, diff=0.3, mask={"size": chunk})}
-    return {"architecture": "Bafavik", "embedding": {"scale": 1.0, "bigram": {"buckets": 32003, "mul_prev": 8191, "mul_cur": 127}},
+    return {"architecture": "Bafavik", "embedding": {"scale": 1.0, "bigram": {"buckets": 32003, "mul_prev": 8191, "mul_cur": 131}},
             "layers": [dict(pair_2, mlp=mlp), dict(pair, mlp=mlp), dict(diff, mlp=mlp)], "loop": {"start": 0, "stop": 1, "times": 2},
             "residual_mult": 0.5, "logit_scale": 1.0, "norm": {"eps": 1e-6}, "vocab": 32000, "width": width}
 
